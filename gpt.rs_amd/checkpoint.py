@@ -168,6 +168,81 @@ class Checkpoint:
         self.close()
 
 
+class SafetensorsFolder:
+    """A model folder, `config.json` beside `model.safetensors`, with the read side of a `Checkpoint`.
+
+    A safetensors file is an 8-byte little-endian length, that many bytes of JSON (name -> dtype, shape, data_offsets) and
+    the data.  `layout` maps a parameter of the model to (tensor name, transpose): matrices are stored [out, in] there and
+    [in, out] in a model.  Entries carry the parameters' names and shapes."""
+
+    _TAG = {"F32": 0, "F16": 1, "BF16": 2, "I32": 3}
+
+    def __init__(self, path: str):
+        import os
+        try:
+            with open(os.path.join(path, "config.json"), "rb") as f:
+                cfg = json.loads(f.read().decode("utf-8"))
+        except (UnicodeDecodeError, json.JSONDecodeError) as e:
+            raise CheckpointError(f"config.json is not valid JSON: {e}") from e
+        if not isinstance(cfg, dict) or "architecture" not in cfg:
+            raise CheckpointError("config.json must be an object that names its `architecture`")
+        self.architecture, self.config, self.runtime = str(cfg["architecture"]), cfg, cfg.get("runtime")
+        self.entries: List[Entry] = []
+        self._by_name: Dict[str, Entry] = {}
+        self._layout: Dict[str, Tuple[str, bool]] = {}
+        self._file = open(os.path.join(path, "model.safetensors"), "rb")
+        try:
+            self._map = mmap.mmap(self._file.fileno(), 0, access=mmap.ACCESS_READ)
+            size = len(self._map)
+            head = _Cursor(self._map, 0, size, "header")
+            n = head.u64()
+            try:
+                index = json.loads(head.take(n).decode("utf-8"))
+            except (UnicodeDecodeError, json.JSONDecodeError) as e:
+                raise CheckpointError(f"safetensors header is not valid JSON: {e}") from e
+            self._tensors: Dict[str, Tuple[int, Tuple[int, ...], int, int]] = {}
+            for name, t in index.items():
+                if name == "__metadata__":
+                    continue
+                if t["dtype"] not in self._TAG:
+                    raise CheckpointError(f"tensor `{name}`: dtype {t['dtype']} is not supported")
+                tag, dims = self._TAG[t["dtype"]], tuple(int(d) for d in t["shape"])
+                a, b = (int(v) for v in t["data_offsets"])
+                count = int(np.prod(dims, dtype=np.int64)) if dims else 1
+                if b - a != count * _NP_OF_TAG[tag].itemsize or a < 0 or 8 + n + b > size:
+                    raise CheckpointError(f"tensor `{name}`: data range does not match its shape or the file")
+                self._tensors[name] = (tag, dims, 8 + n + a, b - a)
+        except Exception:
+            self.close()
+            raise
+
+    def bind_layout(self, layout: Mapping[str, Tuple[str, bool]]):
+        self.entries, self._by_name, self._layout = [], {}, dict(layout)
+        for param, (tensor, transpose) in layout.items():
+            if tensor not in self._tensors:
+                raise CheckpointError(f"tensor `{tensor}` not found in the model folder")
+            tag, dims, off, n = self._tensors[tensor]
+            e = Entry(param, 0, dims[::-1] if transpose else dims, tag, 0, off, n)
+            self.entries.append(e)
+            self._by_name[param] = e
+
+    entry = Checkpoint.entry
+    names = Checkpoint.names
+    __contains__ = Checkpoint.__contains__
+    __iter__ = Checkpoint.__iter__
+    close = Checkpoint.close
+    __enter__ = Checkpoint.__enter__
+    __exit__ = Checkpoint.__exit__
+
+    def array(self, name: str) -> np.ndarray:
+        """The parameter as a view of the file mapping (bf16 as 16-bit words), transposed where the layout says so."""
+        e = self.entry(name)
+        tensor, transpose = self._layout[name]
+        dims = self._tensors[tensor][1]
+        a = np.frombuffer(self._map, dtype=_NP_OF_TAG[e.dtype_tag], count=e.byte_len // _NP_OF_TAG[e.dtype_tag].itemsize, offset=e.offset).reshape(dims)
+        return a.T if transpose else a
+
+
 def _index_bytes(items, data_start: int) -> bytes:
     out = bytearray(struct.pack("<I", len(items)))
     rel = 0

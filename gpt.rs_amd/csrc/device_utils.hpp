@@ -23,6 +23,33 @@ __device__ __forceinline__ uint32_t pack_bf16x2(float lo, float hi) {
     return (uint32_t)f32_to_bf16(lo) | ((uint32_t)f32_to_bf16(hi) << 16);
 }
 
+// A gate / up pair of a feed-forward layer.  kind 0: silu(g) * u (ops/functional/activation.rs:141-162).  kind 1, the
+// clamped unit: g <- min(g, limit), u <- clamp(u, +-limit), g * sigmoid(alpha g) * (u + shift).
+__device__ __forceinline__ float glu_combine(float g, float u, int kind, float limit, float alpha, float shift) {
+    if (kind == 1) {
+        g = fminf(g, limit);
+        u = fminf(fmaxf(u, -limit), limit);
+        return (g / (1.0f + expf(g * -alpha))) * (u + shift);
+    }
+    return (g / (1.0f + expf(g * -1.0f))) * u;
+}
+__device__ __forceinline__ float silu_f32(float x) { return x / (1.0f + expf(-x)); }
+// log(1 + e^x) without overflow and without losing small values
+__device__ __forceinline__ float softplus_f32(float x) { return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x))); }
+
+// Loads / stores as f32 whatever the element type
+template <typename T> struct Elem;
+template <> struct Elem<float> {
+    static __device__ __forceinline__ float ld(const float* p, int64_t i) { return p[i]; }
+    static __device__ __forceinline__ void st(float* p, int64_t i, float v) { p[i] = v; }
+    static __device__ __forceinline__ float round(float v) { return v; }
+};
+template <> struct Elem<bf16_t> {
+    static __device__ __forceinline__ float ld(const bf16_t* p, int64_t i) { return bf16_to_f32(p[i]); }
+    static __device__ __forceinline__ void st(bf16_t* p, int64_t i, float v) { p[i] = f32_to_bf16(v); }
+    static __device__ __forceinline__ float round(float v) { return bf16_to_f32(f32_to_bf16(v)); }
+};
+
 // Sum over the 64 lanes of a wave, result in every lane.  Cross-lane moves use DPP modifiers
 // (register-to-register, VALU rate) instead of ds_bpermute: 16 x 6 bpermutes per thread at the end of
 // a GEMV block kept the LDS pipe busy for ~4 us.  Steps: xor 1 and xor 2 inside quads, mirrored

@@ -322,5 +322,71 @@ struct AttnConcatArgs {
 };
 void attn_concat(hipStream_t s, const AttnConcatArgs& a);
 
+// ---- sequence mixers (kernels_ssm.hip, kernels_latent.hip) ------------------------------------------------------------
+// dtype: 0 f32, 2 bf16, of the tensors called "T" below; everything else is f32.
+
+// cos | sin of positions[r] * freqs[i], times `magnitude`: out f32 [rows, 2 * half]
+void rope_table(hipStream_t s, const int32_t* positions, const float* freqs, float magnitude, float* out, int64_t rows, int64_t half);
+// rotates the pairs (offset + 2i, offset + 2i + 1), i < half, of every head of x T [rows, heads * head_dim]; the rest is copied
+void rope_pairs(hipStream_t s, int dtype, const void* x, const float* table, void* y, int64_t rows, int64_t heads, int64_t head_dim,
+                int64_t offset, int64_t half);
+// raw f32 [rows, rank + 2 * half] -> T: RMS norm with gains over the first `rank` values, pair rotation of the rest
+void latent_rows(hipStream_t s, int dtype, const float* raw, const float* gain, const float* table, void* y, int64_t rows, int64_t rank,
+                 int64_t half, float eps);
+
+// Latent attention over cached rows [latent: rank | rotated key part: rot] (one row per position, shared by all heads).
+// Query t (position start + t) sees rows 0 .. start + t.  Scores q_n . (W_uk c) + q_r . k_r are taken as
+// (W_uk^T q_n) . c + q_r . k_r and the values as W_uv (sum_j p_j c_j): the cache is read as it is.
+struct LatentAttnArgs {
+    int dtype;
+    const void* q;                 // T [t, heads * (dim + rot)], rotated
+    const void* rows;              // T [capacity, rank + rot]
+    const void* w_uk; const void* w_uv;   // T [rank, heads * dim], T [rank, heads * vdim]
+    const int32_t* start;          // si32[1]
+    void* ctx;                     // T [t, heads * vdim]
+    int64_t t, capacity, heads, dim, rot, rank, vdim;
+    float scale;
+};
+void latent_attn(hipStream_t s, const LatentAttnArgs& a);
+// The same with keys and values spelled out per head, k T [l, heads * dim], v T [l, heads * vdim] and the shared part read
+// from rows T [l, ld_rows] at column rank; query t sees keys 0 .. l - t_rows + t.
+struct LatentAttnXArgs {
+    int dtype;
+    const void* q; const void* k; const void* v; const void* rows;
+    void* ctx;
+    int64_t t, l, heads, dim, rot, rank, vdim;
+    float scale;
+};
+void latent_attn_expanded(hipStream_t s, const LatentAttnXArgs& a);
+
+// Depthwise causal convolution with bias and silu over `ch` columns of p f32 [rows, ld] from column `col`; taps f32
+// [taps, ch] (last row meets the current token), state f32 [taps - 1, ch]: the inputs before the first row.  y T [rows, ch].
+struct ConvArgs {
+    int dtype;
+    const float* p; const float* taps; const float* bias; const float* state;
+    void* y;
+    int64_t rows, ld, col, ch, ntaps;
+};
+void conv_silu(hipStream_t s, const ConvArgs& a);
+// the last taps - 1 inputs after `rows` more rows; state_out may be state
+void conv_state(hipStream_t s, const float* p, const float* state, float* state_out, int64_t rows, int64_t ld, int64_t col, int64_t ch, int64_t ntaps);
+
+// Mamba-2 recurrence, head h of group h / (heads / groups): dt = softplus(p[t, dt_col + h] + dt_bias[h]),
+// S <- exp(-exp(A_log[h]) dt) S + dt B x^T, y = S^T C + D[h] x.  xbc T [rows, heads * vdim + 2 groups * n] = x | B | C.
+// y null: only the state; state_out null: only the rows.  state_out may be state.
+struct SsmArgs {
+    int dtype;
+    const void* xbc; const float* p; const float* dt_bias; const float* a_log; const float* d;
+    const float* state; float* state_out; void* y;
+    int64_t rows, ld, dt_col, heads, groups, n, vdim;
+};
+void ssm_scan(hipStream_t s, const SsmArgs& a);
+// y T [rows, n] = rms-normed in `groups` equal parts of (y * silu(p[:, col ..])), times gain[n]
+void gated_rms_norm(hipStream_t s, int dtype, const void* y, const float* p, const float* gain, void* out, int64_t rows, int64_t n, int64_t ld,
+                    int64_t col, int64_t groups, float eps);
+// How a gate / up pair is combined (see glu_combine in device_utils.hpp)
+struct GluParams { int kind = 0; float limit = 0.f, alpha = 1.f, shift = 0.f; };
+void clamped_glu(hipStream_t s, int dtype, const void* gate, const void* up, void* y, int64_t n, const GluParams& p);
+
 }  // namespace k
 }  // namespace gptrs

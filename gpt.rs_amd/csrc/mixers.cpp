@@ -1,0 +1,293 @@
+// Sequence-mixer CustomCall targets of this backend (build-defined; the reference has no counterpart): validation, launch
+// descriptors and launches.  Operands per target (T: f32 or bf16, the model's dtype; everything else f32 unless said):
+//
+//   rope_table(positions si32[R], freqs[half]) {magnitude}                              -> [R, 2 half]   cos | sin
+//   rope_pairs(x T[R, heads * hd], table[R, 2 half]) {heads, offset}                    -> T, x's shape
+//   latent_rows(raw[R, rank + 2 half], gain[rank], table) {eps}                         -> T[R, rank + 2 half]
+//   latent_attention(q T[R, heads * (dim + rot)], cache T[1, C, rank + rot], w_uk T[rank, heads * dim],
+//                    w_uv T[rank, heads * vdim], start si32[1]) {heads, rot, scale}      -> T[R, heads * vdim]
+//   latent_attention_expanded(q T[R, ..], k T[L, heads * dim], v T[L, heads * vdim], rows T[L, rank + rot])
+//                    {heads, rot, scale}                                                -> T[R, heads * vdim]
+//   causal_conv_silu(p[R, W], taps[K, ch], bias[ch], state[K - 1, ch]) {col}            -> T[R, ch]
+//   causal_conv_state(p, state) {col}                                                   -> state's shape
+//   ssm_scan(xbc T[R, ch], p, dt_bias[H], a_log[H], d[H], state[H, N, V]) {groups, dt_col} -> T[R, H * V]
+//   ssm_state(xbc, p, dt_bias, a_log, state) {groups, dt_col}                           -> state's shape
+//   gated_rms_norm(y T[R, n], p[R, W], gain[n]) {groups, col, eps}                      -> T[R, n]
+//   clamped_glu(gate T, up T) {limit, alpha, shift}                                     -> T, gate's shape
+//
+// latent_attention: query i stands at position start + i.  latent_attention_expanded: the queries are the last R of the L
+// positions.  p is the f32 result of an input projection whose columns hold several inputs of the mixer.
+#include <cmath>
+#include <cstring>
+
+#include "runtime.hpp"
+
+namespace gptrs {
+
+namespace {
+const Json* attr(const Instr& in, const char* name) {
+    auto it = in.attrs.find(name);
+    return it == in.attrs.end() ? nullptr : it->second.find("value");
+}
+int64_t attr_int(const Instr& in, const char* name) {
+    const Json* v = attr(in, name);
+    try {
+        if (v) return v->as_int();
+    } catch (const JsonError&) {
+    }
+    fail_spec(in.target + ": attribute `" + name + "` (I64) is missing");
+}
+float attr_float(const Instr& in, const char* name) {
+    const Json* v = attr(in, name);
+    try {
+        if (v) {
+            const double d = v->as_double();
+            if (std::isfinite(d)) return (float)d;
+        }
+    } catch (const JsonError&) {
+    }
+    fail_spec(in.target + ": attribute `" + name + "` (F64) is missing or not finite");
+}
+}  // namespace
+
+void lower_mixer_calls(Function& fn) {
+    bool any = false;
+    for (const Instr& in : fn.body) any = any || (in.op == OpKind::CustomCall && mixer_call_target(in.target) != Mix::None);
+    if (!any) return;
+    std::vector<const Spec*> spec(fn.max_value_id + 1, nullptr);
+    for (size_t i = 0; i < fn.param_ids.size(); ++i) spec[fn.param_ids[i]] = &fn.param_specs[i];
+    for (const Instr& in : fn.body)
+        for (size_t o = 0; o < in.out_ids.size(); ++o) spec[in.out_ids[o]] = &in.out_specs[o];
+
+    for (Instr& in : fn.body) {
+        if (in.op != OpKind::CustomCall) continue;
+        const Mix mix = mixer_call_target(in.target);
+        if (mix == Mix::None) continue;
+        auto need = [&](bool ok, const char* what) { if (!ok) fail_spec(in.target + ": " + what); };
+        static const std::map<Mix, size_t> kArity = {{Mix::RopeTable, 2}, {Mix::RopePairs, 2}, {Mix::LatentRows, 3}, {Mix::LatentAttn, 5},
+                                                     {Mix::LatentAttnX, 4}, {Mix::ConvSilu, 4}, {Mix::ConvState, 2}, {Mix::SsmScan, 6},
+                                                     {Mix::SsmState, 5}, {Mix::GatedNorm, 3}, {Mix::Glu, 2}};
+        need(in.operands.size() == kArity.at(mix), "wrong number of operands");
+        std::vector<const Spec*> s;
+        for (const Operand& o : in.operands) {
+            need(o.value >= 0 && o.value <= fn.max_value_id && spec[o.value], "operands must be values");
+            s.push_back(spec[o.value]);
+        }
+        const Spec& out = in.out_specs[0];
+        auto is = [](const Spec& x, DType d, std::vector<int64_t> dims) { return x.dtype == d && x.dims == dims; };
+        auto f32 = [&](const Spec& x, std::vector<int64_t> dims) { return is(x, DType::F32, std::move(dims)); };
+        auto rows2 = [&](const Spec& x) { return x.rank() == 2 && x.dims[0] >= 1 && x.dims[1] >= 1; };
+        Instr::MixAttrs& m = in.mx;
+        switch (mix) {
+            case Mix::RopeTable:
+                need(s[0]->dtype == DType::SI32 && s[0]->rank() == 1, "positions must be si32[R]");
+                need(s[1]->rank() == 1 && f32(*s[1], s[1]->dims), "freqs must be f32[half]");
+                need(f32(out, {s[0]->dims[0], 2 * s[1]->dims[0]}), "output must be f32[R, 2 half]");
+                in.scale = attr_float(in, "magnitude");
+                break;
+            case Mix::RopePairs: {
+                m.heads = attr_int(in, "heads");
+                m.col = attr_int(in, "offset");
+                need(rows2(*s[0]) && dtype_is_float(s[0]->dtype) && out == *s[0], "x must be a float matrix, the output has its type");
+                need(m.heads > 0 && s[0]->dims[1] % m.heads == 0, "row length must be heads * head_dim");
+                m.dim = s[0]->dims[1] / m.heads;
+                need(s[1]->rank() == 2 && f32(*s[1], {s[0]->dims[0], s[1]->dims[1]}) && s[1]->dims[1] % 2 == 0, "table must be f32[R, 2 half]");
+                m.rot = s[1]->dims[1];
+                need(m.dim % 2 == 0 && m.col % 2 == 0 && m.col >= 0 && m.col + m.rot <= m.dim, "the rotated part must lie in the head, at even places");
+                break;
+            }
+            case Mix::LatentRows:
+                need(rows2(*s[0]) && f32(*s[0], s[0]->dims), "raw must be an f32 matrix");
+                need(s[1]->rank() == 1 && s[1]->dims[0] >= 1 && f32(*s[1], s[1]->dims), "gain must be f32[rank]");
+                m.rank = s[1]->dims[0];
+                m.rot = s[0]->dims[1] - m.rank;
+                need(m.rot >= 0 && m.rot % 2 == 0 && f32(*s[2], {s[0]->dims[0], m.rot}), "table must be f32[R, width - rank]");
+                need(dtype_is_float(out.dtype) && out.dims == s[0]->dims, "output must have raw's shape");
+                in.eps = attr_float(in, "eps");
+                break;
+            case Mix::LatentAttn:
+            case Mix::LatentAttnX: {
+                const bool x = mix == Mix::LatentAttnX;
+                m.heads = attr_int(in, "heads");
+                m.rot = attr_int(in, "rot");
+                in.scale = attr_float(in, "scale");
+                need(m.heads > 0 && m.rot >= 0 && m.rot % 2 == 0, "heads must be positive, rot even");
+                const DType dt = s[0]->dtype;
+                need(dtype_is_float(dt) && rows2(*s[0]), "q must be a float matrix");
+                const Spec& kk = *s[x ? 1 : 2];
+                const Spec& vv = *s[x ? 2 : 3];
+                need(rows2(kk) && rows2(vv) && kk.dtype == dt && vv.dtype == dt && kk.dims[0] == vv.dims[0], "key / value operands must be matrices of q's dtype");
+                need(kk.dims[1] % m.heads == 0 && vv.dims[1] % m.heads == 0, "key / value widths must be multiples of heads");
+                m.dim = kk.dims[1] / m.heads;
+                m.vdim = vv.dims[1] / m.heads;
+                need(s[0]->dims[1] == m.heads * (m.dim + m.rot), "q must be [R, heads * (dim + rot)]");
+                const Spec& rr = *s[x ? 3 : 1];
+                if (x) {
+                    need(rr.dtype == dt && rr.rank() == 2 && rr.dims[0] == kk.dims[0] && rr.dims[1] > m.rot, "rows must be T[L, rank + rot]");
+                    need(kk.dims[0] >= s[0]->dims[0], "at least as many keys as queries");
+                    m.rank = rr.dims[1] - m.rot;
+                } else {
+                    m.rank = kk.dims[0];
+                    need(rr.dtype == dt && rr.rank() == 3 && rr.dims[0] == 1 && rr.dims[1] >= 1 && rr.dims[2] == m.rank + m.rot, "cache must be T[1, C, rank + rot]");
+                    need(is(*s[4], DType::SI32, {1}), "start must be si32[1]");
+                }
+                need(is(out, dt, {s[0]->dims[0], m.heads * m.vdim}), "output must be T[R, heads * vdim]");
+                break;
+            }
+            case Mix::ConvSilu:
+                m.col = attr_int(in, "col");
+                need(rows2(*s[0]) && f32(*s[0], s[0]->dims), "p must be an f32 matrix");
+                need(s[1]->rank() == 2 && s[1]->dims[0] >= 1 && f32(*s[1], s[1]->dims), "taps must be f32[K, ch]");
+                m.taps = s[1]->dims[0];
+                m.dim = s[1]->dims[1];
+                need(f32(*s[2], {m.dim}) && f32(*s[3], {m.taps - 1, m.dim}), "bias must be f32[ch], state f32[K - 1, ch]");
+                need(m.col >= 0 && m.col + m.dim <= s[0]->dims[1], "channels must lie in p's columns");
+                need(dtype_is_float(out.dtype) && out.dims == std::vector<int64_t>{s[0]->dims[0], m.dim}, "output must be T[R, ch]");
+                break;
+            case Mix::ConvState:
+                m.col = attr_int(in, "col");
+                need(rows2(*s[0]) && f32(*s[0], s[0]->dims) && s[1]->rank() == 2 && f32(*s[1], s[1]->dims), "p and state must be f32 matrices");
+                m.taps = s[1]->dims[0] + 1;
+                m.dim = s[1]->dims[1];
+                need(m.col >= 0 && m.col + m.dim <= s[0]->dims[1] && out == *s[1], "channels must lie in p's columns, the output has state's type");
+                break;
+            case Mix::SsmScan:
+            case Mix::SsmState: {
+                const bool scan = mix == Mix::SsmScan;
+                const Spec& st = *s[scan ? 5 : 4];
+                m.groups = attr_int(in, "groups");
+                m.dt_col = attr_int(in, "dt_col");
+                need(st.rank() == 3 && f32(st, st.dims), "state must be f32[H, N, V]");
+                m.heads = st.dims[0]; m.state = st.dims[1]; m.vdim = st.dims[2];
+                need(m.heads >= 1 && m.state >= 1 && m.vdim >= 1 && m.state <= 1024, "state sizes out of range");
+                need(m.groups >= 1 && m.heads % m.groups == 0, "heads must be a multiple of groups");
+                need(dtype_is_float(s[0]->dtype) && s[0]->rank() == 2 && s[0]->dims[0] >= 1 && s[0]->dims[1] == m.heads * m.vdim + 2 * m.groups * m.state,
+                     "xbc must be T[R, H * V + 2 groups * N]");
+                need(rows2(*s[1]) && f32(*s[1], {s[0]->dims[0], s[1]->dims[1]}) && m.dt_col >= 0 && m.dt_col + m.heads <= s[1]->dims[1], "step sizes must lie in p's columns");
+                for (size_t i = 2; i < (scan ? 5u : 4u); ++i) need(f32(*s[i], {m.heads}), "per-head vectors must be f32[H]");
+                if (scan) need(is(out, s[0]->dtype, {s[0]->dims[0], m.heads * m.vdim}), "output must be T[R, H * V]");
+                else need(out == st, "the output has state's type");
+                break;
+            }
+            case Mix::GatedNorm:
+                m.groups = attr_int(in, "groups");
+                m.col = attr_int(in, "col");
+                in.eps = attr_float(in, "eps");
+                need(rows2(*s[0]) && dtype_is_float(s[0]->dtype) && out == *s[0], "y must be a float matrix, the output has its type");
+                m.dim = s[0]->dims[1];
+                need(m.groups >= 1 && m.dim % m.groups == 0, "row length must be a multiple of groups");
+                need(s[1]->rank() == 2 && f32(*s[1], {s[0]->dims[0], s[1]->dims[1]}) && m.col >= 0 && m.col + m.dim <= s[1]->dims[1], "the gate must lie in p's columns");
+                need(f32(*s[2], {m.dim}), "gain must be f32[n]");
+                break;
+            case Mix::Glu:
+                need(*s[0] == *s[1] && *s[0] == out && dtype_is_float(out.dtype), "gate, up and output must be of one float type");
+                in.fparam[0] = attr_float(in, "limit");
+                in.fparam[1] = attr_float(in, "alpha");
+                in.fparam[2] = attr_float(in, "shift");
+                break;
+            default:
+                fail_spec(in.target + ": not a call target");
+        }
+        in.op = OpKind::FMixer;
+        in.mix = mix;
+        in.op_name = "mixer." + in.target.substr(strlen("gpt_rs.hip."));
+    }
+}
+
+size_t mixer_scratch_bytes(const Instr& in, const std::vector<const Spec*>& operands) {
+    (void)in; (void)operands;
+    return 0;
+}
+
+std::vector<std::pair<int, int>> mixer_inplace_pairs(const Instr& in) {
+    (void)in;
+    return {};
+}
+
+void run_mixer(const Plan& plan, const Step& st, ExecCtx& cx) {
+    const Instr& in = st.in;
+    const Instr::MixAttrs& m = in.mx;
+    const Spec& out = in.out_specs[0];
+    hipStream_t s = cx.stream;
+    auto ptr = [&](size_t i) -> const void* { return cx.ptr[st.src[i]]; };
+    auto f = [&](size_t i) { return (const float*)ptr(i); };
+    auto spec = [&](size_t i) -> const Spec& { return plan.values[st.src[i]].spec; };
+    void* dst = cx.ptr[st.dst[0]];
+    const int dt = (int)out.dtype;
+    switch (in.mix) {
+        case Mix::RopeTable:
+            k::rope_table(s, (const int32_t*)ptr(0), f(1), in.scale, (float*)dst, out.dims[0], out.dims[1] / 2);
+            ++cx.launches;
+            break;
+        case Mix::RopePairs:
+            k::rope_pairs(s, dt, ptr(0), f(1), dst, out.dims[0], m.heads, m.dim, m.col, m.rot / 2);
+            ++cx.launches;
+            break;
+        case Mix::LatentRows:
+            k::latent_rows(s, dt, f(0), f(1), f(2), dst, out.dims[0], m.rank, m.rot / 2, in.eps);
+            ++cx.launches;
+            break;
+        case Mix::LatentAttn: {
+            k::LatentAttnArgs a{};
+            a.dtype = dt;
+            a.q = ptr(0); a.rows = ptr(1); a.w_uk = ptr(2); a.w_uv = ptr(3); a.start = (const int32_t*)ptr(4); a.ctx = dst;
+            a.t = out.dims[0]; a.capacity = spec(1).dims[1];
+            a.heads = m.heads; a.dim = m.dim; a.rot = m.rot; a.rank = m.rank; a.vdim = m.vdim; a.scale = in.scale;
+            k::latent_attn(s, a);
+            ++cx.launches;
+            break;
+        }
+        case Mix::LatentAttnX: {
+            k::LatentAttnXArgs a{};
+            a.dtype = dt;
+            a.q = ptr(0); a.k = ptr(1); a.v = ptr(2); a.rows = ptr(3); a.ctx = dst;
+            a.t = out.dims[0]; a.l = spec(1).dims[0];
+            a.heads = m.heads; a.dim = m.dim; a.rot = m.rot; a.rank = m.rank; a.vdim = m.vdim; a.scale = in.scale;
+            k::latent_attn_expanded(s, a);
+            ++cx.launches;
+            break;
+        }
+        case Mix::ConvSilu: {
+            k::ConvArgs a{};
+            a.dtype = dt;
+            a.p = f(0); a.taps = f(1); a.bias = f(2); a.state = f(3); a.y = dst;
+            a.rows = out.dims[0]; a.ld = spec(0).dims[1]; a.col = m.col; a.ch = m.dim; a.ntaps = m.taps;
+            k::conv_silu(s, a);
+            ++cx.launches;
+            break;
+        }
+        case Mix::ConvState:
+            k::conv_state(s, f(0), f(1), (float*)dst, spec(0).dims[0], spec(0).dims[1], m.col, m.dim, m.taps);
+            ++cx.launches;
+            break;
+        case Mix::SsmScan:
+        case Mix::SsmState: {
+            const bool scan = in.mix == Mix::SsmScan;
+            k::SsmArgs a{};
+            a.dtype = (int)spec(0).dtype;
+            a.xbc = ptr(0); a.p = f(1); a.dt_bias = f(2); a.a_log = f(3);
+            if (scan) { a.d = f(4); a.state = f(5); a.y = dst; }
+            else { a.state = f(4); a.state_out = (float*)dst; }
+            a.rows = spec(0).dims[0]; a.ld = spec(1).dims[1]; a.dt_col = m.dt_col;
+            a.heads = m.heads; a.groups = m.groups; a.n = m.state; a.vdim = m.vdim;
+            k::ssm_scan(s, a);
+            ++cx.launches;
+            break;
+        }
+        case Mix::GatedNorm:
+            k::gated_rms_norm(s, dt, ptr(0), f(1), f(2), dst, out.dims[0], m.dim, spec(1).dims[1], m.col, m.groups, in.eps);
+            ++cx.launches;
+            break;
+        case Mix::Glu: {
+            k::GluParams p;
+            p.kind = 1; p.limit = in.fparam[0]; p.alpha = in.fparam[1]; p.shift = in.fparam[2];
+            k::clamped_glu(s, dt, ptr(0), ptr(1), dst, out.count(), p);
+            ++cx.launches;
+            break;
+        }
+        default:
+            fail_unimpl(in.op_name, "no kernel bound to this operation");
+    }
+}
+
+}  // namespace gptrs

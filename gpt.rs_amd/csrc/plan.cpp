@@ -595,6 +595,12 @@ void Builder::describe(Step& st) {
                                         k::chain_attn_part_bytes(in.n_q, in.n_kv, in.head_dim)) * (size_t)std::max<int64_t>(in.batch, 1);
             break;
         }
+        case OpKind::FMixer: {
+            std::vector<const Spec*> ops;
+            for (size_t i = 0; i < in.operands.size(); ++i) ops.push_back(&spec_of(in, i));
+            st.scratch_bytes = mixer_scratch_bytes(in, ops);
+            break;
+        }
         default:
             break;
     }
@@ -704,6 +710,7 @@ void Builder::build() {
                 pairs.push_back({(int)attn_cache_operand(st.in, b), (int)attn_cache_output(b)});
                 pairs.push_back({(int)attn_cache_operand(st.in, b) + 1, (int)attn_cache_output(b) + 1});
             }
+        if (st.in.op == OpKind::FMixer) pairs = mixer_inplace_pairs(st.in);
         bool all_inplace = !pairs.empty();
         for (auto& pr : pairs) {
             const int bv = st.src[pr.first];
@@ -1413,6 +1420,9 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
             cx.launches += 2;
             break;
         }
+        case OpKind::FMixer:
+            run_mixer(plan, st, cx);
+            break;
         default:
             fail_unimpl(in.op_name, "no kernel bound to this operation");
     }

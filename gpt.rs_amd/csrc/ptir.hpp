@@ -72,7 +72,14 @@ enum class OpKind {
     // fused forms produced by the executor's pattern pass (never present on the wire)
     FLayerNorm, FRmsNorm, FSoftmax, FGelu, FSilu, FSwiglu, FLinear, FRope, FAttnDecode, FAttnPrefill, FAttnConcat,
     FEmbed, FQuant,
+    FMixer,   // sequence-mixer targets (mixers.cpp): `Instr::mix` says which
     Unsupported
+};
+// What an FMixer instruction computes.  The first block are CustomCall targets (mixer_call_target); the last three are
+// formed by the fusion pass from those and serve every sequence of a batch.
+enum class Mix {
+    None, RopeTable, RopePairs, LatentRows, LatentAttn, LatentAttnX, ConvSilu, ConvState, SsmScan, SsmState, GatedNorm, Glu,
+    SsmSeq, LatentDecode, LatentPrefill
 };
 enum class UnaryOp { Neg, Abs, Exp, Log, Tanh, Erf, Rsqrt, Reciprocal };
 enum class BinaryOp { Add, Sub, Mul, Div, Maximum, Minimum };
@@ -133,6 +140,18 @@ struct Instr {
     // weight operand is then a (codes, scales) pair: (x, q, s, [q2, s2], [bias], [residual], [gamma]).
     // FQuant: 1 int8 scales, 2 int8 codes, 3 int4 scales, 4 int4 codes, 5 int8 dequantise, 6 int4 dequantise
     int quant = 0;
+    // FLinear with act = 2: how the pair is combined.  0: silu(gate) * up; 1: the clamped unit (CustomCall
+    // gpt_rs.hip.clamped_glu.v1) with fparam = {limit, alpha, shift}
+    int glu = 0;
+    // FLinear: every output column is multiplied by an f32 factor (operand behind the bias, ahead of the residual)
+    bool has_scale = false;
+    // FMixer: attributes of the call (only those of `mix` are meaningful)
+    Mix mix = Mix::None;
+    struct MixAttrs {
+        int64_t heads = 0, groups = 0, state = 0, vdim = 0, dim = 0, rot = 0, rank = 0, taps = 0, col = 0, dt_col = 0, z_col = 0;
+    } mx;
+    std::vector<int64_t> lens;               // FMixer over a batch: rows of each sequence, in order
+    bool append = false;                     // Mix::LatentDecode: the step's cache rows are written by the call itself
     bool scalar_rhs = false;                 // Binary whose rhs is a broadcast scalar literal
     float scalar_val = 0.f;
 };
@@ -158,6 +177,19 @@ inline int norm_call_target(const std::string& t) {
     if (t == "gpt_rs.hip.layer_norm.v1") return 1;
     if (t == "gpt_rs.hip.rms_norm.v1") return 2;
     return 0;
+}
+// CustomCall targets of the sequence mixers and of what goes with them (build-defined; operands in mixers.cpp)
+inline Mix mixer_call_target(const std::string& t) {
+    static const std::pair<const char*, Mix> kTargets[] = {
+        {"gpt_rs.hip.rope_table.v1", Mix::RopeTable}, {"gpt_rs.hip.rope_pairs.v1", Mix::RopePairs},
+        {"gpt_rs.hip.latent_rows.v1", Mix::LatentRows}, {"gpt_rs.hip.latent_attention.v1", Mix::LatentAttn},
+        {"gpt_rs.hip.latent_attention_expanded.v1", Mix::LatentAttnX}, {"gpt_rs.hip.causal_conv_silu.v1", Mix::ConvSilu},
+        {"gpt_rs.hip.causal_conv_state.v1", Mix::ConvState}, {"gpt_rs.hip.ssm_scan.v1", Mix::SsmScan},
+        {"gpt_rs.hip.ssm_state.v1", Mix::SsmState}, {"gpt_rs.hip.gated_rms_norm.v1", Mix::GatedNorm},
+        {"gpt_rs.hip.clamped_glu.v1", Mix::Glu}};
+    for (auto& e : kTargets)
+        if (t == e.first) return e.second;
+    return Mix::None;
 }
 inline int quant_op_target(const std::string& t) {
     if (t == "gpt_rs.hip.quantize_w8_scales.v1") return 1;

@@ -323,6 +323,16 @@ void collapse_broadcast_inputs(Function& fn, const std::vector<BroadcastInput>& 
 // would have formed from the functional's own sequence; their operands are validated here.  Runs on every program,
 // fusion on or off: the targets are part of what the backend executes.
 void lower_norm_calls(Function& fn);
+// mixers.cpp: the sequence-mixer CustomCall targets (mixer_call_target) become FMixer instructions; operands and attributes
+// are validated here.  Runs on every program, fusion on or off.
+void lower_mixer_calls(Function& fn);
+// mixers.cpp: scratch of one launch, and the launch itself.  mixer_inplace_pairs: (operand slot, output slot) of the state
+// that the call may update in place when the caller donates it.
+size_t mixer_scratch_bytes(const Instr& in, const std::vector<const Spec*>& operands);
+std::vector<std::pair<int, int>> mixer_inplace_pairs(const Instr& in);
+struct Plan;
+struct Step;
+void run_mixer(const Plan& plan, const Step& st, ExecCtx& cx);
 // fuse.cpp: the input position whose contents, broadcast along leading axes, are result `r` of the function as written
 // (a chain of BroadcastTo / Reshape instructions that keep the last axis), or -1.
 int result_broadcast_source(const Function& fn, size_t r);

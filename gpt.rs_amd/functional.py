@@ -457,3 +457,92 @@ def dynamic_update_slice_into(base: Tensor, update: Tensor, starts: Tensor) -> T
     if len(update.dims) != len(base.dims) or any(u > b for u, b in zip(update.dims, base.dims)):
         raise ValueError("dynamic_update_slice_into update exceeds base")
     return base.dynamic_update_slice(update, starts, list(update.dims))
+
+
+# --------------------------------------------------------------------------- sequence mixers
+# CustomCall targets of this backend for mixers the reference has no functional for (selective state spaces, latent
+# attention).  Each call has one result, as every PTIR instruction; the backend's fusion pass puts the calls of a layer and of
+# a batch together (csrc/fuse.cpp), csrc/mixers.cpp states operands and attributes.
+def _attrs(**kw) -> dict:
+    return {k: ({"kind": "I64", "value": int(v)} if isinstance(v, (int, np.integer)) else {"kind": "F64", "value": float(v)}) for k, v in kw.items()}
+
+
+def scale_columns(x: Tensor, scale: Tensor) -> Tensor:
+    """x[T, N] times one factor per column."""
+    return x * scale.broadcast_to(x.dims)
+
+
+def clamped_glu(gate: Tensor, up: Tensor, limit: float, alpha: float = 1.702, shift: float = 1.0) -> Tensor:
+    """g * sigmoid(alpha g) * (u + shift) with g = min(gate, limit) and u = clamp(up, -limit, limit)."""
+    if gate.spec != up.spec:
+        raise ValueError("clamped_glu gate/up spec mismatch")
+    return gate.fb.custom_call("gpt_rs.hip.clamped_glu.v1", [gate, up], gate.spec, _attrs(limit=float(limit), alpha=float(alpha), shift=float(shift)))
+
+
+def yarn_pair_frequencies(dims: int, base: float, factor: float, original: float, fast: float, slow: float) -> Tuple[np.ndarray, float]:
+    """(frequencies [dims / 2], magnitude) of a YaRN-scaled rotation whose ramp is at least 0.001 wide.  Unlike
+    `_yarn_inv_freqs`, which restates the reference's f32 arithmetic and its own ramp rule, in f64 and rounded once."""
+    i = np.arange(dims // 2, dtype=np.float64)
+    f = float(base) ** (-2.0 * i / dims)
+
+    def dim_of(turns):
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    lo, hi = max(math.floor(dim_of(fast)), 0), min(math.ceil(dim_of(slow)), dims - 1)
+    ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return (f / factor * ramp + f * (1.0 - ramp)).astype(np.float32), 0.1 * math.log(factor) + 1.0
+
+
+def pair_frequencies(dims: int, base: float) -> np.ndarray:
+    """base^(-2i / dims), i < dims / 2."""
+    return (float(base) ** (-2.0 * np.arange(dims // 2, dtype=np.float64) / dims)).astype(np.float32)
+
+
+def rope_table(positions: Tensor, freqs: Tensor, magnitude: float = 1.0) -> Tensor:
+    """f32 [R, 2 half]: magnitude * cos | magnitude * sin of positions[r] * freqs[i], computed on the device."""
+    return positions.fb.custom_call("gpt_rs.hip.rope_table.v1", [positions, freqs], TensorSpec("F32", (positions.dims[0], 2 * freqs.dims[0])),
+                                    _attrs(magnitude=float(magnitude)))
+
+
+def rope_pairs(x: Tensor, table: Tensor, heads: int, offset: int) -> Tensor:
+    """Interleaved rotation: in every head of x[R, heads * hd] the dimensions (offset + 2i, offset + 2i + 1) turn by angle i of
+    the row's table entry; the others pass."""
+    return x.fb.custom_call("gpt_rs.hip.rope_pairs.v1", [x, table], x.spec, _attrs(heads=heads, offset=offset))
+
+
+def latent_rows(raw: Tensor, gain: Tensor, table: Tensor, eps: float, dtype: str) -> Tensor:
+    """[rms-normed latent | rotated key part] of raw f32 [R, rank + rot]: what a latent-attention cache holds per position."""
+    return raw.fb.custom_call("gpt_rs.hip.latent_rows.v1", [raw, gain, table], TensorSpec(dtype, raw.dims), _attrs(eps=float(eps)))
+
+
+def latent_attention(q: Tensor, cache: Tensor, w_uk: Tensor, w_uv: Tensor, start: Tensor, heads: int, rot: int, scale: float) -> Tensor:
+    """Causal attention of rotated queries at positions start, start + 1, .. over cached rows [1, C, rank + rot]."""
+    return q.fb.custom_call("gpt_rs.hip.latent_attention.v1", [q, cache, w_uk, w_uv, start], TensorSpec(q.dtype, (q.dims[0], w_uv.dims[1])),
+                            _attrs(heads=heads, rot=rot, scale=float(scale)))
+
+
+def latent_attention_expanded(q: Tensor, k: Tensor, v: Tensor, rows: Tensor, heads: int, rot: int, scale: float) -> Tensor:
+    """The same for a prompt, with the unrotated keys k[L, heads * dim] and values v[L, heads * vdim] of all heads spelled out
+    and the shared rotated part read from rows[L, rank + rot]."""
+    return q.fb.custom_call("gpt_rs.hip.latent_attention_expanded.v1", [q, k, v, rows], TensorSpec(q.dtype, (q.dims[0], v.dims[1])),
+                            _attrs(heads=heads, rot=rot, scale=float(scale)))
+
+
+def causal_conv_silu(p: Tensor, taps: Tensor, bias: Tensor, state: Tensor, col: int, dtype: str) -> Tuple[Tensor, Tensor]:
+    """Depthwise causal convolution + silu over the channels p[:, col : col + ch] (f32), taps[K, ch]; `state` holds the K - 1
+    inputs before the first row.  Returns (rows [R, ch], the state after them)."""
+    y = p.fb.custom_call("gpt_rs.hip.causal_conv_silu.v1", [p, taps, bias, state], TensorSpec(dtype, (p.dims[0], taps.dims[1])), _attrs(col=col))
+    return y, p.fb.custom_call("gpt_rs.hip.causal_conv_state.v1", [p, state], state.spec, _attrs(col=col))
+
+
+def ssm_scan(xbc: Tensor, p: Tensor, dt_bias: Tensor, a_log: Tensor, d: Tensor, state: Tensor, groups: int, dt_col: int) -> Tuple[Tensor, Tensor]:
+    """Mamba-2 recurrence over x | B | C rows with the step sizes softplus(p[:, dt_col + h] + dt_bias[h]); state f32
+    [heads, N, V].  Returns (rows [R, heads * V], the state after them)."""
+    at = _attrs(groups=groups, dt_col=dt_col)
+    y = p.fb.custom_call("gpt_rs.hip.ssm_scan.v1", [xbc, p, dt_bias, a_log, d, state], TensorSpec(xbc.dtype, (xbc.dims[0], state.dims[0] * state.dims[2])), at)
+    return y, p.fb.custom_call("gpt_rs.hip.ssm_state.v1", [xbc, p, dt_bias, a_log, state], state.spec, at)
+
+
+def gated_rms_norm(y: Tensor, p: Tensor, gain: Tensor, groups: int, col: int, eps: float) -> Tensor:
+    """RMS norm of y * silu(p[:, col : col + n]) in `groups` equal parts, times gain."""
+    return y.fb.custom_call("gpt_rs.hip.gated_rms_norm.v1", [y, p, gain], y.spec, _attrs(groups=groups, col=col, eps=float(eps)))

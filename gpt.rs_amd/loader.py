@@ -19,12 +19,13 @@ well: streaming trades time for memory, as in the reference.
 """
 from __future__ import annotations
 
+import os
 from dataclasses import dataclass, field
 from typing import Callable, Dict, Iterable, List, Optional, Set
 
 import numpy as np
 
-from .checkpoint import Checkpoint, CheckpointError, Entry
+from .checkpoint import Checkpoint, CheckpointError, Entry, SafetensorsFolder
 from .ptir import TensorSpec, bf16_bits_to_f32, f32_to_bf16_bits
 
 
@@ -254,21 +255,38 @@ class CheckpointParamSource:
         return h
 
 
+def open_checkpoint(path: str):
+    """A GPTRSCHK file, or a model folder (config.json + model.safetensors)."""
+    from . import models
+    if not os.path.isdir(path):
+        return Checkpoint(path)
+    ck = SafetensorsFolder(path)
+    try:
+        ck.kind = models.KIND_OF_ARCHITECTURE.get(ck.architecture)
+        if ck.kind is None:
+            raise CheckpointError(f"unsupported architecture '{ck.architecture}'")
+        cls = models.MODEL_KINDS[ck.kind][0]
+        ck.bind_layout(cls.tensor_layout(cls.config_from_json(ck.config)))
+        return ck
+    except Exception:
+        ck.close()
+        raise
+
+
 def load_model(backend, path: str, dtype: Optional[str] = None, **model_kwargs):
     """loader.rs:238-306: open the checkpoint, read its kind, config and `runtime.weight_streaming`, build the model.
     Not streaming: every parameter is loaded once into the backend's memo.  Streaming: the model resolves every
-    parameter through the source at each forward.  The checkpoint stays open for the life of the model."""
+    parameter through the source at each forward.  The checkpoint stays open for the life of the model.  `path` may also
+    be a model folder (open_checkpoint)."""
     from . import models
-    ck = Checkpoint(path)
+    ck = open_checkpoint(path)
     try:
         ws = WeightStreamingConfig.from_runtime(ck.runtime)
         validate_weight_streaming_config(ws)
-        if ck.kind == "gpt":
-            model = models.Gpt(models.Gpt.config_from_json(ck.config), backend, dtype or "F32")
-        elif ck.kind == "ministral":
-            model = models.Ministral(models.Ministral.config_from_json(ck.config), backend, dtype or "Bf16", **model_kwargs)
-        else:
+        if ck.kind not in models.MODEL_KINDS:
             raise CheckpointError(f"unsupported model kind '{ck.kind}'")
+        cls, default_dtype = models.MODEL_KINDS[ck.kind]
+        model = cls(cls.config_from_json(ck.config), backend, dtype or default_dtype, **model_kwargs)
         expected = model.expected_params()
         for name, dims in expected.items():
             e = ck.entry(name)   # "missing tensor '<name>' in checkpoint"

@@ -43,6 +43,33 @@ class DecodeKvCache:
     capacity: int
 
 
+@dataclass
+class DecodeLatentCache:
+    """One row [latent | rotated key part] per position, shared by all heads: [1, capacity, rank + rot]."""
+
+    rows: object
+    len: int
+    capacity: int
+
+
+@dataclass
+class DecodeSsmState:
+    """What a state-space layer carries from token to token: the convolution's last inputs f32 [taps - 1, channels] and the
+    recurrent state f32 [heads, N, vdim].  Its size does not depend on the position."""
+
+    conv: object
+    state: object
+    len: int
+
+
+@dataclass
+class SharedLayerCache:
+    """A layer that reads the cache of layer `layer` and holds nothing itself."""
+
+    layer: int
+    len: int
+
+
 def _np_to_bytes(arr: np.ndarray, dtype: str) -> bytes:
     if dtype == "Bf16":
         return f32_to_bf16_bits(np.asarray(arr, np.float32)).astype("<u2").tobytes()
@@ -230,8 +257,23 @@ class _ModelBase:
         arr = np.asarray(values, dtype=np.int32)
         return self.backend.materialize(TensorSpec("Si32", arr.shape), arr.tobytes())
 
-    def _zeros(self, dims):
-        return self.backend.materialize(TensorSpec(self.dtype, dims), None)
+    def _zeros(self, dims, dtype: Optional[str] = None):
+        return self.backend.materialize(TensorSpec(dtype or self.dtype, dims), None)
+
+    def _grow_rows(self, handle, dims, capacity: int):
+        """A cache tensor of shape `dims` = [heads, old capacity, width] copied into a zero tensor of `capacity` rows
+        (model/gpt.rs:626-657)."""
+        heads, old_cap, width = dims
+        key = ("grow", heads, old_cap, width, capacity)
+        if key not in self._programs:
+            fb = FunctionBuilder("main", self.dtype)
+            base = fb.param(self.dtype, [heads, capacity, width])
+            old = fb.param(self.dtype, [heads, old_cap, width])
+            st = fb.param("Si32", [3])
+            fb.set_results([F.dynamic_update_slice_into(base, old, st)])
+            self._programs[key] = (Program(fb), {})
+        return self.backend.run_program(self._programs[key][0], [self._zeros([heads, capacity, width]), handle, self._upload_i32([0, 0, 0])],
+                                        [True, False, False])[0]
 
     def _run(self, program: Program, args: list, donate: Optional[list] = None):
         if self.front_end:
@@ -545,23 +587,10 @@ class Gpt(_ModelBase):
 
     def _grow_caches(self, caches, capacity: int):
         """model/gpt.rs:626-657: copy each layer's cache into a larger zero buffer."""
-        hkv, dh = self.attn.num_key_value_heads, self.attn.kv_head_dim
-        old_cap = caches[0][0].capacity
-        key = ("grow", old_cap, capacity)
-        if key not in self._programs:
-            fb = FunctionBuilder("main", self.dtype)
-            base = fb.param(self.dtype, [hkv, capacity, dh])
-            old = fb.param(self.dtype, [hkv, old_cap, dh])
-            st = fb.param("Si32", [3])
-            fb.set_results([F.dynamic_update_slice_into(base, old, st)])
-            self._programs[key] = (Program(fb), {})
-        prog = self._programs[key][0]
-        st = self._upload_i32([0, 0, 0])
+        dims = (self.attn.num_key_value_heads, caches[0][0].capacity, self.attn.kv_head_dim)
         for c in caches:
             for i, slot in enumerate(c):
-                k = self.backend.run_program(prog, [self._zeros([hkv, capacity, dh]), slot.keys, st], [True, False, False])[0]
-                v = self.backend.run_program(prog, [self._zeros([hkv, capacity, dh]), slot.values, st], [True, False, False])[0]
-                c[i] = DecodeKvCache(k, v, slot.len, capacity)
+                c[i] = DecodeKvCache(self._grow_rows(slot.keys, dims, capacity), self._grow_rows(slot.values, dims, capacity), slot.len, capacity)
 
 
 # ================================================================================ Ministral
@@ -889,9 +918,445 @@ class Ministral(_ModelBase):
         return outs[-1]
 
 
+# ================================================================================ Dadupel
+@dataclass
+class SsmMixerConfig:
+    """A Mamba-2 mixer (state-space duality)."""
+
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int
+
+    @property
+    def inner(self): return self.heads * self.vdim
+    @property
+    def channels(self): return self.inner + 2 * self.groups * self.state       # x | B | C
+    @property
+    def projection(self): return self.inner + self.channels + self.heads       # z | x | B | C | dt
+
+
+@dataclass
+class LatentMixerConfig:
+    """A latent-attention mixer.  `kv_from`: the layer whose cached rows it attends to (None: its own)."""
+
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rope_base: float
+    rope_scaling: Optional[Tuple[float, float, float, float]] = None   # YaRN: (factor, original, fast, slow)
+    kv_from: Optional[int] = None
+
+    @property
+    def row_width(self): return self.kv_rank + self.rot_dim
+
+    def frequencies(self) -> Tuple[np.ndarray, float]:
+        if self.rope_scaling is None:
+            return F.pair_frequencies(self.rot_dim, self.rope_base), 1.0
+        return F.yarn_pair_frequencies(self.rot_dim, self.rope_base, *self.rope_scaling)
+
+
+@dataclass
+class DadupelLayer:
+    mixer: object                     # SsmMixerConfig | LatentMixerConfig
+    ffn_dim: Optional[int] = None     # None: no feed-forward
+    glu_limit: float = 0.0
+
+
+@dataclass
+class DadupelConfig:
+    vocab_size: int
+    embed_dim: int
+    eps: float
+    layers: List[DadupelLayer]
+    context_length: int = 1 << 20     # the design states no limit; this one bounds the caches
+
+    @property
+    def num_layers(self): return len(self.layers)
+
+
+class Dadupel(_ModelBase):
+    """Hybrid decoder: Mamba-2 and latent-attention mixers in any order, each beside a clamped gated feed-forward under ONE
+    layer norm (x + scale_1 * mixer(h) + scale_2 * ff(h)), tied embedding and head.
+
+    The residual stream, the norms, the input projections of the mixers' f32 parts and the logits are f32; matmul operands
+    and the latent cache are in the model dtype; recurrent states are f32.  A batch may hold sequences of different lengths:
+    their rows are stacked without padding, the linear layers run over all of them, the mixers sequence by sequence (decode
+    steps: all sequences in one launch)."""
+
+    namespace = "dadupel"
+    ragged_batches = True
+
+    def __init__(self, config: DadupelConfig, backend, dtype: str = "Bf16", context_length: Optional[int] = None):
+        super().__init__(backend, dtype)
+        self.config = config
+        if context_length is not None:
+            config.context_length = int(context_length)
+        for i, L in enumerate(config.layers):
+            m = L.mixer
+            if isinstance(m, SsmMixerConfig):
+                if m.heads % m.groups or m.inner % m.norm_groups:
+                    raise ValueError(f"layer {i}: heads must be a multiple of groups, heads * vdim of norm_groups")
+            elif m.kv_from is not None:
+                src = config.layers[m.kv_from].mixer if 0 <= m.kv_from < i else None
+                if not isinstance(src, LatentMixerConfig) or src.kv_from is not None or (src.kv_rank, src.rot_dim) != (m.kv_rank, m.rot_dim):
+                    raise ValueError(f"layer {i}: kv_from must name an earlier latent-attention layer with a cache of the same sizes")
+
+    # -- configuration and parameters ---------------------------------------------------
+    @staticmethod
+    def config_from_json(c) -> DadupelConfig:
+        layers = []
+        for L in c["layers"]:
+            m = L["mixer"]
+            if L["type"] == "mamba2":
+                mixer = SsmMixerConfig(heads=int(m["heads"]), vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m["groups"]),
+                                       conv=int(m["conv"]), norm_groups=int(m["norm_groups"]))
+            elif L["type"] == "latent_attention":
+                rot, sc = m["rot"], m["rot"].get("scaling")
+                if int(rot["dims"]) != int(m["rot_dim"]):
+                    raise ValueError("latent attention rotates its whole rot_dim part: rot.dims must equal rot_dim")
+                mixer = LatentMixerConfig(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                                          q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), rope_base=float(rot["base"]),
+                                          rope_scaling=None if not sc else tuple(float(sc[k]) for k in ("factor", "original", "fast", "slow")),
+                                          kv_from=None if m.get("kv_from") is None else int(m["kv_from"]))
+            else:
+                raise ValueError(f"unknown layer type {L['type']!r}")
+            mlp = L.get("mlp")
+            if mlp is not None and mlp["kind"] != "dense":
+                raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+            layers.append(DadupelLayer(mixer, None if mlp is None else int(mlp["ff"]), 0.0 if mlp is None else float(mlp["limit"])))
+        return DadupelConfig(vocab_size=int(c["vocab"]), embed_dim=int(c["width"]), eps=float(c["norm"]["eps"]), layers=layers,
+                             context_length=int(c.get("context_length", 1 << 20)))
+
+    def checkpoint_config(self) -> Dict[str, object]:
+        c, layers = self.config, []
+        for L in c.layers:
+            m = L.mixer
+            if isinstance(m, SsmMixerConfig):
+                e = {"type": "mamba2", "mixer": dict(heads=m.heads, vdim=m.vdim, state=m.state, groups=m.groups, conv=m.conv, norm_groups=m.norm_groups)}
+            else:
+                rot = {"dims": m.rot_dim, "base": m.rope_base}
+                if m.rope_scaling is not None:
+                    rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), m.rope_scaling))
+                mix = dict(heads=m.heads, dim=m.dim, rot_dim=m.rot_dim, vdim=m.vdim, q_rank=m.q_rank, kv_rank=m.kv_rank, scale=m.scale, rot=rot)
+                if m.kv_from is not None:
+                    mix["kv_from"] = m.kv_from
+                e = {"type": "latent_attention", "mixer": mix}
+            e["mlp"] = None if L.ffn_dim is None else {"kind": "dense", "ff": L.ffn_dim, "limit": L.glu_limit}
+            layers.append(e)
+        return {"architecture": "Dadupel", "vocab": c.vocab_size, "width": c.embed_dim, "norm": {"eps": c.eps}, "layers": layers}
+
+    @staticmethod
+    def _param_plan(c: DadupelConfig) -> Dict[str, Tuple[tuple, str, bool]]:
+        """parameter -> (shape, tensor of a model folder, transposed there)."""
+        d = c.embed_dim
+        out = {"tok_embeddings.weight": ((c.vocab_size, d), "embed", False)}
+        for i, L in enumerate(c.layers):
+            p, t, m = f"blocks.{i}.", f"l{i}.", L.mixer
+            out[p + "norm_1.gamma"] = ((d,), t + "norm1", False)
+            out[p + "norm_1.beta"] = ((d,), t + "norm1.b", False)
+            q, u = p + "mixer.", t + "mix."
+            if isinstance(m, SsmMixerConfig):
+                out[q + "w_in"] = ((d, m.projection), u + "in", True)
+                out[q + "conv"] = ((m.conv, m.channels), u + "conv", True)
+                out[q + "conv_bias"] = ((m.channels,), u + "conv.b", False)
+                out[q + "dt_bias"] = ((m.heads,), u + "dt_bias", False)
+                out[q + "a_log"] = ((m.heads,), u + "A_log", False)
+                out[q + "d"] = ((m.heads,), u + "D", False)
+                out[q + "norm.gamma"] = ((m.inner,), u + "norm", False)
+                out[q + "w_out"] = ((m.inner, d), u + "o", True)
+            else:
+                out[q + "w_dq"] = ((d, m.q_rank), u + "dq", True)
+                out[q + "q_norm.gamma"] = ((m.q_rank,), u + "dq.norm", False)
+                out[q + "w_uq"] = ((m.q_rank, m.heads * (m.dim + m.rot_dim)), u + "uq", True)
+                if m.kv_from is None:
+                    out[q + "w_dkv"] = ((d, m.row_width), u + "dkv", True)
+                    out[q + "kv_norm.gamma"] = ((m.kv_rank,), u + "dkv.norm", False)
+                out[q + "w_uk"] = ((m.kv_rank, m.heads * m.dim), u + "uk", True)
+                out[q + "w_uv"] = ((m.kv_rank, m.heads * m.vdim), u + "uv", True)
+                out[q + "w_out"] = ((m.heads * m.vdim, d), u + "o", True)
+            out[p + "scale_1"] = ((d,), t + "ls1", False)
+            if L.ffn_dim is not None:
+                out[p + "feed_forward.w_gate"] = ((d, L.ffn_dim), t + "mlp.gate", True)
+                out[p + "feed_forward.w_up"] = ((d, L.ffn_dim), t + "mlp.up", True)
+                out[p + "feed_forward.w_down"] = ((L.ffn_dim, d), t + "mlp.down", True)
+                out[p + "scale_2"] = ((d,), t + "ls2", False)
+        out["final_norm.gamma"] = ((d,), "final.norm", False)
+        out["final_norm.beta"] = ((d,), "final.norm.b", False)
+        out["lm_head"] = ((d, c.vocab_size), "embed", True)     # the tied table once more, as a linear layer reads it
+        return out
+
+    def expected_params(self) -> Dict[str, tuple]:
+        return {n: e[0] for n, e in self._param_plan(self.config).items()}
+
+    @classmethod
+    def tensor_layout(cls, config: DadupelConfig) -> Dict[str, Tuple[str, bool]]:
+        return {n: (e[1], e[2]) for n, e in cls._param_plan(config).items()}
+
+    def param_dtype(self, name: str) -> str:
+        """Matrices that feed products are in the model dtype; gains, scales, taps and per-head constants are f32."""
+        leaf = name.rsplit(".", 1)[-1]
+        return self.dtype if leaf.startswith("w_") or leaf in ("weight", "lm_head") else "F32"
+
+    @classmethod
+    def random(cls, config: DadupelConfig, backend, seed: int = 0, dtype: str = "Bf16", context_length: Optional[int] = None) -> "Dadupel":
+        """Random weights of the right shapes and of sensible sizes, one numpy stream per tensor."""
+        m = cls(config, backend, dtype, context_length)
+        table = None
+        for idx, (name, dims) in enumerate(m.expected_params().items()):
+            rng = np.random.default_rng(np.random.SeedSequence([seed, idx]))
+            leaf = name.rsplit(".", 1)[-1]
+            if leaf == "lm_head":
+                arr = np.ascontiguousarray(table.T)
+            elif leaf == "dt_bias":
+                arr = np.log(np.expm1(np.exp(rng.uniform(np.log(1e-3), np.log(1e-1), dims)))).astype(np.float32)
+            elif leaf == "a_log":
+                arr = np.log(rng.uniform(1.0, 16.0, dims)).astype(np.float32)
+            elif leaf in ("gamma", "d"):
+                arr = (1.0 + 0.1 * rng.standard_normal(dims)).astype(np.float32)
+            elif leaf in ("beta", "conv_bias"):
+                arr = (0.1 * rng.standard_normal(dims)).astype(np.float32)
+            elif leaf in ("scale_1", "scale_2"):
+                arr = rng.uniform(0.3, 1.0, dims).astype(np.float32)
+            else:
+                arr = rng.standard_normal(dims, dtype=np.float32)
+                arr *= np.float32(1.0 if leaf == "weight" else dims[0] ** -0.5)
+            if leaf == "weight":
+                table = arr = bf16_bits_to_f32(f32_to_bf16_bits(arr * np.float32(dims[1] ** -0.5))) if dtype == "Bf16" else arr * np.float32(dims[1] ** -0.5)
+            m.set_param(name, arr, m.param_dtype(name))
+        return m
+
+    @property
+    def num_layers(self): return self.config.num_layers
+    @property
+    def context_length(self): return self.config.context_length
+
+    # -- graph pieces ----------------------------------------------------------------
+    def _norm(self, x: Tensor, P, name: str) -> Tensor:
+        """Layer norm of the f32 stream, handed on in the matmul dtype."""
+        out, *_ = F.layer_norm(x, P[name + ".gamma"], P[name + ".beta"], self.config.eps)
+        return out if self.dtype == "F32" else out.cast(self.dtype)
+
+    def _stack(self, parts: List[Tensor]) -> Tensor:
+        return parts[0] if len(parts) == 1 else Tensor.concat(0, parts)
+
+    def _ssm_mixer(self, P, p: str, m: SsmMixerConfig, proj: Tensor, lens, states):
+        """proj f32 [rows, z | x | B | C | dt] of all sequences; returns (rows in the matmul dtype, new (conv, state) per sequence)."""
+        ys, new, r0 = [], [], 0
+        dt_col = m.inner + m.channels
+        for n, (conv, state) in zip(lens, states):
+            pr = proj if len(lens) == 1 else proj.slice([r0, 0], [n, m.projection])
+            r0 += n
+            xbc, conv2 = F.causal_conv_silu(pr, P[p + "conv"], P[p + "conv_bias"], conv, m.inner, self.dtype)
+            y, state2 = F.ssm_scan(xbc, pr, P[p + "dt_bias"], P[p + "a_log"], P[p + "d"], state, m.groups, dt_col)
+            ys.append(y)
+            new.append((conv2, state2))
+        return F.gated_rms_norm(self._stack(ys), proj, P[p + "norm.gamma"], m.norm_groups, 0, self.config.eps), new
+
+    def _build(self, lens: Tuple[int, ...], capacity: int, decode: bool, last_only: bool = False, n_logit_rows: Optional[int] = None):
+        """One program for a forward of len(lens) sequences, sequence b bringing lens[b] rows (decode: one each).
+        last_only: the head runs on every sequence's last row; n_logit_rows: on that many rows, named by an argument."""
+        last_only = last_only and not decode
+        key = (lens, capacity, decode, last_only, n_logit_rows)
+        if key in self._programs:
+            return self._programs[key]
+        cfg, dt, B, rows = self.config, self.dtype, len(lens), sum(lens)
+        fb = FunctionBuilder("main", dt)
+        tok = fb.param("Si32", [rows])
+        pos = fb.param("Si32", [rows])
+        starts = fb.param("Si32", [3 * B])       # [0, position, 0] of every sequence: where its new cache rows go
+        layout = {"args": ["tokens", "positions", "starts"]}
+        pick = None
+        if n_logit_rows is not None:
+            pick = fb.param("Si32", [n_logit_rows])
+            layout["args"].append("logit_rows")
+        held = []                                # per sequence and layer: the tensors of its slot
+        for _ in range(B):
+            per = []
+            for L in cfg.layers:
+                m = L.mixer
+                if isinstance(m, SsmMixerConfig):
+                    per.append((fb.param("F32", [m.conv - 1, m.channels]), fb.param("F32", [m.heads, m.state, m.vdim])))
+                elif m.kv_from is None:
+                    per.append((fb.param(dt, [1, capacity, m.row_width]),))
+                else:
+                    per.append(())
+            held.append(per)
+        layout["n_args"] = len(fb.params)
+        P = self._declare_params(fb)
+        tables: Dict[tuple, Tensor] = {}
+        new_rows: Dict[int, Tensor] = {}
+
+        def table_of(m: LatentMixerConfig) -> Tensor:
+            f, mag = m.frequencies()
+            k = (f.tobytes(), mag)
+            if k not in tables:
+                tables[k] = F.rope_table(pos, fb.constant(TensorSpec("F32", f.shape), f.astype("<f4").tobytes()), mag)
+            return tables[k]
+
+        def part(t: Tensor, b: int) -> Tensor:   # the rows of sequence b
+            return t if B == 1 else t.slice([sum(lens[:b]), 0], [lens[b], t.dims[1]])
+
+        for L in cfg.layers:
+            if isinstance(L.mixer, LatentMixerConfig):
+                table_of(L.mixer)
+        hidden = F.embedding_lookup(P["tok_embeddings.weight"], tok)
+        if dt != "F32":
+            hidden = hidden.cast("F32")
+        new = [[()] * cfg.num_layers for _ in range(B)]
+        for i, L in enumerate(cfg.layers):
+            p, m = f"blocks.{i}.", L.mixer
+            q = p + "mixer."
+            h = self._norm(hidden, P, p + "norm_1")
+            ssm = isinstance(m, SsmMixerConfig)
+            # everything that reads the normed row comes first, so that a decode step's launches stay together
+            if ssm:
+                proj = F.linear(h, P[q + "w_in"], out_dtype="F32")
+            else:
+                cq = F.linear(h, P[q + "w_dq"], out_dtype="F32")
+                raw = F.linear(h, P[q + "w_dkv"], out_dtype="F32") if m.kv_from is None else None
+            act = None
+            if L.ffn_dim is not None:
+                f = p + "feed_forward."
+                act = F.clamped_glu(F.linear(h, P[f + "w_gate"]), F.linear(h, P[f + "w_up"]), L.glu_limit)
+            if ssm:
+                mixed, states = self._ssm_mixer(P, q, m, proj, lens, [held[b][i] for b in range(B)])
+                for b in range(B):
+                    new[b][i] = states[b]
+            else:
+                table, half = table_of(m), m.rot_dim // 2
+                cqn, *_ = F.rms_norm(cq, P[q + "q_norm.gamma"], cfg.eps)
+                qh = F.linear(cqn if dt == "F32" else cqn.cast(dt), P[q + "w_uq"])
+                qh = F.rope_pairs(qh, table, m.heads, m.dim)
+                src = i if m.kv_from is None else m.kv_from
+                if m.kv_from is None:
+                    new_rows[i] = F.latent_rows(raw, P[q + "kv_norm.gamma"], table, cfg.eps, dt)
+                    for b in range(B):
+                        upd = part(new_rows[i], b).reshape([1, lens[b], m.row_width])
+                        at = starts if B == 1 else starts.slice([3 * b], [3])
+                        new[b][i] = (F.dynamic_update_slice_into(held[b][i][0], upd, at),)
+                ctxs = []
+                if decode:
+                    for b in range(B):
+                        ctxs.append(F.latent_attention(part(qh, b), new[b][src][0], P[q + "w_uk"], P[q + "w_uv"], pos if B == 1 else pos.slice([b], [1]),
+                                                       m.heads, m.rot_dim, m.scale))
+                else:   # a prompt starts at its first token: its keys and values are the rows at hand
+                    lat = new_rows[src].slice([0, 0], [rows, m.kv_rank])
+                    kn, vv = F.linear(lat, P[q + "w_uk"]), F.linear(lat, P[q + "w_uv"])
+                    for b in range(B):
+                        ctxs.append(F.latent_attention_expanded(part(qh, b), part(kn, b), part(vv, b), part(new_rows[src], b), m.heads, m.rot_dim, m.scale))
+                mixed = self._stack(ctxs)
+            hidden = F.scale_columns(F.linear(mixed, P[q + "w_out"], out_dtype="F32"), P[p + "scale_1"]) + hidden
+            if act is not None:
+                hidden = F.scale_columns(F.linear(act, P[p + "feed_forward.w_down"], out_dtype="F32"), P[p + "scale_2"]) + hidden
+        if pick is not None:
+            hidden = hidden.take(pick)
+        elif last_only:
+            hidden = self._stack([hidden.slice([sum(lens[:b + 1]) - 1, 0], [1, cfg.embed_dim]) for b in range(B)])
+        logits = F.linear(self._norm(hidden, P, "final_norm"), P["lm_head"], out_dtype="F32")
+        fb.set_results([t for b in range(B) for slot in new[b] for t in slot] + [logits])
+        prog = Program(fb)
+        self._programs[key] = (prog, layout)
+        return prog, layout
+
+    # -- forward -----------------------------------------------------------------------
+    def forward_with_decode_cache(self, tokens, position_offset, caches, fixed_capacity=None, last_logits_only=False):
+        """See Gpt.forward_with_decode_cache."""
+        return self.forward_batch([list(tokens)], position_offset, [caches], fixed_capacity, last_logits_only=last_logits_only)
+
+    def forward_decode_device_token(self, token_handle, position_offset, caches, fixed_capacity=None):
+        """See Gpt.forward_decode_device_token."""
+        return self.forward_batch([[None]], position_offset, [caches], fixed_capacity, token_handle=token_handle)
+
+    def forward_batch(self, token_rows, position_offset, caches, fixed_capacity=None, token_handle=None, last_logits_only=False,
+                      logit_rows: Optional[Sequence[int]] = None):
+        """Independent sequences of any lengths.  `position_offset`: one for all or one per sequence.  The batch either starts
+        (empty caches, offset 0) or goes on by one token each; `caches[b]` is updated in place.  `logit_rows`: the stacked rows
+        whose logits are wanted (default: all, or each sequence's last with `last_logits_only`)."""
+        cfg, B = self.config, len(token_rows)
+        lens = tuple(len(r) for r in token_rows)
+        if B == 0 or min(lens) == 0:
+            raise ValueError("token sequence must contain at least one element")
+        offs = [int(position_offset)] * B if isinstance(position_offset, (int, np.integer)) else [int(o) for o in position_offset]
+        if len(offs) != B or len(caches) != B or any(len(c) != cfg.num_layers for c in caches):
+            raise ValueError(f"expected an offset and {cfg.num_layers} cache slots (one per layer) for every sequence")
+        have = caches[0][0] is not None
+        if any((slot is not None) != have for c in caches for slot in c):
+            raise ValueError("the sequences of a batch either all start or all go on")
+        if have and max(lens) != 1:
+            raise ValueError("decode with an existing cache supports one token per sequence")
+        if not have and any(offs):
+            raise ValueError("a sequence without a cache starts at position 0")
+        if token_handle is not None and max(lens) != 1:
+            raise ValueError("device tokens feed one step (one token per sequence)")
+        if token_handle is None:
+            for row in token_rows:
+                for t in row:
+                    if not 0 <= t < cfg.vocab_size:
+                        raise ValueError(f"token index {t} out of range")
+        totals = [o + n for o, n in zip(offs, lens)]
+        need = max(totals)
+        if need > cfg.context_length:
+            raise ValueError(f"token sequence length {need} exceeds model context length {cfg.context_length}")
+        if fixed_capacity is not None:
+            if not 0 < fixed_capacity <= cfg.context_length or fixed_capacity < need:
+                raise ValueError(f"decode cache capacity {fixed_capacity} invalid for sequence length {need}")
+            capacity = fixed_capacity
+        else:
+            capacity = decode_cache_capacity(need, cfg.context_length)
+        if have:
+            for c, o in zip(caches, offs):
+                for slot in c:
+                    if slot.len != o:
+                        raise ValueError(f"decode cache length {slot.len} must match position offset {o}")
+            # the sequences of a step share one capacity: the largest any of them has or needs
+            capacity = max([capacity] + [s.capacity for c in caches for s in c if isinstance(s, DecodeLatentCache)])
+            for c in caches:
+                for i, s in enumerate(c):
+                    if isinstance(s, DecodeLatentCache) and s.capacity < capacity:
+                        c[i] = DecodeLatentCache(self._grow_rows(s.rows, (1, s.capacity, cfg.layers[i].mixer.row_width), capacity), s.len, capacity)
+        prog, _ = self._build(lens, capacity, have, last_logits_only, None if logit_rows is None else len(logit_rows))
+        tok_arg = token_handle if token_handle is not None else self._upload_i32([t for row in token_rows for t in row])
+        args = [tok_arg, self._upload_i32([o + j for o, n in zip(offs, lens) for j in range(n)]), self._upload_i32([v for o in offs for v in (0, o, 0)])]
+        if logit_rows is not None:
+            args.append(self._upload_i32(logit_rows))
+        held = []
+        for c in caches:
+            for L, slot in zip(cfg.layers, c):
+                m = L.mixer
+                if isinstance(m, SsmMixerConfig):
+                    held += [slot.conv, slot.state] if have else [self._zeros([m.conv - 1, m.channels], "F32"), self._zeros([m.heads, m.state, m.vdim], "F32")]
+                elif m.kv_from is None:
+                    held.append(slot.rows if have else self._zeros([1, capacity, m.row_width]))
+        outs = self._run(prog, args + held, [False] * len(args) + [True] * len(held))
+        it = iter(outs[:-1])
+        for b in range(B):
+            for i, L in enumerate(cfg.layers):
+                m = L.mixer
+                if isinstance(m, SsmMixerConfig):
+                    caches[b][i] = DecodeSsmState(next(it), next(it), totals[b])
+                elif m.kv_from is None:
+                    caches[b][i] = DecodeLatentCache(next(it), totals[b], capacity)
+                else:
+                    caches[b][i] = SharedLayerCache(m.kv_from, totals[b])
+        return outs[-1]
+
+
+# kind of a checkpoint -> (class, default storage dtype); `architecture` of a model folder's config.json -> kind
+MODEL_KINDS = {"gpt": (Gpt, "F32"), "ministral": (Ministral, "Bf16"), "dadupel": (Dadupel, "Bf16")}
+KIND_OF_ARCHITECTURE = {"Dadupel": "dadupel"}
+
+
 # ================================================================================ BatchGenerator
 class BatchGenerator:
-    """Greedy generation for several independent sequences of equal prompt length at once (the reference decodes one
+    """Greedy generation for several independent sequences at once, of equal prompt length unless the model takes batches of
+    unequal rows (`ragged_batches`) (the reference decodes one
     sequence per model call; its batch is a host-side loop): rows stacked through `forward_batch`, one attention launch
     per layer for all of them.  On a backend with sample_decode_rows_begin / _wait the loop is pipelined like
     `Generator`: the tokens of step t stay on the device as the input of step t + 1, which is queued before the host
@@ -901,7 +1366,9 @@ class BatchGenerator:
     def __init__(self, model, prompts: Sequence[Sequence[int]], kv_cache_capacity: Optional[int] = None):
         if len(prompts) == 0 or len(prompts[0]) == 0:
             raise ValueError("prompts must be non-empty")
-        if any(len(p) != len(prompts[0]) for p in prompts):
+        if any(len(p) == 0 for p in prompts):
+            raise ValueError("prompts must be non-empty")
+        if any(len(p) != len(prompts[0]) for p in prompts) and not getattr(model, "ragged_batches", False):
             raise ValueError("all prompts of a batch must have equal length")
         self.model = model
         self.batch = len(prompts)
@@ -910,7 +1377,16 @@ class BatchGenerator:
         self.caches = [[None] * model.num_layers for _ in prompts]
         self.pipelined = hasattr(model.backend, "sample_decode_rows_begin")
         self.logits = model.forward_batch(self.tokens, 0, self.caches, self.capacity, last_logits_only=True)
-        self.processed_len = len(prompts[0])
+        self.lens = [len(p) for p in prompts]
+
+    @property
+    def processed_len(self) -> int:
+        """Tokens of the longest sequence that have gone through the model."""
+        return max(self.lens)
+
+    def _offset(self):
+        """Positions of the next tokens: one number while all sequences have one length."""
+        return self.lens[0] if min(self.lens) == max(self.lens) else list(self.lens)
 
     def step(self) -> List[int]:
         """Samples one token per sequence and runs the forward that consumes them."""
@@ -919,14 +1395,14 @@ class BatchGenerator:
             raise ValueError("context length reached")
         if self.pipelined:
             ticket = be.sample_decode_rows_begin(self.logits)
-            self.logits = self.model.forward_batch([[None]] * B, self.processed_len, self.caches, self.capacity,
+            self.logits = self.model.forward_batch([[None]] * B, self._offset(), self.caches, self.capacity,
                                                    token_handle=be.decode_rows_tensor(B))
             nxt = be.sample_decode_rows_wait(ticket, B)
         else:
             rows = be.to_numpy(self.logits)
             nxt = [int(np.argmax(rows[b])) for b in range(B)]
-            self.logits = self.model.forward_batch([[t] for t in nxt], self.processed_len, self.caches, self.capacity)
-        self.processed_len += 1
+            self.logits = self.model.forward_batch([[t] for t in nxt], self._offset(), self.caches, self.capacity)
+        self.lens = [n + 1 for n in self.lens]
         for b in range(B):
             self.tokens[b].append(nxt[b])
         return nxt

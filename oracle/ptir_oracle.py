@@ -42,6 +42,8 @@ from typing import Dict, List, Sequence, Tuple
 
 import numpy as np
 
+from . import dadupel_reference as DR
+
 _HERE = os.path.dirname(os.path.abspath(__file__))
 _LIB = None
 
@@ -476,6 +478,88 @@ def _norm_call(target: str, attrs, ins: List[OTensor], out_dtype: str) -> OTenso
     return out
 
 
+# ---- sequence mixers: every target by the mechanism's own function (dadupel_reference.py) in f64, the result rounded once
+def _mx_ssm(at, xbc, p, dt_bias, a_log, d, state):
+    H, N, V = state.shape
+    G, dc, inner = int(at["groups"]), int(at["dt_col"]), state.shape[0] * state.shape[2]
+    T = xbc.shape[0]
+    dt = DR.softplus(p[:, dc:dc + H] + dt_bias)
+    return DR.selective_state_scan(xbc[:, :inner].reshape(T, H, V), xbc[:, inner:inner + G * N].reshape(T, G, N),
+                                   xbc[:, inner + G * N:].reshape(T, G, N), dt, a_log, d, state)
+
+
+def _mx_split_q(at, q, dim):
+    q = q.reshape(q.shape[0], int(at["heads"]), -1)
+    return q[..., :dim], q[..., dim:]
+
+
+def _mx_attend(at, q, rows, w_uk, w_uv, start):
+    rank, H = w_uk.shape[0], int(at["heads"])
+    m = {"dim": w_uk.shape[1] // H, "vdim": w_uv.shape[1] // H, "scale": at["scale"]}
+    qn, qr = _mx_split_q(at, q, m["dim"])
+    return DR.latent_attend(qn, qr, rows[0, :, :rank], rows[0, :, rank:], w_uk.T, w_uv.T, m, int(start[0]))
+
+
+def _mx_attend_x(at, q, k, v, rows):
+    H = int(at["heads"])
+    m = {"dim": k.shape[1] // H, "vdim": v.shape[1] // H, "scale": at["scale"]}
+    qn, qr = _mx_split_q(at, q, m["dim"])
+    # keys and values are given: the identity takes the place of W_uk / W_uv over [k | v]
+    kv = np.concatenate([k, v], axis=1)
+    eye = np.eye(kv.shape[1])
+    return DR.latent_attend(qn, qr, kv, rows[:, rows.shape[1] - int(at["rot"]):], eye[:k.shape[1]], eye[k.shape[1]:], m, k.shape[0] - q.shape[0])
+
+
+def _mx_rope_pairs(at, x, table):
+    H, off, half = int(at["heads"]), int(at["offset"]), table.shape[1] // 2
+    y = x.reshape(x.shape[0], H, -1).copy()
+    y[..., off:off + 2 * half] = DR.rotate_pairs(y[..., off:off + 2 * half], table[:, :half], table[:, half:])
+    return y
+
+
+def _mx_latent_rows(at, raw, gain, table):
+    r, half = gain.shape[0], table.shape[1] // 2
+    return np.concatenate([DR.rms_norm(raw[:, :r], gain, at["eps"]), DR.rotate_pairs(raw[:, r:], table[:, :half], table[:, half:])], axis=1)
+
+
+def _mx_rope_table(at, pos, freqs):
+    ang = pos.astype(np.float64)[:, None] * freqs[None, :]
+    return np.concatenate([np.cos(ang), np.sin(ang)], axis=1) * at["magnitude"]
+
+
+def _mx_conv(at, p, state, taps=None, bias=None):
+    c = int(at["col"])
+    x = p[:, c:c + state.shape[1]]
+    if taps is None:
+        return np.concatenate([state, x], axis=0)[x.shape[0]:]
+    return DR.causal_conv_silu(x, taps.T, bias, state)[0]
+
+
+def _mx_gated(at, y, p, gain):
+    c, n = int(at["col"]), y.shape[1]
+    return DR.grouped_rms_norm(y * DR.silu(p[:, c:c + n]), gain, int(at["groups"]), at["eps"])
+
+
+def _mx_glu(at, g, u):
+    g = np.minimum(g, at["limit"])
+    return g * DR.sigmoid(at["alpha"] * g) * (np.clip(u, -at["limit"], at["limit"]) + at["shift"])
+
+
+_MIXER_CALLS = {
+    "gpt_rs.hip.rope_table.v1": _mx_rope_table,
+    "gpt_rs.hip.rope_pairs.v1": _mx_rope_pairs,
+    "gpt_rs.hip.latent_rows.v1": _mx_latent_rows,
+    "gpt_rs.hip.latent_attention.v1": _mx_attend,
+    "gpt_rs.hip.latent_attention_expanded.v1": _mx_attend_x,
+    "gpt_rs.hip.causal_conv_silu.v1": lambda at, p, taps, bias, state: _mx_conv(at, p, state, taps, bias),
+    "gpt_rs.hip.causal_conv_state.v1": lambda at, p, state: _mx_conv(at, p, state),
+    "gpt_rs.hip.ssm_scan.v1": lambda at, *v: _mx_ssm(at, *v)[0],
+    "gpt_rs.hip.ssm_state.v1": lambda at, xbc, p, dt_bias, a_log, state: _mx_ssm(at, xbc, p, dt_bias, a_log, np.zeros_like(a_log), state)[1],
+    "gpt_rs.hip.gated_rms_norm.v1": _mx_gated,
+    "gpt_rs.hip.clamped_glu.v1": _mx_glu,
+}
+
+
 def _custom_call(target: str, attrs, ins: List[OTensor], out_dtype: str, out_dims) -> OTensor:
     if target in ("gpt_rs.hip.layer_norm.v1", "gpt_rs.hip.rms_norm.v1"):
         return _norm_call(target, attrs, ins, out_dtype)
@@ -497,6 +581,10 @@ def _custom_call(target: str, attrs, ins: List[OTensor], out_dtype: str, out_dim
         return _finish(out_dtype, dequantize_int8(ins[0].a, ins[1].a))
     elif target == "gpt_rs.hip.dequantize_w4g128.v1":
         return _finish(out_dtype, dequantize_int4_g128(ins[0].a, ins[1].a))
+    elif target in _MIXER_CALLS:
+        vals = [x.a.astype(np.float64) if x.dtype in ("F32", "Bf16") else x.a for x in ins]
+        at = {k: v["value"] for k, v in (attrs or {}).items()}
+        return _finish(out_dtype, np.asarray(_MIXER_CALLS[target](at, *vals), np.float32).reshape(out_dims))
     else:
         raise OracleError("unimplemented", f"custom_call target {target}")
     # reference semantics for "dequantize + dot_general": f32 accumulate, output rounded
