@@ -1263,7 +1263,8 @@ int gptrs_hip_fusion_report(const char* program_json, size_t json_len, const int
                 if (in.norm) text += in.norm_ln ? "+layer_norm" : "+rms_norm";
                 if (in.has_bias) text += "+bias";
                 if (in.act == 1) text += "+gelu";
-                if (in.act == 2) text += "+swiglu";
+                if (in.act == 2) text += in.glu ? "+clamped_glu" : "+swiglu";
+                if (in.has_scale) text += "+colscale";
                 if (in.has_residual) text += "+residual";
                 text += in.mfma ? " [gemm]" : in.tiled ? " [stream]" : " [generic]";
             }

@@ -310,7 +310,7 @@ struct Fuser {
             const int src = in.operands[0].value;
             if (src < 0 || def[src] < 0 || uses[src] != 1) continue;
             Instr& nrm = fn.body[def[src]];
-            if (nrm.dead || nrm.op != OpKind::FRmsNorm || nrm.out_specs[0].dtype != DType::F32) continue;
+            if (nrm.dead || (nrm.op != OpKind::FRmsNorm && nrm.op != OpKind::FLayerNorm) || nrm.out_specs[0].dtype != DType::F32) continue;
             Instr ni = nrm;
             ni.out_ids = in.out_ids;
             ni.out_specs = in.out_specs;
@@ -859,7 +859,7 @@ struct Fuser {
                     // bias: Add(linear, BroadcastTo(b[N]))  (tensor_ops.rs:42-56)
                     Instr* lin = linear_of(a);
                     int vec;
-                    if (lin && !lin->has_bias && !lin->has_residual && lin->act == 0 && !lin->out_f32 &&
+                    if (lin && !lin->has_bias && !lin->has_scale && !lin->has_residual && lin->act == 0 && !lin->out_f32 &&
                         vector_bcast_last(b, in.out_specs[0].dims.back(), vec)) {
                         Instr ni = *lin;
                         Operand o; o.value = vec;
@@ -893,9 +893,27 @@ struct Fuser {
                         reindex();
                         changed = true;
                     }
+                } else if (in.op == OpKind::Binary && in.binary == BinaryOp::Mul && !in.scalar_rhs) {
+                    // factors per column: Mul(linear, BroadcastTo(s[N])) of f32 results on the weight-streaming and matrix-core kernels
+                    for (int side = 0; side < 2 && !changed; ++side) {
+                        Instr* lin = linear_of(in.operands[side].value);
+                        int vec;
+                        if (!lin || lin->quant || lin->has_scale || lin->has_residual || lin->act != 0 || in.out_specs[0].dtype != DType::F32 ||
+                            !fast_linear(*lin) || !vector_bcast_last(in.operands[1 - side].value, in.out_specs[0].dims.back(), vec))
+                            continue;
+                        Instr ni = *lin;
+                        Operand o; o.value = vec;
+                        ni.operands.push_back(o);
+                        ni.has_scale = true;
+                        ni.out_ids = {v};
+                        lin->dead = true;
+                        fn.body[i] = ni;
+                        reindex();
+                        changed = true;
+                    }
                 } else if (in.op == OpKind::FGelu) {
                     Instr* lin = linear_of(in.operands[0].value);
-                    if (lin && lin->act == 0 && !lin->has_residual && !lin->out_f32 && in.fparam[0] == 0.5f && in.fparam[1] == 1.41421354f &&
+                    if (lin && lin->act == 0 && !lin->has_scale && !lin->has_residual && !lin->out_f32 && in.fparam[0] == 0.5f && in.fparam[1] == 1.41421354f &&
                         in.fparam[2] == 1.0f) {
                         Instr ni = *lin;
                         ni.act = 1;
@@ -905,7 +923,7 @@ struct Fuser {
                         reindex();
                         changed = true;
                     }
-                } else if (in.op == OpKind::FSwiglu) {
+                } else if (in.op == OpKind::FSwiglu || (in.op == OpKind::FMixer && in.mix == Mix::Glu)) {
                     Instr* lg = linear_of(in.operands[0].value);
                     Instr* lu = linear_of(in.operands[1].value);
                     if (lg && lu && lg != lu && lg->act == 0 && lu->act == 0 && !lg->has_bias && !lu->has_bias &&
@@ -920,6 +938,11 @@ struct Fuser {
                             if (lg->quant) ni.operands.push_back(lu->operands[2]);
                             ni.act = 2;
                             ni.out_ids = {v};
+                            if (in.op == OpKind::FMixer) {   // the clamped pair: the kernels that stream or tile the weights know it
+                                ni.glu = 1;
+                                for (int q = 0; q < 3; ++q) ni.fparam[q] = in.fparam[q];
+                                if (ni.quant || !fast_linear(ni)) continue;
+                            }
                             lg->dead = true;
                             lu->dead = true;
                             fn.body[i] = ni;
@@ -960,7 +983,7 @@ struct Fuser {
                 for (size_t o = 0; o < c.operands.size(); ++o) {
                     if (c.operands[o].value != nv) continue;
                     ++found;
-                    if (c.op == OpKind::FLinear && c.tiled && !c.norm && o == 0 && !(ln && c.quant) && !(ln && xf32)) cons.push_back(&c);
+                    if (c.op == OpKind::FLinear && c.tiled && !c.norm && o == 0 && !(ln && c.quant)) cons.push_back(&c);
                 }
             }
             if (cons.empty() || (int)cons.size() != found || found != uses[nv]) continue;

@@ -75,11 +75,20 @@ bool argmax_rows_noalloc(hipStream_t s, int device, int dtype, const void* logit
 void sample_temperature_last_row(hipStream_t s, int dtype, const void* logits, int64_t rows, int64_t vocab,
                                  float temperature, float u, int64_t* out);
 
+// How a gate / up pair is combined (see glu_combine in device_utils.hpp)
+struct GluParams { int kind = 0; float limit = 0.f, alpha = 1.f, shift = 0.f; };
+// What the unquantised linear kernels apply besides bias, GELU and residual: factors per output column (f32, between bias and
+// residual) and the kind of pair
+struct EpiExtra { const float* colscale = nullptr; GluParams glu; };
+
 // ---- fused kernels (kernels_fused.hip) --------------------------------------------------
 // y[r] = LN(x[r]) * gamma + beta over the last axis, two-pass (mean, then centred variance):
 // ops/functional/normalization.rs:123-174.  inv_n is the f32-rounded 1/N multiplier.
 void layer_norm(hipStream_t s, int dtype, const void* x, const void* gamma, const void* beta, void* y,
                 int64_t rows, int64_t n, float inv_n, float eps);
+// the same over f32 rows, gains and offsets with a bf16 result (the f32 value rounded once)
+void layer_norm_f32_to_bf16(hipStream_t s, const void* x, const void* gamma, const void* beta, void* y, int64_t rows, int64_t n,
+                            float inv_n, float eps);
 // y = x * rsqrt(mean(x^2)+eps) * gamma: normalization.rs:183-217
 void rms_norm(hipStream_t s, int dtype, const void* x, const void* gamma, void* y, int64_t rows, int64_t n,
               float inv_n, float eps);
@@ -119,7 +128,8 @@ struct TiledLinearArgs {
     const void* beta;   // with gamma: LayerNorm (normalization.rs:123-174) instead of RMSNorm
     // bf16 weights only.  out_f32: y and residual are f32 (the accumulator leaves unrounded).  x_f32 (with gamma, RMSNorm):
     // x and gamma are f32, the normalised row is rounded to bf16 once as it is staged.
-    int out_f32 = 0, x_f32 = 0;
+    int out_f32 = 0, x_f32 = 0;   // (x_f32 with beta: the f32 LayerNorm, beta f32)
+    EpiExtra extra;
 };
 size_t tiled_weight_bytes(int dtype, int64_t k, int64_t n);
 void tile_weights(hipStream_t s, int dtype, const void* w, void* wt, int64_t k, int64_t n);
@@ -141,6 +151,7 @@ struct SkinnyLinearArgs {
     // the code copies of skinny_pack_codes, scale / scale2 the scale tensors as the program holds them (bf16)
     int quant; const void* scale; const void* scale2;
     int out_f32 = 0;   // bf16 only: y and residual are f32
+    EpiExtra extra;    // unquantised only
 };
 bool skinny_quant_supported(int dtype, int64_t m, int64_t k, int64_t n, int qf);
 size_t skinny_codes_bytes(int64_t k, int64_t n, int qf);
@@ -181,9 +192,9 @@ constexpr int kChainMaxXsWords = 12288;   // staged activation words (48 KiB): K
 constexpr size_t kChainBarrierBytes = (kChainCounters * 64 + 64) * sizeof(unsigned);  // zero-initialised once
 // kChainOutF32: y and the residual are f32.  kChainXF32 (with kChainNorm): x and gamma are f32, the normalised row is
 // rounded to bf16 once as it is staged.
-// kChainLayerNorm (with kChainNorm, f32 phases only): LayerNorm with gains `gamma` and offsets `beta` instead of RMSNorm.
+// kChainLayerNorm (with kChainNorm, f32 phases or kChainXF32): LayerNorm with gains `gamma` and offsets `beta` instead of RMSNorm.
 enum : int { kChainNorm = 1, kChainDual = 2, kChainGelu = 4, kChainResidual = 8, kChainBias = 16, kChainOutF32 = 32, kChainXF32 = 64,
-             kChainLayerNorm = 128, kChainAttnFinal = 256 };
+             kChainLayerNorm = 128, kChainAttnFinal = 256, kChainColScale = 512, kChainClampedGlu = 1024 };
 // weight format of a linear phase; kChainW32: f32 weights (16-byte word = 4 columns x 1 k) with f32 activations,
 // bias, residual and output (the launch's attention phases then read f32 rows and caches as well)
 enum : int { kChainW16 = 0, kChainW8 = 1, kChainW4 = 2, kChainW32 = 3 };
@@ -211,8 +222,10 @@ struct ChainPhase {
     float* part;                               // [n_q][nch][head_dim + 2] f32
     int n_q, n_kv, head_dim, capacity, rot_half, nch;
     float scale;
-    int pad;
+    float glu_limit;                           // kChainClampedGlu (with kChainDual): see glu_combine
     const void* beta;                          // LayerNorm offsets (kChainLayerNorm)
+    const void* colscale;                      // kChainColScale: f32 factor per output column, between bias and residual
+    float glu_alpha, glu_shift;
 };
 int chain_grid();  // workgroups per launch (one per CU), 0 when no device is current
 bool chain_supported(int dtype, int64_t m, int64_t k, int64_t n, bool dual, bool norm, int wfmt = kChainW16, bool x_f32 = false, bool plain = false);
@@ -260,6 +273,7 @@ struct MfmaLinearArgs {
     // counters, zero before and after every launch); without them every tile runs whole
     void* part = nullptr; size_t part_bytes = 0; unsigned* tickets = nullptr;
     int out_f32 = 0;   // bf16 only: y and residual are f32
+    EpiExtra extra;    // unquantised only
     int lds_direct = 1;   // unquantised bf16: the LDS-direct kernel where it applies (0: the register-staged one)
 };
 size_t mfma_workspace_bytes(int dtype, int64_t m, int64_t k, int64_t n, bool dual, int quant);
@@ -384,8 +398,6 @@ void ssm_scan(hipStream_t s, const SsmArgs& a);
 // y T [rows, n] = rms-normed in `groups` equal parts of (y * silu(p[:, col ..])), times gain[n]
 void gated_rms_norm(hipStream_t s, int dtype, const void* y, const float* p, const float* gain, void* out, int64_t rows, int64_t n, int64_t ld,
                     int64_t col, int64_t groups, float eps);
-// How a gate / up pair is combined (see glu_combine in device_utils.hpp)
-struct GluParams { int kind = 0; float limit = 0.f, alpha = 1.f, shift = 0.f; };
 void clamped_glu(hipStream_t s, int dtype, const void* gate, const void* up, void* y, int64_t n, const GluParams& p);
 
 }  // namespace k

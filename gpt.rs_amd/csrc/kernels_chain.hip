@@ -157,29 +157,31 @@ __device__ __forceinline__ void wg_barrier() {
 // way nothing is fetched between the barrier and the first use.
 struct PhaseRegs {
     int K, N, Kw, ntiles, upb, units, lds_bytes, flags, wfmt;
-    float inv_n, eps;
-    const void *x, *gamma, *beta, *bias, *residual, *wscale, *wscale2;
+    float inv_n, eps, glu_limit, glu_alpha, glu_shift;   // (the last three: control wave only)
+    const void *x, *gamma, *beta, *bias, *residual, *wscale, *wscale2, *colscale;
     void* y;
 };
-// (F32: the launch has f32 phases; only those read the LayerNorm offsets, and a register pair that nobody reads is not kept)
-template <bool F32>
+// (LN: phases of the launch's weight format may read LayerNorm offsets; a register pair that nobody reads is not kept)
+template <bool LN>
 __device__ __forceinline__ void regs_from_table(PhaseRegs& R, const GPTRS_CONST ChainPhase* D) {
     R.K = uni(D->K); R.N = uni(D->N); R.Kw = uni(D->Kw); R.ntiles = uni(D->ntiles); R.upb = uni(D->upb); R.units = uni(D->units);
     R.lds_bytes = uni(D->lds_bytes); R.flags = uni(D->flags); R.wfmt = uni(D->wfmt);
     R.inv_n = __int_as_float(uni(__float_as_int(D->inv_n))); R.eps = __int_as_float(uni(__float_as_int(D->eps)));
-    R.x = uni_ptr(D->x); R.gamma = uni_ptr(D->gamma); R.beta = F32 ? uni_ptr(D->beta) : nullptr; R.bias = uni_ptr(D->bias); R.residual = uni_ptr(D->residual);
+    R.x = uni_ptr(D->x); R.gamma = uni_ptr(D->gamma); R.beta = LN ? uni_ptr(D->beta) : nullptr; R.bias = uni_ptr(D->bias); R.residual = uni_ptr(D->residual);
     R.wscale = uni_ptr(D->wscale); R.wscale2 = uni_ptr(D->wscale2); R.y = uni_ptr(D->y);
 }
 #define GPTRS_PD_INT(field) __builtin_amdgcn_readlane(pd, (int)(offsetof(ChainPhase, field) / 4))
 #define GPTRS_PD_PTR(field) ((const void*)(((unsigned long long)(unsigned)__builtin_amdgcn_readlane(pd, (int)(offsetof(ChainPhase, field) / 4) + 1) << 32) | \
                                           (unsigned)__builtin_amdgcn_readlane(pd, (int)(offsetof(ChainPhase, field) / 4))))
-template <bool F32>
+template <bool LN>
 __device__ __forceinline__ void regs_from_lanes(PhaseRegs& R, int pd) {   // pd: dword `lane` of the descriptor
     R.K = GPTRS_PD_INT(K); R.N = GPTRS_PD_INT(N); R.Kw = GPTRS_PD_INT(Kw); R.ntiles = GPTRS_PD_INT(ntiles); R.upb = GPTRS_PD_INT(upb);
     R.units = GPTRS_PD_INT(units); R.lds_bytes = GPTRS_PD_INT(lds_bytes); R.flags = GPTRS_PD_INT(flags); R.wfmt = GPTRS_PD_INT(wfmt);
     R.inv_n = __int_as_float(GPTRS_PD_INT(inv_n)); R.eps = __int_as_float(GPTRS_PD_INT(eps));
-    R.x = GPTRS_PD_PTR(x); R.gamma = GPTRS_PD_PTR(gamma); R.beta = F32 ? GPTRS_PD_PTR(beta) : nullptr; R.bias = GPTRS_PD_PTR(bias); R.residual = GPTRS_PD_PTR(residual);
+    R.x = GPTRS_PD_PTR(x); R.gamma = GPTRS_PD_PTR(gamma); R.beta = LN ? GPTRS_PD_PTR(beta) : nullptr; R.bias = GPTRS_PD_PTR(bias); R.residual = GPTRS_PD_PTR(residual);
     R.wscale = GPTRS_PD_PTR(wscale); R.wscale2 = GPTRS_PD_PTR(wscale2); R.y = const_cast<void*>(GPTRS_PD_PTR(y));
+    R.colscale = GPTRS_PD_PTR(colscale); R.glu_limit = __int_as_float(GPTRS_PD_INT(glu_limit));
+    R.glu_alpha = __int_as_float(GPTRS_PD_INT(glu_alpha)); R.glu_shift = __int_as_float(GPTRS_PD_INT(glu_shift));
 }
 
 // ---------------------------------------------------------------------------- staging (all waves)
@@ -211,7 +213,59 @@ __device__ __forceinline__ void stage_block(const PhaseRegs& P, unsigned* xs, fl
             sv[u] = i < sc_n ? gload2(sc_src + i) : make_uint2(0u, 0u);
         }
     }
-    if ((P.flags & (kChainNorm | kChainXF32)) == (kChainNorm | kChainXF32)) {
+    if (FMT == kChainW16 && (P.flags & (kChainNorm | kChainXF32 | kChainLayerNorm)) == (kChainNorm | kChainXF32 | kChainLayerNorm)) {
+        // LayerNorm of an f32 row (f32 gains and offsets), rounded to bf16 once: mean, then the variance of the centred row
+        constexpr int MF = MAXI / 2;
+        f32x4 v[MF], gg[MF];
+#pragma unroll
+        for (int u = 0; u < MF; ++u) {
+            const int i = u * NT + t;
+            v[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+            gg[u] = v[u];
+            if (u * NT < n && i < n) {
+                const unsigned long long a = cload8(x + 16 * (size_t)i), b = cload8(x + 16 * (size_t)i + 8);
+                v[u] = f32x4{__uint_as_float((unsigned)a), __uint_as_float((unsigned)(a >> 32)), __uint_as_float((unsigned)b), __uint_as_float((unsigned)(b >> 32))};
+                gg[u] = *(const GPTRS_GLOBAL f32x4*)((const char*)P.gamma + 16 * (size_t)i);
+            }
+        }
+        float s = 0.f;
+#pragma unroll
+        for (int u = 0; u < MF; ++u)
+            if (u * NT < n) { s += v[u].x; s += v[u].y; s += v[u].z; s += v[u].w; }
+        const float ws = wave_sum(s);
+        if (lane == 0) ssq[wave] = ws;
+        wg_barrier();
+        float tot = 0.f;
+#pragma unroll
+        for (int w = 0; w < NT / 64; ++w) tot += ssq[w];
+        const float mean = tot * P.inv_n;
+        float q = 0.f;
+#pragma unroll
+        for (int u = 0; u < MF; ++u) {
+            if (u * NT < n) {
+                if (u * NT + t < n) { v[u].x -= mean; v[u].y -= mean; v[u].z -= mean; v[u].w -= mean; }   // (padding stays zero)
+                q += v[u].x * v[u].x; q += v[u].y * v[u].y; q += v[u].z * v[u].z; q += v[u].w * v[u].w;
+            }
+        }
+        const float wq = wave_sum(q);
+        if (lane == 0) ssq[16 + wave] = wq;
+        wg_barrier();
+        float var = 0.f;
+#pragma unroll
+        for (int w = 0; w < NT / 64; ++w) var += ssq[16 + w];
+        const float inv_std = 1.0f / sqrtf(var * P.inv_n + P.eps);
+#pragma unroll
+        for (int u = 0; u < MF; ++u) {
+            const int i = u * NT + t;
+            if (u * NT < npad && i < npad) {
+                f32x4 bb = {0.f, 0.f, 0.f, 0.f};
+                if (i < n) bb = *(const GPTRS_GLOBAL f32x4*)((const char*)P.beta + 16 * (size_t)i);
+                const unsigned o0 = pack_hw((v[u].x * inv_std) * gg[u].x + bb.x, (v[u].y * inv_std) * gg[u].y + bb.y);
+                const unsigned o1 = pack_hw((v[u].z * inv_std) * gg[u].z + bb.z, (v[u].w * inv_std) * gg[u].w + bb.w);
+                *reinterpret_cast<uint2*>(&xs[2 * i]) = make_uint2(o0, o1);
+            }
+        }
+    } else if ((P.flags & (kChainNorm | kChainXF32)) == (kChainNorm | kChainXF32)) {
         // f32 row and gains (a bf16 model whose residual stream is f32): the f32 norm, rounded to bf16 once
         constexpr int MF = MAXI / 2;   // 16-byte items per thread: K <= 4 * MF * NT
         const char* g = (const char*)P.gamma;
@@ -1072,9 +1126,10 @@ __device__ __forceinline__ bool run_attn_phase(const GPTRS_CONST ChainPhase* php
 }
 
 // ---------------------------------------------------------------------------- control wave
-__device__ __forceinline__ float finish(float v, int flags, float bias, float res) {
+__device__ __forceinline__ float finish(float v, int flags, float bias, float res, float colscale) {
     if (flags & kChainBias) v += bias;                                           // tensor_ops.rs:42-56
     if (flags & kChainGelu) v = (v * 0.5f) * (erff(v / 1.41421354f) + 1.0f);     // activation.rs:96-113
+    if (flags & kChainColScale) v *= colscale;
     if (flags & kChainResidual) v += res;
     return v;
 }
@@ -1122,7 +1177,7 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
         } else if (u0 < u1) {
             if (lane == 0) lds_st(&sh.go, ph);
             PhaseRegs P;
-            regs_from_lanes<FMT == kChainW32>(P, pd);
+            regs_from_lanes<FMT == kChainW32 || FMT == kChainW16>(P, pd);
             const int flags = P.flags, ntiles = P.ntiles, N = P.N;
             const bool dual = flags & kChainDual;
             const int cpt = dual ? 2 : 4;              // output columns per tile
@@ -1136,6 +1191,8 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
             constexpr int wfmt = FMT;   // every linear phase of a launch has the kernel's weight format
             const unsigned* sg = wfmt == kChainW8 ? (const unsigned*)P.wscale : nullptr;
             const unsigned* su = wfmt == kChainW8 ? (const unsigned*)P.wscale2 : nullptr;
+            const char* cscale = (wfmt == kChainW16 || wfmt == kChainW32) && (flags & kChainColScale) ? (const char*)P.colscale : nullptr;
+            unsigned long long e_cs = 0ull;              // two column factors
             const bool out_f32 = flags & kChainOutF32;   // y and the residual are f32
             unsigned long long e_rf = 0ull;              // two f32 residual values
             unsigned long long e_bf = 0ull;              // two f32 bias values (f32 phases)
@@ -1150,6 +1207,10 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
                 bw = (bias && in) ? gload(bias + (col >> 1)) : 0u;
                 if (out_f32) e_rf = (resid && in) ? cload8(resid + 4 * (size_t)col) : 0ull;
                 rw = (resid && in && !out_f32) ? cload4(resid + 2 * (size_t)col) : 0u;
+                if (cscale && in) {
+                    const u32x2 c2 = *(const GPTRS_GLOBAL u32x2*)(cscale + 4 * (size_t)col);
+                    e_cs = (unsigned long long)c2.x | ((unsigned long long)c2.y << 32);
+                }
                 ga = (sg && in) ? gload(sg + (col >> 1)) : 0u;
                 gb = (su && in) ? gload(su + (col >> 1)) : 0u;
             };
@@ -1161,12 +1222,13 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
                     *reinterpret_cast<float2*>(&sh.epi_res[i]) = out_f32 ? make_float2(__uint_as_float((unsigned)e_rf), __uint_as_float((unsigned)(e_rf >> 32)))
                                                                           : make_float2(bf16lo(rw), bf16hi(rw));
                 }
+                if (cscale) *reinterpret_cast<float2*>(&sh.epi_s[i]) = make_float2(__uint_as_float((unsigned)e_cs), __uint_as_float((unsigned)(e_cs >> 32)));
                 if (sg) {
                     *reinterpret_cast<float2*>(&sh.epi_s[i]) = make_float2(bf16lo(ga), bf16hi(ga));
                     *reinterpret_cast<float2*>(&sh.epi_s[EPI_MAX + i]) = make_float2(bf16lo(gb), bf16hi(gb));
                 }
             };
-            const bool has_epi = bias || resid || sg;
+            const bool has_epi = bias || resid || sg || cscale;
             unsigned e_bw = 0u, e_rw = 0u, e_ga = 0u, e_gb = 0u;
             if (has_epi) epi_load(lane * 2, e_bw, e_rw, e_ga, e_gb);
             if (wfmt == kChainW32) stage_block_f32(P, xs, sh.ssq);
@@ -1215,6 +1277,10 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
                             sc[0] = a.x; sc[1] = a.y; sc[2] = a.z; sc[3] = a.w;
                         }
                     }
+                    if (cscale) {   // (never a pair)
+                        const float4 a = *reinterpret_cast<const float4*>(&sh.epi_s[e]);
+                        sc[0] = a.x; sc[1] = a.y; sc[2] = a.z; sc[3] = a.w;
+                    }
                     if (flags & (kChainBias | kChainResidual)) {   // both arrays are staged when either is present
                         if (dual) {
                             const float2 b = *reinterpret_cast<const float2*>(&sh.epi_bias[e]), r = *reinterpret_cast<const float2*>(&sh.epi_res[e]);
@@ -1230,13 +1296,14 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
                         for (int c = 0; c < 4; ++c) s[c] *= sc[c];
                     }
                     if (dual) {   // columns interleaved (gate, up, gate, up): activation.rs:141-162
-                        const float a0 = finish((s[0] / (1.0f + expf(s[0] * -1.0f))) * s[1], flags, bi[0], re[0]);
-                        const float a1 = finish((s[2] / (1.0f + expf(s[2] * -1.0f))) * s[3], flags, bi[1], re[1]);
+                        const int kind = flags & kChainClampedGlu ? 1 : 0;
+                        const float a0 = finish(glu_combine(s[0], s[1], kind, P.glu_limit, P.glu_alpha, P.glu_shift), flags, bi[0], re[0], 1.0f);
+                        const float a1 = finish(glu_combine(s[2], s[3], kind, P.glu_limit, P.glu_alpha, P.glu_shift), flags, bi[1], re[1], 1.0f);
                         cstore4(out + 2 * (size_t)(tile * 2), pack_hw(a0, a1));
                     } else {
                         float o[4];
 #pragma unroll
-                        for (int c = 0; c < 4; ++c) o[c] = finish(s[c], flags, bi[c], re[c]);
+                        for (int c = 0; c < 4; ++c) o[c] = finish(s[c], flags, bi[c], re[c], sc[c]);
                         if (tile * 4 + 4 > N) {   // the last tile of a width that is not a multiple of 4: its real columns one by one
 #pragma unroll
                             for (int c = 0; c < 4; ++c) {
@@ -1433,7 +1500,7 @@ __device__ void compute_waves(Shared& sh, const unsigned* xs, PhaseTable table, 
             c_Kv = (uni(D->K) + kpw - 1) / kpw;
             c_sidx = 0;   // int4: entry of the unit's first tile and group in the staged scales ...
             c_soff = uni(D->lds_bytes) >> 2;   // ... which sit behind the activations
-            regs_from_table<FMT == kChainW32>(R, D);
+            regs_from_table<FMT == kChainW32 || FMT == kChainW16>(R, D);
             return true;   // (the caller waits for the phase to open and stages its input)
         }
     };

@@ -19,12 +19,12 @@ template <> __device__ __forceinline__ void stf<bf16_t>(bf16_t* p, int64_t i, fl
 // ------------------------------------------------------------------------------ layer_norm
 // normalization.rs:123-174: mean = sum*(1/N); c = x-mean; var = sum(c*c)*(1/N); y = c*rsqrt(var+eps)*g+b
 // One block per row; the row stays in registers between the passes (up to 16 values/thread).
-template <typename T, int PER>
+template <typename T, typename TO, int PER>
 __global__ void layer_norm_kernel(const T* __restrict__ x, const T* __restrict__ gamma, const T* __restrict__ beta,
-                                  T* __restrict__ y, int64_t n, float inv_n, float eps) {
+                                  TO* __restrict__ y, int64_t n, float inv_n, float eps) {
     __shared__ float red[16];
     const T* row = x + (int64_t)blockIdx.x * n;
-    T* out = y + (int64_t)blockIdx.x * n;
+    TO* out = y + (int64_t)blockIdx.x * n;
     float v[PER];
     float s = 0.f;
 #pragma unroll
@@ -51,12 +51,12 @@ __global__ void layer_norm_kernel(const T* __restrict__ x, const T* __restrict__
     }
 }
 // rows longer than 16*blockDim: re-read from memory on each pass
-template <typename T>
+template <typename T, typename TO>
 __global__ void layer_norm_long_kernel(const T* __restrict__ x, const T* __restrict__ gamma, const T* __restrict__ beta,
-                                       T* __restrict__ y, int64_t n, float inv_n, float eps) {
+                                       TO* __restrict__ y, int64_t n, float inv_n, float eps) {
     __shared__ float red[16];
     const T* row = x + (int64_t)blockIdx.x * n;
-    T* out = y + (int64_t)blockIdx.x * n;
+    TO* out = y + (int64_t)blockIdx.x * n;
     float s = 0.f;
     for (int64_t i = threadIdx.x; i < n; i += blockDim.x) s += ldf(row, i);
     const float mean = block_sum(s, red) * inv_n;
@@ -67,21 +67,27 @@ __global__ void layer_norm_long_kernel(const T* __restrict__ x, const T* __restr
         stf(out, i, ((ldf(row, i) - mean) * inv_std) * ldf(gamma, i) + ldf(beta, i));
 }
 
-template <typename T>
-static void layer_norm_t(hipStream_t s, const T* x, const T* g, const T* b, T* y, int64_t rows, int64_t n, float inv_n,
+template <typename T, typename TO>
+static void layer_norm_t(hipStream_t s, const T* x, const T* g, const T* b, TO* y, int64_t rows, int64_t n, float inv_n,
                          float eps) {
     const int block = n <= 256 ? 64 : (n <= 1024 ? 256 : 1024);  // decode has ONE row: spread it over many lanes
     const int64_t per = cdiv(n, block);
     const unsigned grid = (unsigned)rows;
-    if (per <= 4) layer_norm_kernel<T, 4><<<grid, block, 0, s>>>(x, g, b, y, n, inv_n, eps);
-    else if (per <= 16) layer_norm_kernel<T, 16><<<grid, block, 0, s>>>(x, g, b, y, n, inv_n, eps);
-    else layer_norm_long_kernel<T><<<grid, 1024, 0, s>>>(x, g, b, y, n, inv_n, eps);
+    if (per <= 4) layer_norm_kernel<T, TO, 4><<<grid, block, 0, s>>>(x, g, b, y, n, inv_n, eps);
+    else if (per <= 16) layer_norm_kernel<T, TO, 16><<<grid, block, 0, s>>>(x, g, b, y, n, inv_n, eps);
+    else layer_norm_long_kernel<T, TO><<<grid, 1024, 0, s>>>(x, g, b, y, n, inv_n, eps);
 }
 void layer_norm(hipStream_t s, int dtype, const void* x, const void* gamma, const void* beta, void* y, int64_t rows,
                 int64_t n, float inv_n, float eps) {
     if (rows <= 0 || n <= 0) return;
-    if (dtype == 0) layer_norm_t<float>(s, (const float*)x, (const float*)gamma, (const float*)beta, (float*)y, rows, n, inv_n, eps);
-    else layer_norm_t<bf16_t>(s, (const bf16_t*)x, (const bf16_t*)gamma, (const bf16_t*)beta, (bf16_t*)y, rows, n, inv_n, eps);
+    if (dtype == 0) layer_norm_t<float, float>(s, (const float*)x, (const float*)gamma, (const float*)beta, (float*)y, rows, n, inv_n, eps);
+    else layer_norm_t<bf16_t, bf16_t>(s, (const bf16_t*)x, (const bf16_t*)gamma, (const bf16_t*)beta, (bf16_t*)y, rows, n, inv_n, eps);
+}
+
+void layer_norm_f32_to_bf16(hipStream_t s, const void* x, const void* gamma, const void* beta, void* y, int64_t rows, int64_t n,
+                            float inv_n, float eps) {
+    if (rows <= 0 || n <= 0) return;
+    layer_norm_t<float, bf16_t>(s, (const float*)x, (const float*)gamma, (const float*)beta, (bf16_t*)y, rows, n, inv_n, eps);
 }
 
 // ------------------------------------------------------------------------------ rms_norm

@@ -72,10 +72,11 @@ void tile_weights(hipStream_t s, int dtype, const void* w, void* wt, int64_t k, 
 // ------------------------------------------------------------------------------ GEMV
 constexpr int kXsBytes = 32768;  // LDS bytes for the staged activations
 
-__device__ __forceinline__ float tiled_finish(float v, float v2, bool dual, int act, float bias, bool has_res, float res) {
-    if (dual) v = (v / (1.0f + expf(v * -1.0f))) * v2;              // activation.rs:141-162
+__device__ __forceinline__ float tiled_finish(float v, float v2, bool dual, int act, float bias, bool has_res, float res, const GluParams& glu, float colscale) {
+    if (dual) v = glu_combine(v, v2, glu.kind, glu.limit, glu.alpha, glu.shift);   // activation.rs:141-162
     v += bias;                                                      // tensor_ops.rs:42-56
     if (act == 1) v = (v * 0.5f) * (erff(v / 1.41421354f) + 1.0f);  // activation.rs:96-113
+    v *= colscale;
     if (has_res) v += res;
     return v;
 }
@@ -86,7 +87,7 @@ __global__ __launch_bounds__(256) void gemv_tiled_kernel(const T* __restrict__ x
                                                          const T* __restrict__ beta,
                                                          const T* __restrict__ bias, const T* __restrict__ residual,
                                                          T* __restrict__ y, int M, int64_t K, int64_t N, int64_t ntiles,
-                                                         float inv_n, float eps, int act, int out_f32, int x_f32) {
+                                                         float inv_n, float eps, int act, int out_f32, int x_f32, EpiExtra extra) {
     constexpr int VEC = Word<T>::VEC;
     constexpr int KT = kXsBytes / (int)sizeof(T) / MT;   // rows of x staged at a time (kept as T)
     constexpr int PLANE = TP * MT * VEC;                 // outputs per block (per weight stream set)
@@ -130,7 +131,7 @@ __global__ __launch_bounds__(256) void gemv_tiled_kernel(const T* __restrict__ x
     // pass below then touches only LDS and gamma.
     // LayerNorm (beta given; normalization.rs:123-174): mean first, then the variance of the centred values, as the
     // stand-alone kernel takes them.
-    // x_f32 (RMSNorm only): x and gamma are f32; the staged row is their f32 norm rounded to T once
+    // x_f32: x, gamma and beta are f32; the staged row is their f32 norm rounded to T once
     const float* xf = reinterpret_cast<const float*>(x);
     const float* gf = reinterpret_cast<const float*>(gamma);
     const bool one_chunk = K <= KT && !x_f32;
@@ -139,11 +140,11 @@ __global__ __launch_bounds__(256) void gemv_tiled_kernel(const T* __restrict__ x
             float q = 0.f, mean = 0.f;
             if (beta) {
                 float sm = 0.f;
-                for (int64_t kk = t; kk < K; kk += 256) sm += ldf(x, (int64_t)m * K + kk);
+                for (int64_t kk = t; kk < K; kk += 256) sm += x_f32 ? xf[(int64_t)m * K + kk] : ldf(x, (int64_t)m * K + kk);
                 mean = block_sum(sm, s_tmp) * inv_n;
             }
             for (int64_t kk = t; kk < K; kk += 256) {
-                if (x_f32) { const float v = xf[(int64_t)m * K + kk]; q += v * v; continue; }
+                if (x_f32) { const float v = xf[(int64_t)m * K + kk] - mean; q += v * v; continue; }
                 const T raw = x[(int64_t)m * K + kk];
                 const float v = ldf(&raw, 0) - mean;
                 if (one_chunk) xs[m][kk] = raw;
@@ -177,7 +178,7 @@ __global__ __launch_bounds__(256) void gemv_tiled_kernel(const T* __restrict__ x
                 // the value the stand-alone norm kernel would have stored: (x*inv_rms)*gamma, rounded to T
                 if (NORM) {
                     v = ((v - s_mean[m]) * s_scale[m]) * (x_f32 ? gf[k0 + kk] : ldf(gamma, k0 + kk));
-                    if (beta) v += ldf(beta, k0 + kk);
+                    if (beta) v += x_f32 ? reinterpret_cast<const float*>(beta)[k0 + kk] : ldf(beta, k0 + kk);
                 }
                 stf(&xs[m][0], kk, v);
             }
@@ -243,10 +244,11 @@ __global__ __launch_bounds__(256) void gemv_tiled_kernel(const T* __restrict__ x
         const float tot = red[0][o] + red[1][o] + red[2][o] + red[3][o];
         const float tot2 = DUAL ? red[0][PLANE + o] + red[1][PLANE + o] + red[2][PLANE + o] + red[3][PLANE + o] : 0.f;
         const float b = bias ? ldf(bias, col) : 0.f;
+        const float cs = extra.colscale ? extra.colscale[col] : 1.0f;
         // out_f32: the f32 accumulator (plus an f32 residual) is stored as it is
         const float r = residual ? (out_f32 ? reinterpret_cast<const float*>(residual)[(int64_t)m * N + col]
                                             : ldf(residual, (int64_t)m * N + col)) : 0.f;
-        const float res = tiled_finish(tot, tot2, DUAL, act, b, residual != nullptr, r);
+        const float res = tiled_finish(tot, tot2, DUAL, act, b, residual != nullptr, r, extra.glu, cs);
         if (out_f32) reinterpret_cast<float*>(y)[(int64_t)m * N + col] = res;
         else stf(y, (int64_t)m * N + col, res);
     }
@@ -264,7 +266,7 @@ static void launch_tiled(hipStream_t s, const TiledLinearArgs& a) {
 #define GPTRS_GT(DUAL, NORM)                                                                                          \
     gemv_tiled_kernel<T, MT, TP, U, DUAL, NORM><<<grid, 256, 0, s>>>((const T*)a.x, (const T*)a.wt, (const T*)a.wt2,         \
         (const T*)a.gamma, (const T*)a.beta, (const T*)a.bias, (const T*)a.residual, (T*)a.y, (int)a.m, a.k, a.n, ntiles, a.inv_n, a.eps, a.act, \
-        sizeof(T) == 2 ? a.out_f32 : 0, sizeof(T) == 2 ? a.x_f32 : 0)
+        sizeof(T) == 2 ? a.out_f32 : 0, sizeof(T) == 2 ? a.x_f32 : 0, a.extra)
     if (a.wt2) { if (a.gamma) GPTRS_GT(true, true); else GPTRS_GT(true, false); }
     else { if (a.gamma) GPTRS_GT(false, true); else GPTRS_GT(false, false); }
 #undef GPTRS_GT

@@ -133,10 +133,11 @@ __device__ __forceinline__ uint32_t mfma_pack_bf16(float lo, float hi) {
     return __builtin_bit_cast(uint32_t, __builtin_convertvector(f, bf16x2_t));   // round to nearest even
 }
 
-__device__ __forceinline__ float mfma_finish(float v, float v2, bool dual, int act, float bias, bool has_res, float res) {
-    if (dual) v = (v / (1.0f + expf(v * -1.0f))) * v2;        // activation.rs:141-162
+__device__ __forceinline__ float mfma_finish(float v, float v2, bool dual, int act, float bias, bool has_res, float res, const GluParams& glu, float colscale) {
+    if (dual) v = glu_combine(v, v2, glu.kind, glu.limit, glu.alpha, glu.shift);   // activation.rs:141-162
     v += bias;                                                // tensor_ops.rs:42-56
     if (act == 1) v = (v * 0.5f) * (erff(v / 1.41421354f) + 1.0f);  // activation.rs:96-113
+    v *= colscale;
     if (has_res) v += res;
     return v;
 }
@@ -173,7 +174,7 @@ __global__ __launch_bounds__(256 * KW) void gemm_mfma_kernel(const T* __restrict
                                                         int M, int K, int N, int Npad, int act, int NT, int MT,
                                                         const T* __restrict__ scale, const T* __restrict__ scale2,
                                                         int full_tiles, int splits, float* __restrict__ part,
-                                                        unsigned* __restrict__ tickets, int out_f32) {
+                                                        unsigned* __restrict__ tickets, int out_f32, EpiExtra extra) {
     constexpr int KPC = Mma<T>::KPC;
     constexpr int kBK = kKb * KPC;                            // k per tile
     typedef typename Mma<T>::frag frag_t;
@@ -484,6 +485,7 @@ __global__ __launch_bounds__(256 * KW) void gemm_mfma_kernel(const T* __restrict
             const int n = n0 + wn * (NREAL / 2) + j * 32 + (lane & 31);
             if (n >= N) continue;
             const float bv = bias ? Mma<T>::ld(bias, n) : 0.f;
+            const float cs = extra.colscale ? extra.colscale[n] : 1.0f;
 #pragma unroll
             for (int v = 0; v < 16; ++v) {
                 const int m = m0 + wm * (BM / 2) + i * 32 + 8 * (v >> 2) + 4 * (lane >> 5) + (v & 3);
@@ -493,7 +495,7 @@ __global__ __launch_bounds__(256 * KW) void gemm_mfma_kernel(const T* __restrict
                                                     : Mma<T>::ld(residual, (int64_t)m * N + n)) : 0.f;
                 const float g = acc[i][j][v];
                 const float u = DUAL ? acc[i][DUAL ? j + TN / 2 : j][v] : 0.f;
-                const float o = mfma_finish(g, u, DUAL, act, bv, residual != nullptr, r);
+                const float o = mfma_finish(g, u, DUAL, act, bv, residual != nullptr, r, extra.glu, cs);
                 if (out_f32) reinterpret_cast<float*>(y)[(int64_t)m * N + n] = o;
                 else Mma<T>::st(y, (int64_t)m * N + n, o);
             }
@@ -540,7 +542,7 @@ __global__ __launch_bounds__(64 * WM * WN * KW) void gemm_dma_kernel(const bf16_
                                                                    const bf16_t* __restrict__ wk2, const bf16_t* __restrict__ bias,
                                                                    const bf16_t* __restrict__ residual, bf16_t* __restrict__ y,
                                                                    int M, int K, int N, int Npad, int act, int NT, int MT, int out_f32,
-                                                                   int splits, float* __restrict__ part, unsigned* __restrict__ tickets) {
+                                                                   int splits, float* __restrict__ part, unsigned* __restrict__ tickets, EpiExtra extra) {
     constexpr int BK = 64, KG = 8, ROWB = 128;
     constexpr int BM = 64 * WM, BN = 32 * TN * WN, NW = WM * WN * KW;
     constexpr int NREAL = DUAL ? BN / 2 : BN;                          // output columns per tile
@@ -784,7 +786,7 @@ __global__ __launch_bounds__(64 * WM * WN * KW) void gemm_dma_kernel(const bf16_
             *reinterpret_cast<f32x4_t*>(u) = *reinterpret_cast<const f32x4_t*>(area + 32 * RSF + r * RSF + cc * 8);
             *reinterpret_cast<f32x4_t*>(u + 4) = *reinterpret_cast<const f32x4_t*>(area + 32 * RSF + r * RSF + cc * 8 + 4);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) o[e] = (o[e] / (1.0f + expf(o[e] * -1.0f))) * u[e];   // activation.rs:141-162
+            for (int e = 0; e < 8; ++e) o[e] = glu_combine(o[e], u[e], extra.glu.kind, extra.glu.limit, extra.glu.alpha, extra.glu.shift);   // activation.rs:141-162
         }
         const int64_t at = (int64_t)m * N + n;
         if (vec) {
@@ -799,6 +801,11 @@ __global__ __launch_bounds__(64 * WM * WN * KW) void gemm_dma_kernel(const bf16_
             if (act == 1) {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) o[e] = (o[e] * 0.5f) * (erff(o[e] / 1.41421354f) + 1.0f);   // activation.rs:96-113
+            }
+            if (extra.colscale) {
+                const f32x4_t c0 = *reinterpret_cast<const f32x4_t*>(extra.colscale + n), c1 = *reinterpret_cast<const f32x4_t*>(extra.colscale + n + 4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { o[e] *= c0[e]; o[4 + e] *= c1[e]; }
             }
             if (residual) {
                 if (out_f32) {
@@ -830,7 +837,7 @@ __global__ __launch_bounds__(64 * WM * WN * KW) void gemm_dma_kernel(const bf16_
                 if (n + e >= N) break;
                 const float bv = bias ? bf16_to_f32(bias[n + e]) : 0.f;
                 const float rv = residual ? (out_f32 ? reinterpret_cast<const float*>(residual)[at + e] : bf16_to_f32(residual[at + e])) : 0.f;
-                const float f = mfma_finish(o[e], 0.f, false, act, bv, residual != nullptr, rv);
+                const float f = mfma_finish(o[e], 0.f, false, act, bv, residual != nullptr, rv, extra.glu, extra.colscale ? extra.colscale[n + e] : 1.0f);
                 if (out_f32) reinterpret_cast<float*>(y)[at + e] = f;
                 else y[at + e] = f32_to_bf16(f);
             }
@@ -858,7 +865,7 @@ static void launch_dma(hipStream_t s, const MfmaLinearArgs& a, int splits = 1) {
     kern<<<grid, 64 * WM * WN * KW, lds_bytes, s>>>((const bf16_t*)a.x, (const bf16_t*)a.wk, (const bf16_t*)a.wk2, (const bf16_t*)a.bias,
                                                    (const bf16_t*)a.residual, (bf16_t*)a.y, (int)a.m, (int)a.k, (int)a.n,
                                                    (int)mfma_padded_n(a.n), a.act, (int)nt, (int)mt, a.out_f32, splits, (float*)a.part,
-                                                   a.tickets);
+                                                   a.tickets, a.extra);
 }
 
 // Which tiles an unquantised bf16 launch of the LDS-direct kernel takes: 128 x 192 (`wide`), 128 x 96, or 128 x 192 with
@@ -957,7 +964,7 @@ static void launch_mfma(hipStream_t s, const MfmaLinearArgs& a) {
     const unsigned grid = (unsigned)(cdiv(full, 8) * 8 + (nt * mt - full) * splits);
     kern<<<grid, 256 * KW, lds_bytes, s>>>((const T*)a.x, (const T*)a.wk, (const T*)a.wk2, (const T*)a.bias, (const T*)a.residual, (T*)a.y,
                                       (int)a.m, (int)a.k, (int)a.n, (int)npad, a.act, (int)nt, (int)mt, (const T*)a.scale, (const T*)a.scale2,
-                                      (int)full, splits, (float*)a.part, a.tickets, a.dtype == 2 ? a.out_f32 : 0);
+                                      (int)full, splits, (float*)a.part, a.tickets, a.dtype == 2 ? a.out_f32 : 0, a.extra);
 }
 
 void mfma_gemm(hipStream_t s, const MfmaLinearArgs& a) {

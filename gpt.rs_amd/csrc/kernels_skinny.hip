@@ -82,10 +82,11 @@ __global__ __launch_bounds__(256) void skinny_pack_kernel(const T* __restrict__ 
     }
 }
 
-__device__ __forceinline__ float skinny_finish(float v, float v2, bool dual, int act, float bias, bool has_res, float res) {
-    if (dual) v = (v / (1.0f + expf(v * -1.0f))) * v2;              // activation.rs:141-162
+__device__ __forceinline__ float skinny_finish(float v, float v2, bool dual, int act, float bias, bool has_res, float res, const GluParams& glu = GluParams(), float colscale = 1.0f) {
+    if (dual) v = glu_combine(v, v2, glu.kind, glu.limit, glu.alpha, glu.shift);   // activation.rs:141-162
     v += bias;                                                      // tensor_ops.rs:42-56
     if (act == 1) v = (v * 0.5f) * (erff(v / 1.41421354f) + 1.0f);  // activation.rs:96-113
+    v *= colscale;
     if (has_res) v += res;
     return v;
 }
@@ -95,7 +96,7 @@ __global__ __launch_bounds__(256) void skinny_gemm_kernel(const T* __restrict__ 
                                                           const T* __restrict__ ws2, const T* __restrict__ bias,
                                                           const T* __restrict__ residual, T* __restrict__ y, int M, int K,
                                                           int N, int act, float* __restrict__ part, unsigned* __restrict__ tickets,
-                                                          int out_f32) {
+                                                          int out_f32, EpiExtra extra) {
     constexpr int U = 4;                         // steps per wave and round, all requested before the first is used
     constexpr int KPC = SkinnyT<T>::KPC, KSTEP = 4 * KPC;
     __shared__ float red[4][DUAL ? 2 : 1][64][4];
@@ -177,6 +178,7 @@ __global__ __launch_bounds__(256) void skinny_gemm_kernel(const T* __restrict__ 
     const int n = tile * 16 + c;
     if (n >= N) return;
     const float bv = bias ? SkinnyT<T>::ld(bias, n) : 0.f;
+    const float cs = extra.colscale ? extra.colscale[n] : 1.0f;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         const int m = 4 * kg + i;                // D: lane holds rows 4 kg .. 4 kg + 3 of column c
@@ -184,7 +186,7 @@ __global__ __launch_bounds__(256) void skinny_gemm_kernel(const T* __restrict__ 
         // out_f32: the f32 accumulator (plus an f32 residual) is stored as it is
         const float r = residual ? (out_f32 ? reinterpret_cast<const float*>(residual)[(int64_t)m * N + n]
                                             : SkinnyT<T>::ld(residual, (int64_t)m * N + n)) : 0.f;
-        const float o = skinny_finish(g[i], up[i], DUAL, act, bv, residual != nullptr, r);
+        const float o = skinny_finish(g[i], up[i], DUAL, act, bv, residual != nullptr, r, extra.glu, cs);
         if (out_f32) reinterpret_cast<float*>(y)[(int64_t)m * N + n] = o;
         else SkinnyT<T>::st(y, (int64_t)m * N + n, o);
     }
@@ -445,7 +447,7 @@ void skinny_gemm(hipStream_t s, const SkinnyLinearArgs& a) {
     const dim3 grid((unsigned)cdiv_s(a.n, 16), (unsigned)ks);
 #define GPTRS_LAUNCH(T, DUAL)                                                                                               \
     skinny_gemm_kernel<T, DUAL><<<grid, 256, 0, s>>>((const T*)a.x, (const T*)a.ws, (const T*)a.ws2, (const T*)a.bias,          \
-        (const T*)a.residual, (T*)a.y, (int)a.m, (int)a.k, (int)a.n, a.act, (float*)a.part, a.tickets, a.dtype == 2 ? a.out_f32 : 0)
+        (const T*)a.residual, (T*)a.y, (int)a.m, (int)a.k, (int)a.n, a.act, (float*)a.part, a.tickets, a.dtype == 2 ? a.out_f32 : 0, a.extra)
     if (a.dtype == 0) { if (a.ws2) GPTRS_LAUNCH(float, true); else GPTRS_LAUNCH(float, false); }
     else { if (a.ws2) GPTRS_LAUNCH(bf16_t, true); else GPTRS_LAUNCH(bf16_t, false); }
 #undef GPTRS_LAUNCH

@@ -800,9 +800,9 @@ void Builder::build() {
         const bool dual = in.act == 2;
         const DType ldt = linear_dtype(in, w, in.quant ? &plan.values[st.src[2]].spec : nullptr);
         const int wfmt = chain_format(in, ldt);
-        if (in.norm_ln && wfmt != k::kChainW32) return 0;   // LayerNorm is staged for f32 phases only
+        if (in.norm_ln && wfmt != k::kChainW32 && !(wfmt == k::kChainW16 && in.x_f32)) return 0;   // LayerNorm is staged from f32 rows only
         if (wfmt == k::kChainW32 && (in.norm && !in.norm_ln)) return 0;   // ... and RMSNorm for the others
-        if (!k::chain_supported((int)ldt, x.dims[0], x.dims[1], w.dims[1], dual, in.norm, wfmt, in.x_f32, !in.has_bias && !in.has_residual)) return 0;
+        if (!k::chain_supported((int)ldt, x.dims[0], x.dims[1], w.dims[1], dual, in.norm, wfmt, in.x_f32, !in.has_bias && !in.has_residual && !in.has_scale)) return 0;
         k::ChainPhase p{};
         return k::chain_fill_phase(p, x.dims[1], w.dims[1], dual, wfmt) ? 1 : 0;
     };
@@ -852,6 +852,12 @@ void build_plan(Plan& plan, const std::vector<bool>& donated) {
 // ------------------------------------------------------------------------------ execution
 static inline const void* src_ptr(const Step& st, const ExecCtx& cx, size_t i) {
     return st.src[i] >= 0 ? cx.ptr[st.src[i]] : (const void*)(cx.consts + st.src_const[i]);
+}
+
+static k::GluParams linear_glu(const Instr& in) {
+    k::GluParams p;
+    if (in.act == 2 && in.glu) { p.kind = in.glu; p.limit = in.fparam[0]; p.alpha = in.fparam[1]; p.shift = in.fparam[2]; }
+    return p;
 }
 
 // algorithmic bytes of the weights an FLinear reads once: codes and scales when quantised
@@ -939,14 +945,16 @@ static bool run_chain(const Plan& plan, const Step& head, ExecCtx& cx) {
         }
         size_t oi = linear_extra_pos(in);
         if (in.has_bias) { p.bias = src_ptr(st, cx, oi++); p.flags |= k::kChainBias; }
+        if (in.has_scale) { p.colscale = src_ptr(st, cx, oi++); p.flags |= k::kChainColScale; }
         if (in.has_residual) { p.residual = src_ptr(st, cx, oi++); p.flags |= k::kChainResidual; }
         if (in.norm) { p.gamma = src_ptr(st, cx, oi++); p.inv_n = in.scale; p.eps = in.eps; p.flags |= k::kChainNorm; }
         if (in.norm && in.norm_ln) { p.beta = src_ptr(st, cx, oi++); p.flags |= k::kChainLayerNorm; }
         if (in.act == 1) p.flags |= k::kChainGelu;
+        if (in.act == 2 && in.glu) { p.flags |= k::kChainClampedGlu; p.glu_limit = in.fparam[0]; p.glu_alpha = in.fparam[1]; p.glu_shift = in.fparam[2]; }
         if (in.out_f32 || wfmt == k::kChainW32) p.flags |= k::kChainOutF32;
         if (in.x_f32 || wfmt == k::kChainW32) p.flags |= k::kChainXF32;
         p.y = cx.ptr[st.dst[0]];
-        aligned8({p.x, p.y, p.residual, p.bias, p.gamma, p.beta});
+        aligned8({p.x, p.y, p.residual, p.bias, p.gamma, p.beta, p.colscale});
         if ((p.flags & k::kChainXF32) && (((uintptr_t)p.gamma | (uintptr_t)p.beta | (uintptr_t)p.x) & 15))
             fail_exec("decode chain: f32 rows, gains and offsets must be 16-byte aligned");
         lds_bytes = std::max(lds_bytes, p.lds_total);
@@ -1078,7 +1086,10 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
         case OpKind::FLayerNorm: {
             const Spec& x = in_spec(0);
             const int64_t n = x.dims.back();
-            k::layer_norm(s, (int)out.dtype, src_ptr(st, cx, 0), src_ptr(st, cx, 1), src_ptr(st, cx, 2), dst, n ? x.count() / n : 0, n, in.scale, in.eps);
+            if (x.dtype == DType::F32 && out.dtype == DType::BF16)   // Cast(bf16)(layer_norm(x f32)) folded
+                k::layer_norm_f32_to_bf16(s, src_ptr(st, cx, 0), src_ptr(st, cx, 1), src_ptr(st, cx, 2), dst, n ? x.count() / n : 0, n, in.scale, in.eps);
+            else
+                k::layer_norm(s, (int)out.dtype, src_ptr(st, cx, 0), src_ptr(st, cx, 1), src_ptr(st, cx, 2), dst, n ? x.count() / n : 0, n, in.scale, in.eps);
             ++cx.launches;
             break;
         }
@@ -1144,6 +1155,8 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                     if (in.quant) ma.scale2 = cx.input_bufs[st.tiled_s2_input]->ptr;
                 }
                 if (in.has_bias) ma.bias = src_ptr(st, cx, oi++);
+                if (in.has_scale) ma.extra.colscale = (const float*)src_ptr(st, cx, oi++);
+                ma.extra.glu = linear_glu(in);
                 if (in.has_residual) ma.residual = src_ptr(st, cx, oi++);
                 ma.y = dst;
                 ma.act = in.act == 1 ? 1 : 0;
@@ -1190,12 +1203,15 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                     if (in.quant) sa.scale2 = src_ptr(st, cx, 4);
                 }
                 if (in.has_bias) sa.bias = src_ptr(st, cx, oi++);
+                if (in.has_scale) sa.extra.colscale = (const float*)src_ptr(st, cx, oi++);
+                sa.extra.glu = linear_glu(in);
                 if (in.has_residual) sa.residual = src_ptr(st, cx, oi++);
                 const size_t norm_bytes = in.norm ? align_up((size_t)x.count() * dtype_size(x.dtype)) : 0;
                 if (in.norm) {
                     void* xn = cx.ws + st.scratch_off;
                     if (in.norm_ln) {
-                        k::layer_norm(s, (int)ldt, sa.x, src_ptr(st, cx, oi), src_ptr(st, cx, oi + 1), xn, sa.m, sa.k, in.scale, in.eps);
+                        if (in.x_f32) k::layer_norm_f32_to_bf16(s, sa.x, src_ptr(st, cx, oi), src_ptr(st, cx, oi + 1), xn, sa.m, sa.k, in.scale, in.eps);
+                        else k::layer_norm(s, (int)ldt, sa.x, src_ptr(st, cx, oi), src_ptr(st, cx, oi + 1), xn, sa.m, sa.k, in.scale, in.eps);
                         oi += 2;
                         ++cx.launches;
                     } else {
@@ -1243,6 +1259,8 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                     ++oi;
                 }
                 if (in.has_bias) ta.bias = src_ptr(st, cx, oi++);
+                if (in.has_scale) ta.extra.colscale = (const float*)src_ptr(st, cx, oi++);
+                ta.extra.glu = linear_glu(in);
                 if (in.has_residual) ta.residual = src_ptr(st, cx, oi++);
                 if (in.norm) { ta.gamma = src_ptr(st, cx, oi++); ta.inv_n = in.scale; ta.eps = in.eps; }
                 if (in.norm_ln) ta.beta = src_ptr(st, cx, oi++);
@@ -1264,6 +1282,8 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                 ++cx.launches;
                 break;
             }
+            // (an absorbed column factor or clamped pair runs on the kernels above only: the fusion pass sees to it)
+            if (in.has_scale || in.glu) fail_exec("linear: column factors or a clamped pair on the generic kernel");
             k::LinearArgs a{};
             a.dtype = (int)ldt;
             a.x = src_ptr(st, cx, 0);
