@@ -772,6 +772,232 @@ struct Fuser {
         }
     }
 
+    // ---------------------------------------------------------------- sequence mixers
+    // The calls of one mixer layer, for one sequence or for every sequence of a batch, become one instruction.
+    const Instr* mixer(int v, Mix mix) const {
+        const Instr* p = producer(v);
+        return p && !p->dead && p->op == OpKind::FMixer && p->mix == mix && p->out_ids[0] == v ? p : nullptr;
+    }
+    // v = rows [r0, r0 + n) of src (all columns); src itself counts as rows [0, n)
+    bool rows_of(int v, int src, int64_t& r0, int64_t& n) const {
+        const Spec* vs = spec_of(v);
+        if (!vs || vs->rank() != 2) return false;
+        n = vs->dims[0];
+        r0 = 0;
+        if (v == src) return true;
+        const Instr* p = producer(v);
+        const Spec* ss = spec_of(src);
+        if (!p || p->op != OpKind::Slice || p->operands[0].value != src || !ss || ss->rank() != 2) return false;
+        r0 = p->a[0];
+        return p->a[1] == 0 && p->b[1] == ss->dims[1];
+    }
+    int rows_source(int v) const {
+        const Instr* p = producer(v);
+        return p && p->op == OpKind::Slice ? p->operands[0].value : v;
+    }
+    // elements [at, at + n) of a vector
+    bool elements_of(int v, int src, int64_t at, int64_t n) const {
+        const Spec* vs = spec_of(v);
+        if (!vs || vs->dims != std::vector<int64_t>{n}) return false;
+        if (v == src) return at == 0;
+        const Instr* p = producer(v);
+        return p && p->op == OpKind::Slice && p->operands[0].value == src && p->a == std::vector<int64_t>{at};
+    }
+    int vector_source(int v) const { return rows_source(v); }
+    // the values stacked into v: the operands of Concat_0, or v alone
+    std::vector<int> stacked(int v) const {
+        std::vector<int> out;
+        const Instr* p = producer(v);
+        if (p && !p->dead && p->op == OpKind::Concat && p->axis == 0) {
+            for (const Operand& o : p->operands) {
+                if (o.value < 0) return {};
+                out.push_back(o.value);
+            }
+            return out;
+        }
+        return {v};
+    }
+    int find_mixer(Mix mix, const std::vector<int>& operands) const {   // value of a live call with these operands, or -1
+        for (const Instr& in : fn.body) {
+            if (in.dead || in.op != OpKind::FMixer || in.mix != mix || in.operands.size() != operands.size()) continue;
+            bool same = true;
+            for (size_t i = 0; i < operands.size() && same; ++i) same = in.operands[i].value == operands[i];
+            if (same) return in.out_ids[0];
+        }
+        return -1;
+    }
+    static void add_out(Instr& ni, int id, const Spec& s) { ni.out_ids.push_back(id); ni.out_specs.push_back(s); }
+
+    // Gated norm over the stacked rows of scans over convolutions of rows of one projection, with the calls that leave the
+    // new states -> Mix::SsmSeq (p, taps, bias, dt_bias, a_log, d, gain, conv_0, state_0, conv_1, ..) -> (rows, conv'_0,
+    // state'_0, ..)
+    void pass_ssm() {
+        for (size_t gi = 0; gi < fn.body.size(); ++gi) {
+            if (fn.body[gi].dead || fn.body[gi].op != OpKind::FMixer || fn.body[gi].mix != Mix::GatedNorm) continue;
+            const Instr g = fn.body[gi];
+            const std::vector<int> uses = count_uses();
+            const int y = g.operands[0].value, P = g.operands[1].value;
+            const std::vector<int> parts = stacked(y);
+            if (parts.empty() || uses[y] != 1) continue;
+            Instr ni = make(OpKind::FMixer, "fused.ssm_mixer", {P}, g.out_ids[0], g.out_specs[0]);
+            ni.mix = Mix::SsmSeq;
+            std::vector<int> dead;
+            int64_t row = 0;
+            bool ok = true;
+            const Instr *s0 = nullptr, *c0 = nullptr;
+            for (size_t b = 0; b < parts.size() && ok; ++b) {
+                const Instr* sc = mixer(parts[b], Mix::SsmScan);
+                ok = sc && uses[parts[b]] == 1;
+                if (!ok) break;
+                const int xbc = sc->operands[0].value, pb = sc->operands[1].value;
+                const Instr* cv = mixer(xbc, Mix::ConvSilu);
+                int64_t r0, n;
+                ok = cv && uses[xbc] == 2 && cv->operands[0].value == pb && rows_of(pb, P, r0, n) && r0 == row;
+                if (!ok) break;
+                row += n;
+                const int st = sc->operands[5].value, cs = cv->operands[3].value;
+                const int cs2 = find_mixer(Mix::ConvState, {pb, cs});
+                const int st2 = find_mixer(Mix::SsmState, {xbc, pb, sc->operands[2].value, sc->operands[3].value, st});
+                ok = cs2 >= 0 && st2 >= 0;
+                if (!ok) break;
+                const Instr *ic = producer(cs2), *is = producer(st2);
+                ok = ic->mx.col == cv->mx.col && is->mx.groups == sc->mx.groups && is->mx.dt_col == sc->mx.dt_col;
+                if (b == 0) {
+                    s0 = sc; c0 = cv;
+                    for (int v : {cv->operands[1].value, cv->operands[2].value, sc->operands[2].value, sc->operands[3].value, sc->operands[4].value, g.operands[2].value}) {
+                        Operand o; o.value = v;
+                        ni.operands.push_back(o);
+                    }
+                }
+                for (size_t o = 1; o < 3 && ok; ++o) ok = cv->operands[o].value == c0->operands[o].value;
+                for (size_t o = 2; o < 5 && ok; ++o) ok = sc->operands[o].value == s0->operands[o].value;
+                ok = ok && cv->mx.col == c0->mx.col && sc->mx.groups == s0->mx.groups && sc->mx.dt_col == s0->mx.dt_col &&
+                     ic->out_specs[0] == *spec_of(cs) && sc->mx.heads == s0->mx.heads && sc->mx.state == s0->mx.state && sc->mx.vdim == s0->mx.vdim;
+                if (!ok) break;
+                for (int v : {cs, st}) { Operand o; o.value = v; ni.operands.push_back(o); }
+                add_out(ni, cs2, ic->out_specs[0]);
+                add_out(ni, st2, is->out_specs[0]);
+                ni.lens.push_back(n);
+                for (int v : {parts[b], xbc, cs2, st2}) dead.push_back(v);
+            }
+            if (!ok || row != g.out_specs[0].dims[0]) continue;
+            ni.mx = s0->mx;
+            ni.mx.taps = c0->mx.taps; ni.mx.dim = c0->mx.dim; ni.mx.col = c0->mx.col;
+            ni.mx.z_col = g.mx.col; ni.mx.rank = g.mx.groups;
+            ni.eps = g.eps;
+            if (ni.mx.dim != ni.mx.heads * ni.mx.vdim + 2 * ni.mx.groups * ni.mx.state || g.mx.dim != ni.mx.heads * ni.mx.vdim) continue;
+            for (int v : dead) kill(v);
+            if (parts[0] != y) kill(y);
+            fn.body[gi] = ni;
+            ++fused;
+            reindex();
+        }
+    }
+
+    // Latent attention.  Decode (one row per sequence): the attentions of a batch, the rotation of their queries and, where
+    // the layer has a cache of its own, the forming and writing of the step's cache rows -> Mix::LatentDecode
+    //   (x, table, w_uk, w_uv, pos, [raw, gain, starts,] cache_0, cache_1, ..) -> (ctx[, cache'_0, ..])
+    // Prompts: Mix::LatentPrefill (x, table, k, v, rows) -> ctx, x the unrotated queries.
+    void pass_latent() {
+        for (size_t ai = 0; ai < fn.body.size(); ++ai) {
+            if (fn.body[ai].dead) continue;
+            const Instr root = fn.body[ai];
+            const bool lone = root.op == OpKind::FMixer && (root.mix == Mix::LatentAttn || root.mix == Mix::LatentAttnX);
+            if (!lone && !(root.op == OpKind::Concat && root.axis == 0)) continue;
+            const std::vector<int> uses = count_uses();
+            const int rv = root.out_ids[0];
+            if (lone) {   // an attention that a Concat stacks is taken with its batch
+                bool stacked_by = false;
+                for (const Instr& in : fn.body)
+                    if (!in.dead && in.op == OpKind::Concat && in.axis == 0)
+                        for (const Operand& o : in.operands) stacked_by = stacked_by || o.value == rv;
+                if (stacked_by) continue;
+            }
+            const std::vector<int> parts = lone ? std::vector<int>{rv} : stacked(rv);
+            if (parts.empty()) continue;
+            const Instr* a0 = producer(parts[0]);
+            if (!a0 || a0->op != OpKind::FMixer || (a0->mix != Mix::LatentAttn && a0->mix != Mix::LatentAttnX)) continue;
+            const bool x = a0->mix == Mix::LatentAttnX;
+            const int Q = rows_source(a0->operands[0].value);
+            const Instr* rp = mixer(Q, Mix::RopePairs);
+            if (!rp || rp->mx.col != a0->mx.dim || rp->mx.heads != a0->mx.heads || rp->mx.rot != a0->mx.rot) continue;
+            const int table = rp->operands[1].value;
+            bool ok = true;
+            int64_t row = 0;
+            std::vector<int64_t> lens;
+            int K = -1, V = -1, R = -1, pos = -1, starts = -1, lr = -1;
+            std::vector<int> caches, bases, dead;
+            bool append = !x;
+            for (size_t b = 0; b < parts.size() && ok; ++b) {
+                const Instr* at = mixer(parts[b], a0->mix);
+                ok = at && (lone || uses[parts[b]] == 1) && at->mx.heads == a0->mx.heads && at->mx.rot == a0->mx.rot && at->scale == a0->scale;
+                int64_t r0, n, r1, m;
+                ok = ok && rows_of(at->operands[0].value, Q, r0, n) && r0 == row;
+                if (!ok) break;
+                if (x) {
+                    if (b == 0) { K = rows_source(at->operands[1].value); V = rows_source(at->operands[2].value); R = rows_source(at->operands[3].value); }
+                    for (int o = 1; o < 4 && ok; ++o) ok = rows_of(at->operands[o].value, o == 1 ? K : (o == 2 ? V : R), r1, m) && r1 == row && m == n;
+                } else {
+                    ok = n == 1 && at->operands[2].value == a0->operands[2].value && at->operands[3].value == a0->operands[3].value;
+                    if (b == 0) pos = vector_source(at->operands[4].value);
+                    ok = ok && elements_of(at->operands[4].value, pos, (int64_t)b, 1);
+                    const Spec* ps = spec_of(pos);
+                    ok = ok && ps && ps->dims == std::vector<int64_t>{(int64_t)parts.size()};
+                    const int cv = at->operands[1].value;
+                    ok = ok && spec_of(cv) && *spec_of(cv) == *spec_of(a0->operands[1].value);
+                    caches.push_back(cv);
+                    // the cache as a DynamicUpdateSlice of this step's row
+                    const Instr* du = producer(cv);
+                    append = append && du && !du->dead && du->op == OpKind::DynamicUpdateSlice && du->out_ids[0] == cv && du->operands[0].value >= 0 &&
+                             du->a == std::vector<int64_t>{1, 1, at->mx.rank + at->mx.rot};
+                    int rs = -1;
+                    append = append && reshape_of(du->operands[1].value, rs) && uses[du->operands[1].value] == 1;
+                    if (append) {
+                        if (b == 0) { lr = rows_source(rs); starts = vector_source(du->operands[2].value); }
+                        const Instr* li = mixer(lr, Mix::LatentRows);
+                        const Spec* ss = spec_of(starts);
+                        append = li && li->operands[2].value == table && rows_of(rs, lr, r1, m) && r1 == (int64_t)b && m == 1 &&
+                                 elements_of(du->operands[2].value, starts, 3 * (int64_t)b, 3) && ss && ss->dims == std::vector<int64_t>{3 * (int64_t)parts.size()} &&
+                                 uses[lr] == (int)parts.size();
+                        bases.push_back(du->operands[0].value);
+                    }
+                }
+                row += n;
+                lens.push_back(n);
+                if (!lone) dead.push_back(parts[b]);
+            }
+            if (!ok || row != root.out_specs[0].dims[0]) continue;
+            Instr ni = make(OpKind::FMixer, x ? "fused.latent_prefill" : "fused.latent_decode", {rp->operands[0].value, table}, rv, root.out_specs[0]);
+            ni.mix = x ? Mix::LatentPrefill : Mix::LatentDecode;
+            ni.mx = a0->mx;
+            ni.scale = a0->scale;
+            ni.lens = lens;
+            auto add = [&](int v) { Operand o; o.value = v; ni.operands.push_back(o); };
+            if (x) {
+                add(K); add(V); add(R);
+            } else {
+                add(a0->operands[2].value); add(a0->operands[3].value); add(pos);
+                ni.append = append;
+                if (append) {
+                    const Instr* li = producer(lr);
+                    ni.eps = li->eps;
+                    add(li->operands[0].value); add(li->operands[1].value); add(starts);
+                    for (size_t b = 0; b < parts.size(); ++b) {
+                        add(bases[b]);
+                        add_out(ni, caches[b], *spec_of(caches[b]));
+                    }
+                    for (int v : caches) dead.push_back(v);
+                } else {
+                    for (int v : caches) add(v);
+                }
+            }
+            for (int v : dead) kill(v);
+            fn.body[ai] = ni;
+            ++fused;
+            reindex();
+        }
+    }
+
     // ---------------------------------------------------------------- linear layers
     std::vector<int> count_uses() const {
         std::vector<int> uses(fn.max_value_id + 1, 0);
@@ -1276,6 +1502,9 @@ int fuse_function(Function& fn) {
     f.pass_rope_into_attention();
     f.dce();
     f.pass_attention_batch();
+    f.dce();
+    f.pass_ssm();
+    f.pass_latent();
     f.dce();
     f.pass_linear();
     f.dce();

@@ -398,6 +398,54 @@ void ssm_scan(hipStream_t s, const SsmArgs& a);
 // y T [rows, n] = rms-normed in `groups` equal parts of (y * silu(p[:, col ..])), times gain[n]
 void gated_rms_norm(hipStream_t s, int dtype, const void* y, const float* p, const float* gain, void* out, int64_t rows, int64_t n, int64_t ld,
                     int64_t col, int64_t groups, float eps);
+// The whole mixer for up to kMixerBatch sequences of one launch series (Mix::SsmSeq): sequence b owns the rows [row0[b],
+// row0[b] + len[b]) of p and y.  out T [rows, inner].  scratch: ssm_seq_scratch_bytes().  Returns the number of launches.
+constexpr int kMixerBatch = 16;
+struct SsmSeqArgs {
+    int dtype;
+    const float* p; const float* taps; const float* bias; const float* dt_bias; const float* a_log; const float* d; const float* gain;
+    void* out;
+    int64_t rows, ld, col, ch, ntaps, dt_col, z_col, heads, groups, n, vdim, norm_groups;
+    float eps;
+    int nseq;
+    int row0[kMixerBatch], len[kMixerBatch];
+    const float* conv_in[kMixerBatch]; float* conv_out[kMixerBatch];
+    const float* state_in[kMixerBatch]; float* state_out[kMixerBatch];
+    void* scratch;
+};
+size_t ssm_seq_scratch_bytes(int dtype, int64_t rows, int64_t heads, int64_t groups, int64_t n, int64_t vdim);
+int ssm_seq(hipStream_t s, const SsmSeqArgs& a);
+
+// One decode step of latent attention for up to kMixerBatch sequences (Mix::LatentDecode): x T [nseq, heads * (dim + rot)]
+// unrotated queries, table f32 [nseq, rot]; with raw the step's row is formed (latent_rows) and written at row
+// starts[3 b + 1] of cache b first.  Sequence b attends rows 0 .. pos[b].
+struct LatentDecodeArgs {
+    int dtype;
+    const void* x; const float* table; const void* w_uk; const void* w_uv; const int32_t* pos;
+    const float* raw; const float* gain; const int32_t* starts;
+    void* cache[kMixerBatch];
+    void* ctx;
+    int64_t nseq, capacity, heads, dim, rot, rank, vdim;
+    float scale, eps;
+    void* scratch;
+};
+size_t latent_decode_scratch_bytes(int dtype, int64_t nseq, int64_t capacity, int64_t heads, int64_t dim, int64_t rot, int64_t rank);
+int latent_decode(hipStream_t s, const LatentDecodeArgs& a);
+
+// Causal latent attention of whole prompts (Mix::LatentPrefill), nseq sequences stacked: x T [rows, heads * (dim + rot)]
+// unrotated queries, k / v / rows as in LatentAttnXArgs.
+struct LatentPrefillArgs {
+    int dtype;
+    const void* x; const float* table; const void* k; const void* v; const void* rows;
+    void* ctx;
+    int64_t total, heads, dim, rot, rank, vdim;
+    float scale;
+    int nseq;
+    int row0[kMixerBatch], len[kMixerBatch];
+    void* scratch;
+};
+size_t latent_prefill_scratch_bytes(int dtype, int64_t total, int64_t heads, int64_t dim, int64_t rot, int64_t vdim);
+int latent_prefill(hipStream_t s, const LatentPrefillArgs& a);
 void clamped_glu(hipStream_t s, int dtype, const void* gate, const void* up, void* y, int64_t n, const GluParams& p);
 
 }  // namespace k

@@ -1,7 +1,12 @@
 // Latent attention: keys and values of all heads are linear images of one cached row per position, [latent | rotated key
 // part].  Also the rotation tables and the interleaved (pairwise) rotation it uses.
 //
+// The second part are the launches of Mix::LatentDecode and Mix::LatentPrefill (bf16; f32 and sizes outside their tilings run
+// the stand-alone kernels sequence by sequence).
+//
 // This file's first part are the stand-alone kernels of the CustomCall targets, for any sizes and either element type.
+#include <algorithm>
+
 #include "kernels.hpp"
 #include "device_utils.hpp"
 
@@ -40,15 +45,18 @@ __global__ __launch_bounds__(256) void rope_pairs_kernel(const T* __restrict__ x
     Elem<T>::st(y, 2 * i + 1, v);
 }
 
-// Workgroup = row.
+// Workgroup = row.  starts (one row): the row goes to place starts[1] of y, which holds `capacity` rows.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_rows_kernel(const float* __restrict__ raw, const float* __restrict__ gain, const float* __restrict__ table,
-                                                          T* __restrict__ y, int64_t rank, int64_t half, float eps) {
+                                                          T* __restrict__ y, int64_t rank, int64_t half, float eps, const int32_t* __restrict__ starts,
+                                                          int64_t capacity) {
     __shared__ float red[16];
     const int64_t w = rank + 2 * half;
     const float* row = raw + (int64_t)blockIdx.x * w;
     const float* tab = table + (int64_t)blockIdx.x * 2 * half;
-    T* out = y + (int64_t)blockIdx.x * w;
+    int64_t at = blockIdx.x;
+    if (starts) at = starts[1] < 0 ? 0 : (starts[1] > capacity - 1 ? capacity - 1 : starts[1]);
+    T* out = y + at * w;
     float q = 0.f;
     for (int64_t i = threadIdx.x; i < rank; i += 256) q += row[i] * row[i];
     const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)rank + eps);
@@ -160,6 +168,266 @@ __global__ __launch_bounds__(256) void latent_attn_x_kernel(LatentAttnXArgs a) {
     for (int64_t v = t; v < a.vdim; v += 256) Elem<T>::st((T*)a.ctx, (i * a.heads + h) * a.vdim + v, acc[v] * inv);
 }
 
+// ---------------------------------------------------------------------------- decode (bf16)
+typedef __bf16 bf16x8_l __attribute__((ext_vector_type(8)));
+typedef float f32x4_l __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4_l __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ f32x4_l mma16(const u32x4_l& a, const u32x4_l& b, f32x4_l c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_l, a), __builtin_bit_cast(bf16x8_l, b), c, 0, 0, 0);
+}
+// sum over the 16 lanes of a row, in every lane of it
+__device__ __forceinline__ float row16_sum(float v) {
+    int x = __float_as_int(v);
+#define GPTRS_DPP_ADD(ctrl) x = __float_as_int(__int_as_float(x) + __int_as_float(__builtin_amdgcn_update_dpp(0, x, (ctrl), 0xf, 0xf, false)))
+    GPTRS_DPP_ADD(0xB1);    // quad_perm [1,0,3,2]
+    GPTRS_DPP_ADD(0x4E);    // quad_perm [2,3,0,1]
+    GPTRS_DPP_ADD(0x141);   // row_half_mirror
+    GPTRS_DPP_ADD(0x140);   // row_mirror
+#undef GPTRS_DPP_ADD
+    return __int_as_float(x);
+}
+__device__ __forceinline__ float row16_max(float v) {
+    int x = __float_as_int(v);
+#define GPTRS_DPP_MAX(ctrl) x = __float_as_int(fmaxf(__int_as_float(x), __int_as_float(__builtin_amdgcn_update_dpp(0, x, (ctrl), 0xf, 0xf, false))))
+    GPTRS_DPP_MAX(0xB1);
+    GPTRS_DPP_MAX(0x4E);
+    GPTRS_DPP_MAX(0x141);
+    GPTRS_DPP_MAX(0x140);
+#undef GPTRS_DPP_MAX
+    return __int_as_float(x);
+}
+
+constexpr int kPrepRows = 64;    // latent dimensions per workgroup of the query part
+constexpr int kTileP = 64;       // cache rows per step of the attention part
+constexpr int kHeadTile = 16;
+
+// Blocks [0, heads * rank / 64): W_uk^T q_n of one head and 64 latent dimensions, for every sequence (the first of a head
+// also rotates the q_r part); blocks behind them, one per sequence: the step's cache row.
+// ql bf16 [nseq][heads][rank + rot].
+__global__ __launch_bounds__(256) void latent_prep_kernel(LatentDecodeArgs a, bf16_t* __restrict__ ql) {
+    extern __shared__ float lat_lds[];
+    const int t = threadIdx.x;
+    const int rank = (int)a.rank, rot = (int)a.rot, dim = (int)a.dim, H = (int)a.heads, hd = dim + rot, w = rank + rot;
+    const int rc = (rank + kPrepRows - 1) / kPrepRows;
+    if ((int)blockIdx.x >= H * rc) {
+        float* red = lat_lds;
+        const int b = blockIdx.x - H * rc;
+        const float* raw = a.raw + (int64_t)b * w;
+        const float* tab = a.table + (int64_t)b * rot;
+        int64_t at = a.starts[3 * b + 1];
+        at = at < 0 ? 0 : (at > a.capacity - 1 ? a.capacity - 1 : at);
+        bf16_t* out = (bf16_t*)a.cache[b] + at * w;
+        float q = 0.f;
+        for (int i = t; i < rank; i += 256) q += raw[i] * raw[i];
+        const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)rank + a.eps);
+        for (int i = t; i < rank; i += 256) out[i] = f32_to_bf16((raw[i] * inv) * a.gain[i]);
+        for (int i = t; i < rot / 2; i += 256) {
+            const float u = raw[rank + 2 * i], v = raw[rank + 2 * i + 1], c = tab[i], s = tab[rot / 2 + i];
+            out[rank + 2 * i] = f32_to_bf16(u * c - v * s);
+            out[rank + 2 * i + 1] = f32_to_bf16(v * c + u * s);
+        }
+        return;
+    }
+    const int h = blockIdx.x / rc, r0 = (blockIdx.x % rc) * kPrepRows;
+    const int l16 = t & 15, g = t >> 4;          // 16 groups of 16 lanes; a group takes latent dimensions r0 + g + 16 j
+    float* q = lat_lds;                          // [nseq][dim]
+    for (int i = t; i < (int)a.nseq * dim; i += 256)
+        q[i] = bf16_to_f32(((const bf16_t*)a.x)[((int64_t)(i / dim) * H + h) * hd + i % dim]);
+    if (r0 == 0)
+        for (int i = t; i < (int)a.nseq * (rot / 2); i += 256) {
+            const int b = i / (rot / 2), j = i % (rot / 2);
+            const bf16_t* xr = (const bf16_t*)a.x + ((int64_t)b * H + h) * hd + dim;
+            const float u = bf16_to_f32(xr[2 * j]), v = bf16_to_f32(xr[2 * j + 1]);
+            const float c = a.table[(int64_t)b * rot + j], s = a.table[(int64_t)b * rot + rot / 2 + j];
+            bf16_t* o = ql + ((int64_t)b * H + h) * w + rank;
+            o[2 * j] = f32_to_bf16(u * c - v * s);
+            o[2 * j + 1] = f32_to_bf16(v * c + u * s);
+        }
+    __syncthreads();
+    const bf16_t* wk = (const bf16_t*)a.w_uk;
+    const int64_t ldw = (int64_t)H * dim;
+    constexpr int J = kPrepRows / 16;
+    for (int b = 0; b < (int)a.nseq; ++b) {
+        float s[J];
+#pragma unroll
+        for (int j = 0; j < J; ++j) s[j] = 0.f;
+        for (int d = l16 * 8; d < dim; d += 128) {
+            float qv[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) qv[e] = q[b * dim + d + e];
+#pragma unroll
+            for (int j = 0; j < J; ++j) {
+                const int r = r0 + g + 16 * j;
+                if (r >= rank) continue;
+                const uint4 v = *reinterpret_cast<const uint4*>(wk + r * ldw + (int64_t)h * dim + d);
+                const uint32_t vw[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { s[j] += qv[2 * e] * bf16lo(vw[e]); s[j] += qv[2 * e + 1] * bf16hi(vw[e]); }
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const float tot = row16_sum(s[j]);
+            const int r = r0 + g + 16 * j;
+            if (l16 == 0 && r < rank) ql[((int64_t)b * H + h) * w + r] = f32_to_bf16(tot);
+        }
+    }
+}
+
+// Workgroup = slice of the positions x 16 heads x sequence.  Tiles of 64 cache rows in LDS; scores on the matrix cores (wave w:
+// rows 16 w ..), softmax over the tile, weights split into a bf16 value and its remainder, weighted rows on the matrix cores
+// (wave w: latent dimensions 16 (w + 4 i) ..).  part f32 [nseq][heads][nsplit][rank + 2]: sums, maximum, weight.
+template <int RT>
+__global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ ql, float* __restrict__ part, int nsplit) {
+    extern __shared__ __align__(16) unsigned char lat_smem[];
+    const int rank = (int)a.rank, w = rank + (int)a.rot, H = (int)a.heads, ws = w + 8;   // LDS row stride
+    bf16_t* rows = reinterpret_cast<bf16_t*>(lat_smem);               // [64][ws]
+    bf16_t* qs = rows + kTileP * ws;                                  // [16][ws]
+    constexpr int PS = kTileP + 8;
+    bf16_t* ph = qs + kHeadTile * ws;                                 // [16][PS] weights
+    bf16_t* pl = ph + kHeadTile * PS;                                 // [16][PS] their remainders
+    float* sc = reinterpret_cast<float*>(pl + kHeadTile * PS);        // [16][64 + 1]
+    float* corr = sc + kHeadTile * (kTileP + 1);                      // [16]
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, c = lane & 15, kg = lane >> 4;
+    const int b = blockIdx.z, h0 = blockIdx.y * kHeadTile, sp = blockIdx.x;
+    const int n = min(max(a.pos[b], 0) + 1, (int)a.capacity);
+    const int per = ((n + nsplit - 1) / nsplit + 15) / 16 * 16;
+    const int p0 = sp * per, p1 = min(p0 + per, n);
+    const int hr = H - h0 < kHeadTile ? H - h0 : kHeadTile;           // heads that exist
+    float* rec = part + (((int64_t)b * H + h0) * nsplit + sp) * (rank + 2);
+    const int64_t rec_h = (int64_t)nsplit * (rank + 2);
+    if (p0 >= p1) {   // nothing falls to this slice: an empty record
+        for (int i = t; i < hr; i += 256) { rec[i * rec_h + rank] = -INFINITY; rec[i * rec_h + rank + 1] = 0.f; }
+        return;
+    }
+    const int wv = w / 8;                                             // 16-byte words per row
+    for (int i = t; i < kHeadTile * wv; i += 256) {
+        const int r = i / wv, k = i % wv;
+        const uint4 v = *reinterpret_cast<const uint4*>(ql + ((int64_t)b * H + h0 + (r < hr ? r : 0)) * w + 8 * k);
+        *reinterpret_cast<uint4*>(qs + r * ws + 8 * k) = v;
+    }
+    f32x4_l acc[RT];
+#pragma unroll
+    for (int i = 0; i < RT; ++i) acc[i] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.f;                             // of head 4 * wave + kg, in all its 16 lanes
+    const bf16_t* cache = (const bf16_t*)a.cache[b];
+    for (int q0 = p0; q0 < p1; q0 += kTileP) {
+        const int np = min(kTileP, p1 - q0);
+        const int npad = (np + 31) / 32 * 32;                         // the matrix cores take 32 rows at a time
+        __syncthreads();
+        for (int i = t; i < npad * wv; i += 256) {
+            const int r = i / wv, k = i % wv;
+            uint4 v = make_uint4(0u, 0u, 0u, 0u);
+            if (r < np) v = *reinterpret_cast<const uint4*>(cache + (int64_t)(q0 + r) * w + 8 * k);
+            *reinterpret_cast<uint4*>(rows + r * ws + 8 * k) = v;
+        }
+        __syncthreads();
+        if (wave * 16 < npad) {
+            f32x4_l s = {0.f, 0.f, 0.f, 0.f};
+            for (int k = 0; k < w; k += 32)
+                s = mma16(*reinterpret_cast<const u32x4_l*>(qs + c * ws + k + 8 * kg), *reinterpret_cast<const u32x4_l*>(rows + (wave * 16 + c) * ws + k + 8 * kg), s);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) sc[(4 * kg + i) * (kTileP + 1) + wave * 16 + c] = s[i] * a.scale;
+        }
+        __syncthreads();
+        {   // head 4 * wave + kg: lanes c take rows c, c + 16, ..
+            const int h = 4 * wave + kg;
+            float v[4], mx = -INFINITY;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                v[i] = c + 16 * i < np ? sc[h * (kTileP + 1) + c + 16 * i] : -INFINITY;
+                mx = fmaxf(mx, v[i]);
+            }
+            const float mn = fmaxf(m_run, row16_max(mx));
+            float sum = 0.f;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const float p = expf(v[i] - mn);
+                const bf16_t hi = f32_to_bf16(p);
+                ph[h * PS + c + 16 * i] = hi;
+                pl[h * PS + c + 16 * i] = f32_to_bf16(p - bf16_to_f32(hi));
+                sum += p;
+            }
+            const float cr = expf(m_run - mn);
+            l_run = l_run * cr + row16_sum(sum);
+            m_run = mn;
+            if (c == 0) corr[h] = cr;
+        }
+        __syncthreads();
+        float cr[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) cr[i] = corr[4 * kg + i];
+#pragma unroll
+        for (int i = 0; i < RT; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) acc[i][e] *= cr[e];
+        for (int k = 0; k < npad; k += 32) {
+            const u32x4_l ah = *reinterpret_cast<const u32x4_l*>(ph + c * PS + k + 8 * kg), al = *reinterpret_cast<const u32x4_l*>(pl + c * PS + k + 8 * kg);
+#pragma unroll
+            for (int i = 0; i < RT; ++i) {
+                const int r = (wave + 4 * i) * 16;
+                if (r >= rank) break;
+                // column r + c of 8 consecutive rows
+                const bf16_t* src = rows + (k + 8 * kg) * ws + r + c;
+                u32x4_l bv;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) bv[e] = (uint32_t)src[2 * e * ws] | ((uint32_t)src[(2 * e + 1) * ws] << 16);
+                acc[i] = mma16(ah, bv, acc[i]);
+                acc[i] = mma16(al, bv, acc[i]);
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+        const int r = (wave + 4 * i) * 16 + c;
+        if (r >= rank) break;
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            if (4 * kg + e < hr) rec[(4 * kg + e) * rec_h + r] = acc[i][e];
+    }
+    if (c == 0 && 4 * wave + kg < hr) {
+        rec[(4 * wave + kg) * rec_h + rank] = m_run;
+        rec[(4 * wave + kg) * rec_h + rank + 1] = l_run;
+    }
+}
+
+constexpr int kOutV = 32;        // values per workgroup of the output part
+// Workgroup = head x 32 values x sequence: the slices' records merged into the weighted latent, times W_uv.
+__global__ __launch_bounds__(256) void latent_combine_kernel(LatentDecodeArgs a, const float* __restrict__ part, int nsplit) {
+    extern __shared__ float lat_lds[];
+    const int rank = (int)a.rank, vdim = (int)a.vdim, H = (int)a.heads;
+    float* lat = lat_lds;                        // [rank]
+    float* wgt = lat + rank;                     // [nsplit]
+    float* red = wgt + nsplit;                   // [256 / kOutV][kOutV]
+    const int t = threadIdx.x, h = blockIdx.x, v0 = blockIdx.y * kOutV, b = blockIdx.z;
+    const float* rec = part + ((int64_t)b * H + h) * nsplit * (rank + 2);
+    float m = -INFINITY, l = 0.f;
+    for (int s = 0; s < nsplit; ++s) m = fmaxf(m, rec[(int64_t)s * (rank + 2) + rank]);
+    for (int s = 0; s < nsplit; ++s) l += expf(rec[(int64_t)s * (rank + 2) + rank] - m) * rec[(int64_t)s * (rank + 2) + rank + 1];
+    if (t < nsplit) wgt[t] = expf(rec[(int64_t)t * (rank + 2) + rank] - m) / l;
+    __syncthreads();
+    for (int r = t; r < rank; r += 256) {
+        float v = 0.f;
+        for (int s = 0; s < nsplit; ++s)
+            if (wgt[s] != 0.f) v += wgt[s] * rec[(int64_t)s * (rank + 2) + r];   // (an empty slice left its sums unset)
+        lat[r] = v;
+    }
+    __syncthreads();
+    const int v = t % kOutV, g = t / kOutV;
+    const bf16_t* wv = (const bf16_t*)a.w_uv + (int64_t)h * vdim + v0 + v;
+    float s = 0.f;
+    if (v0 + v < vdim)
+        for (int r = g; r < rank; r += 256 / kOutV) s += lat[r] * bf16_to_f32(wv[(int64_t)r * H * vdim]);
+    red[g * kOutV + v] = s;
+    __syncthreads();
+    if (t < kOutV && v0 + t < vdim) {
+        float o = 0.f;
+        for (int q = 0; q < 256 / kOutV; ++q) o += red[q * kOutV + t];
+        ((bf16_t*)a.ctx)[((int64_t)b * H + h) * vdim + v0 + t] = f32_to_bf16(o);
+    }
+}
+
 template <typename F>
 void with_lds(F kern, size_t bytes) { (void)hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes); }
 
@@ -180,8 +448,13 @@ void rope_pairs(hipStream_t s, int dtype, const void* x, const float* table, voi
 void latent_rows(hipStream_t s, int dtype, const float* raw, const float* gain, const float* table, void* y, int64_t rows, int64_t rank, int64_t half,
                  float eps) {
     if (rows <= 0) return;
-    if (dtype == 0) latent_rows_kernel<float><<<(unsigned)rows, 256, 0, s>>>(raw, gain, table, (float*)y, rank, half, eps);
-    else latent_rows_kernel<bf16_t><<<(unsigned)rows, 256, 0, s>>>(raw, gain, table, (bf16_t*)y, rank, half, eps);
+    if (dtype == 0) latent_rows_kernel<float><<<(unsigned)rows, 256, 0, s>>>(raw, gain, table, (float*)y, rank, half, eps, nullptr, 0);
+    else latent_rows_kernel<bf16_t><<<(unsigned)rows, 256, 0, s>>>(raw, gain, table, (bf16_t*)y, rank, half, eps, nullptr, 0);
+}
+static void latent_append(hipStream_t s, int dtype, const float* raw, const float* gain, const float* table, const int32_t* starts, void* cache,
+                          int64_t capacity, int64_t rank, int64_t half, float eps) {
+    if (dtype == 0) latent_rows_kernel<float><<<1, 256, 0, s>>>(raw, gain, table, (float*)cache, rank, half, eps, starts, capacity);
+    else latent_rows_kernel<bf16_t><<<1, 256, 0, s>>>(raw, gain, table, (bf16_t*)cache, rank, half, eps, starts, capacity);
 }
 void latent_attn(hipStream_t s, const LatentAttnArgs& a) {
     if (a.t <= 0) return;
@@ -196,6 +469,95 @@ void latent_attn_expanded(hipStream_t s, const LatentAttnXArgs& a) {
     const dim3 grid((unsigned)a.t, (unsigned)a.heads);
     if (a.dtype == 0) { with_lds(latent_attn_x_kernel<float>, lds); latent_attn_x_kernel<float><<<grid, 256, lds, s>>>(a); }
     else { with_lds(latent_attn_x_kernel<bf16_t>, lds); latent_attn_x_kernel<bf16_t><<<grid, 256, lds, s>>>(a); }
+}
+
+
+static size_t lat_align(size_t n) { return (n + 255) / 256 * 256; }
+// slices of the positions: 32 rows each up to 32 of them, fewer where the batch fills the chip by itself
+static int latent_nsplit(int64_t nseq, int64_t capacity, int64_t heads) {
+    const int64_t blocks = nseq * cdiv_l(heads, kHeadTile);
+    int64_t n = std::min<int64_t>(cdiv_l(capacity, 32), 32);
+    while (n > 4 && blocks * n > 1024) n = (n + 1) / 2;
+    return (int)std::max<int64_t>(n, 1);
+}
+static size_t latent_partial_lds(int64_t w) {
+    return (size_t)((kTileP + kHeadTile) * (w + 8) + 2 * kHeadTile * (kTileP + 8)) * 2 + (kHeadTile * (kTileP + 1) + kHeadTile) * 4;
+}
+static bool latent_fast(int dtype, int64_t heads, int64_t dim, int64_t rot, int64_t rank) {
+    return dtype == 2 && heads >= 1 && dim % 8 == 0 && rot % 2 == 0 && rank % 16 == 0 && (rank + rot) % 32 == 0 && rank <= 1024 && dim <= 512 &&
+           latent_partial_lds(rank + rot) <= 160 * 1024;
+}
+size_t latent_decode_scratch_bytes(int dtype, int64_t nseq, int64_t capacity, int64_t heads, int64_t dim, int64_t rot, int64_t rank) {
+    if (latent_fast(dtype, heads, dim, rot, rank))
+        return lat_align((size_t)(nseq * heads * (rank + rot)) * 2) + (size_t)(nseq * heads * (rank + 2)) * 32 * sizeof(float);
+    const size_t es = dtype == 0 ? 4 : 2;
+    return lat_align((size_t)(nseq * heads * (dim + rot)) * es);
+}
+int latent_decode(hipStream_t s, const LatentDecodeArgs& a) {
+    const size_t es = a.dtype == 0 ? 4 : 2;
+    const int64_t w = a.rank + a.rot;
+    if (latent_fast(a.dtype, a.heads, a.dim, a.rot, a.rank)) {
+        bf16_t* ql = (bf16_t*)a.scratch;
+        float* part = (float*)((char*)a.scratch + lat_align((size_t)(a.nseq * a.heads * w) * 2));
+        const int ns = latent_nsplit(a.nseq, a.capacity, a.heads);
+        const int64_t rc = cdiv_l(a.rank, kPrepRows);
+        latent_prep_kernel<<<(unsigned)(a.heads * rc + (a.raw ? a.nseq : 0)), 256, (size_t)std::max<int64_t>(a.nseq * a.dim, 16) * 4, s>>>(a, ql);
+        const size_t lds = latent_partial_lds(w);
+        const dim3 grid((unsigned)ns, (unsigned)cdiv_l(a.heads, kHeadTile), (unsigned)a.nseq);
+        const int64_t rt = cdiv_l(a.rank / 16, 4);
+#define GPTRS_PARTIAL(RT) do { with_lds(latent_partial_kernel<RT>, lds); latent_partial_kernel<RT><<<grid, 256, lds, s>>>(a, ql, part, ns); } while (0)
+        if (rt <= 2) GPTRS_PARTIAL(2);
+        else if (rt <= 4) GPTRS_PARTIAL(4);
+        else if (rt <= 8) GPTRS_PARTIAL(8);
+        else GPTRS_PARTIAL(16);
+#undef GPTRS_PARTIAL
+        latent_combine_kernel<<<dim3((unsigned)a.heads, (unsigned)cdiv_l(a.vdim, kOutV), (unsigned)a.nseq), 256, (size_t)(a.rank + ns + 256) * 4, s>>>(a, part, ns);
+        return 3;
+    }
+    rope_pairs(s, a.dtype, a.x, a.table, a.scratch, a.nseq, a.heads, a.dim + a.rot, a.dim, a.rot / 2);
+    int n = 1;
+    for (int64_t b = 0; b < a.nseq; ++b) {
+        if (a.raw) {
+            latent_append(s, a.dtype, a.raw + b * w, a.gain, a.table + b * a.rot, a.starts + 3 * b, a.cache[b], a.capacity, a.rank, a.rot / 2, a.eps);
+            ++n;
+        }
+        LatentAttnArgs q{};
+        q.dtype = a.dtype;
+        q.q = (const char*)a.scratch + (size_t)(b * a.heads * (a.dim + a.rot)) * es;
+        q.rows = a.cache[b]; q.w_uk = a.w_uk; q.w_uv = a.w_uv; q.start = a.pos + b;
+        q.ctx = (char*)a.ctx + (size_t)(b * a.heads * a.vdim) * es;
+        q.t = 1; q.capacity = a.capacity; q.heads = a.heads; q.dim = a.dim; q.rot = a.rot; q.rank = a.rank; q.vdim = a.vdim; q.scale = a.scale;
+        latent_attn(s, q);
+        ++n;
+    }
+    return n;
+}
+
+size_t latent_prefill_scratch_bytes(int dtype, int64_t total, int64_t heads, int64_t dim, int64_t rot, int64_t vdim) {
+    (void)vdim;
+    return lat_align((size_t)(total * heads * (dim + rot)) * (dtype == 0 ? 4 : 2));
+}
+int latent_prefill(hipStream_t s, const LatentPrefillArgs& a) {
+    const size_t es = a.dtype == 0 ? 4 : 2;
+    const int64_t hd = a.heads * (a.dim + a.rot), w = a.rank + a.rot;
+    int n = 0;
+    for (int b = 0; b < a.nseq; ++b) {
+        const int64_t r = a.row0[b];
+        char* q = (char*)a.scratch + (size_t)(r * hd) * es;
+        rope_pairs(s, a.dtype, (const char*)a.x + (size_t)(r * hd) * es, a.table + r * a.rot, q, a.len[b], a.heads, a.dim + a.rot, a.dim, a.rot / 2);
+        LatentAttnXArgs x{};
+        x.dtype = a.dtype;
+        x.q = q;
+        x.k = (const char*)a.k + (size_t)(r * a.heads * a.dim) * es;
+        x.v = (const char*)a.v + (size_t)(r * a.heads * a.vdim) * es;
+        x.rows = (const char*)a.rows + (size_t)(r * w) * es;
+        x.ctx = (char*)a.ctx + (size_t)(r * a.heads * a.vdim) * es;
+        x.t = x.l = a.len[b];
+        x.heads = a.heads; x.dim = a.dim; x.rot = a.rot; x.rank = a.rank; x.vdim = a.vdim; x.scale = a.scale;
+        latent_attn_expanded(s, x);
+        n += 2;
+    }
+    return n;
 }
 
 }  // namespace k

@@ -17,6 +17,7 @@
 //
 // latent_attention: query i stands at position start + i.  latent_attention_expanded: the queries are the last R of the L
 // positions.  p is the f32 result of an input projection whose columns hold several inputs of the mixer.
+#include <algorithm>
 #include <cmath>
 #include <cstring>
 
@@ -195,13 +196,23 @@ void lower_mixer_calls(Function& fn) {
 }
 
 size_t mixer_scratch_bytes(const Instr& in, const std::vector<const Spec*>& operands) {
-    (void)in; (void)operands;
+    const Instr::MixAttrs& m = in.mx;
+    const int dt = (int)in.out_specs[0].dtype;
+    const int64_t rows = in.out_specs[0].rank() == 2 ? in.out_specs[0].dims[0] : 0;
+    if (in.mix == Mix::SsmSeq) return k::ssm_seq_scratch_bytes(dt, rows, m.heads, m.groups, m.state, m.vdim);
+    if (in.mix == Mix::LatentDecode)
+        return k::latent_decode_scratch_bytes(dt, std::min<int64_t>(rows, k::kMixerBatch), operands[in.append ? 8 : 5]->dims[1], m.heads, m.dim, m.rot, m.rank);
+    if (in.mix == Mix::LatentPrefill) return k::latent_prefill_scratch_bytes(dt, rows, m.heads, m.dim, m.rot, m.vdim);
     return 0;
 }
 
 std::vector<std::pair<int, int>> mixer_inplace_pairs(const Instr& in) {
-    (void)in;
-    return {};
+    std::vector<std::pair<int, int>> out;
+    if (in.mix == Mix::SsmSeq)
+        for (int b = 0; b < (int)in.lens.size(); ++b) { out.push_back({7 + 2 * b, 1 + 2 * b}); out.push_back({8 + 2 * b, 2 + 2 * b}); }
+    if (in.mix == Mix::LatentDecode && in.append)
+        for (int b = 0; b < (int)in.lens.size(); ++b) out.push_back({8 + b, 1 + b});
+    return out;
 }
 
 void run_mixer(const Plan& plan, const Step& st, ExecCtx& cx) {
@@ -283,6 +294,75 @@ void run_mixer(const Plan& plan, const Step& st, ExecCtx& cx) {
             p.kind = 1; p.limit = in.fparam[0]; p.alpha = in.fparam[1]; p.shift = in.fparam[2];
             k::clamped_glu(s, dt, ptr(0), ptr(1), dst, out.count(), p);
             ++cx.launches;
+            break;
+        }
+        case Mix::SsmSeq: {
+            int64_t row = 0;
+            for (size_t b0 = 0; b0 < in.lens.size(); b0 += k::kMixerBatch) {   // rows of the scratch are the rows of the batch
+                k::SsmSeqArgs a{};
+                a.dtype = dt;
+                a.p = f(0); a.taps = f(1); a.bias = f(2); a.dt_bias = f(3); a.a_log = f(4); a.d = f(5); a.gain = f(6);
+                a.out = dst;
+                a.ld = spec(0).dims[1]; a.col = m.col; a.ch = m.dim; a.ntaps = m.taps; a.dt_col = m.dt_col; a.z_col = m.z_col;
+                a.heads = m.heads; a.groups = m.groups; a.n = m.state; a.vdim = m.vdim; a.norm_groups = m.rank;
+                a.eps = in.eps;
+                a.nseq = (int)std::min<size_t>(in.lens.size() - b0, k::kMixerBatch);
+                for (int b = 0; b < a.nseq; ++b) {
+                    const int q = (int)b0 + b;
+                    a.row0[b] = (int)row;
+                    a.len[b] = (int)in.lens[q];
+                    row += in.lens[q];
+                    a.conv_in[b] = f(7 + 2 * q); a.state_in[b] = f(8 + 2 * q);
+                    a.conv_out[b] = (float*)cx.ptr[st.dst[1 + 2 * q]]; a.state_out[b] = (float*)cx.ptr[st.dst[2 + 2 * q]];
+                }
+                a.rows = row - a.row0[0];
+                a.scratch = cx.ws + st.scratch_off;
+                cx.launches += k::ssm_seq(s, a);
+            }
+            break;
+        }
+        case Mix::LatentDecode: {
+            const size_t c0 = in.append ? 8 : 5;
+            for (size_t b0 = 0; b0 < in.lens.size(); b0 += k::kMixerBatch) {
+                k::LatentDecodeArgs a{};
+                a.dtype = dt;
+                a.heads = m.heads; a.dim = m.dim; a.rot = m.rot; a.rank = m.rank; a.vdim = m.vdim; a.scale = in.scale; a.eps = in.eps;
+                a.nseq = (int64_t)std::min<size_t>(in.lens.size() - b0, k::kMixerBatch);
+                a.capacity = spec(c0).dims[1];
+                const size_t es = dtype_size(out.dtype);
+                a.x = (const char*)ptr(0) + b0 * (size_t)spec(0).dims[1] * es;
+                a.table = f(1) + b0 * m.rot;
+                a.w_uk = ptr(2); a.w_uv = ptr(3);
+                a.pos = (const int32_t*)ptr(4) + b0;
+                a.ctx = (char*)dst + b0 * (size_t)out.dims[1] * es;
+                if (in.append) { a.raw = f(5) + b0 * (m.rank + m.rot); a.gain = f(6); a.starts = (const int32_t*)ptr(7) + 3 * b0; }
+                for (int64_t b = 0; b < a.nseq; ++b) {
+                    const void* from = ptr(c0 + b0 + b);
+                    void* to = in.append ? cx.ptr[st.dst[1 + b0 + b]] : const_cast<void*>(from);
+                    if (to != from) {   // a cache that was not donated is copied first
+                        GPTRS_HIP_CHECK(hipMemcpyAsync(to, from, spec(c0).bytes(), hipMemcpyDeviceToDevice, s));
+                        ++cx.launches;
+                    }
+                    a.cache[b] = to;
+                }
+                a.scratch = cx.ws + st.scratch_off;
+                cx.launches += k::latent_decode(s, a);
+            }
+            break;
+        }
+        case Mix::LatentPrefill: {
+            int64_t row = 0;
+            for (size_t b0 = 0; b0 < in.lens.size(); b0 += k::kMixerBatch) {
+                k::LatentPrefillArgs a{};
+                a.dtype = dt;
+                a.x = ptr(0); a.table = f(1); a.k = ptr(2); a.v = ptr(3); a.rows = ptr(4); a.ctx = dst;
+                a.heads = m.heads; a.dim = m.dim; a.rot = m.rot; a.rank = m.rank; a.vdim = m.vdim; a.scale = in.scale;
+                a.total = out.dims[0];
+                a.nseq = (int)std::min<size_t>(in.lens.size() - b0, k::kMixerBatch);
+                for (int b = 0; b < a.nseq; ++b) { a.row0[b] = (int)row; a.len[b] = (int)in.lens[b0 + b]; row += in.lens[b0 + b]; }
+                a.scratch = cx.ws + st.scratch_off;
+                cx.launches += k::latent_prefill(s, a);
+            }
             break;
         }
         default:
