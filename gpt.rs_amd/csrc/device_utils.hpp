@@ -50,6 +50,59 @@ template <> struct Elem<bf16_t> {
     static __device__ __forceinline__ float round(float v) { return bf16_to_f32(f32_to_bf16(v)); }
 };
 
+// ---- 16 x 16 x 32 bf16 matrix-core tiles.  Operand: lane = 16 * k-group + row (A) or column (B) holds 8 consecutive k;
+// result: lane = 16 * kg + column holds rows 4 kg .. 4 kg + 3.
+typedef __bf16 bf16x8_m __attribute__((ext_vector_type(8)));
+typedef float f32x4_m __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4_m __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x2_m __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ f32x4_m mma16(const u32x4_m& a, const u32x4_m& b, f32x4_m c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_m, a), __builtin_bit_cast(bf16x8_m, b), c, 0, 0, 0);
+}
+// Operand whose k runs DOWN the rows of an LDS matrix m[k][..] (stride in elements, a multiple of 4; m 8-byte aligned): the
+// lane's row / column is m's column.  ds_read_b64_tr_b16 hands lane i of 16 the column i of 4 rows; lane 4 e + j of the 16 names
+// columns 4 j .. 4 j + 3 of row e.
+__device__ __forceinline__ u32x4_m lds_operand_t(const bf16_t* m, int stride, int lane) {
+    typedef short s16x4 __attribute__((ext_vector_type(4)));
+    typedef __attribute__((address_space(3))) s16x4* lds_p;
+    const int c = lane & 15, kg = lane >> 4;
+    const bf16_t* p = m + (8 * kg + (c >> 2)) * stride + 4 * (c & 3);
+    const u32x2_m lo = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)(p)));
+    const u32x2_m hi = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)(p + 4 * stride)));
+    u32x4_m r;
+    r.x = lo.x; r.y = lo.y; r.z = hi.x; r.w = hi.y;
+    return r;
+}
+// bf16 pair by the hardware converter (round to nearest even)
+__device__ __forceinline__ uint32_t pack_bf16_hw(float lo, float hi) {
+    typedef float f32x2_p __attribute__((ext_vector_type(2)));
+    typedef __bf16 bf16x2_p __attribute__((ext_vector_type(2)));
+    f32x2_p f;
+    f.x = lo; f.y = hi;
+    return __builtin_bit_cast(uint32_t, __builtin_convertvector(f, bf16x2_p));
+}
+// Sum / maximum over the 16 lanes of a row, in every lane of it
+__device__ __forceinline__ float row16_sum(float v) {
+    int x = __float_as_int(v);
+#define GPTRS_DPP_ADD(ctrl) x = __float_as_int(__int_as_float(x) + __int_as_float(__builtin_amdgcn_update_dpp(0, x, (ctrl), 0xf, 0xf, false)))
+    GPTRS_DPP_ADD(0xB1);    // quad_perm [1,0,3,2]
+    GPTRS_DPP_ADD(0x4E);    // quad_perm [2,3,0,1]
+    GPTRS_DPP_ADD(0x141);   // row_half_mirror
+    GPTRS_DPP_ADD(0x140);   // row_mirror
+#undef GPTRS_DPP_ADD
+    return __int_as_float(x);
+}
+__device__ __forceinline__ float row16_max(float v) {
+    int x = __float_as_int(v);
+#define GPTRS_DPP_MAX(ctrl) x = __float_as_int(fmaxf(__int_as_float(x), __int_as_float(__builtin_amdgcn_update_dpp(0, x, (ctrl), 0xf, 0xf, false))))
+    GPTRS_DPP_MAX(0xB1);
+    GPTRS_DPP_MAX(0x4E);
+    GPTRS_DPP_MAX(0x141);
+    GPTRS_DPP_MAX(0x140);
+#undef GPTRS_DPP_MAX
+    return __int_as_float(x);
+}
+
 // Sum over the 64 lanes of a wave, result in every lane.  Cross-lane moves use DPP modifiers
 // (register-to-register, VALU rate) instead of ds_bpermute: 16 x 6 bpermutes per thread at the end of
 // a GEMV block kept the LDS pipe busy for ~4 us.  Steps: xor 1 and xor 2 inside quads, mirrored

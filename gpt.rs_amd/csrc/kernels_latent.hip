@@ -169,35 +169,6 @@ __global__ __launch_bounds__(256) void latent_attn_x_kernel(LatentAttnXArgs a) {
 }
 
 // ---------------------------------------------------------------------------- decode (bf16)
-typedef __bf16 bf16x8_l __attribute__((ext_vector_type(8)));
-typedef float f32x4_l __attribute__((ext_vector_type(4)));
-typedef uint32_t u32x4_l __attribute__((ext_vector_type(4)));
-
-__device__ __forceinline__ f32x4_l mma16(const u32x4_l& a, const u32x4_l& b, f32x4_l c) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_l, a), __builtin_bit_cast(bf16x8_l, b), c, 0, 0, 0);
-}
-// sum over the 16 lanes of a row, in every lane of it
-__device__ __forceinline__ float row16_sum(float v) {
-    int x = __float_as_int(v);
-#define GPTRS_DPP_ADD(ctrl) x = __float_as_int(__int_as_float(x) + __int_as_float(__builtin_amdgcn_update_dpp(0, x, (ctrl), 0xf, 0xf, false)))
-    GPTRS_DPP_ADD(0xB1);    // quad_perm [1,0,3,2]
-    GPTRS_DPP_ADD(0x4E);    // quad_perm [2,3,0,1]
-    GPTRS_DPP_ADD(0x141);   // row_half_mirror
-    GPTRS_DPP_ADD(0x140);   // row_mirror
-#undef GPTRS_DPP_ADD
-    return __int_as_float(x);
-}
-__device__ __forceinline__ float row16_max(float v) {
-    int x = __float_as_int(v);
-#define GPTRS_DPP_MAX(ctrl) x = __float_as_int(fmaxf(__int_as_float(x), __int_as_float(__builtin_amdgcn_update_dpp(0, x, (ctrl), 0xf, 0xf, false))))
-    GPTRS_DPP_MAX(0xB1);
-    GPTRS_DPP_MAX(0x4E);
-    GPTRS_DPP_MAX(0x141);
-    GPTRS_DPP_MAX(0x140);
-#undef GPTRS_DPP_MAX
-    return __int_as_float(x);
-}
-
 constexpr int kPrepRows = 64;    // latent dimensions per workgroup of the query part
 constexpr int kTileP = 64;       // cache rows per step of the attention part
 constexpr int kHeadTile = 16;
@@ -307,9 +278,9 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a,
         const uint4 v = *reinterpret_cast<const uint4*>(ql + ((int64_t)b * H + h0 + (r < hr ? r : 0)) * w + 8 * k);
         *reinterpret_cast<uint4*>(qs + r * ws + 8 * k) = v;
     }
-    f32x4_l acc[RT];
+    f32x4_m acc[RT];
 #pragma unroll
-    for (int i = 0; i < RT; ++i) acc[i] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < RT; ++i) acc[i] = f32x4_m{0.f, 0.f, 0.f, 0.f};
     float m_run = -INFINITY, l_run = 0.f;                             // of head 4 * wave + kg, in all its 16 lanes
     const bf16_t* cache = (const bf16_t*)a.cache[b];
     for (int q0 = p0; q0 < p1; q0 += kTileP) {
@@ -324,9 +295,9 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a,
         }
         __syncthreads();
         if (wave * 16 < npad) {
-            f32x4_l s = {0.f, 0.f, 0.f, 0.f};
+            f32x4_m s = {0.f, 0.f, 0.f, 0.f};
             for (int k = 0; k < w; k += 32)
-                s = mma16(*reinterpret_cast<const u32x4_l*>(qs + c * ws + k + 8 * kg), *reinterpret_cast<const u32x4_l*>(rows + (wave * 16 + c) * ws + k + 8 * kg), s);
+                s = mma16(*reinterpret_cast<const u32x4_m*>(qs + c * ws + k + 8 * kg), *reinterpret_cast<const u32x4_m*>(rows + (wave * 16 + c) * ws + k + 8 * kg), s);
 #pragma unroll
             for (int i = 0; i < 4; ++i) sc[(4 * kg + i) * (kTileP + 1) + wave * 16 + c] = s[i] * a.scale;
         }
@@ -363,16 +334,12 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a,
 #pragma unroll
             for (int e = 0; e < 4; ++e) acc[i][e] *= cr[e];
         for (int k = 0; k < npad; k += 32) {
-            const u32x4_l ah = *reinterpret_cast<const u32x4_l*>(ph + c * PS + k + 8 * kg), al = *reinterpret_cast<const u32x4_l*>(pl + c * PS + k + 8 * kg);
+            const u32x4_m ah = *reinterpret_cast<const u32x4_m*>(ph + c * PS + k + 8 * kg), al = *reinterpret_cast<const u32x4_m*>(pl + c * PS + k + 8 * kg);
 #pragma unroll
             for (int i = 0; i < RT; ++i) {
                 const int r = (wave + 4 * i) * 16;
                 if (r >= rank) break;
-                // column r + c of 8 consecutive rows
-                const bf16_t* src = rows + (k + 8 * kg) * ws + r + c;
-                u32x4_l bv;
-#pragma unroll
-                for (int e = 0; e < 4; ++e) bv[e] = (uint32_t)src[2 * e * ws] | ((uint32_t)src[(2 * e + 1) * ws] << 16);
+                const u32x4_m bv = lds_operand_t(rows + k * ws + r, ws, lane);
                 acc[i] = mma16(ah, bv, acc[i]);
                 acc[i] = mma16(al, bv, acc[i]);
             }
@@ -426,6 +393,161 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentDecodeArgs a,
         for (int q = 0; q < 256 / kOutV; ++q) o += red[q * kOutV + t];
         ((bf16_t*)a.ctx)[((int64_t)b * H + h) * vdim + v0 + t] = f32_to_bf16(o);
     }
+}
+
+// ---------------------------------------------------------------------------- prompts (bf16)
+constexpr int kQTile = 128;      // queries per workgroup: 32 per wave, two 16-row operands that share every key operand
+constexpr int kKTile = 64;       // keys per step
+
+// Workgroup = 128 queries x head x sequence.  Keys [unrotated | shared rotated part] and values of 64 positions in LDS; scores,
+// online softmax in f32, weights as a bf16 value and its remainder, so that the products with the values see the f32
+// weights to 16 bits.  KS: dim + rot in steps of 32 (zero padded), VT: vdim in tiles of 16 (zero padded).
+template <int KS, int VT>
+__global__ __launch_bounds__(256, 1) void latent_prefill_kernel(LatentPrefillArgs a) {
+    extern __shared__ __align__(16) unsigned char lat_smem[];
+    constexpr int KSTR = KS * 32 + 8, VSTR = VT * 16 + 8, PSTR = kKTile + 8;
+    bf16_t* kt = reinterpret_cast<bf16_t*>(lat_smem);      // [64][KSTR]
+    bf16_t* vt = kt + kKTile * KSTR;                       // [64][VSTR]
+    bf16_t* pw = vt + kKTile * VSTR;                       // per wave: [2][32][PSTR]
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, c = lane & 15, kg = lane >> 4;
+    const int b = blockIdx.z, h = blockIdx.y, T = a.len[b], r0 = a.row0[b];
+    const int q0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * kQTile;   // the longest workgroups first
+    if (q0 >= T) return;
+    const int dim = (int)a.dim, rot = (int)a.rot, hd = dim + rot, vdim = (int)a.vdim, H = (int)a.heads, w = (int)(a.rank + a.rot);
+    bf16_t* ph = pw + wave * 2 * 32 * PSTR;
+    bf16_t* pl = ph + 32 * PSTR;
+
+    // queries: rotated on the way in, rounded once; rows behind the prompt repeat its last row and are not stored
+    u32x4_m q[2][KS];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int row = r0 + min(q0 + wave * 32 + i * 16 + c, T - 1);
+        const bf16_t* src = (const bf16_t*)a.x + ((int64_t)row * H + h) * hd;
+        const float* tab = a.table + (int64_t)row * rot;
+#pragma unroll
+        for (int k = 0; k < KS; ++k) {
+            const int d = 32 * k + 8 * kg;
+            u32x4_m v = {0u, 0u, 0u, 0u};
+            if (d < hd) {
+                v = *reinterpret_cast<const u32x4_m*>(src + d);
+                if (d >= dim) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        const float cs = tab[(d - dim) / 2 + e], sn = tab[rot / 2 + (d - dim) / 2 + e];
+                        const float x0 = bf16lo(v[e]), x1 = bf16hi(v[e]);
+                        v[e] = pack_bf16_hw(x0 * cs - x1 * sn, x1 * cs + x0 * sn);
+                    }
+                }
+            }
+            q[i][k] = v;
+        }
+    }
+    f32x4_m o[2][VT];
+    float m[2][4], l[2][4];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+#pragma unroll
+        for (int v = 0; v < VT; ++v) o[i][v] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { m[i][e] = -INFINITY; l[i][e] = 0.f; }
+    }
+    const float scale2 = a.scale * 1.44269504f;            // weights as powers of two
+    const int kend = min(q0 + kQTile, T);
+    const int myq = q0 + wave * 32;                        // the wave's first query
+    constexpr int KW = KS * 4, VW = VT * 2;                // 16-byte words per staged row
+    for (int k0 = 0; k0 < kend; k0 += kKTile) {
+        __syncthreads();
+        for (int i = t; i < kKTile * KW; i += 256) {
+            const int r = i / KW, d = (i % KW) * 8, pos = k0 + r;
+            uint4 v = make_uint4(0u, 0u, 0u, 0u);
+            if (pos < kend && d < hd)
+                v = d < dim ? *reinterpret_cast<const uint4*>((const bf16_t*)a.k + ((int64_t)(r0 + pos) * H + h) * dim + d)
+                            : *reinterpret_cast<const uint4*>((const bf16_t*)a.rows + (int64_t)(r0 + pos) * w + (int)a.rank + d - dim);
+            *reinterpret_cast<uint4*>(kt + r * KSTR + d) = v;
+        }
+        for (int i = t; i < kKTile * VW; i += 256) {
+            const int r = i / VW, d = (i % VW) * 8, pos = k0 + r;
+            uint4 v = make_uint4(0u, 0u, 0u, 0u);
+            if (pos < kend && d < vdim) v = *reinterpret_cast<const uint4*>((const bf16_t*)a.v + ((int64_t)(r0 + pos) * H + h) * vdim + d);
+            *reinterpret_cast<uint4*>(vt + r * VSTR + d) = v;
+        }
+        __syncthreads();
+        if (k0 > myq + 31) continue;                       // all keys of the step lie ahead of the wave's queries
+        f32x4_m s[2][4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            s[0][j] = s[1][j] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int k = 0; k < KS; ++k) {
+                const u32x4_m kv = *reinterpret_cast<const u32x4_m*>(kt + (16 * j + c) * KSTR + 32 * k + 8 * kg);
+                s[0][j] = mma16(q[0][k], kv, s[0][j]);
+                s[1][j] = mma16(q[1][k], kv, s[1][j]);
+            }
+        }
+        const bool edge = k0 + kKTile - 1 > myq;           // some key lies ahead of some query (or behind the prompt)
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int qi = myq + i * 16 + 4 * kg + e;
+                float x[4], mx = -INFINITY;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    x[j] = s[i][j][e] * scale2;
+                    if (edge && k0 + 16 * j + c > qi) x[j] = -INFINITY;
+                    mx = fmaxf(mx, x[j]);
+                }
+                const float mn = fmaxf(m[i][e], row16_max(mx));   // finite: key k0 <= myq + 31 may lie ahead of qi only after key 0 was seen
+                const float corr = __builtin_amdgcn_exp2f(m[i][e] - mn);
+                float sum = 0.f;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const float p = __builtin_amdgcn_exp2f(x[j] - mn);
+                    sum += p;
+                    const uint32_t hi = pack_bf16_hw(p, 0.f) & 0xFFFFu;
+                    ph[(i * 16 + 4 * kg + e) * PSTR + 16 * j + c] = (bf16_t)hi;
+                    pl[(i * 16 + 4 * kg + e) * PSTR + 16 * j + c] = (bf16_t)(pack_bf16_hw(p - __uint_as_float(hi << 16), 0.f) & 0xFFFFu);
+                }
+                l[i][e] = l[i][e] * corr + row16_sum(sum);
+                m[i][e] = mn;
+#pragma unroll
+                for (int v = 0; v < VT; ++v) o[i][v][e] *= corr;
+            }
+        }
+        // (the weights are the wave's own: its LDS operations complete in order)
+        asm volatile("" ::: "memory");
+#pragma unroll
+        for (int k = 0; k < kKTile / 32; ++k) {
+            u32x4_m p0[2], p1[2];
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                p0[i] = *reinterpret_cast<const u32x4_m*>(ph + (i * 16 + c) * PSTR + 32 * k + 8 * kg);
+                p1[i] = *reinterpret_cast<const u32x4_m*>(pl + (i * 16 + c) * PSTR + 32 * k + 8 * kg);
+            }
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const u32x4_m vv = lds_operand_t(vt + 32 * k * VSTR + 16 * v, VSTR, lane);
+#pragma unroll
+                for (int i = 0; i < 2; ++i) {
+                    o[i][v] = mma16(p0[i], vv, o[i][v]);
+                    o[i][v] = mma16(p1[i], vv, o[i][v]);
+                }
+            }
+        }
+        asm volatile("" ::: "memory");
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int qi = myq + i * 16 + 4 * kg + e;
+            if (qi >= T) continue;
+            const float inv = 1.0f / l[i][e];
+            bf16_t* out = (bf16_t*)a.ctx + ((int64_t)(r0 + qi) * H + h) * vdim;
+#pragma unroll
+            for (int v = 0; v < VT; ++v)
+                if (16 * v + c < vdim) out[16 * v + c] = f32_to_bf16(o[i][v][e] * inv);
+        }
 }
 
 template <typename F>
@@ -537,7 +659,31 @@ size_t latent_prefill_scratch_bytes(int dtype, int64_t total, int64_t heads, int
     (void)vdim;
     return lat_align((size_t)(total * heads * (dim + rot)) * (dtype == 0 ? 4 : 2));
 }
+template <int KS, int VT>
+static void launch_prefill(hipStream_t s, const LatentPrefillArgs& a, int64_t longest) {
+    constexpr int lds = (kKTile * (KS * 32 + 8) + kKTile * (VT * 16 + 8) + 4 * 2 * 32 * (kKTile + 8)) * 2;
+    static_assert(lds <= 160 * 1024, "LDS of one CU");
+    with_lds(latent_prefill_kernel<KS, VT>, lds);
+    latent_prefill_kernel<KS, VT><<<dim3((unsigned)cdiv_l(longest, kQTile), (unsigned)a.heads, (unsigned)a.nseq), 256, lds, s>>>(a);
+}
+template <int KS>
+static void launch_prefill_v(hipStream_t s, const LatentPrefillArgs& a, int64_t longest) {
+    if (a.vdim <= 64) launch_prefill<KS, 4>(s, a, longest);
+    else if (a.vdim <= 128) launch_prefill<KS, 8>(s, a, longest);
+    else launch_prefill<KS, 16>(s, a, longest);
+}
 int latent_prefill(hipStream_t s, const LatentPrefillArgs& a) {
+    if (a.dtype == 2 && a.dim % 8 == 0 && a.rot % 8 == 0 && a.rank % 8 == 0 && a.vdim % 8 == 0 && a.dim + a.rot <= 256 && a.vdim <= 256) {
+        int64_t longest = 0;
+        for (int b = 0; b < a.nseq; ++b) longest = std::max<int64_t>(longest, a.len[b]);
+        const int64_t ks = cdiv_l(a.dim + a.rot, 32);
+        if (ks <= 2) launch_prefill_v<2>(s, a, longest);
+        else if (ks <= 3) launch_prefill_v<3>(s, a, longest);
+        else if (ks <= 4) launch_prefill_v<4>(s, a, longest);
+        else if (ks <= 6) launch_prefill_v<6>(s, a, longest);
+        else launch_prefill_v<8>(s, a, longest);
+        return 1;
+    }
     const size_t es = a.dtype == 0 ? 4 : 2;
     const int64_t hd = a.heads * (a.dim + a.rot), w = a.rank + a.rot;
     int n = 0;

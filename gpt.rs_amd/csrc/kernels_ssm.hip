@@ -4,7 +4,7 @@
 //   * one row per sequence (decode): a step kernel (convolution of the channels it needs, recurrence, un-gated rows) and a
 //     finish kernel (gated norm, the convolution's new history); both read the old history, so the caller may donate it;
 //   * prompts: convolution, then the recurrence in chunks of 64 tokens on the matrix cores (bf16; ssd_kernel), gated norm.
-//     f32 runs the token-by-token kernel.
+//     f32 (and sizes outside its tiling) runs the token-by-token kernel.
 //
 // This file's first part are the stand-alone kernels of the CustomCall targets, one per target, for any sizes and either
 // element type.  Rows of the input projection stay f32 (step sizes enter the recurrence from them); the state is f32.
@@ -231,6 +231,259 @@ __global__ __launch_bounds__(256) void ssm_finish_kernel(SsmSeqArgs a, const flo
     for (; i < part; i += 256) Elem<T>::st(out, i, ((y[i] * silu_f32(z[i])) * inv) * a.gain[g0 + i]);
 }
 
+// ---------------------------------------------------------------------------- prompts
+// The convolution over whole prompts: a thread takes 4 channels of kConvRows rows and slides its window of taps along them.
+constexpr int kConvRows = 16;
+template <typename T, int K>
+__global__ __launch_bounds__(256) void conv_rows_kernel(SsmSeqArgs a, T* __restrict__ xbc) {
+    const int b = blockIdx.z;
+    const int64_t c = 4 * ((int64_t)blockIdx.x * 256 + threadIdx.x), t0 = (int64_t)blockIdx.y * kConvRows;
+    if (c >= a.ch || t0 >= a.len[b]) return;
+    const float* p = a.p + (int64_t)a.row0[b] * a.ld + a.col + c;
+    T* out = xbc + ((int64_t)(a.row0[b] - a.row0[0])) * a.ch + c;
+    float4 tap[K], win[K];
+#pragma unroll
+    for (int k = 0; k < K; ++k) tap[k] = *reinterpret_cast<const float4*>(a.taps + k * a.ch + c);
+    const float4 bias = *reinterpret_cast<const float4*>(a.bias + c);
+#pragma unroll
+    for (int k = 0; k + 1 < K; ++k) {
+        const int64_t r = t0 + k - (K - 1);
+        win[k + 1] = r >= 0 ? *reinterpret_cast<const float4*>(p + r * a.ld) : *reinterpret_cast<const float4*>(a.conv_in[b] + (r + K - 1) * a.ch + c);
+    }
+    const int64_t t1 = t0 + kConvRows < a.len[b] ? t0 + kConvRows : a.len[b];
+    for (int64_t t = t0; t < t1; ++t) {
+#pragma unroll
+        for (int k = 0; k + 1 < K; ++k) win[k] = win[k + 1];
+        win[K - 1] = *reinterpret_cast<const float4*>(p + t * a.ld);
+        float4 v = bias;
+#pragma unroll
+        for (int k = 0; k < K; ++k) { v.x += tap[k].x * win[k].x; v.y += tap[k].y * win[k].y; v.z += tap[k].z * win[k].z; v.w += tap[k].w * win[k].w; }
+        v.x = silu_f32(v.x); v.y = silu_f32(v.y); v.z = silu_f32(v.z); v.w = silu_f32(v.w);
+        if (sizeof(T) == 2) *reinterpret_cast<uint2*>(out + t * a.ch) = make_uint2(pack_bf16_hw(v.x, v.y), pack_bf16_hw(v.z, v.w));
+        else *reinterpret_cast<float4*>(out + t * a.ch) = v;
+    }
+}
+
+// The recurrence in chunks of 64 tokens (state-space duality).  With cum_t the running sum of the log decays inside a chunk,
+//     y_t = sum_{s <= t} (C_t . B_s) exp(cum_t - cum_s) dt_s x_s  +  exp(cum_t) S^T C_t  +  D x_t
+//     S  <- exp(cum_end) S + sum_s exp(cum_end - cum_s) dt_s B_s x_s^T
+// so a chunk is four small matrix products.  Workgroup = head x slice of 16 VT values x sequence, 4 waves; it walks the chunks of
+// its sequence.  Wave w owns the rows t = 16 w .. of a chunk and the states n = 16 (w + 4 i) .., i < NPW, which it keeps in f32
+// accumulators as S^T (rows: values, columns: states) from the first chunk to the last.  Factors that are not bf16 already (the
+// decayed scores, the weighted x, the state as an operand) enter the products as a bf16 value plus its remainder.
+constexpr int kChunk = 64;
+template <int NPW, int VT>
+__global__ __launch_bounds__(256) void ssd_kernel(SsmSeqArgs a, const bf16_t* __restrict__ xbc, bf16_t* __restrict__ y) {
+    constexpr int NP = 64 * NPW, NSTR = NP + 8, VS = 16 * VT, XSTR = VS + 8, MSTR = kChunk + 8;
+    extern __shared__ __align__(16) unsigned char ssd_smem[];
+    bf16_t* Bm = reinterpret_cast<bf16_t*>(ssd_smem);   // [64][NSTR] token rows of B
+    bf16_t* Cm = Bm + kChunk * NSTR;                    // [64][NSTR]
+    bf16_t* xm = Cm + kChunk * NSTR;                    // [64][XSTR]
+    bf16_t* sh = xm + kChunk * XSTR;                    // [VS][NSTR] S^T
+    bf16_t* sl = sh + VS * NSTR;                        // [VS][NSTR] its remainder
+    bf16_t* mm = sl + VS * NSTR;                        // per wave: [2][16][MSTR]
+    float* cum = reinterpret_cast<float*>(mm + 4 * 2 * 16 * MSTR);   // [64]
+    float* dts = cum + kChunk;                          // [64] step sizes
+    float* wgt = dts + kChunk;                          // [64] exp(cum_end - cum_s) dt_s
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, kg = lane >> 4;
+    const int h = blockIdx.x, v0 = blockIdx.y * VS, b = blockIdx.z, T = a.len[b];
+    const int N = (int)a.n, vdim = (int)a.vdim, inner = (int)(a.heads * a.vdim), grp = h / (int)(a.heads / a.groups);
+    const int64_t ch = a.ch;
+    const bf16_t* rows = xbc + (int64_t)(a.row0[b] - a.row0[0]) * ch;
+    bf16_t* yout = y + (int64_t)(a.row0[b] - a.row0[0]) * inner + (int64_t)h * vdim + v0;
+    const float* p = a.p + (int64_t)a.row0[b] * a.ld + a.dt_col + h;
+    const bf16_t* bsrc = rows + inner + (int64_t)grp * N;
+    const bf16_t* csrc = bsrc + a.groups * (int64_t)N;
+    const bf16_t* xsrc = rows + (int64_t)h * vdim + v0;
+    const float rate = expf(a.a_log[h]), dtb = a.dt_bias[h], dd = a.d[h];
+    bf16_t* mh = mm + wave * 2 * 16 * MSTR;
+    bf16_t* ml = mh + 16 * MSTR;
+
+    // state in, columns n of rows v
+    f32x4_m S[VT][NPW];
+#pragma unroll
+    for (int i = 0; i < VT; ++i)
+#pragma unroll
+        for (int j = 0; j < NPW; ++j)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int n = 16 * (wave + 4 * j) + c, v = v0 + 16 * i + 4 * kg + e;
+                S[i][j][e] = n < N && v < vdim ? a.state_in[b][((int64_t)h * N + n) * vdim + v] : 0.f;
+            }
+    // columns that no token fills stay zero
+    for (int i = tid; i < kChunk * (NP / 8); i += 256) {
+        const int r = i / (NP / 8), n = (i % (NP / 8)) * 8;
+        if (n >= N) {
+            *reinterpret_cast<uint4*>(Bm + r * NSTR + n) = make_uint4(0u, 0u, 0u, 0u);
+            *reinterpret_cast<uint4*>(Cm + r * NSTR + n) = make_uint4(0u, 0u, 0u, 0u);
+        }
+    }
+    const int nw = N / 8;                               // 16-byte words per row of B and C
+    constexpr int BU = (kChunk * (NP / 8) + 255) / 256, XW = VS / 8, XU = (kChunk * XW + 255) / 256;
+    uint4 rb[BU], rc[BU], rx[XU];
+    float rdt = 0.f;
+    auto fetch = [&](int t0) {                          // a chunk's words into registers; tokens behind the prompt are zero
+#pragma unroll
+        for (int u = 0; u < BU; ++u) {
+            const int i = tid + 256 * u, r = i / nw, k = i % nw;
+            rb[u] = rc[u] = make_uint4(0u, 0u, 0u, 0u);
+            if (i < kChunk * nw && t0 + r < T) {
+                rb[u] = *reinterpret_cast<const uint4*>(bsrc + (int64_t)(t0 + r) * ch + 8 * k);
+                rc[u] = *reinterpret_cast<const uint4*>(csrc + (int64_t)(t0 + r) * ch + 8 * k);
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < XU; ++u) {
+            const int i = tid + 256 * u, r = i / XW, k = i % XW;
+            rx[u] = make_uint4(0u, 0u, 0u, 0u);
+            if (i < kChunk * XW && t0 + r < T && v0 + 8 * k < vdim) rx[u] = *reinterpret_cast<const uint4*>(xsrc + (int64_t)(t0 + r) * ch + 8 * k);
+        }
+        if (wave == 0) rdt = t0 + lane < T ? p[(int64_t)(t0 + lane) * a.ld] : 0.f;
+    };
+    fetch(0);
+    for (int t0 = 0; t0 < T; t0 += kChunk) {
+        __syncthreads();                                // the previous chunk has been read
+#pragma unroll
+        for (int u = 0; u < BU; ++u) {
+            const int i = tid + 256 * u, r = i / nw, k = i % nw;
+            if (i < kChunk * nw) {
+                *reinterpret_cast<uint4*>(Bm + r * NSTR + 8 * k) = rb[u];
+                *reinterpret_cast<uint4*>(Cm + r * NSTR + 8 * k) = rc[u];
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < XU; ++u) {
+            const int i = tid + 256 * u, r = i / XW, k = i % XW;
+            if (i < kChunk * XW) *reinterpret_cast<uint4*>(xm + r * XSTR + 8 * k) = rx[u];
+        }
+#pragma unroll
+        for (int i = 0; i < VT; ++i)
+#pragma unroll
+            for (int j = 0; j < NPW; ++j)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int at = (16 * i + 4 * kg + e) * NSTR + 16 * (wave + 4 * j) + c;
+                    const uint32_t hi = pack_bf16_hw(S[i][j][e], 0.f) & 0xFFFFu;
+                    sh[at] = (bf16_t)hi;
+                    sl[at] = (bf16_t)(pack_bf16_hw(S[i][j][e] - __uint_as_float(hi << 16), 0.f) & 0xFFFFu);
+                }
+        if (wave == 0) {
+            const bool live = t0 + lane < T;            // behind the prompt: no step, no decay
+            const float dt = live ? softplus_f32(rdt + dtb) : 0.f;
+            float s = -rate * dt;
+#pragma unroll
+            for (int off = 1; off < 64; off <<= 1) {
+                const float o = __shfl_up(s, off, 64);
+                if (lane >= off) s += o;
+            }
+            const float end = __shfl(s, 63, 64);
+            cum[lane] = s;
+            dts[lane] = dt;
+            wgt[lane] = expf(end - s) * dt;
+        }
+        __syncthreads();
+        if (t0 + kChunk < T) fetch(t0 + kChunk);
+
+        // scores of the wave's 16 tokens against tokens 0 .. 16 wave + 15 of the chunk
+        u32x4_m ca[2 * NPW];
+#pragma unroll
+        for (int k = 0; k < 2 * NPW; ++k) ca[k] = *reinterpret_cast<const u32x4_m*>(Cm + (16 * wave + c) * NSTR + 32 * k + 8 * kg);
+        float ct[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ct[e] = cum[16 * wave + 4 * kg + e];
+        const int ksteps = wave / 2 + 1;                // steps of 32 tokens that reach the wave's rows
+        for (int j = 0; j < 2 * ksteps; ++j) {
+            f32x4_m g = {0.f, 0.f, 0.f, 0.f};
+            if (j <= wave) {
+#pragma unroll
+                for (int k = 0; k < 2 * NPW; ++k)
+                    g = mma16(ca[k], *reinterpret_cast<const u32x4_m*>(Bm + (16 * j + c) * NSTR + 32 * k + 8 * kg), g);
+            }
+            const float cs = cum[16 * j + c], ds = dts[16 * j + c];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float f = 16 * j + c <= 16 * wave + 4 * kg + e ? g[e] * (expf(ct[e] - cs) * ds) : 0.f;
+                const uint32_t hi = pack_bf16_hw(f, 0.f) & 0xFFFFu;
+                mh[(4 * kg + e) * MSTR + 16 * j + c] = (bf16_t)hi;
+                ml[(4 * kg + e) * MSTR + 16 * j + c] = (bf16_t)(pack_bf16_hw(f - __uint_as_float(hi << 16), 0.f) & 0xFFFFu);
+            }
+        }
+        asm volatile("" ::: "memory");                // (the wave's own values: its LDS operations complete in order)
+        f32x4_m yi[VT], ys[VT];
+#pragma unroll
+        for (int i = 0; i < VT; ++i) {
+            yi[i] = ys[i] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int k = 0; k < 2 * NPW; ++k) {
+                ys[i] = mma16(ca[k], *reinterpret_cast<const u32x4_m*>(sh + (16 * i + c) * NSTR + 32 * k + 8 * kg), ys[i]);
+                ys[i] = mma16(ca[k], *reinterpret_cast<const u32x4_m*>(sl + (16 * i + c) * NSTR + 32 * k + 8 * kg), ys[i]);
+            }
+        }
+        for (int k = 0; k < ksteps; ++k) {
+            const u32x4_m m0 = *reinterpret_cast<const u32x4_m*>(mh + c * MSTR + 32 * k + 8 * kg), m1 = *reinterpret_cast<const u32x4_m*>(ml + c * MSTR + 32 * k + 8 * kg);
+#pragma unroll
+            for (int i = 0; i < VT; ++i) {
+                const u32x4_m xv = lds_operand_t(xm + 32 * k * XSTR + 16 * i, XSTR, lane);
+                yi[i] = mma16(m0, xv, yi[i]);
+                yi[i] = mma16(m1, xv, yi[i]);
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int t = 16 * wave + 4 * kg + e;
+            const float et = expf(ct[e]);
+            if (t0 + t < T) {
+#pragma unroll
+                for (int i = 0; i < VT; ++i)
+                    if (v0 + 16 * i + c < vdim)
+                        yout[(int64_t)(t0 + t) * inner + 16 * i + c] = f32_to_bf16(yi[i][e] + et * ys[i][e] + dd * bf16_to_f32(xm[t * XSTR + 16 * i + c]));
+            }
+        }
+        // the state after the chunk
+        const float edecay = expf(cum[kChunk - 1]);
+#pragma unroll
+        for (int i = 0; i < VT; ++i)
+#pragma unroll
+            for (int j = 0; j < NPW; ++j)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) S[i][j][e] *= edecay;
+#pragma unroll
+        for (int k = 0; k < kChunk / 32; ++k) {
+            u32x4_m bv[NPW];
+#pragma unroll
+            for (int j = 0; j < NPW; ++j) bv[j] = lds_operand_t(Bm + 32 * k * NSTR + 16 * (wave + 4 * j), NSTR, lane);
+            float ws[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ws[e] = wgt[32 * k + 8 * kg + e];
+#pragma unroll
+            for (int i = 0; i < VT; ++i) {
+                const u32x4_m xv = lds_operand_t(xm + 32 * k * XSTR + 16 * i, XSTR, lane);
+                u32x4_m xh, xl;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const float f0 = bf16lo(xv[e]) * ws[2 * e], f1 = bf16hi(xv[e]) * ws[2 * e + 1];
+                    xh[e] = pack_bf16_hw(f0, f1);
+                    xl[e] = pack_bf16_hw(f0 - bf16lo(xh[e]), f1 - bf16hi(xh[e]));
+                }
+#pragma unroll
+                for (int j = 0; j < NPW; ++j) {
+                    S[i][j] = mma16(xh, bv[j], S[i][j]);
+                    S[i][j] = mma16(xl, bv[j], S[i][j]);
+                }
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < VT; ++i)
+#pragma unroll
+        for (int j = 0; j < NPW; ++j)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int n = 16 * (wave + 4 * j) + c, v = v0 + 16 * i + 4 * kg + e;
+                if (n < N && v < vdim) a.state_out[b][((int64_t)h * N + n) * vdim + v] = S[i][j][e];
+            }
+}
+
 }  // namespace
 
 void conv_silu(hipStream_t s, const ConvArgs& a) {
@@ -309,25 +562,61 @@ int ssm_seq(hipStream_t s, const SsmSeqArgs& a) {
     const size_t es = a.dtype == 0 ? 4 : 2;
     const int64_t inner = a.heads * a.vdim;
     char* xbc = (char*)a.scratch;
-    char* y = xbc;   // behind the convolved rows of this launch series
-    y += ssm_align((size_t)a.rows * a.ch * es);
-    int n = 0;
+    char* y = xbc + ssm_align((size_t)a.rows * a.ch * es);   // behind the convolved rows of this launch series
+    int n = 0, longest = 0;
+    for (int b = 0; b < a.nseq; ++b) longest = std::max(longest, a.len[b]);
+    auto row = [&](int b) { return (int64_t)(a.row0[b] - a.row0[0]); };
+    // convolution of all prompts in one launch where 4 channels go together, else prompt by prompt
+    if (a.ch % 4 == 0 && a.ld % 4 == 0 && a.col % 4 == 0 && a.ntaps >= 2 && a.ntaps <= 4) {
+        const dim3 grid((unsigned)cdiv_m(a.ch / 4, 256), (unsigned)cdiv_m(longest, kConvRows), (unsigned)a.nseq);
+#define GPTRS_CONV(T) do { if (a.ntaps == 2) conv_rows_kernel<T, 2><<<grid, 256, 0, s>>>(a, (T*)xbc); \
+                           else if (a.ntaps == 3) conv_rows_kernel<T, 3><<<grid, 256, 0, s>>>(a, (T*)xbc); \
+                           else conv_rows_kernel<T, 4><<<grid, 256, 0, s>>>(a, (T*)xbc); } while (0)
+        if (a.dtype == 0) GPTRS_CONV(float);
+        else GPTRS_CONV(bf16_t);
+#undef GPTRS_CONV
+        ++n;
+    } else {
+        for (int b = 0; b < a.nseq; ++b) {
+            ConvArgs c{};
+            c.dtype = a.dtype;
+            c.p = a.p + (int64_t)a.row0[b] * a.ld; c.taps = a.taps; c.bias = a.bias; c.state = a.conv_in[b];
+            c.y = xbc + (size_t)(row(b) * a.ch) * es;
+            c.rows = a.len[b]; c.ld = a.ld; c.col = a.col; c.ch = a.ch; c.ntaps = a.ntaps;
+            conv_silu(s, c);
+            ++n;
+        }
+    }
     for (int b = 0; b < a.nseq; ++b) {
-        const int64_t r = a.row0[b] - a.row0[0];
-        ConvArgs c{};
-        c.dtype = a.dtype;
-        c.p = a.p + (int64_t)a.row0[b] * a.ld; c.taps = a.taps; c.bias = a.bias; c.state = a.conv_in[b];
-        c.y = xbc + (size_t)(r * a.ch) * es;
-        c.rows = a.len[b]; c.ld = a.ld; c.col = a.col; c.ch = a.ch; c.ntaps = a.ntaps;
-        conv_silu(s, c);
-        conv_state(s, c.p, a.conv_in[b], a.conv_out[b], a.len[b], a.ld, a.col, a.ch, a.ntaps);
-        SsmArgs m{};
-        m.dtype = a.dtype;
-        m.xbc = c.y; m.p = c.p; m.dt_bias = a.dt_bias; m.a_log = a.a_log; m.d = a.d;
-        m.state = a.state_in[b]; m.state_out = a.state_out[b]; m.y = y + (size_t)(r * inner) * es;
-        m.rows = a.len[b]; m.ld = a.ld; m.dt_col = a.dt_col; m.heads = a.heads; m.groups = a.groups; m.n = a.n; m.vdim = a.vdim;
-        ssm_scan(s, m);
-        n += 3;
+        conv_state(s, a.p + (int64_t)a.row0[b] * a.ld, a.conv_in[b], a.conv_out[b], a.len[b], a.ld, a.col, a.ch, a.ntaps);
+        ++n;
+    }
+    if (a.dtype == 2 && a.n % 8 == 0 && a.n <= 256 && a.vdim % 8 == 0) {
+        // slices of 32 values, or of 16 where the slices are too few for the chip
+#define GPTRS_SSD(NPW, VT)                                                                                                       \
+        do {                                                                                                                     \
+            constexpr int NS = 64 * NPW + 8, VS = 16 * VT;                                                                       \
+            constexpr int lds = (2 * kChunk * NS + kChunk * (VS + 8) + 2 * VS * NS + 4 * 2 * 16 * (kChunk + 8)) * 2 + 3 * kChunk * 4; \
+            static_assert(lds <= 160 * 1024, "LDS of one CU");                                                                   \
+            (void)hipFuncSetAttribute((const void*)ssd_kernel<NPW, VT>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);        \
+            ssd_kernel<NPW, VT><<<dim3((unsigned)a.heads, (unsigned)cdiv_m(a.vdim, VS), (unsigned)a.nseq), 256, lds, s>>>(a, (const bf16_t*)xbc, (bf16_t*)y); \
+        } while (0)
+        const bool wide = a.vdim > 16 && a.heads * cdiv_m(a.vdim, 32) * a.nseq >= 160;
+        if (a.n <= 64) { if (wide) GPTRS_SSD(1, 2); else GPTRS_SSD(1, 1); }
+        else if (a.n <= 128) { if (wide) GPTRS_SSD(2, 2); else GPTRS_SSD(2, 1); }
+        else { if (wide) GPTRS_SSD(4, 2); else GPTRS_SSD(4, 1); }
+#undef GPTRS_SSD
+        ++n;
+    } else {
+        for (int b = 0; b < a.nseq; ++b) {
+            SsmArgs m{};
+            m.dtype = a.dtype;
+            m.xbc = xbc + (size_t)(row(b) * a.ch) * es; m.p = a.p + (int64_t)a.row0[b] * a.ld; m.dt_bias = a.dt_bias; m.a_log = a.a_log; m.d = a.d;
+            m.state = a.state_in[b]; m.state_out = a.state_out[b]; m.y = y + (size_t)(row(b) * inner) * es;
+            m.rows = a.len[b]; m.ld = a.ld; m.dt_col = a.dt_col; m.heads = a.heads; m.groups = a.groups; m.n = a.n; m.vdim = a.vdim;
+            ssm_scan(s, m);
+            ++n;
+        }
     }
     gated_rms_norm(s, a.dtype, y, a.p + (int64_t)a.row0[0] * a.ld, a.gain, (char*)a.out + (size_t)a.row0[0] * inner * es, a.rows, inner, a.ld, a.z_col,
                    a.norm_groups, a.eps);

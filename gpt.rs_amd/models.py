@@ -1107,14 +1107,15 @@ class Dadupel(_ModelBase):
     @classmethod
     def random(cls, config: DadupelConfig, backend, seed: int = 0, dtype: str = "Bf16", context_length: Optional[int] = None) -> "Dadupel":
         """Random weights of the right shapes and of sensible sizes, one numpy stream per tensor."""
+        from concurrent.futures import ThreadPoolExecutor
         m = cls(config, backend, dtype, context_length)
-        table = None
-        for idx, (name, dims) in enumerate(m.expected_params().items()):
+        plan = [(n, d) for n, d in m.expected_params().items() if n != "lm_head"]
+
+        def make(idx):
+            name, dims = plan[idx]
             rng = np.random.default_rng(np.random.SeedSequence([seed, idx]))
             leaf = name.rsplit(".", 1)[-1]
-            if leaf == "lm_head":
-                arr = np.ascontiguousarray(table.T)
-            elif leaf == "dt_bias":
+            if leaf == "dt_bias":
                 arr = np.log(np.expm1(np.exp(rng.uniform(np.log(1e-3), np.log(1e-1), dims)))).astype(np.float32)
             elif leaf == "a_log":
                 arr = np.log(rng.uniform(1.0, 16.0, dims)).astype(np.float32)
@@ -1126,10 +1127,21 @@ class Dadupel(_ModelBase):
                 arr = rng.uniform(0.3, 1.0, dims).astype(np.float32)
             else:
                 arr = rng.standard_normal(dims, dtype=np.float32)
-                arr *= np.float32(1.0 if leaf == "weight" else dims[0] ** -0.5)
-            if leaf == "weight":
-                table = arr = bf16_bits_to_f32(f32_to_bf16_bits(arr * np.float32(dims[1] ** -0.5))) if dtype == "Bf16" else arr * np.float32(dims[1] ** -0.5)
-            m.set_param(name, arr, m.param_dtype(name))
+                arr *= np.float32((dims[1] if leaf == "weight" else dims[0]) ** -0.5)
+            dt = m.param_dtype(name)
+            return name, dims, dt, _np_to_bytes(arr, dt), arr if leaf == "weight" else None
+
+        workers = max(1, min(16, os.cpu_count() or 1))
+        with ThreadPoolExecutor(max_workers=workers) as ex:
+            pending, nxt, table = [], 0, None
+            while nxt < len(plan) or pending:   # bounded look-ahead: a few tensors of host memory in flight
+                while nxt < len(plan) and len(pending) < 2 * workers:
+                    pending.append(ex.submit(make, nxt))
+                    nxt += 1
+                name, dims, dt, data, arr = pending.pop(0).result()
+                m.set_param_bytes(name, TensorSpec(dt, dims), data)
+                table = arr if arr is not None else table
+        m.set_param("lm_head", np.ascontiguousarray(table.T), m.param_dtype("lm_head"))
         return m
 
     @property
