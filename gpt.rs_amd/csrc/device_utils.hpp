@@ -73,6 +73,32 @@ __device__ __forceinline__ u32x4_m lds_operand_t(const bf16_t* m, int stride, in
     r.x = lo.x; r.y = lo.y; r.z = hi.x; r.w = hi.y;
     return r;
 }
+// The same for an operand whose k slots are the rows 4 kg .. 4 kg + 3 and 16 + 4 kg .. 16 + 4 kg + 3 of m: what the results of
+// two stacked 16 x 16 tiles hold per lane, so that such results feed the next product from registers.
+__device__ __forceinline__ u32x4_m lds_operand_t2(const bf16_t* m, int stride, int lane) {
+    typedef short s16x4 __attribute__((ext_vector_type(4)));
+    typedef __attribute__((address_space(3))) s16x4* lds_p;
+    const int c = lane & 15, kg = lane >> 4;
+    const bf16_t* p = m + (4 * kg + (c >> 2)) * stride + 4 * (c & 3);
+    const u32x2_m lo = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)(p)));
+    const u32x2_m hi = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)(p + 16 * stride)));
+    u32x4_m r;
+    r.x = lo.x; r.y = lo.y; r.z = hi.x; r.w = hi.y;
+    return r;
+}
+// Sum / maximum over the four lanes that share a column (lane, lane ^ 16, lane ^ 32, lane ^ 48)
+__device__ __forceinline__ float col4_sum(float v) {
+    const u32x2_m a = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false));
+    v = __uint_as_float(a.x) + __uint_as_float(a.y);
+    const u32x2_m b = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false));
+    return __uint_as_float(b.x) + __uint_as_float(b.y);
+}
+__device__ __forceinline__ float col4_max(float v) {
+    const u32x2_m a = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false));
+    v = fmaxf(__uint_as_float(a.x), __uint_as_float(a.y));
+    const u32x2_m b = __builtin_bit_cast(u32x2_m, __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false));
+    return fmaxf(__uint_as_float(b.x), __uint_as_float(b.y));
+}
 // bf16 pair by the hardware converter (round to nearest even)
 __device__ __forceinline__ uint32_t pack_bf16_hw(float lo, float hi) {
     typedef float f32x2_p __attribute__((ext_vector_type(2)));
@@ -80,6 +106,11 @@ __device__ __forceinline__ uint32_t pack_bf16_hw(float lo, float hi) {
     f32x2_p f;
     f.x = lo; f.y = hi;
     return __builtin_bit_cast(uint32_t, __builtin_convertvector(f, bf16x2_p));
+}
+// (a, b) as a pair of bf16 values plus the pair of their remainders: together 16 bits of each
+__device__ __forceinline__ void split_bf16_hw(float a, float b, uint32_t& hi, uint32_t& lo) {
+    hi = pack_bf16_hw(a, b);
+    lo = pack_bf16_hw(a - bf16lo(hi), b - bf16hi(hi));
 }
 // Sum / maximum over the 16 lanes of a row, in every lane of it
 __device__ __forceinline__ float row16_sum(float v) {

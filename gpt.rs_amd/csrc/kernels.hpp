@@ -429,7 +429,7 @@ struct LatentDecodeArgs {
     float scale, eps;
     void* scratch;
 };
-size_t latent_decode_scratch_bytes(int dtype, int64_t nseq, int64_t capacity, int64_t heads, int64_t dim, int64_t rot, int64_t rank);
+size_t latent_decode_scratch_bytes(int dtype, int64_t nseq, int64_t capacity, int64_t heads, int64_t dim, int64_t rot, int64_t rank, int64_t vdim);
 int latent_decode(hipStream_t s, const LatentDecodeArgs& a);
 
 // Causal latent attention of whole prompts (Mix::LatentPrefill), nseq sequences stacked: x T [rows, heads * (dim + rot)]

@@ -170,7 +170,7 @@ __global__ __launch_bounds__(256) void latent_attn_x_kernel(LatentAttnXArgs a) {
 
 // ---------------------------------------------------------------------------- decode (bf16)
 constexpr int kPrepRows = 64;    // latent dimensions per workgroup of the query part
-constexpr int kTileP = 64;       // cache rows per step of the attention part
+constexpr int kTileP = 32;       // cache rows per step of the attention part
 constexpr int kHeadTile = 16;
 
 // Blocks [0, heads * rank / 64): W_uk^T q_n of one head and 64 latent dimensions, for every sequence (the first of a head
@@ -218,144 +218,154 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentDecodeArgs a, bf
     __syncthreads();
     const bf16_t* wk = (const bf16_t*)a.w_uk;
     const int64_t ldw = (int64_t)H * dim;
-    constexpr int J = kPrepRows / 16;
-    for (int b = 0; b < (int)a.nseq; ++b) {
-        float s[J];
+    constexpr int J = kPrepRows / 16, BT = 8;    // a word of W_uk serves up to 8 sequences
+    for (int b0 = 0; b0 < (int)a.nseq; b0 += BT) {
+        float s[BT][J];
 #pragma unroll
-        for (int j = 0; j < J; ++j) s[j] = 0.f;
+        for (int b = 0; b < BT; ++b)
+#pragma unroll
+            for (int j = 0; j < J; ++j) s[b][j] = 0.f;
         for (int d = l16 * 8; d < dim; d += 128) {
-            float qv[8];
+            u32x4_m x[J];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) qv[e] = q[b * dim + d + e];
+            for (int j = 0; j < J; ++j) x[j] = *reinterpret_cast<const u32x4_m*>(wk + (int64_t)min(r0 + g + 16 * j, rank - 1) * ldw + (int64_t)h * dim + d);
 #pragma unroll
-            for (int j = 0; j < J; ++j) {
-                const int r = r0 + g + 16 * j;
-                if (r >= rank) continue;
-                const uint4 v = *reinterpret_cast<const uint4*>(wk + r * ldw + (int64_t)h * dim + d);
-                const uint32_t vw[4] = {v.x, v.y, v.z, v.w};
+            for (int b = 0; b < BT; ++b) {
+                if (b0 + b >= (int)a.nseq) break;
+                const float4 qa = *reinterpret_cast<const float4*>(q + (b0 + b) * dim + d), qb = *reinterpret_cast<const float4*>(q + (b0 + b) * dim + d + 4);
 #pragma unroll
-                for (int e = 0; e < 4; ++e) { s[j] += qv[2 * e] * bf16lo(vw[e]); s[j] += qv[2 * e + 1] * bf16hi(vw[e]); }
+                for (int j = 0; j < J; ++j) {
+                    float v = s[b][j];
+                    v += qa.x * bf16lo(x[j][0]); v += qa.y * bf16hi(x[j][0]);
+                    v += qa.z * bf16lo(x[j][1]); v += qa.w * bf16hi(x[j][1]);
+                    v += qb.x * bf16lo(x[j][2]); v += qb.y * bf16hi(x[j][2]);
+                    v += qb.z * bf16lo(x[j][3]); v += qb.w * bf16hi(x[j][3]);
+                    s[b][j] = v;
+                }
             }
         }
 #pragma unroll
-        for (int j = 0; j < J; ++j) {
-            const float tot = row16_sum(s[j]);
-            const int r = r0 + g + 16 * j;
-            if (l16 == 0 && r < rank) ql[((int64_t)b * H + h) * w + r] = f32_to_bf16(tot);
+        for (int b = 0; b < BT; ++b) {
+            if (b0 + b >= (int)a.nseq) break;
+#pragma unroll
+            for (int j = 0; j < J; ++j) {
+                const float tot = row16_sum(s[b][j]);
+                const int r = r0 + g + 16 * j;
+                if (l16 == 0 && r < rank) ql[((int64_t)(b0 + b) * H + h) * w + r] = f32_to_bf16(tot);
+            }
         }
     }
 }
 
-// Workgroup = slice of the positions x 16 heads x sequence.  Tiles of 64 cache rows in LDS; scores on the matrix cores (wave w:
-// rows 16 w ..), softmax over the tile, weights split into a bf16 value and its remainder, weighted rows on the matrix cores
-// (wave w: latent dimensions 16 (w + 4 i) ..).  part f32 [nseq][heads][nsplit][rank + 2]: sums, maximum, weight.
+// Workgroup = ONE wave: slice of the positions x 16 heads (and 16 RT latent dimensions of the result) x sequence.  32 cache rows
+// at a time in LDS, all their words requested before the first is stored; scores transposed (rows: positions, columns: heads),
+// so a lane holds 8 positions of one head: softmax in registers, and the weights (a bf16 value and its remainder) feed the
+// product with the cached latents from there.  part f32 [nseq][heads][nsplit][rank + 2]: sums, maximum (base 2), weight.
 template <int RT>
-__global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ ql, float* __restrict__ part, int nsplit) {
+__global__ __launch_bounds__(64) void latent_partial_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ ql, float* __restrict__ part, int nsplit) {
     extern __shared__ __align__(16) unsigned char lat_smem[];
     const int rank = (int)a.rank, w = rank + (int)a.rot, H = (int)a.heads, ws = w + 8;   // LDS row stride
-    bf16_t* rows = reinterpret_cast<bf16_t*>(lat_smem);               // [64][ws]
+    bf16_t* rows = reinterpret_cast<bf16_t*>(lat_smem);               // [32][ws]
     bf16_t* qs = rows + kTileP * ws;                                  // [16][ws]
-    constexpr int PS = kTileP + 8;
-    bf16_t* ph = qs + kHeadTile * ws;                                 // [16][PS] weights
-    bf16_t* pl = ph + kHeadTile * PS;                                 // [16][PS] their remainders
-    float* sc = reinterpret_cast<float*>(pl + kHeadTile * PS);        // [16][64 + 1]
-    float* corr = sc + kHeadTile * (kTileP + 1);                      // [16]
-    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, c = lane & 15, kg = lane >> 4;
-    const int b = blockIdx.z, h0 = blockIdx.y * kHeadTile, sp = blockIdx.x;
+    const int lane = threadIdx.x, c = lane & 15, kg = lane >> 4;
+    const int rparts = (rank + 16 * RT - 1) / (16 * RT);
+    const int b = blockIdx.z, h0 = ((int)blockIdx.y / rparts) * kHeadTile, rp0 = ((int)blockIdx.y % rparts) * 16 * RT, sp = blockIdx.x;
     const int n = min(max(a.pos[b], 0) + 1, (int)a.capacity);
     const int per = ((n + nsplit - 1) / nsplit + 15) / 16 * 16;
     const int p0 = sp * per, p1 = min(p0 + per, n);
     const int hr = H - h0 < kHeadTile ? H - h0 : kHeadTile;           // heads that exist
     float* rec = part + (((int64_t)b * H + h0) * nsplit + sp) * (rank + 2);
     const int64_t rec_h = (int64_t)nsplit * (rank + 2);
-    if (p0 >= p1) {   // nothing falls to this slice: an empty record
-        for (int i = t; i < hr; i += 256) { rec[i * rec_h + rank] = -INFINITY; rec[i * rec_h + rank + 1] = 0.f; }
+    if (p0 >= p1) {   // nothing falls to this slice: its weight is zero, and whoever merges does not use its sums
+        if (lane < hr) { rec[lane * rec_h + rank] = -INFINITY; rec[lane * rec_h + rank + 1] = 0.f; }
         return;
     }
-    const int wv = w / 8;                                             // 16-byte words per row
-    for (int i = t; i < kHeadTile * wv; i += 256) {
-        const int r = i / wv, k = i % wv;
-        const uint4 v = *reinterpret_cast<const uint4*>(ql + ((int64_t)b * H + h0 + (r < hr ? r : 0)) * w + 8 * k);
-        *reinterpret_cast<uint4*>(qs + r * ws + 8 * k) = v;
-    }
-    f32x4_m acc[RT];
+    const int wv = w / 8;                                             // 16-byte words per row (a multiple of 4)
+    const bf16_t* cache = (const bf16_t*)a.cache[b];
+    // rows go 8 at a time, 8 lanes to a row: a lane takes every eighth word of rows (lane >> 3), + 8, ..; kept as R x U words
+    constexpr int U = 10, RQ = kHeadTile / 8, RR = kTileP / 8;
+    const int lr = lane >> 3, lk = lane & 7;
+    u32x4_m vq[RQ][U], vr[RR][U];
+    auto request = [&](const bf16_t* src, int last, int k0, u32x4_m* v, int R) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+            const u32x4_m* from = reinterpret_cast<const u32x4_m*>(src + (int64_t)min(lr + 8 * i, last) * w);
+#pragma unroll
+            for (int u = 0; u < U; ++u) v[i * U + u] = from[min(k0 + lk + 8 * u, wv - 1)];
+        }
+    };
+    auto store = [&](bf16_t* dst, int k0, const u32x4_m* v, int R) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+            u32x4_m* to = reinterpret_cast<u32x4_m*>(dst + (lr + 8 * i) * ws);
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+                if (k0 + lk + 8 * u < wv) to[k0 + lk + 8 * u] = v[i * U + u];
+        }
+    };
+    f32x4_m acc[RT];                                                  // rows: latent dimensions, column: head c
 #pragma unroll
     for (int i = 0; i < RT; ++i) acc[i] = f32x4_m{0.f, 0.f, 0.f, 0.f};
-    float m_run = -INFINITY, l_run = 0.f;                             // of head 4 * wave + kg, in all its 16 lanes
-    const bf16_t* cache = (const bf16_t*)a.cache[b];
+    float m_run = -INFINITY, l_run = 0.f;                             // of head c, in its four lanes
+    const float scale2 = a.scale * 1.44269504f;
     for (int q0 = p0; q0 < p1; q0 += kTileP) {
         const int np = min(kTileP, p1 - q0);
-        const int npad = (np + 31) / 32 * 32;                         // the matrix cores take 32 rows at a time
-        __syncthreads();
-        for (int i = t; i < npad * wv; i += 256) {
-            const int r = i / wv, k = i % wv;
-            uint4 v = make_uint4(0u, 0u, 0u, 0u);
-            if (r < np) v = *reinterpret_cast<const uint4*>(cache + (int64_t)(q0 + r) * w + 8 * k);
-            *reinterpret_cast<uint4*>(rows + r * ws + 8 * k) = v;
+        asm volatile("" ::: "memory");
+        for (int k0 = 0; k0 < wv; k0 += 8 * U) {
+            if (q0 == p0) request(ql + ((int64_t)b * H + h0) * w, hr - 1, k0, &vq[0][0], RQ);
+            request(cache + (int64_t)q0 * w, np - 1, k0, &vr[0][0], RR);
+            if (q0 == p0) store(qs, k0, &vq[0][0], RQ);
+            store(rows, k0, &vr[0][0], RR);
         }
-        __syncthreads();
-        if (wave * 16 < npad) {
-            f32x4_m s = {0.f, 0.f, 0.f, 0.f};
-            for (int k = 0; k < w; k += 32)
-                s = mma16(*reinterpret_cast<const u32x4_m*>(qs + c * ws + k + 8 * kg), *reinterpret_cast<const u32x4_m*>(rows + (wave * 16 + c) * ws + k + 8 * kg), s);
-#pragma unroll
-            for (int i = 0; i < 4; ++i) sc[(4 * kg + i) * (kTileP + 1) + wave * 16 + c] = s[i] * a.scale;
+        asm volatile("" ::: "memory");
+        f32x4_m s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
+        for (int k = 0; k < w; k += 32) {
+            const u32x4_m qv = *reinterpret_cast<const u32x4_m*>(qs + c * ws + k + 8 * kg);
+            s0 = mma16(*reinterpret_cast<const u32x4_m*>(rows + c * ws + k + 8 * kg), qv, s0);
+            s1 = mma16(*reinterpret_cast<const u32x4_m*>(rows + (16 + c) * ws + k + 8 * kg), qv, s1);
         }
-        __syncthreads();
-        {   // head 4 * wave + kg: lanes c take rows c, c + 16, ..
-            const int h = 4 * wave + kg;
-            float v[4], mx = -INFINITY;
+        float x[8], mx = -INFINITY;
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                v[i] = c + 16 * i < np ? sc[h * (kTileP + 1) + c + 16 * i] : -INFINITY;
-                mx = fmaxf(mx, v[i]);
-            }
-            const float mn = fmaxf(m_run, row16_max(mx));
-            float sum = 0.f;
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const float p = expf(v[i] - mn);
-                const bf16_t hi = f32_to_bf16(p);
-                ph[h * PS + c + 16 * i] = hi;
-                pl[h * PS + c + 16 * i] = f32_to_bf16(p - bf16_to_f32(hi));
-                sum += p;
-            }
-            const float cr = expf(m_run - mn);
-            l_run = l_run * cr + row16_sum(sum);
-            m_run = mn;
-            if (c == 0) corr[h] = cr;
+        for (int e = 0; e < 4; ++e) {
+            x[e] = 4 * kg + e < np ? s0[e] * scale2 : -INFINITY;
+            x[4 + e] = 16 + 4 * kg + e < np ? s1[e] * scale2 : -INFINITY;
+            mx = fmaxf(mx, fmaxf(x[e], x[4 + e]));
         }
-        __syncthreads();
-        float cr[4];
+        const float mn = fmaxf(m_run, col4_max(mx)), corr = __builtin_amdgcn_exp2f(m_run - mn);
+        float sum = 0.f;
+        u32x4_m ph, pl;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) cr[i] = corr[4 * kg + i];
+        for (int e = 0; e < 4; ++e) {
+            const float u = __builtin_amdgcn_exp2f(x[2 * e] - mn), v = __builtin_amdgcn_exp2f(x[2 * e + 1] - mn);
+            sum += u + v;
+            uint32_t hi, lo;
+            split_bf16_hw(u, v, hi, lo);
+            ph[e] = hi; pl[e] = lo;
+        }
+        l_run = l_run * corr + col4_sum(sum);
+        m_run = mn;
 #pragma unroll
-        for (int i = 0; i < RT; ++i)
+        for (int i = 0; i < RT; ++i) {
+            if (rp0 + 16 * i >= rank) break;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) acc[i][e] *= cr[e];
-        for (int k = 0; k < npad; k += 32) {
-            const u32x4_m ah = *reinterpret_cast<const u32x4_m*>(ph + c * PS + k + 8 * kg), al = *reinterpret_cast<const u32x4_m*>(pl + c * PS + k + 8 * kg);
-#pragma unroll
-            for (int i = 0; i < RT; ++i) {
-                const int r = (wave + 4 * i) * 16;
-                if (r >= rank) break;
-                const u32x4_m bv = lds_operand_t(rows + k * ws + r, ws, lane);
-                acc[i] = mma16(ah, bv, acc[i]);
-                acc[i] = mma16(al, bv, acc[i]);
-            }
+            for (int e = 0; e < 4; ++e) acc[i][e] *= corr;
+            const u32x4_m rv = lds_operand_t2(rows + rp0 + 16 * i, ws, lane);
+            acc[i] = mma16(rv, ph, acc[i]);
+            acc[i] = mma16(rv, pl, acc[i]);
         }
     }
+    if (c < hr) {
 #pragma unroll
-    for (int i = 0; i < RT; ++i) {
-        const int r = (wave + 4 * i) * 16 + c;
-        if (r >= rank) break;
+        for (int i = 0; i < RT; ++i) {
+            if (rp0 + 16 * i >= rank) break;
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-            if (4 * kg + e < hr) rec[(4 * kg + e) * rec_h + r] = acc[i][e];
-    }
-    if (c == 0 && 4 * wave + kg < hr) {
-        rec[(4 * wave + kg) * rec_h + rank] = m_run;
-        rec[(4 * wave + kg) * rec_h + rank + 1] = l_run;
+            for (int e = 0; e < 2; ++e)   // (records are 8-byte aligned: rank is even)
+                *reinterpret_cast<float2*>(rec + c * rec_h + rp0 + 16 * i + 4 * kg + 2 * e) = make_float2(acc[i][2 * e], acc[i][2 * e + 1]);
+        }
+        if (kg == 0 && rp0 == 0) {
+            rec[c * rec_h + rank] = m_run;
+            rec[c * rec_h + rank + 1] = l_run;
+        }
     }
 }
 
@@ -365,63 +375,131 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentDecodeArgs a,
     extern __shared__ float lat_lds[];
     const int rank = (int)a.rank, vdim = (int)a.vdim, H = (int)a.heads;
     float* lat = lat_lds;                        // [rank]
-    float* wgt = lat + rank;                     // [nsplit]
-    float* red = wgt + nsplit;                   // [256 / kOutV][kOutV]
-    const int t = threadIdx.x, h = blockIdx.x, v0 = blockIdx.y * kOutV, b = blockIdx.z;
-    const float* rec = part + ((int64_t)b * H + h) * nsplit * (rank + 2);
-    float m = -INFINITY, l = 0.f;
-    for (int s = 0; s < nsplit; ++s) m = fmaxf(m, rec[(int64_t)s * (rank + 2) + rank]);
-    for (int s = 0; s < nsplit; ++s) l += expf(rec[(int64_t)s * (rank + 2) + rank] - m) * rec[(int64_t)s * (rank + 2) + rank + 1];
-    if (t < nsplit) wgt[t] = expf(rec[(int64_t)t * (rank + 2) + rank] - m) / l;
-    __syncthreads();
-    for (int r = t; r < rank; r += 256) {
-        float v = 0.f;
-        for (int s = 0; s < nsplit; ++s)
-            if (wgt[s] != 0.f) v += wgt[s] * rec[(int64_t)s * (rank + 2) + r];   // (an empty slice left its sums unset)
-        lat[r] = v;
+    float* wgt = lat + rank;                     // [32]
+    float* red = wgt + 32;                       // [4][kOutV]
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, h = blockIdx.x, v0 = blockIdx.y * kOutV, b = blockIdx.z;
+    const int rs = rank + 2;
+    const float* rec = part + ((int64_t)b * H + h) * nsplit * rs;
+    // 4 lanes of 8 values, 64 groups of latent dimensions; the first words of W_uv and the first records are requested at once
+    const int v8 = 8 * (t & 3), g = t >> 2;
+    const bool vlive = v0 + v8 < vdim;
+    const int64_t ldw = (int64_t)H * vdim;
+    const bf16_t* wv = (const bf16_t*)a.w_uv + (int64_t)h * vdim + (vlive ? v0 + v8 : 0);
+    constexpr int U = 8;
+    u32x4_m x[U];
+    auto request = [&](int r0) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) x[u] = *reinterpret_cast<const u32x4_m*>(wv + (int64_t)min(r0 + 64 * u, rank - 1) * ldw);
+    };
+    request(g);
+    const float mv = lane < nsplit ? rec[(int64_t)lane * rs + rank] : -INFINITY, lv = lane < nsplit ? rec[(int64_t)lane * rs + rank + 1] : 0.f;
+    constexpr int SU = 16;
+    float2 y[2][SU];
+    auto records = [&](int r, int s0, float2* dst) __attribute__((always_inline)) {   // (clamped: what is not there is not used)
+#pragma unroll
+        for (int u = 0; u < SU; ++u) dst[u] = *reinterpret_cast<const float2*>(rec + (int64_t)min(s0 + u, nsplit - 1) * rs + min(r, rank - 2));
+    };
+    records(2 * t, 0, y[0]);
+    records(2 * t, SU, y[1]);
+    {   // every wave finds the weights of the (at most 32) slices; wave 0 leaves them in LDS
+        const float m = wave_max(mv), e = __builtin_amdgcn_exp2f(mv - m);
+        const float l = wave_sum(e * lv);
+        if (wave == 0 && lane < 32) wgt[lane] = e / l;
     }
     __syncthreads();
-    const int v = t % kOutV, g = t / kOutV;
-    const bf16_t* wv = (const bf16_t*)a.w_uv + (int64_t)h * vdim + v0 + v;
-    float s = 0.f;
-    if (v0 + v < vdim)
-        for (int r = g; r < rank; r += 256 / kOutV) s += lat[r] * bf16_to_f32(wv[(int64_t)r * H * vdim]);
-    red[g * kOutV + v] = s;
-    __syncthreads();
-    if (t < kOutV && v0 + t < vdim) {
-        float o = 0.f;
-        for (int q = 0; q < 256 / kOutV; ++q) o += red[q * kOutV + t];
-        ((bf16_t*)a.ctx)[((int64_t)b * H + h) * vdim + v0 + t] = f32_to_bf16(o);
+    for (int r = 2 * t; r < rank; r += 512) {
+        if (r != 2 * t) { records(r, 0, y[0]); records(r, SU, y[1]); }
+        float2 v = make_float2(0.f, 0.f);
+#pragma unroll
+        for (int q = 0; q < 2; ++q)
+#pragma unroll
+            for (int u = 0; u < SU; ++u) {
+                const float f = wgt[q * SU + u];   // zero behind the last slice, and for an empty one, whose sums are unset
+                v.x += f != 0.f ? f * y[q][u].x : 0.f;
+                v.y += f != 0.f ? f * y[q][u].y : 0.f;
+            }
+        lat[r] = v.x;
+        lat[r + 1] = v.y;
     }
+    __syncthreads();
+    float o[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) o[e] = 0.f;
+    for (int r0 = g; r0 < rank; r0 += 64 * U) {
+        if (r0 != g) request(r0);
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const float f = r0 + 64 * u < rank ? lat[r0 + 64 * u] : 0.f;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { o[2 * e] += f * bf16lo(x[u][e]); o[2 * e + 1] += f * bf16hi(x[u][e]); }
+        }
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {   // over the 16 groups of the wave: lanes 4 apart
+        float x = o[e];
+        x += __shfl_xor(x, 4, 64);
+        x += __shfl_xor(x, 8, 64);
+        x = col4_sum(x);
+        if (lane < 4) red[wave * kOutV + v8 + e] = x;
+    }
+    __syncthreads();
+    if (t < kOutV && v0 + t < vdim)
+        ((bf16_t*)a.ctx)[((int64_t)b * H + h) * vdim + v0 + t] = f32_to_bf16(red[t] + red[kOutV + t] + red[2 * kOutV + t] + red[3 * kOutV + t]);
 }
 
 // ---------------------------------------------------------------------------- prompts (bf16)
-constexpr int kQTile = 128;      // queries per workgroup: 32 per wave, two 16-row operands that share every key operand
+constexpr int kQTile = 128;      // queries per workgroup: 16 per wave
 constexpr int kKTile = 64;       // keys per step
 
-// Workgroup = 128 queries x head x sequence.  Keys [unrotated | shared rotated part] and values of 64 positions in LDS; scores,
-// online softmax in f32, weights as a bf16 value and its remainder, so that the products with the values see the f32
-// weights to 16 bits.  KS: dim + rot in steps of 32 (zero padded), VT: vdim in tiles of 16 (zero padded).
+// Workgroup = 128 queries x head x sequence, 8 waves.  Keys [unrotated | shared rotated part] and values of a step in LDS, the
+// next step's words in registers meanwhile.  Everything is transposed (scores: rows = keys, columns = queries; result:
+// rows = values), so a lane works on one query: softmax in f32 registers, the weights go from there into the product with the
+// values, as a bf16 value and its remainder.  KS: dim + rot in steps of 32, VT: vdim in tiles of 16 (both zero padded).
 template <int KS, int VT>
-__global__ __launch_bounds__(256, 1) void latent_prefill_kernel(LatentPrefillArgs a) {
+__global__ __launch_bounds__(512) void latent_prefill_kernel(LatentPrefillArgs a) {
     extern __shared__ __align__(16) unsigned char lat_smem[];
-    constexpr int KSTR = KS * 32 + 8, VSTR = VT * 16 + 8, PSTR = kKTile + 8;
-    bf16_t* kt = reinterpret_cast<bf16_t*>(lat_smem);      // [64][KSTR]
-    bf16_t* vt = kt + kKTile * KSTR;                       // [64][VSTR]
-    bf16_t* pw = vt + kKTile * VSTR;                       // per wave: [2][32][PSTR]
+    constexpr int KSTR = KS * 32 + 8, VSTR = VT * 16 + 8;
+    bf16_t* kt = reinterpret_cast<bf16_t*>(lat_smem);                 // [64][KSTR]
+    bf16_t* vt = kt + kKTile * KSTR;                                  // [64][VSTR]
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, c = lane & 15, kg = lane >> 4;
     const int b = blockIdx.z, h = blockIdx.y, T = a.len[b], r0 = a.row0[b];
     const int q0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * kQTile;   // the longest workgroups first
     if (q0 >= T) return;
     const int dim = (int)a.dim, rot = (int)a.rot, hd = dim + rot, vdim = (int)a.vdim, H = (int)a.heads, w = (int)(a.rank + a.rot);
-    bf16_t* ph = pw + wave * 2 * 32 * PSTR;
-    bf16_t* pl = ph + 32 * PSTR;
+    const int kend = min(q0 + kQTile, T);
+    const int myq = q0 + wave * 16, qi = myq + c;                     // the wave's first query, the lane's
 
-    // queries: rotated on the way in, rounded once; rows behind the prompt repeat its last row and are not stored
-    u32x4_m q[2][KS];
+    // A thread's words of a step, by 32-bit offsets from uniform bases.  Nothing is loaded conditionally: keys behind the last
+    // one repeat it (their scores are masked), columns behind a row's end repeat its start (the queries are zero there, or the
+    // result is not stored).
+    constexpr int KW = KS * 4, VW = VT * 2;                           // 16-byte words per staged row
+    constexpr int KU = kKTile * KW / 512, VU = (kKTile * VW + 511) / 512;   // ... per thread
+    static_assert(kKTile * KW % 512 == 0 && kKTile * VW % 512 == 0, "whole rounds of the workgroup");
+    u32x4_m rk[KU], rv[VU];
+    const char* kbase = (const char*)a.k + ((int64_t)r0 * H + h) * dim * 2;
+    const char* rbase = (const char*)a.rows + ((int64_t)r0 * w + a.rank) * 2;
+    const char* vbase = (const char*)a.v + ((int64_t)r0 * H + h) * vdim * 2;
+    auto fetch = [&](int k0) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-        const int row = r0 + min(q0 + wave * 32 + i * 16 + c, T - 1);
+        for (int u = 0; u < KU; ++u) {
+            const int i = t + 512 * u, d = (i % KW) * 8, pos = min(k0 + i / KW, kend - 1);
+            const bool un = d < dim || d >= hd;                       // an unrotated column
+            const char* base = un ? kbase : rbase;
+            const unsigned off = un ? (unsigned)pos * (unsigned)(H * dim * 2) + (unsigned)((d < dim ? d : 0) * 2) : (unsigned)pos * (unsigned)(w * 2) + (unsigned)((d - dim) * 2);
+            rk[u] = *reinterpret_cast<const u32x4_m*>(base + off);
+        }
+#pragma unroll
+        for (int u = 0; u < VU; ++u) {
+            const int i = t + 512 * u, d = (i % VW) * 8, pos = min(k0 + i / VW, kend - 1);
+            rv[u] = *reinterpret_cast<const u32x4_m*>(vbase + ((unsigned)pos * (unsigned)(H * vdim * 2) + (unsigned)((d < vdim ? d : 0) * 2)));
+        }
+    };
+    fetch(0);
+
+    // queries: rotated on the way in, rounded once; columns behind the prompt repeat its last query and are not stored
+    u32x4_m q[KS];
+    {
+        const int row = r0 + min(qi, T - 1);
         const bf16_t* src = (const bf16_t*)a.x + ((int64_t)row * H + h) * hd;
         const float* tab = a.table + (int64_t)row * rot;
 #pragma unroll
@@ -439,115 +517,89 @@ __global__ __launch_bounds__(256, 1) void latent_prefill_kernel(LatentPrefillArg
                     }
                 }
             }
-            q[i][k] = v;
+            q[k] = v;
         }
     }
-    f32x4_m o[2][VT];
-    float m[2][4], l[2][4];
+    f32x4_m o[VT];
+    float m = -INFINITY, l = 0.f;
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-#pragma unroll
-        for (int v = 0; v < VT; ++v) o[i][v] = f32x4_m{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int e = 0; e < 4; ++e) { m[i][e] = -INFINITY; l[i][e] = 0.f; }
-    }
-    const float scale2 = a.scale * 1.44269504f;            // weights as powers of two
-    const int kend = min(q0 + kQTile, T);
-    const int myq = q0 + wave * 32;                        // the wave's first query
-    constexpr int KW = KS * 4, VW = VT * 2;                // 16-byte words per staged row
+    for (int v = 0; v < VT; ++v) o[v] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+    const float scale2 = a.scale * 1.44269504f;                       // weights as powers of two
     for (int k0 = 0; k0 < kend; k0 += kKTile) {
         __syncthreads();
-        for (int i = t; i < kKTile * KW; i += 256) {
-            const int r = i / KW, d = (i % KW) * 8, pos = k0 + r;
-            uint4 v = make_uint4(0u, 0u, 0u, 0u);
-            if (pos < kend && d < hd)
-                v = d < dim ? *reinterpret_cast<const uint4*>((const bf16_t*)a.k + ((int64_t)(r0 + pos) * H + h) * dim + d)
-                            : *reinterpret_cast<const uint4*>((const bf16_t*)a.rows + (int64_t)(r0 + pos) * w + (int)a.rank + d - dim);
-            *reinterpret_cast<uint4*>(kt + r * KSTR + d) = v;
+#pragma unroll
+        for (int u = 0; u < KU; ++u) {
+            const int i = t + 512 * u;
+            *reinterpret_cast<u32x4_m*>(kt + (i / KW) * KSTR + (i % KW) * 8) = rk[u];
         }
-        for (int i = t; i < kKTile * VW; i += 256) {
-            const int r = i / VW, d = (i % VW) * 8, pos = k0 + r;
-            uint4 v = make_uint4(0u, 0u, 0u, 0u);
-            if (pos < kend && d < vdim) v = *reinterpret_cast<const uint4*>((const bf16_t*)a.v + ((int64_t)(r0 + pos) * H + h) * vdim + d);
-            *reinterpret_cast<uint4*>(vt + r * VSTR + d) = v;
+#pragma unroll
+        for (int u = 0; u < VU; ++u) {
+            const int i = t + 512 * u;
+            *reinterpret_cast<u32x4_m*>(vt + (i / VW) * VSTR + (i % VW) * 8) = rv[u];
         }
         __syncthreads();
-        if (k0 > myq + 31) continue;                       // all keys of the step lie ahead of the wave's queries
-        f32x4_m s[2][4];
+        if (k0 + kKTile < kend) fetch(k0 + kKTile);
+        if (k0 > myq + 15) continue;                                  // all keys of the step lie ahead of the wave's queries
+        f32x4_m s[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            s[0][j] = s[1][j] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+            s[j] = f32x4_m{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int k = 0; k < KS; ++k) {
-                const u32x4_m kv = *reinterpret_cast<const u32x4_m*>(kt + (16 * j + c) * KSTR + 32 * k + 8 * kg);
-                s[0][j] = mma16(q[0][k], kv, s[0][j]);
-                s[1][j] = mma16(q[1][k], kv, s[1][j]);
-            }
+            for (int k = 0; k < KS; ++k) s[j] = mma16(*reinterpret_cast<const u32x4_m*>(kt + (16 * j + c) * KSTR + 32 * k + 8 * kg), q[k], s[j]);
         }
-        const bool edge = k0 + kKTile - 1 > myq;           // some key lies ahead of some query (or behind the prompt)
+        const bool edge = k0 + kKTile - 1 > myq;                      // some key lies ahead of some query
+        float mx = -INFINITY;
 #pragma unroll
-        for (int i = 0; i < 2; ++i) {
+        for (int j = 0; j < 4; ++j)
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                const int qi = myq + i * 16 + 4 * kg + e;
-                float x[4], mx = -INFINITY;
-#pragma unroll
-                for (int j = 0; j < 4; ++j) {
-                    x[j] = s[i][j][e] * scale2;
-                    if (edge && k0 + 16 * j + c > qi) x[j] = -INFINITY;
-                    mx = fmaxf(mx, x[j]);
-                }
-                const float mn = fmaxf(m[i][e], row16_max(mx));   // finite: key k0 <= myq + 31 may lie ahead of qi only after key 0 was seen
-                const float corr = __builtin_amdgcn_exp2f(m[i][e] - mn);
-                float sum = 0.f;
-#pragma unroll
-                for (int j = 0; j < 4; ++j) {
-                    const float p = __builtin_amdgcn_exp2f(x[j] - mn);
-                    sum += p;
-                    const uint32_t hi = pack_bf16_hw(p, 0.f) & 0xFFFFu;
-                    ph[(i * 16 + 4 * kg + e) * PSTR + 16 * j + c] = (bf16_t)hi;
-                    pl[(i * 16 + 4 * kg + e) * PSTR + 16 * j + c] = (bf16_t)(pack_bf16_hw(p - __uint_as_float(hi << 16), 0.f) & 0xFFFFu);
-                }
-                l[i][e] = l[i][e] * corr + row16_sum(sum);
-                m[i][e] = mn;
-#pragma unroll
-                for (int v = 0; v < VT; ++v) o[i][v][e] *= corr;
+                float x = s[j][e] * scale2;
+                if (edge && k0 + 16 * j + 4 * kg + e > qi) x = -INFINITY;
+                s[j][e] = x;
+                mx = fmaxf(mx, x);
             }
-        }
-        // (the weights are the wave's own: its LDS operations complete in order)
-        asm volatile("" ::: "memory");
+        // k0 and myq are multiples of 16 and k0 <= myq + 15, so every query sees key k0: the maximum is finite
+        const float mn = fmaxf(m, col4_max(mx));
+        float sum = 0.f;
+        u32x4_m ph[2], pl[2];
 #pragma unroll
-        for (int k = 0; k < kKTile / 32; ++k) {
-            u32x4_m p0[2], p1[2];
+        for (int j = 0; j < 4; ++j)
 #pragma unroll
-            for (int i = 0; i < 2; ++i) {
-                p0[i] = *reinterpret_cast<const u32x4_m*>(ph + (i * 16 + c) * PSTR + 32 * k + 8 * kg);
-                p1[i] = *reinterpret_cast<const u32x4_m*>(pl + (i * 16 + c) * PSTR + 32 * k + 8 * kg);
+            for (int e = 0; e < 2; ++e) {
+                const float u = __builtin_amdgcn_exp2f(s[j][2 * e] - mn), v = __builtin_amdgcn_exp2f(s[j][2 * e + 1] - mn);
+                sum += u + v;
+                uint32_t hi, lo;
+                split_bf16_hw(u, v, hi, lo);
+                ph[j / 2][2 * (j & 1) + e] = hi;
+                pl[j / 2][2 * (j & 1) + e] = lo;
             }
-#pragma unroll
-            for (int v = 0; v < VT; ++v) {
-                const u32x4_m vv = lds_operand_t(vt + 32 * k * VSTR + 16 * v, VSTR, lane);
-#pragma unroll
-                for (int i = 0; i < 2; ++i) {
-                    o[i][v] = mma16(p0[i], vv, o[i][v]);
-                    o[i][v] = mma16(p1[i], vv, o[i][v]);
-                }
-            }
-        }
-        asm volatile("" ::: "memory");
-    }
-#pragma unroll
-    for (int i = 0; i < 2; ++i)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int qi = myq + i * 16 + 4 * kg + e;
-            if (qi >= T) continue;
-            const float inv = 1.0f / l[i][e];
-            bf16_t* out = (bf16_t*)a.ctx + ((int64_t)(r0 + qi) * H + h) * vdim;
+        sum = col4_sum(sum);
+        if (__builtin_amdgcn_ballot_w64(mn > m) != 0) {               // some column's maximum has moved
+            const float corr = __builtin_amdgcn_exp2f(m - mn);
+            l *= corr;
 #pragma unroll
             for (int v = 0; v < VT; ++v)
-                if (16 * v + c < vdim) out[16 * v + c] = f32_to_bf16(o[i][v][e] * inv);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) o[v][e] *= corr;
+            m = mn;
         }
+        l += sum;
+#pragma unroll
+        for (int k = 0; k < kKTile / 32; ++k)
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const u32x4_m vv = lds_operand_t2(vt + 32 * k * VSTR + 16 * v, VSTR, lane);
+                o[v] = mma16(vv, ph[k], o[v]);
+                o[v] = mma16(vv, pl[k], o[v]);
+            }
+    }
+    if (qi >= T) return;
+    const float inv = 1.0f / l;
+    bf16_t* out = (bf16_t*)a.ctx + ((int64_t)(r0 + qi) * H + h) * vdim + 4 * kg;
+#pragma unroll
+    for (int v = 0; v < VT; ++v)
+        if (16 * v + 4 * kg < vdim)
+            *reinterpret_cast<uint2*>(out + 16 * v) = make_uint2(pack_bf16_hw(o[v][0] * inv, o[v][1] * inv), pack_bf16_hw(o[v][2] * inv, o[v][3] * inv));
 }
 
 template <typename F>
@@ -599,18 +651,18 @@ static size_t lat_align(size_t n) { return (n + 255) / 256 * 256; }
 static int latent_nsplit(int64_t nseq, int64_t capacity, int64_t heads) {
     const int64_t blocks = nseq * cdiv_l(heads, kHeadTile);
     int64_t n = std::min<int64_t>(cdiv_l(capacity, 32), 32);
-    while (n > 4 && blocks * n > 1024) n = (n + 1) / 2;
+    while (n > 4 && blocks * n > 512) n = (n + 1) / 2;
     return (int)std::max<int64_t>(n, 1);
 }
 static size_t latent_partial_lds(int64_t w) {
-    return (size_t)((kTileP + kHeadTile) * (w + 8) + 2 * kHeadTile * (kTileP + 8)) * 2 + (kHeadTile * (kTileP + 1) + kHeadTile) * 4;
+    return (size_t)(kTileP + kHeadTile) * (w + 8) * 2;
 }
-static bool latent_fast(int dtype, int64_t heads, int64_t dim, int64_t rot, int64_t rank) {
-    return dtype == 2 && heads >= 1 && dim % 8 == 0 && rot % 2 == 0 && rank % 16 == 0 && (rank + rot) % 32 == 0 && rank <= 1024 && dim <= 512 &&
+static bool latent_fast(int dtype, int64_t heads, int64_t dim, int64_t rot, int64_t rank, int64_t vdim) {
+    return dtype == 2 && heads >= 1 && dim % 8 == 0 && vdim % 8 == 0 && rot % 2 == 0 && rank % 16 == 0 && (rank + rot) % 32 == 0 && rank <= 1024 && dim <= 512 &&
            latent_partial_lds(rank + rot) <= 160 * 1024;
 }
-size_t latent_decode_scratch_bytes(int dtype, int64_t nseq, int64_t capacity, int64_t heads, int64_t dim, int64_t rot, int64_t rank) {
-    if (latent_fast(dtype, heads, dim, rot, rank))
+size_t latent_decode_scratch_bytes(int dtype, int64_t nseq, int64_t capacity, int64_t heads, int64_t dim, int64_t rot, int64_t rank, int64_t vdim) {
+    if (latent_fast(dtype, heads, dim, rot, rank, vdim))
         return lat_align((size_t)(nseq * heads * (rank + rot)) * 2) + (size_t)(nseq * heads * (rank + 2)) * 32 * sizeof(float);
     const size_t es = dtype == 0 ? 4 : 2;
     return lat_align((size_t)(nseq * heads * (dim + rot)) * es);
@@ -618,22 +670,20 @@ size_t latent_decode_scratch_bytes(int dtype, int64_t nseq, int64_t capacity, in
 int latent_decode(hipStream_t s, const LatentDecodeArgs& a) {
     const size_t es = a.dtype == 0 ? 4 : 2;
     const int64_t w = a.rank + a.rot;
-    if (latent_fast(a.dtype, a.heads, a.dim, a.rot, a.rank)) {
+    if (latent_fast(a.dtype, a.heads, a.dim, a.rot, a.rank, a.vdim)) {
         bf16_t* ql = (bf16_t*)a.scratch;
         float* part = (float*)((char*)a.scratch + lat_align((size_t)(a.nseq * a.heads * w) * 2));
         const int ns = latent_nsplit(a.nseq, a.capacity, a.heads);
         const int64_t rc = cdiv_l(a.rank, kPrepRows);
         latent_prep_kernel<<<(unsigned)(a.heads * rc + (a.raw ? a.nseq : 0)), 256, (size_t)std::max<int64_t>(a.nseq * a.dim, 16) * 4, s>>>(a, ql);
         const size_t lds = latent_partial_lds(w);
-        const dim3 grid((unsigned)ns, (unsigned)cdiv_l(a.heads, kHeadTile), (unsigned)a.nseq);
-        const int64_t rt = cdiv_l(a.rank / 16, 4);
-#define GPTRS_PARTIAL(RT) do { with_lds(latent_partial_kernel<RT>, lds); latent_partial_kernel<RT><<<grid, 256, lds, s>>>(a, ql, part, ns); } while (0)
-        if (rt <= 2) GPTRS_PARTIAL(2);
-        else if (rt <= 4) GPTRS_PARTIAL(4);
-        else if (rt <= 8) GPTRS_PARTIAL(8);
+        const int64_t rt = a.rank / 16;
+        const dim3 grid((unsigned)ns, (unsigned)(cdiv_l(a.heads, kHeadTile) * cdiv_l(rt, 16)), (unsigned)a.nseq);
+#define GPTRS_PARTIAL(RT) do { with_lds(latent_partial_kernel<RT>, lds); latent_partial_kernel<RT><<<grid, 64, lds, s>>>(a, ql, part, ns); } while (0)
+        if (rt <= 8) GPTRS_PARTIAL(8);
         else GPTRS_PARTIAL(16);
 #undef GPTRS_PARTIAL
-        latent_combine_kernel<<<dim3((unsigned)a.heads, (unsigned)cdiv_l(a.vdim, kOutV), (unsigned)a.nseq), 256, (size_t)(a.rank + ns + 256) * 4, s>>>(a, part, ns);
+        latent_combine_kernel<<<dim3((unsigned)a.heads, (unsigned)cdiv_l(a.vdim, kOutV), (unsigned)a.nseq), 256, (size_t)(a.rank + 32 + 4 * kOutV) * 4, s>>>(a, part, ns);
         return 3;
     }
     rope_pairs(s, a.dtype, a.x, a.table, a.scratch, a.nseq, a.heads, a.dim + a.rot, a.dim, a.rot / 2);
@@ -661,10 +711,10 @@ size_t latent_prefill_scratch_bytes(int dtype, int64_t total, int64_t heads, int
 }
 template <int KS, int VT>
 static void launch_prefill(hipStream_t s, const LatentPrefillArgs& a, int64_t longest) {
-    constexpr int lds = (kKTile * (KS * 32 + 8) + kKTile * (VT * 16 + 8) + 4 * 2 * 32 * (kKTile + 8)) * 2;
+    constexpr int lds = kKTile * (KS * 32 + 8 + VT * 16 + 8) * 2;
     static_assert(lds <= 160 * 1024, "LDS of one CU");
     with_lds(latent_prefill_kernel<KS, VT>, lds);
-    latent_prefill_kernel<KS, VT><<<dim3((unsigned)cdiv_l(longest, kQTile), (unsigned)a.heads, (unsigned)a.nseq), 256, lds, s>>>(a);
+    latent_prefill_kernel<KS, VT><<<dim3((unsigned)cdiv_l(longest, kQTile), (unsigned)a.heads, (unsigned)a.nseq), 512, lds, s>>>(a);
 }
 template <int KS>
 static void launch_prefill_v(hipStream_t s, const LatentPrefillArgs& a, int64_t longest) {
@@ -673,12 +723,12 @@ static void launch_prefill_v(hipStream_t s, const LatentPrefillArgs& a, int64_t 
     else launch_prefill<KS, 16>(s, a, longest);
 }
 int latent_prefill(hipStream_t s, const LatentPrefillArgs& a) {
-    if (a.dtype == 2 && a.dim % 8 == 0 && a.rot % 8 == 0 && a.rank % 8 == 0 && a.vdim % 8 == 0 && a.dim + a.rot <= 256 && a.vdim <= 256) {
+    if (a.dtype == 2 && a.dim % 8 == 0 && a.rot % 8 == 0 && a.rank % 8 == 0 && a.vdim % 8 == 0 && a.dim + a.rot <= 256 && a.vdim <= 256 &&
+        a.total * std::max(a.heads * std::max(a.dim, a.vdim), a.rank + a.rot) < (1ll << 30)) {   // 32-bit offsets
         int64_t longest = 0;
         for (int b = 0; b < a.nseq; ++b) longest = std::max<int64_t>(longest, a.len[b]);
         const int64_t ks = cdiv_l(a.dim + a.rot, 32);
         if (ks <= 2) launch_prefill_v<2>(s, a, longest);
-        else if (ks <= 3) launch_prefill_v<3>(s, a, longest);
         else if (ks <= 4) launch_prefill_v<4>(s, a, longest);
         else if (ks <= 6) launch_prefill_v<6>(s, a, longest);
         else launch_prefill_v<8>(s, a, longest);

@@ -251,10 +251,16 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(SsmSeqArgs a, T* __restr
         win[k + 1] = r >= 0 ? *reinterpret_cast<const float4*>(p + r * a.ld) : *reinterpret_cast<const float4*>(a.conv_in[b] + (r + K - 1) * a.ch + c);
     }
     const int64_t t1 = t0 + kConvRows < a.len[b] ? t0 + kConvRows : a.len[b];
-    for (int64_t t = t0; t < t1; ++t) {
+    float4 in[kConvRows];   // all rows requested before the first is used
+#pragma unroll
+    for (int u = 0; u < kConvRows; ++u) in[u] = *reinterpret_cast<const float4*>(p + (t0 + u < t1 ? t0 + u : t1 - 1) * a.ld);
+#pragma unroll
+    for (int u = 0; u < kConvRows; ++u) {
+        const int64_t t = t0 + u;
+        if (t >= t1) break;
 #pragma unroll
         for (int k = 0; k + 1 < K; ++k) win[k] = win[k + 1];
-        win[K - 1] = *reinterpret_cast<const float4*>(p + t * a.ld);
+        win[K - 1] = in[u];
         float4 v = bias;
 #pragma unroll
         for (int k = 0; k < K; ++k) { v.x += tap[k].x * win[k].x; v.y += tap[k].y * win[k].y; v.z += tap[k].z * win[k].z; v.w += tap[k].w * win[k].w; }
@@ -268,23 +274,22 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(SsmSeqArgs a, T* __restr
 //     y_t = sum_{s <= t} (C_t . B_s) exp(cum_t - cum_s) dt_s x_s  +  exp(cum_t) S^T C_t  +  D x_t
 //     S  <- exp(cum_end) S + sum_s exp(cum_end - cum_s) dt_s B_s x_s^T
 // so a chunk is four small matrix products.  Workgroup = head x slice of 16 VT values x sequence, 4 waves; it walks the chunks of
-// its sequence.  Wave w owns the rows t = 16 w .. of a chunk and the states n = 16 (w + 4 i) .., i < NPW, which it keeps in f32
-// accumulators as S^T (rows: values, columns: states) from the first chunk to the last.  Factors that are not bf16 already (the
-// decayed scores, the weighted x, the state as an operand) enter the products as a bf16 value plus its remainder.
+// its sequence, the next chunk's words in registers while one is worked on.  Wave w owns the tokens t = 16 w .. of a chunk and
+// the states n = 16 (w + 4 i) .., i < NPW, which it keeps in f32 accumulators (rows: states, columns: values) from the first
+// chunk to the last.  Products are taken transposed (scores: rows = s, columns = t; result: rows = values, columns = t): the
+// decayed scores feed the second product from registers.  Factors that are not bf16 already (the decayed scores, the
+// weighted x, the state as an operand) enter the products as a bf16 value plus its remainder.  Logarithms are to base 2.
 constexpr int kChunk = 64;
 template <int NPW, int VT>
 __global__ __launch_bounds__(256) void ssd_kernel(SsmSeqArgs a, const bf16_t* __restrict__ xbc, bf16_t* __restrict__ y) {
-    constexpr int NP = 64 * NPW, NSTR = NP + 8, VS = 16 * VT, XSTR = VS + 8, MSTR = kChunk + 8;
+    constexpr int NP = 64 * NPW, NSTR = NP + 8, VS = 16 * VT, XSTR = VS + 8;
     extern __shared__ __align__(16) unsigned char ssd_smem[];
     bf16_t* Bm = reinterpret_cast<bf16_t*>(ssd_smem);   // [64][NSTR] token rows of B
     bf16_t* Cm = Bm + kChunk * NSTR;                    // [64][NSTR]
     bf16_t* xm = Cm + kChunk * NSTR;                    // [64][XSTR]
     bf16_t* sh = xm + kChunk * XSTR;                    // [VS][NSTR] S^T
     bf16_t* sl = sh + VS * NSTR;                        // [VS][NSTR] its remainder
-    bf16_t* mm = sl + VS * NSTR;                        // per wave: [2][16][MSTR]
-    float* cum = reinterpret_cast<float*>(mm + 4 * 2 * 16 * MSTR);   // [64]
-    float* dts = cum + kChunk;                          // [64] step sizes
-    float* wgt = dts + kChunk;                          // [64] exp(cum_end - cum_s) dt_s
+    float* steps = reinterpret_cast<float*>(sl + VS * NSTR);   // two buffers of cum | dt | exp(cum_end - cum_s) dt_s, [64] each
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, kg = lane >> 4;
     const int h = blockIdx.x, v0 = blockIdx.y * VS, b = blockIdx.z, T = a.len[b];
     const int N = (int)a.n, vdim = (int)a.vdim, inner = (int)(a.heads * a.vdim), grp = h / (int)(a.heads / a.groups);
@@ -295,20 +300,17 @@ __global__ __launch_bounds__(256) void ssd_kernel(SsmSeqArgs a, const bf16_t* __
     const bf16_t* bsrc = rows + inner + (int64_t)grp * N;
     const bf16_t* csrc = bsrc + a.groups * (int64_t)N;
     const bf16_t* xsrc = rows + (int64_t)h * vdim + v0;
-    const float rate = expf(a.a_log[h]), dtb = a.dt_bias[h], dd = a.d[h];
-    bf16_t* mh = mm + wave * 2 * 16 * MSTR;
-    bf16_t* ml = mh + 16 * MSTR;
+    const float rate2 = expf(a.a_log[h]) * 1.44269504f, dtb = a.dt_bias[h], dd = a.d[h];
 
-    // state in, columns n of rows v
-    f32x4_m S[VT][NPW];
+    f32x4_m S[NPW][VT];                                 // rows n = 16 (wave + 4 j) + 4 kg + e, column v = 16 i + c
 #pragma unroll
-    for (int i = 0; i < VT; ++i)
+    for (int j = 0; j < NPW; ++j)
 #pragma unroll
-        for (int j = 0; j < NPW; ++j)
+        for (int i = 0; i < VT; ++i)
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                const int n = 16 * (wave + 4 * j) + c, v = v0 + 16 * i + 4 * kg + e;
-                S[i][j][e] = n < N && v < vdim ? a.state_in[b][((int64_t)h * N + n) * vdim + v] : 0.f;
+                const int n = 16 * (wave + 4 * j) + 4 * kg + e, v = v0 + 16 * i + c;
+                S[j][i][e] = n < N && v < vdim ? a.state_in[b][((int64_t)h * N + n) * vdim + v] : 0.f;
             }
     // columns that no token fills stay zero
     for (int i = tid; i < kChunk * (NP / 8); i += 256) {
@@ -318,18 +320,20 @@ __global__ __launch_bounds__(256) void ssd_kernel(SsmSeqArgs a, const bf16_t* __
             *reinterpret_cast<uint4*>(Cm + r * NSTR + n) = make_uint4(0u, 0u, 0u, 0u);
         }
     }
-    const int nw = N / 8;                               // 16-byte words per row of B and C
-    constexpr int BU = (kChunk * (NP / 8) + 255) / 256, XW = VS / 8, XU = (kChunk * XW + 255) / 256;
+    // a thread's words of a chunk: the same place of rows BR apart
+    constexpr int NW = NP / 8, BR = 256 / NW, BU = kChunk / BR, XW = VS / 8, XU = (kChunk * XW + 255) / 256;
+    const int br = tid / NW, bk = 8 * (tid % NW);
+    const bool bl = bk < N;
     uint4 rb[BU], rc[BU], rx[XU];
     float rdt = 0.f;
-    auto fetch = [&](int t0) {                          // a chunk's words into registers; tokens behind the prompt are zero
+    auto fetch = [&](int t0) {                          // tokens behind the prompt are zero
 #pragma unroll
         for (int u = 0; u < BU; ++u) {
-            const int i = tid + 256 * u, r = i / nw, k = i % nw;
+            const int r = t0 + br + BR * u;
             rb[u] = rc[u] = make_uint4(0u, 0u, 0u, 0u);
-            if (i < kChunk * nw && t0 + r < T) {
-                rb[u] = *reinterpret_cast<const uint4*>(bsrc + (int64_t)(t0 + r) * ch + 8 * k);
-                rc[u] = *reinterpret_cast<const uint4*>(csrc + (int64_t)(t0 + r) * ch + 8 * k);
+            if (bl && r < T) {
+                rb[u] = *reinterpret_cast<const uint4*>(bsrc + (int64_t)r * ch + bk);
+                rc[u] = *reinterpret_cast<const uint4*>(csrc + (int64_t)r * ch + bk);
             }
         }
 #pragma unroll
@@ -340,15 +344,31 @@ __global__ __launch_bounds__(256) void ssd_kernel(SsmSeqArgs a, const bf16_t* __
         }
         if (wave == 0) rdt = t0 + lane < T ? p[(int64_t)(t0 + lane) * a.ld] : 0.f;
     };
-    fetch(0);
-    for (int t0 = 0; t0 < T; t0 += kChunk) {
-        __syncthreads();                                // the previous chunk has been read
+    auto decays = [&](int t0, float* st) {              // wave 0: step sizes and running decays of a chunk
+        const bool live = t0 + lane < T;                // behind the prompt: no step, no decay
+        const float dt = live ? softplus_f32(rdt + dtb) : 0.f;
+        float s = -rate2 * dt;
 #pragma unroll
-        for (int u = 0; u < BU; ++u) {
-            const int i = tid + 256 * u, r = i / nw, k = i % nw;
-            if (i < kChunk * nw) {
-                *reinterpret_cast<uint4*>(Bm + r * NSTR + 8 * k) = rb[u];
-                *reinterpret_cast<uint4*>(Cm + r * NSTR + 8 * k) = rc[u];
+        for (int off = 1; off < 64; off <<= 1) {
+            const float o = __shfl_up(s, off, 64);
+            if (lane >= off) s += o;
+        }
+        const float end = __shfl(s, 63, 64);
+        st[lane] = s;
+        st[kChunk + lane] = dt;
+        st[2 * kChunk + lane] = __builtin_amdgcn_exp2f(end - s) * dt;
+    };
+    fetch(0);
+    if (wave == 0) decays(0, steps);
+    int buf = 0;
+    for (int t0 = 0; t0 < T; t0 += kChunk, buf ^= 1) {
+        const float* cum = steps + buf * 3 * kChunk;
+        __syncthreads();                                // the previous chunk has been read
+        if (bl) {
+#pragma unroll
+            for (int u = 0; u < BU; ++u) {
+                *reinterpret_cast<uint4*>(Bm + (br + BR * u) * NSTR + bk) = rb[u];
+                *reinterpret_cast<uint4*>(Cm + (br + BR * u) * NSTR + bk) = rc[u];
             }
         }
 #pragma unroll
@@ -357,131 +377,165 @@ __global__ __launch_bounds__(256) void ssd_kernel(SsmSeqArgs a, const bf16_t* __
             if (i < kChunk * XW) *reinterpret_cast<uint4*>(xm + r * XSTR + 8 * k) = rx[u];
         }
 #pragma unroll
-        for (int i = 0; i < VT; ++i)
+        for (int j = 0; j < NPW; ++j)
 #pragma unroll
-            for (int j = 0; j < NPW; ++j)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const int at = (16 * i + 4 * kg + e) * NSTR + 16 * (wave + 4 * j) + c;
-                    const uint32_t hi = pack_bf16_hw(S[i][j][e], 0.f) & 0xFFFFu;
-                    sh[at] = (bf16_t)hi;
-                    sl[at] = (bf16_t)(pack_bf16_hw(S[i][j][e] - __uint_as_float(hi << 16), 0.f) & 0xFFFFu);
-                }
-        if (wave == 0) {
-            const bool live = t0 + lane < T;            // behind the prompt: no step, no decay
-            const float dt = live ? softplus_f32(rdt + dtb) : 0.f;
-            float s = -rate * dt;
-#pragma unroll
-            for (int off = 1; off < 64; off <<= 1) {
-                const float o = __shfl_up(s, off, 64);
-                if (lane >= off) s += o;
+            for (int i = 0; i < VT; ++i) {
+                const int at = (16 * i + c) * NSTR + 16 * (wave + 4 * j) + 4 * kg;
+                uint2 hi, lo;
+                split_bf16_hw(S[j][i][0], S[j][i][1], hi.x, lo.x);
+                split_bf16_hw(S[j][i][2], S[j][i][3], hi.y, lo.y);
+                *reinterpret_cast<uint2*>(sh + at) = hi;
+                *reinterpret_cast<uint2*>(sl + at) = lo;
             }
-            const float end = __shfl(s, 63, 64);
-            cum[lane] = s;
-            dts[lane] = dt;
-            wgt[lane] = expf(end - s) * dt;
-        }
         __syncthreads();
-        if (t0 + kChunk < T) fetch(t0 + kChunk);
+        const bool more = t0 + kChunk < T;
+        if (more) fetch(t0 + kChunk);
 
-        // scores of the wave's 16 tokens against tokens 0 .. 16 wave + 15 of the chunk
+        // columns: the wave's 16 tokens
         u32x4_m ca[2 * NPW];
 #pragma unroll
         for (int k = 0; k < 2 * NPW; ++k) ca[k] = *reinterpret_cast<const u32x4_m*>(Cm + (16 * wave + c) * NSTR + 32 * k + 8 * kg);
-        float ct[4];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) ct[e] = cum[16 * wave + 4 * kg + e];
-        const int ksteps = wave / 2 + 1;                // steps of 32 tokens that reach the wave's rows
-        for (int j = 0; j < 2 * ksteps; ++j) {
-            f32x4_m g = {0.f, 0.f, 0.f, 0.f};
-            if (j <= wave) {
-#pragma unroll
-                for (int k = 0; k < 2 * NPW; ++k)
-                    g = mma16(ca[k], *reinterpret_cast<const u32x4_m*>(Bm + (16 * j + c) * NSTR + 32 * k + 8 * kg), g);
-            }
-            const float cs = cum[16 * j + c], ds = dts[16 * j + c];
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float f = 16 * j + c <= 16 * wave + 4 * kg + e ? g[e] * (expf(ct[e] - cs) * ds) : 0.f;
-                const uint32_t hi = pack_bf16_hw(f, 0.f) & 0xFFFFu;
-                mh[(4 * kg + e) * MSTR + 16 * j + c] = (bf16_t)hi;
-                ml[(4 * kg + e) * MSTR + 16 * j + c] = (bf16_t)(pack_bf16_hw(f - __uint_as_float(hi << 16), 0.f) & 0xFFFFu);
-            }
-        }
-        asm volatile("" ::: "memory");                // (the wave's own values: its LDS operations complete in order)
-        f32x4_m yi[VT], ys[VT];
+        const float ct = cum[16 * wave + c];
+        f32x4_m yt[VT];
+        const float et = __builtin_amdgcn_exp2f(ct);
 #pragma unroll
         for (int i = 0; i < VT; ++i) {
-            yi[i] = ys[i] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+            yt[i] = f32x4_m{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int k = 0; k < 2 * NPW; ++k) {
-                ys[i] = mma16(ca[k], *reinterpret_cast<const u32x4_m*>(sh + (16 * i + c) * NSTR + 32 * k + 8 * kg), ys[i]);
-                ys[i] = mma16(ca[k], *reinterpret_cast<const u32x4_m*>(sl + (16 * i + c) * NSTR + 32 * k + 8 * kg), ys[i]);
+                yt[i] = mma16(*reinterpret_cast<const u32x4_m*>(sh + (16 * i + c) * NSTR + 32 * k + 8 * kg), ca[k], yt[i]);
+                yt[i] = mma16(*reinterpret_cast<const u32x4_m*>(sl + (16 * i + c) * NSTR + 32 * k + 8 * kg), ca[k], yt[i]);
             }
+#pragma unroll
+            for (int e = 0; e < 4; ++e) yt[i][e] *= et;
         }
-        for (int k = 0; k < ksteps; ++k) {
-            const u32x4_m m0 = *reinterpret_cast<const u32x4_m*>(mh + c * MSTR + 32 * k + 8 * kg), m1 = *reinterpret_cast<const u32x4_m*>(ml + c * MSTR + 32 * k + 8 * kg);
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {                   // steps of 32 tokens s
+            if (k > wave / 2) break;
+            u32x4_m mh, ml;
+#pragma unroll
+            for (int jj = 0; jj < 2; ++jj) {
+                const int j = 2 * k + jj;
+                f32x4_m g = {0.f, 0.f, 0.f, 0.f};
+                if (j <= wave) {                        // later tokens do not reach the wave's
+#pragma unroll
+                    for (int q = 0; q < 2 * NPW; ++q)
+                        g = mma16(*reinterpret_cast<const u32x4_m*>(Bm + (16 * j + c) * NSTR + 32 * q + 8 * kg), ca[q], g);
+                }
+                const f32x4_m cs = *reinterpret_cast<const f32x4_m*>(cum + 16 * j + 4 * kg), ds = *reinterpret_cast<const f32x4_m*>(cum + kChunk + 16 * j + 4 * kg);
+                float f[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    f[e] = 16 * j + 4 * kg + e <= 16 * wave + c ? g[e] * (__builtin_amdgcn_exp2f(ct - cs[e]) * ds[e]) : 0.f;
+                uint32_t hi, lo;
+                split_bf16_hw(f[0], f[1], hi, lo);
+                mh[2 * jj] = hi; ml[2 * jj] = lo;
+                split_bf16_hw(f[2], f[3], hi, lo);
+                mh[2 * jj + 1] = hi; ml[2 * jj + 1] = lo;
+            }
 #pragma unroll
             for (int i = 0; i < VT; ++i) {
-                const u32x4_m xv = lds_operand_t(xm + 32 * k * XSTR + 16 * i, XSTR, lane);
-                yi[i] = mma16(m0, xv, yi[i]);
-                yi[i] = mma16(m1, xv, yi[i]);
+                const u32x4_m xv = lds_operand_t2(xm + 32 * k * XSTR + 16 * i, XSTR, lane);
+                yt[i] = mma16(xv, mh, yt[i]);
+                yt[i] = mma16(xv, ml, yt[i]);
             }
         }
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int t = 16 * wave + 4 * kg + e;
-            const float et = expf(ct[e]);
+        {
+            const int t = 16 * wave + c;
             if (t0 + t < T) {
 #pragma unroll
-                for (int i = 0; i < VT; ++i)
-                    if (v0 + 16 * i + c < vdim)
-                        yout[(int64_t)(t0 + t) * inner + 16 * i + c] = f32_to_bf16(yi[i][e] + et * ys[i][e] + dd * bf16_to_f32(xm[t * XSTR + 16 * i + c]));
+                for (int i = 0; i < VT; ++i) {
+                    if (v0 + 16 * i + 4 * kg >= vdim) continue;
+                    const uint2 xw = *reinterpret_cast<const uint2*>(xm + t * XSTR + 16 * i + 4 * kg);
+                    *reinterpret_cast<uint2*>(yout + (int64_t)(t0 + t) * inner + 16 * i + 4 * kg) =
+                        make_uint2(pack_bf16_hw(yt[i][0] + dd * bf16lo(xw.x), yt[i][1] + dd * bf16hi(xw.x)),
+                                   pack_bf16_hw(yt[i][2] + dd * bf16lo(xw.y), yt[i][3] + dd * bf16hi(xw.y)));
+                }
             }
         }
         // the state after the chunk
-        const float edecay = expf(cum[kChunk - 1]);
+        const float edecay = __builtin_amdgcn_exp2f(cum[kChunk - 1]);
 #pragma unroll
-        for (int i = 0; i < VT; ++i)
+        for (int j = 0; j < NPW; ++j)
 #pragma unroll
-            for (int j = 0; j < NPW; ++j)
+            for (int i = 0; i < VT; ++i)
 #pragma unroll
-                for (int e = 0; e < 4; ++e) S[i][j][e] *= edecay;
+                for (int e = 0; e < 4; ++e) S[j][i][e] *= edecay;
 #pragma unroll
         for (int k = 0; k < kChunk / 32; ++k) {
             u32x4_m bv[NPW];
 #pragma unroll
             for (int j = 0; j < NPW; ++j) bv[j] = lds_operand_t(Bm + 32 * k * NSTR + 16 * (wave + 4 * j), NSTR, lane);
-            float ws[8];
-#pragma unroll
-            for (int e = 0; e < 8; ++e) ws[e] = wgt[32 * k + 8 * kg + e];
+            const f32x4_m w0 = *reinterpret_cast<const f32x4_m*>(cum + 2 * kChunk + 32 * k + 8 * kg), w1 = *reinterpret_cast<const f32x4_m*>(cum + 2 * kChunk + 32 * k + 8 * kg + 4);
+            const float ws[8] = {w0[0], w0[1], w0[2], w0[3], w1[0], w1[1], w1[2], w1[3]};
 #pragma unroll
             for (int i = 0; i < VT; ++i) {
                 const u32x4_m xv = lds_operand_t(xm + 32 * k * XSTR + 16 * i, XSTR, lane);
                 u32x4_m xh, xl;
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    const float f0 = bf16lo(xv[e]) * ws[2 * e], f1 = bf16hi(xv[e]) * ws[2 * e + 1];
-                    xh[e] = pack_bf16_hw(f0, f1);
-                    xl[e] = pack_bf16_hw(f0 - bf16lo(xh[e]), f1 - bf16hi(xh[e]));
+                    uint32_t hi, lo;
+                    split_bf16_hw(bf16lo(xv[e]) * ws[2 * e], bf16hi(xv[e]) * ws[2 * e + 1], hi, lo);
+                    xh[e] = hi; xl[e] = lo;
                 }
 #pragma unroll
                 for (int j = 0; j < NPW; ++j) {
-                    S[i][j] = mma16(xh, bv[j], S[i][j]);
-                    S[i][j] = mma16(xl, bv[j], S[i][j]);
+                    S[j][i] = mma16(bv[j], xh, S[j][i]);
+                    S[j][i] = mma16(bv[j], xl, S[j][i]);
                 }
             }
         }
+        if (more && wave == 0) decays(t0 + kChunk, steps + (buf ^ 1) * 3 * kChunk);
     }
 #pragma unroll
-    for (int i = 0; i < VT; ++i)
+    for (int j = 0; j < NPW; ++j)
 #pragma unroll
-        for (int j = 0; j < NPW; ++j)
+        for (int i = 0; i < VT; ++i)
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                const int n = 16 * (wave + 4 * j) + c, v = v0 + 16 * i + 4 * kg + e;
-                if (n < N && v < vdim) a.state_out[b][((int64_t)h * N + n) * vdim + v] = S[i][j][e];
+                const int n = 16 * (wave + 4 * j) + 4 * kg + e, v = v0 + 16 * i + c;
+                if (n < N && v < vdim) a.state_out[b][((int64_t)h * N + n) * vdim + v] = S[j][i][e];
             }
+}
+
+// Gated norm of bf16 rows whose parts are multiples of 8: a wave per row and part of up to 64 * 8 * KEEP values, each formed once.
+constexpr int kNormKeep = 4;
+__global__ __launch_bounds__(256) void gated_norm_wave_kernel(const bf16_t* __restrict__ y, const float* __restrict__ p, const float* __restrict__ gain,
+                                                              bf16_t* __restrict__ out, int64_t rows, int64_t n, int64_t ld, int64_t col, int part,
+                                                              int groups, float eps) {
+    const int lane = threadIdx.x & 63;
+    const int64_t job = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (job >= rows * groups) return;
+    const int64_t r = job / groups, g0 = (job % groups) * part;
+    float v[kNormKeep][8];
+    float q = 0.f;
+#pragma unroll
+    for (int u = 0; u < kNormKeep; ++u) {
+        const int i = 8 * (lane + 64 * u);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[u][e] = 0.f;
+        if (i < part) {
+            const uint4 yw = *reinterpret_cast<const uint4*>(y + r * n + g0 + i);
+            const float* z = p + r * ld + col + g0 + i;
+            const float4 z0 = *reinterpret_cast<const float4*>(z), z1 = *reinterpret_cast<const float4*>(z + 4);
+            v[u][0] = bf16lo(yw.x) * silu_f32(z0.x); v[u][1] = bf16hi(yw.x) * silu_f32(z0.y);
+            v[u][2] = bf16lo(yw.y) * silu_f32(z0.z); v[u][3] = bf16hi(yw.y) * silu_f32(z0.w);
+            v[u][4] = bf16lo(yw.z) * silu_f32(z1.x); v[u][5] = bf16hi(yw.z) * silu_f32(z1.y);
+            v[u][6] = bf16lo(yw.w) * silu_f32(z1.z); v[u][7] = bf16hi(yw.w) * silu_f32(z1.w);
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) q += v[u][e] * v[u][e];
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(q) / (float)part + eps);
+#pragma unroll
+    for (int u = 0; u < kNormKeep; ++u) {
+        const int i = 8 * (lane + 64 * u);
+        if (i >= part) continue;
+        const float4 a = *reinterpret_cast<const float4*>(gain + g0 + i), b = *reinterpret_cast<const float4*>(gain + g0 + i + 4);
+        *reinterpret_cast<uint4*>(out + r * n + g0 + i) =
+            make_uint4(pack_bf16_hw((v[u][0] * inv) * a.x, (v[u][1] * inv) * a.y), pack_bf16_hw((v[u][2] * inv) * a.z, (v[u][3] * inv) * a.w),
+                       pack_bf16_hw((v[u][4] * inv) * b.x, (v[u][5] * inv) * b.y), pack_bf16_hw((v[u][6] * inv) * b.z, (v[u][7] * inv) * b.w));
+    }
 }
 
 }  // namespace
@@ -518,6 +572,12 @@ void ssm_scan(hipStream_t s, const SsmArgs& a) {
 void gated_rms_norm(hipStream_t s, int dtype, const void* y, const float* p, const float* gain, void* out, int64_t rows, int64_t n, int64_t ld,
                     int64_t col, int64_t groups, float eps) {
     if (rows <= 0 || n <= 0) return;
+    const int64_t part = n / groups;
+    if (dtype == 2 && part % 8 == 0 && part <= 64 * 8 * kNormKeep && ld % 4 == 0 && col % 4 == 0 && rows * groups < (1ll << 31)) {
+        gated_norm_wave_kernel<<<(unsigned)cdiv_m(rows * groups, 4), 256, 0, s>>>((const bf16_t*)y, p, gain, (bf16_t*)out, rows, n, ld, col, (int)part,
+                                                                                 (int)groups, eps);
+        return;
+    }
     const dim3 grid((unsigned)rows, (unsigned)groups);
     if (dtype == 0) gated_rms_norm_kernel<float><<<grid, 256, 0, s>>>((const float*)y, p, gain, (float*)out, n, ld, col, n / groups, eps);
     else gated_rms_norm_kernel<bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)y, p, gain, (bf16_t*)out, n, ld, col, n / groups, eps);
@@ -596,7 +656,7 @@ int ssm_seq(hipStream_t s, const SsmSeqArgs& a) {
 #define GPTRS_SSD(NPW, VT)                                                                                                       \
         do {                                                                                                                     \
             constexpr int NS = 64 * NPW + 8, VS = 16 * VT;                                                                       \
-            constexpr int lds = (2 * kChunk * NS + kChunk * (VS + 8) + 2 * VS * NS + 4 * 2 * 16 * (kChunk + 8)) * 2 + 3 * kChunk * 4; \
+            constexpr int lds = (2 * kChunk * NS + kChunk * (VS + 8) + 2 * VS * NS) * 2 + 6 * kChunk * 4;                        \
             static_assert(lds <= 160 * 1024, "LDS of one CU");                                                                   \
             (void)hipFuncSetAttribute((const void*)ssd_kernel<NPW, VT>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);        \
             ssd_kernel<NPW, VT><<<dim3((unsigned)a.heads, (unsigned)cdiv_m(a.vdim, VS), (unsigned)a.nseq), 256, lds, s>>>(a, (const bf16_t*)xbc, (bf16_t*)y); \

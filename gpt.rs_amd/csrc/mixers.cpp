@@ -201,7 +201,7 @@ size_t mixer_scratch_bytes(const Instr& in, const std::vector<const Spec*>& oper
     const int64_t rows = in.out_specs[0].rank() == 2 ? in.out_specs[0].dims[0] : 0;
     if (in.mix == Mix::SsmSeq) return k::ssm_seq_scratch_bytes(dt, rows, m.heads, m.groups, m.state, m.vdim);
     if (in.mix == Mix::LatentDecode)
-        return k::latent_decode_scratch_bytes(dt, std::min<int64_t>(rows, k::kMixerBatch), operands[in.append ? 8 : 5]->dims[1], m.heads, m.dim, m.rot, m.rank);
+        return k::latent_decode_scratch_bytes(dt, std::min<int64_t>(rows, k::kMixerBatch), operands[in.append ? 8 : 5]->dims[1], m.heads, m.dim, m.rot, m.rank, m.vdim);
     if (in.mix == Mix::LatentPrefill) return k::latent_prefill_scratch_bytes(dt, rows, m.heads, m.dim, m.rot, m.vdim);
     return 0;
 }
