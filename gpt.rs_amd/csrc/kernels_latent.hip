@@ -257,52 +257,53 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentDecodeArgs a, bf
     }
 }
 
-// Workgroup = ONE wave: slice of the positions x 16 heads (and 16 RT latent dimensions of the result) x sequence.  32 cache rows
-// at a time in LDS, all their words requested before the first is stored; scores transposed (rows: positions, columns: heads),
-// so a lane holds 8 positions of one head: softmax in registers, and the weights (a bf16 value and its remainder) feed the
-// product with the cached latents from there.  part f32 [nseq][heads][nsplit][rank + 2]: sums, maximum (base 2), weight.
+// Workgroup = slice of the positions x sequence x up to 4 waves; a wave = 16 heads and 16 RT latent dimensions of their result, and
+// all waves share the cache rows, 32 at a time in LDS.  Scores transposed (rows: positions, columns: heads), so a lane holds 8
+// positions of one head: softmax in registers, and the weights (a bf16 value and its remainder) feed the product with the
+// cached latents from there.  part f32 [nseq][heads][nsplit][rank + 2]: sums, maximum (base 2), weight.
 template <int RT>
-__global__ __launch_bounds__(64) void latent_partial_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ ql, float* __restrict__ part, int nsplit) {
+__global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ ql, float* __restrict__ part, int nsplit) {
     extern __shared__ __align__(16) unsigned char lat_smem[];
     const int rank = (int)a.rank, w = rank + (int)a.rot, H = (int)a.heads, ws = w + 8;   // LDS row stride
     bf16_t* rows = reinterpret_cast<bf16_t*>(lat_smem);               // [32][ws]
-    bf16_t* qs = rows + kTileP * ws;                                  // [16][ws]
-    const int lane = threadIdx.x, c = lane & 15, kg = lane >> 4;
-    const int rparts = (rank + 16 * RT - 1) / (16 * RT);
-    const int b = blockIdx.z, h0 = ((int)blockIdx.y / rparts) * kHeadTile, rp0 = ((int)blockIdx.y % rparts) * 16 * RT, sp = blockIdx.x;
+    bf16_t* q0s = rows + kTileP * ws;                                 // queries of the workgroup's tiles of 16 heads, [16][ws] each
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, W = (int)blockDim.x >> 6, c = lane & 15, kg = lane >> 4;
+    const int rparts = (rank + 16 * RT - 1) / (16 * RT), units = (H + kHeadTile - 1) / kHeadTile * rparts;
+    const int unit = (int)blockIdx.y * W + wave;
+    const bool live = unit < units;
+    const int ht0 = (int)blockIdx.y * W / rparts, ht1 = min((int)blockIdx.y * W + W - 1, units - 1) / rparts;   // the workgroup's tiles of heads
+    const int ht = live ? unit / rparts : ht0, rp0 = live ? (unit % rparts) * 16 * RT : 0;
+    const int b = blockIdx.z, h0 = ht * kHeadTile, sp = blockIdx.x;
     const int n = min(max(a.pos[b], 0) + 1, (int)a.capacity);
     const int per = ((n + nsplit - 1) / nsplit + 15) / 16 * 16;
     const int p0 = sp * per, p1 = min(p0 + per, n);
-    const int hr = H - h0 < kHeadTile ? H - h0 : kHeadTile;           // heads that exist
+    const int hr = !live ? 0 : (H - h0 < kHeadTile ? H - h0 : kHeadTile);   // heads that exist
     float* rec = part + (((int64_t)b * H + h0) * nsplit + sp) * (rank + 2);
     const int64_t rec_h = (int64_t)nsplit * (rank + 2);
     if (p0 >= p1) {   // nothing falls to this slice: its weight is zero, and whoever merges does not use its sums
-        if (lane < hr) { rec[lane * rec_h + rank] = -INFINITY; rec[lane * rec_h + rank + 1] = 0.f; }
+        if (lane < hr && rp0 == 0) { rec[lane * rec_h + rank] = -INFINITY; rec[lane * rec_h + rank + 1] = 0.f; }
         return;
     }
     const int wv = w / 8;                                             // 16-byte words per row (a multiple of 4)
     const bf16_t* cache = (const bf16_t*)a.cache[b];
-    // rows go 8 at a time, 8 lanes to a row: a lane takes every eighth word of rows (lane >> 3), + 8, ..; kept as R x U words
-    constexpr int U = 10, RQ = kHeadTile / 8, RR = kTileP / 8;
-    const int lr = lane >> 3, lk = lane & 7;
-    u32x4_m vq[RQ][U], vr[RR][U];
-    auto request = [&](const bf16_t* src, int last, int k0, u32x4_m* v, int R) __attribute__((always_inline)) {
+    // 8 threads to a row: a thread takes every eighth word of it
+    auto stage = [&](const bf16_t* src, bf16_t* dst, int nrows, int last) {   // rows behind `last` repeat it
+        constexpr int U = 10;                                         // words per thread requested before the first is stored
+        for (int r = tid >> 3; r < nrows; r += 8 * W) {
+            const u32x4_m* from = reinterpret_cast<const u32x4_m*>(src + (int64_t)min(r, last) * w);
+            u32x4_m* to = reinterpret_cast<u32x4_m*>(dst + r * ws);
+            for (int k0 = tid & 7; k0 < wv; k0 += 8 * U) {
+                u32x4_m v[U];
 #pragma unroll
-        for (int i = 0; i < R; ++i) {
-            const u32x4_m* from = reinterpret_cast<const u32x4_m*>(src + (int64_t)min(lr + 8 * i, last) * w);
+                for (int u = 0; u < U; ++u) v[u] = from[min(k0 + 8 * u, wv - 1)];
 #pragma unroll
-            for (int u = 0; u < U; ++u) v[i * U + u] = from[min(k0 + lk + 8 * u, wv - 1)];
+                for (int u = 0; u < U; ++u)
+                    if (k0 + 8 * u < wv) to[k0 + 8 * u] = v[u];
+            }
         }
     };
-    auto store = [&](bf16_t* dst, int k0, const u32x4_m* v, int R) __attribute__((always_inline)) {
-#pragma unroll
-        for (int i = 0; i < R; ++i) {
-            u32x4_m* to = reinterpret_cast<u32x4_m*>(dst + (lr + 8 * i) * ws);
-#pragma unroll
-            for (int u = 0; u < U; ++u)
-                if (k0 + lk + 8 * u < wv) to[k0 + lk + 8 * u] = v[i * U + u];
-        }
-    };
+    stage(ql + ((int64_t)b * H + ht0 * kHeadTile) * w, q0s, (ht1 - ht0 + 1) * kHeadTile, H - 1 - ht0 * kHeadTile);
+    const bf16_t* qs = q0s + (ht - ht0) * kHeadTile * ws;
     f32x4_m acc[RT];                                                  // rows: latent dimensions, column: head c
 #pragma unroll
     for (int i = 0; i < RT; ++i) acc[i] = f32x4_m{0.f, 0.f, 0.f, 0.f};
@@ -310,14 +311,9 @@ __global__ __launch_bounds__(64) void latent_partial_kernel(LatentDecodeArgs a, 
     const float scale2 = a.scale * 1.44269504f;
     for (int q0 = p0; q0 < p1; q0 += kTileP) {
         const int np = min(kTileP, p1 - q0);
-        asm volatile("" ::: "memory");
-        for (int k0 = 0; k0 < wv; k0 += 8 * U) {
-            if (q0 == p0) request(ql + ((int64_t)b * H + h0) * w, hr - 1, k0, &vq[0][0], RQ);
-            request(cache + (int64_t)q0 * w, np - 1, k0, &vr[0][0], RR);
-            if (q0 == p0) store(qs, k0, &vq[0][0], RQ);
-            store(rows, k0, &vr[0][0], RR);
-        }
-        asm volatile("" ::: "memory");
+        __syncthreads();
+        stage(cache + (int64_t)q0 * w, rows, kTileP, np - 1);
+        __syncthreads();
         f32x4_m s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
         for (int k = 0; k < w; k += 32) {
             const u32x4_m qv = *reinterpret_cast<const u32x4_m*>(qs + c * ws + k + 8 * kg);
@@ -654,8 +650,8 @@ static int latent_nsplit(int64_t nseq, int64_t capacity, int64_t heads) {
     while (n > 4 && blocks * n > 512) n = (n + 1) / 2;
     return (int)std::max<int64_t>(n, 1);
 }
-static size_t latent_partial_lds(int64_t w) {
-    return (size_t)(kTileP + kHeadTile) * (w + 8) * 2;
+static size_t latent_partial_lds(int64_t w, int64_t head_tiles = 1) {
+    return (size_t)(kTileP + head_tiles * kHeadTile) * (w + 8) * 2;
 }
 static bool latent_fast(int dtype, int64_t heads, int64_t dim, int64_t rot, int64_t rank, int64_t vdim) {
     return dtype == 2 && heads >= 1 && dim % 8 == 0 && vdim % 8 == 0 && rot % 2 == 0 && rank % 16 == 0 && (rank + rot) % 32 == 0 && rank <= 1024 && dim <= 512 &&
@@ -676,10 +672,15 @@ int latent_decode(hipStream_t s, const LatentDecodeArgs& a) {
         const int ns = latent_nsplit(a.nseq, a.capacity, a.heads);
         const int64_t rc = cdiv_l(a.rank, kPrepRows);
         latent_prep_kernel<<<(unsigned)(a.heads * rc + (a.raw ? a.nseq : 0)), 256, (size_t)std::max<int64_t>(a.nseq * a.dim, 16) * 4, s>>>(a, ql);
-        const size_t lds = latent_partial_lds(w);
-        const int64_t rt = a.rank / 16;
-        const dim3 grid((unsigned)ns, (unsigned)(cdiv_l(a.heads, kHeadTile) * cdiv_l(rt, 16)), (unsigned)a.nseq);
-#define GPTRS_PARTIAL(RT) do { with_lds(latent_partial_kernel<RT>, lds); latent_partial_kernel<RT><<<grid, 64, lds, s>>>(a, ql, part, ns); } while (0)
+        const int64_t rt = a.rank / 16, parts = cdiv_l(rt, 16), units = cdiv_l(a.heads, kHeadTile) * parts;
+        // waves per workgroup, as many as have work and whose queries fit beside the rows (a workgroup of W consecutive units
+        // meets at most (W - 2) / parts + 2 tiles of heads)
+        int64_t W = std::min<int64_t>(units, 4);
+        auto tiles = [&](int64_t n) { return n <= 1 ? 1 : std::min<int64_t>((n - 2) / parts + 2, n); };
+        while (W > 1 && latent_partial_lds(w, tiles(W)) > 160 * 1024) --W;
+        const size_t lds = latent_partial_lds(w, tiles(W));
+        const dim3 grid((unsigned)ns, (unsigned)cdiv_l(units, W), (unsigned)a.nseq);
+#define GPTRS_PARTIAL(RT) do { with_lds(latent_partial_kernel<RT>, lds); latent_partial_kernel<RT><<<grid, (unsigned)(64 * W), lds, s>>>(a, ql, part, ns); } while (0)
         if (rt <= 8) GPTRS_PARTIAL(8);
         else GPTRS_PARTIAL(16);
 #undef GPTRS_PARTIAL
