@@ -170,7 +170,7 @@ __global__ __launch_bounds__(256) void latent_attn_x_kernel(LatentAttnXArgs a) {
 
 // ---------------------------------------------------------------------------- decode (bf16)
 constexpr int kPrepRows = 64;    // latent dimensions per workgroup of the query part
-constexpr int kTileP = 32;       // cache rows per step of the attention part
+constexpr int kTileP = 64;       // cache rows per step of the attention part
 constexpr int kHeadTile = 16;
 
 // Blocks [0, heads * rank / 64): W_uk^T q_n of one head and 64 latent dimensions, for every sequence (the first of a head
@@ -258,7 +258,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentDecodeArgs a, bf
 }
 
 // Workgroup = slice of the positions x sequence x up to 4 waves; a wave = 16 heads and 16 RT latent dimensions of their result, and
-// all waves share the cache rows, 32 at a time in LDS.  Scores transposed (rows: positions, columns: heads), so a lane holds 8
+// all waves share the cache rows, 64 at a time in LDS.  Scores transposed (rows: positions, columns: heads), so a lane holds 16
 // positions of one head: softmax in registers, and the weights (a bf16 value and its remainder) feed the product with the
 // cached latents from there.  part f32 [nseq][heads][nsplit][rank + 2]: sums, maximum (base 2), weight.
 template <int RT>
@@ -288,19 +288,24 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a,
     const bf16_t* cache = (const bf16_t*)a.cache[b];
     // 8 threads to a row: a thread takes every eighth word of it
     auto stage = [&](const bf16_t* src, bf16_t* dst, int nrows, int last) {   // rows behind `last` repeat it
-        constexpr int U = 10;                                         // words per thread requested before the first is stored
-        for (int r = tid >> 3; r < nrows; r += 8 * W) {
-            const u32x4_m* from = reinterpret_cast<const u32x4_m*>(src + (int64_t)min(r, last) * w);
-            u32x4_m* to = reinterpret_cast<u32x4_m*>(dst + r * ws);
+        constexpr int R = 2, U = 10;                                  // rows x words per thread requested before the first is stored
+        for (int r0 = tid >> 3; r0 < nrows; r0 += 8 * W * R)
             for (int k0 = tid & 7; k0 < wv; k0 += 8 * U) {
-                u32x4_m v[U];
+                u32x4_m v[R][U];
 #pragma unroll
-                for (int u = 0; u < U; ++u) v[u] = from[min(k0 + 8 * u, wv - 1)];
+                for (int i = 0; i < R; ++i) {
+                    const u32x4_m* from = reinterpret_cast<const u32x4_m*>(src + (int64_t)min(r0 + 8 * W * i, last) * w);
 #pragma unroll
-                for (int u = 0; u < U; ++u)
-                    if (k0 + 8 * u < wv) to[k0 + 8 * u] = v[u];
+                    for (int u = 0; u < U; ++u) v[i][u] = from[min(k0 + 8 * u, wv - 1)];
+                }
+#pragma unroll
+                for (int i = 0; i < R; ++i) {
+                    u32x4_m* to = reinterpret_cast<u32x4_m*>(dst + (r0 + 8 * W * i) * ws);
+#pragma unroll
+                    for (int u = 0; u < U; ++u)
+                        if (r0 + 8 * W * i < nrows && k0 + 8 * u < wv) to[k0 + 8 * u] = v[i][u];
+                }
             }
-        }
     };
     stage(ql + ((int64_t)b * H + ht0 * kHeadTile) * w, q0s, (ht1 - ht0 + 1) * kHeadTile, H - 1 - ht0 * kHeadTile);
     const bf16_t* qs = q0s + (ht - ht0) * kHeadTile * ws;
@@ -314,30 +319,37 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a,
         __syncthreads();
         stage(cache + (int64_t)q0 * w, rows, kTileP, np - 1);
         __syncthreads();
-        f32x4_m s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
+        constexpr int PT = kTileP / 16;
+        f32x4_m sc[PT];
+#pragma unroll
+        for (int j = 0; j < PT; ++j) sc[j] = f32x4_m{0.f, 0.f, 0.f, 0.f};
         for (int k = 0; k < w; k += 32) {
             const u32x4_m qv = *reinterpret_cast<const u32x4_m*>(qs + c * ws + k + 8 * kg);
-            s0 = mma16(*reinterpret_cast<const u32x4_m*>(rows + c * ws + k + 8 * kg), qv, s0);
-            s1 = mma16(*reinterpret_cast<const u32x4_m*>(rows + (16 + c) * ws + k + 8 * kg), qv, s1);
-        }
-        float x[8], mx = -INFINITY;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            x[e] = 4 * kg + e < np ? s0[e] * scale2 : -INFINITY;
-            x[4 + e] = 16 + 4 * kg + e < np ? s1[e] * scale2 : -INFINITY;
-            mx = fmaxf(mx, fmaxf(x[e], x[4 + e]));
+            for (int j = 0; j < PT; ++j) sc[j] = mma16(*reinterpret_cast<const u32x4_m*>(rows + (16 * j + c) * ws + k + 8 * kg), qv, sc[j]);
         }
+        float mx = -INFINITY;
+#pragma unroll
+        for (int j = 0; j < PT; ++j)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                sc[j][e] = 16 * j + 4 * kg + e < np ? sc[j][e] * scale2 : -INFINITY;
+                mx = fmaxf(mx, sc[j][e]);
+            }
         const float mn = fmaxf(m_run, col4_max(mx)), corr = __builtin_amdgcn_exp2f(m_run - mn);
         float sum = 0.f;
-        u32x4_m ph, pl;
+        u32x4_m ph[PT / 2], pl[PT / 2];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const float u = __builtin_amdgcn_exp2f(x[2 * e] - mn), v = __builtin_amdgcn_exp2f(x[2 * e + 1] - mn);
-            sum += u + v;
-            uint32_t hi, lo;
-            split_bf16_hw(u, v, hi, lo);
-            ph[e] = hi; pl[e] = lo;
-        }
+        for (int j = 0; j < PT; ++j)
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+                const float u = __builtin_amdgcn_exp2f(sc[j][2 * e] - mn), v = __builtin_amdgcn_exp2f(sc[j][2 * e + 1] - mn);
+                sum += u + v;
+                uint32_t hi, lo;
+                split_bf16_hw(u, v, hi, lo);
+                ph[j / 2][2 * (j & 1) + e] = hi;
+                pl[j / 2][2 * (j & 1) + e] = lo;
+            }
         l_run = l_run * corr + col4_sum(sum);
         m_run = mn;
 #pragma unroll
@@ -345,9 +357,12 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a,
             if (rp0 + 16 * i >= rank) break;
 #pragma unroll
             for (int e = 0; e < 4; ++e) acc[i][e] *= corr;
-            const u32x4_m rv = lds_operand_t2(rows + rp0 + 16 * i, ws, lane);
-            acc[i] = mma16(rv, ph, acc[i]);
-            acc[i] = mma16(rv, pl, acc[i]);
+#pragma unroll
+            for (int k = 0; k < PT / 2; ++k) {
+                const u32x4_m rv = lds_operand_t2(rows + 32 * k * ws + rp0 + 16 * i, ws, lane);
+                acc[i] = mma16(rv, ph[k], acc[i]);
+                acc[i] = mma16(rv, pl[k], acc[i]);
+            }
         }
     }
     if (c < hr) {
@@ -365,19 +380,20 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentDecodeArgs a,
     }
 }
 
-constexpr int kOutV = 32;        // values per workgroup of the output part
-// Workgroup = head x 32 values x sequence: the slices' records merged into the weighted latent, times W_uv.
+// Workgroup = head x OV values x sequence (narrow where there are few heads and sequences): the slices' records merged into the weighted latent, times W_uv.
+template <int OV>
 __global__ __launch_bounds__(256) void latent_combine_kernel(LatentDecodeArgs a, const float* __restrict__ part, int nsplit) {
     extern __shared__ float lat_lds[];
     const int rank = (int)a.rank, vdim = (int)a.vdim, H = (int)a.heads;
     float* lat = lat_lds;                        // [rank]
     float* wgt = lat + rank;                     // [32]
-    float* red = wgt + 32;                       // [4][kOutV]
-    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, h = blockIdx.x, v0 = blockIdx.y * kOutV, b = blockIdx.z;
+    float* red = wgt + 32;                       // [4][OV]
+    constexpr int VL = OV / 8, GR = 256 / VL;    // lanes of 8 values, groups of latent dimensions
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, h = blockIdx.x, v0 = blockIdx.y * OV, b = blockIdx.z;
     const int rs = rank + 2;
     const float* rec = part + ((int64_t)b * H + h) * nsplit * rs;
-    // 4 lanes of 8 values, 64 groups of latent dimensions; the first words of W_uv and the first records are requested at once
-    const int v8 = 8 * (t & 3), g = t >> 2;
+    // the first words of W_uv and the first records are requested at once
+    const int v8 = 8 * (t % VL), g = t / VL;
     const bool vlive = v0 + v8 < vdim;
     const int64_t ldw = (int64_t)H * vdim;
     const bf16_t* wv = (const bf16_t*)a.w_uv + (int64_t)h * vdim + (vlive ? v0 + v8 : 0);
@@ -385,7 +401,7 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentDecodeArgs a,
     u32x4_m x[U];
     auto request = [&](int r0) {
 #pragma unroll
-        for (int u = 0; u < U; ++u) x[u] = *reinterpret_cast<const u32x4_m*>(wv + (int64_t)min(r0 + 64 * u, rank - 1) * ldw);
+        for (int u = 0; u < U; ++u) x[u] = *reinterpret_cast<const u32x4_m*>(wv + (int64_t)min(r0 + GR * u, rank - 1) * ldw);
     };
     request(g);
     const float mv = lane < nsplit ? rec[(int64_t)lane * rs + rank] : -INFINITY, lv = lane < nsplit ? rec[(int64_t)lane * rs + rank + 1] : 0.f;
@@ -421,26 +437,26 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentDecodeArgs a,
     float o[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) o[e] = 0.f;
-    for (int r0 = g; r0 < rank; r0 += 64 * U) {
+    for (int r0 = g; r0 < rank; r0 += GR * U) {
         if (r0 != g) request(r0);
 #pragma unroll
         for (int u = 0; u < U; ++u) {
-            const float f = r0 + 64 * u < rank ? lat[r0 + 64 * u] : 0.f;
+            const float f = r0 + GR * u < rank ? lat[r0 + GR * u] : 0.f;
 #pragma unroll
             for (int e = 0; e < 4; ++e) { o[2 * e] += f * bf16lo(x[u][e]); o[2 * e + 1] += f * bf16hi(x[u][e]); }
         }
     }
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {   // over the 16 groups of the wave: lanes 4 apart
+    for (int e = 0; e < 8; ++e) {   // over the groups of the wave: lanes VL apart
         float x = o[e];
-        x += __shfl_xor(x, 4, 64);
-        x += __shfl_xor(x, 8, 64);
+        if (VL == 4) { x += __shfl_xor(x, 4, 64); x += __shfl_xor(x, 8, 64); }
         x = col4_sum(x);
-        if (lane < 4) red[wave * kOutV + v8 + e] = x;
+        if (lane < VL) red[wave * OV + v8 + e] = x;
     }
     __syncthreads();
-    if (t < kOutV && v0 + t < vdim)
-        ((bf16_t*)a.ctx)[((int64_t)b * H + h) * vdim + v0 + t] = f32_to_bf16(red[t] + red[kOutV + t] + red[2 * kOutV + t] + red[3 * kOutV + t]);
+    static_assert(VL == 4 || VL == 16, "reduction above");
+    if (t < OV && v0 + t < vdim)
+        ((bf16_t*)a.ctx)[((int64_t)b * H + h) * vdim + v0 + t] = f32_to_bf16(red[t] + red[OV + t] + red[2 * OV + t] + red[3 * OV + t]);
 }
 
 // ---------------------------------------------------------------------------- prompts (bf16)
@@ -643,10 +659,10 @@ void latent_attn_expanded(hipStream_t s, const LatentAttnXArgs& a) {
 
 
 static size_t lat_align(size_t n) { return (n + 255) / 256 * 256; }
-// slices of the positions: 32 rows each up to 32 of them, fewer where the batch fills the chip by itself
+// slices of the positions: 64 rows each up to 32 of them, fewer where the batch fills the chip by itself
 static int latent_nsplit(int64_t nseq, int64_t capacity, int64_t heads) {
     const int64_t blocks = nseq * cdiv_l(heads, kHeadTile);
-    int64_t n = std::min<int64_t>(cdiv_l(capacity, 32), 32);
+    int64_t n = std::min<int64_t>(cdiv_l(capacity, kTileP), 32);
     while (n > 4 && blocks * n > 512) n = (n + 1) / 2;
     return (int)std::max<int64_t>(n, 1);
 }
@@ -684,7 +700,10 @@ int latent_decode(hipStream_t s, const LatentDecodeArgs& a) {
         if (rt <= 8) GPTRS_PARTIAL(8);
         else GPTRS_PARTIAL(16);
 #undef GPTRS_PARTIAL
-        latent_combine_kernel<<<dim3((unsigned)a.heads, (unsigned)cdiv_l(a.vdim, kOutV), (unsigned)a.nseq), 256, (size_t)(a.rank + 32 + 4 * kOutV) * 4, s>>>(a, part, ns);
+#define GPTRS_COMBINE(OV) latent_combine_kernel<OV><<<dim3((unsigned)a.heads, (unsigned)cdiv_l(a.vdim, OV), (unsigned)a.nseq), 256, (size_t)(a.rank + 32 + 4 * OV) * 4, s>>>(a, part, ns)
+        if (a.vdim > 64 && a.heads * a.nseq >= 192) GPTRS_COMBINE(128);
+        else GPTRS_COMBINE(32);
+#undef GPTRS_COMBINE
         return 3;
     }
     rope_pairs(s, a.dtype, a.x, a.table, a.scratch, a.nseq, a.heads, a.dim + a.rot, a.dim, a.rot / 2);

@@ -118,7 +118,7 @@ def latent_args(seed, T, heads, dim, rot, rank, vdim, dt, n=None):
             (rn(seed + 2, len(pos), heads * vdim), dt), (0.1 * rn(seed + 3, len(pos), rank + rot), dt)]
 
 
-SHAPES = [(2, 16, 8, 24, 24), (1, 32, 32, 64, 32), (3, 128, 64, 32, 128), (2, 64, 24, 16, 136), (1, 10, 6, 11, 7)]
+SHAPES = [(2, 16, 8, 24, 24), (1, 32, 32, 64, 32), (3, 128, 64, 32, 128), (2, 64, 24, 16, 136), (1, 200, 56, 32, 256), (1, 10, 6, 11, 7)]
 
 
 @pytest.mark.parametrize("dt", ["F32", "Bf16"])
@@ -142,14 +142,14 @@ def test_prompt_attention_and_single_keys(hip, dt, shape, T):
 
 @pytest.mark.parametrize("dt", ["F32", "Bf16"])
 @pytest.mark.parametrize("shape", [(3, 16, 8, 24, 24), (5, 32, 32, 64, 32), (24, 16, 32, 96, 8), (32, 128, 64, 512, 128), (2, 40, 24, 360, 40), (1, 10, 6, 11, 7)])
-@pytest.mark.parametrize("lens", [[1], [2, 31, 32, 33], [500, 1, 257], list(range(1, 19))])
+@pytest.mark.parametrize("lens", [[1], [2, 63, 64, 65], [500, 1, 257], [4000, 2049, 66], list(range(1, 19))])
 def test_decode_attention_of_a_batch(hip, dt, shape, lens):
     """One step of unequal sequences (more than one launch's worth in the last case), caches written in place of nothing but the
     new row; one far row, the row before and the new row itself stand out in turn."""
     heads, dim, rot, rank, vdim = shape
-    if len(lens) > 4 and rank > 96:
-        pytest.skip("one size of long batch is enough")
-    B, C = len(lens), 512
+    B, C = len(lens), 512 if max(lens) <= 512 else 4096
+    if (len(lens) > 4 and rank > 96) or (C > 512 and (rank == 512 or heads < 2)):
+        pytest.skip("a few sizes of long batches and long caches are enough")
     pos = np.array([n - 1 for n in lens], np.int32)
     starts = np.array([v for n in lens for v in (0, n - 1, 0)], np.int32)
     caches = [0.3 * rn(20 + b, 1, C, rank + rot) for b in range(B)]
