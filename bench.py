@@ -22,6 +22,7 @@ from __future__ import annotations
 
 import argparse
 import ctypes
+import gc
 import hashlib
 import json
 import os
@@ -544,11 +545,18 @@ def _time_model(be, model, prompt_len: int, vocab: int, batch: int, steps: int, 
         for _ in range(warmup):
             g.step()
         be.synchronize()
-        t0 = time.perf_counter()
-        for _ in range(steps):
-            g.step()
-        be.synchronize()
-        return (time.perf_counter() - t0) / steps
+        # whether a full collection of the interpreter's garbage falls into the timed steps depends on what ran before, and one
+        # of some milliseconds shows in 64 steps: collect first, and not while the steps are timed
+        gc.collect()
+        gc.disable()
+        try:
+            t0 = time.perf_counter()
+            for _ in range(steps):
+                g.step()
+            be.synchronize()
+            return (time.perf_counter() - t0) / steps
+        finally:
+            gc.enable()
     one = decode(gen)
     launches = be.counter("last_program_launches")
     del gen
