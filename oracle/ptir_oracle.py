@@ -43,6 +43,7 @@ from typing import Dict, List, Sequence, Tuple
 import numpy as np
 
 from . import dadupel_reference as DR
+from . import fuzazen_reference as FR
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 _LIB = None
@@ -478,7 +479,8 @@ def _norm_call(target: str, attrs, ins: List[OTensor], out_dtype: str) -> OTenso
     return out
 
 
-# ---- sequence mixers: every target by the mechanism's own function (dadupel_reference.py) in f64, the result rounded once
+# ---- sequence mixers: every target by the mechanism's own function (dadupel_reference.py, fuzazen_reference.py) in f64, the result
+# rounded once
 def _mx_ssm(at, xbc, p, dt_bias, a_log, d, state):
     H, N, V = state.shape
     G, dc, inner = int(at["groups"]), int(at["dt_col"]), state.shape[0] * state.shape[2]
@@ -545,6 +547,30 @@ def _mx_glu(at, g, u):
     return g * DR.sigmoid(at["alpha"] * g) * (np.clip(u, -at["limit"], at["limit"]) + at["shift"])
 
 
+def _mx_heads(x, heads):
+    return x.reshape(x.shape[0], int(heads), -1)
+
+
+def _mx_head_norm(at, x):
+    return FR.over_rms(_mx_heads(x, at["heads"]), at["eps"])
+
+
+def _mx_head_gate(at, x, g):
+    return _mx_heads(x, at["heads"]) * FR.sigmoid(g)[:, :, None]
+
+
+def _mx_chunk_attend(at, q, k, v, sink):
+    chunk = int(at["chunk"]) or q.shape[0]
+    return FR.chunk_attend(_mx_heads(q, at["heads"]), _mx_heads(k, at["kv_heads"]), _mx_heads(v, at["kv_heads"]), sink, at["scale"], chunk, 0)
+
+
+def _mx_chunk_attend_cache(at, q, kc, vc, sink, position):
+    n = int(position[0])
+    n = n % int(at["chunk"]) if int(at["chunk"]) else n
+    k, v = kc[:, :n + 1].transpose(1, 0, 2), vc[:, :n + 1].transpose(1, 0, 2)   # the chunk's rows as a sequence of their own
+    return FR.chunk_attend(_mx_heads(q, at["heads"]), k, v, sink, at["scale"], n + 1, n)
+
+
 _MIXER_CALLS = {
     "gpt_rs.hip.rope_table.v1": _mx_rope_table,
     "gpt_rs.hip.rope_pairs.v1": _mx_rope_pairs,
@@ -557,6 +583,10 @@ _MIXER_CALLS = {
     "gpt_rs.hip.ssm_state.v1": lambda at, xbc, p, dt_bias, a_log, state: _mx_ssm(at, xbc, p, dt_bias, a_log, np.zeros_like(a_log), state)[1],
     "gpt_rs.hip.gated_rms_norm.v1": _mx_gated,
     "gpt_rs.hip.clamped_glu.v1": _mx_glu,
+    "gpt_rs.hip.head_rms_norm.v1": _mx_head_norm,
+    "gpt_rs.hip.head_gate.v1": _mx_head_gate,
+    "gpt_rs.hip.chunk_attention.v1": _mx_chunk_attend,
+    "gpt_rs.hip.chunk_attention_cache.v1": _mx_chunk_attend_cache,
 }
 
 
