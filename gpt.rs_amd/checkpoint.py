@@ -173,7 +173,8 @@ class SafetensorsFolder:
 
     A safetensors file is an 8-byte little-endian length, that many bytes of JSON (name -> dtype, shape, data_offsets) and
     the data.  `layout` maps a parameter of the model to (tensor name, transpose): matrices are stored [out, in] there and
-    [in, out] in a model.  Entries carry the parameters' names and shapes."""
+    [in, out] in a model.  A tuple of names stands for the tensors stacked along their first axis (projections of one input
+    that a model holds as one matrix).  Entries carry the parameters' names and shapes."""
 
     _TAG = {"F32": 0, "F16": 1, "BF16": 2, "I32": 3}
 
@@ -189,7 +190,7 @@ class SafetensorsFolder:
         self.architecture, self.config, self.runtime = str(cfg["architecture"]), cfg, cfg.get("runtime")
         self.entries: List[Entry] = []
         self._by_name: Dict[str, Entry] = {}
-        self._layout: Dict[str, Tuple[str, bool]] = {}
+        self._layout: Dict[str, Tuple[Tuple[str, ...], bool]] = {}
         self._file = open(os.path.join(path, "model.safetensors"), "rb")
         try:
             self._map = mmap.mmap(self._file.fileno(), 0, access=mmap.ACCESS_READ)
@@ -216,15 +217,23 @@ class SafetensorsFolder:
             self.close()
             raise
 
-    def bind_layout(self, layout: Mapping[str, Tuple[str, bool]]):
-        self.entries, self._by_name, self._layout = [], {}, dict(layout)
-        for param, (tensor, transpose) in layout.items():
-            if tensor not in self._tensors:
-                raise CheckpointError(f"tensor `{tensor}` not found in the model folder")
-            tag, dims, off, n = self._tensors[tensor]
+    def bind_layout(self, layout: Mapping[str, Tuple[object, bool]]):
+        self.entries, self._by_name, self._layout = [], {}, {}
+        for param, (names, transpose) in layout.items():
+            names = (names,) if isinstance(names, str) else tuple(names)
+            for tensor in names:
+                if tensor not in self._tensors:
+                    raise CheckpointError(f"tensor `{tensor}` not found in the model folder")
+            tag, dims, off, n = self._tensors[names[0]]
+            for tensor in names[1:]:
+                t2, d2, _, n2 = self._tensors[tensor]
+                if t2 != tag or d2[1:] != dims[1:]:
+                    raise CheckpointError(f"tensor `{tensor}` cannot be stacked behind `{names[0]}`")
+                dims, n = (dims[0] + d2[0],) + dims[1:], n + n2
             e = Entry(param, 0, dims[::-1] if transpose else dims, tag, 0, off, n)
             self.entries.append(e)
             self._by_name[param] = e
+            self._layout[param] = (names, transpose)
 
     entry = Checkpoint.entry
     names = Checkpoint.names
@@ -235,11 +244,15 @@ class SafetensorsFolder:
     __exit__ = Checkpoint.__exit__
 
     def array(self, name: str) -> np.ndarray:
-        """The parameter as a view of the file mapping (bf16 as 16-bit words), transposed where the layout says so."""
-        e = self.entry(name)
-        tensor, transpose = self._layout[name]
-        dims = self._tensors[tensor][1]
-        a = np.frombuffer(self._map, dtype=_NP_OF_TAG[e.dtype_tag], count=e.byte_len // _NP_OF_TAG[e.dtype_tag].itemsize, offset=e.offset).reshape(dims)
+        """The parameter (bf16 as 16-bit words), transposed where the layout says so: a view of the file mapping, a copy where
+        tensors are stacked."""
+        self.entry(name)   # "tensor not found"
+        names, transpose = self._layout[name]
+        parts = []
+        for tensor in names:
+            tag, dims, off, n = self._tensors[tensor]
+            parts.append(np.frombuffer(self._map, dtype=_NP_OF_TAG[tag], count=n // _NP_OF_TAG[tag].itemsize, offset=off).reshape(dims))
+        a = parts[0] if len(parts) == 1 else np.concatenate(parts)
         return a.T if transpose else a
 
 

@@ -461,7 +461,7 @@ def dynamic_update_slice_into(base: Tensor, update: Tensor, starts: Tensor) -> T
 
 # --------------------------------------------------------------------------- sequence mixers
 # CustomCall targets of this backend for mixers the reference has no functional for (selective state spaces, latent
-# attention).  Each call has one result, as every PTIR instruction; the backend's fusion pass puts the calls of a layer and of
+# attention, chunked attention with sinks).  Each call has one result, as every PTIR instruction; the backend's fusion pass puts the calls of a layer and of
 # a batch together (csrc/fuse.cpp), csrc/mixers.cpp states operands and attributes.
 def _attrs(**kw) -> dict:
     return {k: ({"kind": "I64", "value": int(v)} if isinstance(v, (int, np.integer)) else {"kind": "F64", "value": float(v)}) for k, v in kw.items()}
@@ -477,6 +477,17 @@ def clamped_glu(gate: Tensor, up: Tensor, limit: float, alpha: float = 1.702, sh
     if gate.spec != up.spec:
         raise ValueError("clamped_glu gate/up spec mismatch")
     return gate.fb.custom_call("gpt_rs.hip.clamped_glu.v1", [gate, up], gate.spec, _attrs(limit=float(limit), alpha=float(alpha), shift=float(shift)))
+
+
+def post_norm_add(x: Tensor, y: Tensor, gain: Tensor, mult: float, eps: float) -> Tensor:
+    """Residual update of a sublayer whose output is normed: x + mult * rms_norm(y)."""
+    out, *_ = rms_norm(y, gain, eps)
+    return x + (out if mult == 1.0 else out * float(mult))
+
+
+def softcap(x: Tensor, cap: float) -> Tensor:
+    """cap * tanh(x / cap)."""
+    return (x / float(cap)).tanh() * float(cap)
 
 
 def yarn_pair_frequencies(dims: int, base: float, factor: float, original: float, fast: float, slow: float) -> Tuple[np.ndarray, float]:
@@ -546,3 +557,28 @@ def ssm_scan(xbc: Tensor, p: Tensor, dt_bias: Tensor, a_log: Tensor, d: Tensor, 
 def gated_rms_norm(y: Tensor, p: Tensor, gain: Tensor, groups: int, col: int, eps: float) -> Tensor:
     """RMS norm of y * silu(p[:, col : col + n]) in `groups` equal parts, times gain."""
     return y.fb.custom_call("gpt_rs.hip.gated_rms_norm.v1", [y, p, gain], y.spec, _attrs(groups=groups, col=col, eps=float(eps)))
+
+
+def head_rms_norm(x: Tensor, heads: int, eps: float, dtype: Optional[str] = None) -> Tensor:
+    """Every head of x[R, heads * hd] divided by its root mean square (no gain)."""
+    return x.fb.custom_call("gpt_rs.hip.head_rms_norm.v1", [x], TensorSpec(dtype or x.dtype, x.dims), _attrs(heads=heads, eps=float(eps)))
+
+
+def head_gate(x: Tensor, gate: Tensor, heads: int) -> Tensor:
+    """Every head of x[R, heads * vd] times sigmoid of its column of gate f32 [R, heads]."""
+    return x.fb.custom_call("gpt_rs.hip.head_gate.v1", [x, gate], x.spec, _attrs(heads=heads))
+
+
+def chunk_attention(q: Tensor, k: Tensor, v: Tensor, sink: Tensor, heads: int, kv_heads: int, chunk: int, scale: float) -> Tensor:
+    """Grouped-query attention of a prompt that starts at position 0, q[R, heads * D], k[R, kv_heads * D], v[R, kv_heads * V]:
+    position i sees the positions up to i of its own chunk of `chunk` positions (0: of the whole prompt); the softmax
+    denominator of head h also holds exp(sink[h])."""
+    return q.fb.custom_call("gpt_rs.hip.chunk_attention.v1", [q, k, v, sink], TensorSpec(q.dtype, (q.dims[0], v.dims[1] // kv_heads * heads)),
+                            _attrs(heads=heads, kv_heads=kv_heads, chunk=chunk, scale=float(scale)))
+
+
+def chunk_attention_cache(q: Tensor, keys: Tensor, values: Tensor, sink: Tensor, position: Tensor, heads: int, chunk: int, scale: float) -> Tensor:
+    """The same for one query q[1, heads * D] at `position` si32[1] over caches [kv_heads, C, D] and [kv_heads, C, V] that hold the
+    positions of its chunk from row 0 on: the rows 0 .. position % chunk are seen."""
+    return q.fb.custom_call("gpt_rs.hip.chunk_attention_cache.v1", [q, keys, values, sink, position], TensorSpec(q.dtype, (1, heads * values.dims[2])),
+                            _attrs(heads=heads, chunk=chunk, scale=float(scale)))

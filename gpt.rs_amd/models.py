@@ -918,6 +918,130 @@ class Ministral(_ModelBase):
         return outs[-1]
 
 
+# ================================================================================ ragged batches
+class _RaggedModel(_ModelBase):
+    """Forward passes over batches of sequences of different lengths.  The rows of a batch are stacked without padding: linear
+    layers run over all of them, mixers sequence by sequence (decode steps: all sequences in one launch).  A model says what a
+    layer keeps per sequence (`_fresh_slot`, `_slot_handles`, `_grown_slot`, `_new_slot`), which arguments its programs take
+    beside tokens and positions (`_position_args`) and builds the program (`_build`)."""
+
+    ragged_batches = True
+
+    @property
+    def num_layers(self): return self.config.num_layers
+    @property
+    def context_length(self): return self.config.context_length
+
+    def _stack(self, parts: List[Tensor]) -> Tensor:
+        return parts[0] if len(parts) == 1 else Tensor.concat(0, parts)
+
+    def expected_params(self) -> Dict[str, tuple]:
+        return {n: e[0] for n, e in self._param_plan(self.config).items()}
+
+    @classmethod
+    def tensor_layout(cls, config) -> Dict[str, Tuple[object, bool]]:
+        return {n: (e[1], e[2]) for n, e in cls._param_plan(config).items()}
+
+    def param_dtype(self, name: str) -> str:
+        """Matrices that feed products are in the model dtype; gains, scales, taps and per-head constants are f32."""
+        leaf = name.rsplit(".", 1)[-1]
+        return self.dtype if leaf.startswith("w_") or leaf in ("weight", "lm_head") else "F32"
+
+    def _fill_random(self, names: Sequence[str], seed: int, draw, keep: Sequence[str] = ()) -> Dict[str, np.ndarray]:
+        """Sets the parameters `names` to draw(rng, name, dims), one numpy stream per tensor; returns those in `keep`."""
+        from concurrent.futures import ThreadPoolExecutor
+        dims_of, names, kept = self.expected_params(), list(names), {}
+
+        def make(idx):
+            name = names[idx]
+            arr = draw(np.random.default_rng(np.random.SeedSequence([seed, idx])), name, dims_of[name])
+            dt = self.param_dtype(name)
+            return name, dt, _np_to_bytes(arr, dt), arr if name in keep else None
+
+        workers = max(1, min(16, os.cpu_count() or 1))
+        with ThreadPoolExecutor(max_workers=workers) as ex:
+            pending, nxt = [], 0
+            while nxt < len(names) or pending:   # bounded look-ahead: a few tensors of host memory in flight
+                while nxt < len(names) and len(pending) < 2 * workers:
+                    pending.append(ex.submit(make, nxt))
+                    nxt += 1
+                name, dt, data, arr = pending.pop(0).result()
+                self.set_param_bytes(name, TensorSpec(dt, dims_of[name]), data)
+                if arr is not None:
+                    kept[name] = arr
+        return kept
+
+    # -- forward -----------------------------------------------------------------------
+    def forward_with_decode_cache(self, tokens, position_offset, caches, fixed_capacity=None, last_logits_only=False):
+        """See Gpt.forward_with_decode_cache."""
+        return self.forward_batch([list(tokens)], position_offset, [caches], fixed_capacity, last_logits_only=last_logits_only)
+
+    def forward_decode_device_token(self, token_handle, position_offset, caches, fixed_capacity=None):
+        """See Gpt.forward_decode_device_token."""
+        return self.forward_batch([[None]], position_offset, [caches], fixed_capacity, token_handle=token_handle)
+
+    def forward_batch(self, token_rows, position_offset, caches, fixed_capacity=None, token_handle=None, last_logits_only=False,
+                      logit_rows: Optional[Sequence[int]] = None):
+        """Independent sequences of any lengths.  `position_offset`: one for all or one per sequence.  The batch either starts
+        (empty caches, offset 0) or goes on by one token each; `caches[b]` is updated in place.  `logit_rows`: the stacked rows
+        whose logits are wanted (default: all, or each sequence's last with `last_logits_only`)."""
+        cfg, B = self.config, len(token_rows)
+        lens = tuple(len(r) for r in token_rows)
+        if B == 0 or min(lens) == 0:
+            raise ValueError("token sequence must contain at least one element")
+        offs = [int(position_offset)] * B if isinstance(position_offset, (int, np.integer)) else [int(o) for o in position_offset]
+        if len(offs) != B or len(caches) != B or any(len(c) != cfg.num_layers for c in caches):
+            raise ValueError(f"expected an offset and {cfg.num_layers} cache slots (one per layer) for every sequence")
+        have = caches[0][0] is not None
+        if any((slot is not None) != have for c in caches for slot in c):
+            raise ValueError("the sequences of a batch either all start or all go on")
+        if have and max(lens) != 1:
+            raise ValueError("decode with an existing cache supports one token per sequence")
+        if not have and any(offs):
+            raise ValueError("a sequence without a cache starts at position 0")
+        if token_handle is not None and max(lens) != 1:
+            raise ValueError("device tokens feed one step (one token per sequence)")
+        if token_handle is None:
+            for row in token_rows:
+                for t in row:
+                    if not 0 <= t < cfg.vocab_size:
+                        raise ValueError(f"token index {t} out of range")
+        totals = [o + n for o, n in zip(offs, lens)]
+        need = max(totals)
+        if need > cfg.context_length:
+            raise ValueError(f"token sequence length {need} exceeds model context length {cfg.context_length}")
+        if fixed_capacity is not None:
+            if not 0 < fixed_capacity <= cfg.context_length or fixed_capacity < need:
+                raise ValueError(f"decode cache capacity {fixed_capacity} invalid for sequence length {need}")
+            capacity = fixed_capacity
+        else:
+            capacity = decode_cache_capacity(need, cfg.context_length)
+        if have:
+            for c, o in zip(caches, offs):
+                for slot in c:
+                    if slot.len != o:
+                        raise ValueError(f"decode cache length {slot.len} must match position offset {o}")
+            # the sequences of a step share one capacity: the largest any of them has or needs
+            capacity = max([capacity] + [getattr(s, "capacity", 0) for c in caches for s in c])
+            for c in caches:
+                for i, s in enumerate(c):
+                    c[i] = self._grown_slot(i, s, capacity)
+        if logit_rows is not None and list(logit_rows) == list(range(sum(lens))):
+            logit_rows = None
+        prog, _ = self._build(lens, capacity, have, last_logits_only and logit_rows is None, None if logit_rows is None else len(logit_rows))
+        tok_arg = token_handle if token_handle is not None else self._upload_i32([t for row in token_rows for t in row])
+        args = [tok_arg, self._upload_i32([o + j for o, n in zip(offs, lens) for j in range(n)])] + self._position_args(offs)
+        if logit_rows is not None:
+            args.append(self._upload_i32(logit_rows))
+        held = [h for c in caches for i, slot in enumerate(c) for h in (self._slot_handles(slot) if have else self._fresh_slot(i, capacity))]
+        outs = self._run(prog, args + held, [False] * len(args) + [True] * len(held))
+        it = iter(outs[:-1])
+        for b in range(B):
+            for i in range(cfg.num_layers):
+                caches[b][i] = self._new_slot(i, it, totals[b], capacity)
+        return outs[-1]
+
+
 # ================================================================================ Dadupel
 @dataclass
 class SsmMixerConfig:
@@ -981,7 +1105,7 @@ class DadupelConfig:
     def num_layers(self): return len(self.layers)
 
 
-class Dadupel(_ModelBase):
+class Dadupel(_RaggedModel):
     """Hybrid decoder: Mamba-2 and latent-attention mixers in any order, each beside a clamped gated feed-forward under ONE
     layer norm (x + scale_1 * mixer(h) + scale_2 * ff(h)), tied embedding and head.
 
@@ -991,7 +1115,6 @@ class Dadupel(_ModelBase):
     steps: all sequences in one launch)."""
 
     namespace = "dadupel"
-    ragged_batches = True
 
     def __init__(self, config: DadupelConfig, backend, dtype: str = "Bf16", context_length: Optional[int] = None):
         super().__init__(backend, dtype)
@@ -1092,71 +1215,36 @@ class Dadupel(_ModelBase):
         out["lm_head"] = ((d, c.vocab_size), "embed", True)     # the tied table once more, as a linear layer reads it
         return out
 
-    def expected_params(self) -> Dict[str, tuple]:
-        return {n: e[0] for n, e in self._param_plan(self.config).items()}
-
-    @classmethod
-    def tensor_layout(cls, config: DadupelConfig) -> Dict[str, Tuple[str, bool]]:
-        return {n: (e[1], e[2]) for n, e in cls._param_plan(config).items()}
-
-    def param_dtype(self, name: str) -> str:
-        """Matrices that feed products are in the model dtype; gains, scales, taps and per-head constants are f32."""
-        leaf = name.rsplit(".", 1)[-1]
-        return self.dtype if leaf.startswith("w_") or leaf in ("weight", "lm_head") else "F32"
-
     @classmethod
     def random(cls, config: DadupelConfig, backend, seed: int = 0, dtype: str = "Bf16", context_length: Optional[int] = None) -> "Dadupel":
         """Random weights of the right shapes and of sensible sizes, one numpy stream per tensor."""
-        from concurrent.futures import ThreadPoolExecutor
         m = cls(config, backend, dtype, context_length)
-        plan = [(n, d) for n, d in m.expected_params().items() if n != "lm_head"]
 
-        def make(idx):
-            name, dims = plan[idx]
-            rng = np.random.default_rng(np.random.SeedSequence([seed, idx]))
+        def draw(rng, name, dims):
             leaf = name.rsplit(".", 1)[-1]
             if leaf == "dt_bias":
-                arr = np.log(np.expm1(np.exp(rng.uniform(np.log(1e-3), np.log(1e-1), dims)))).astype(np.float32)
-            elif leaf == "a_log":
-                arr = np.log(rng.uniform(1.0, 16.0, dims)).astype(np.float32)
-            elif leaf in ("gamma", "d"):
-                arr = (1.0 + 0.1 * rng.standard_normal(dims)).astype(np.float32)
-            elif leaf in ("beta", "conv_bias"):
-                arr = (0.1 * rng.standard_normal(dims)).astype(np.float32)
-            elif leaf in ("scale_1", "scale_2"):
-                arr = rng.uniform(0.3, 1.0, dims).astype(np.float32)
-            else:
-                arr = rng.standard_normal(dims, dtype=np.float32)
-                arr *= np.float32((dims[1] if leaf == "weight" else dims[0]) ** -0.5)
-            dt = m.param_dtype(name)
-            return name, dims, dt, _np_to_bytes(arr, dt), arr if leaf == "weight" else None
+                return np.log(np.expm1(np.exp(rng.uniform(np.log(1e-3), np.log(1e-1), dims)))).astype(np.float32)
+            if leaf == "a_log":
+                return np.log(rng.uniform(1.0, 16.0, dims)).astype(np.float32)
+            if leaf in ("gamma", "d"):
+                return (1.0 + 0.1 * rng.standard_normal(dims)).astype(np.float32)
+            if leaf in ("beta", "conv_bias"):
+                return (0.1 * rng.standard_normal(dims)).astype(np.float32)
+            if leaf in ("scale_1", "scale_2"):
+                return rng.uniform(0.3, 1.0, dims).astype(np.float32)
+            arr = rng.standard_normal(dims, dtype=np.float32)
+            arr *= np.float32((dims[1] if leaf == "weight" else dims[0]) ** -0.5)
+            return arr
 
-        workers = max(1, min(16, os.cpu_count() or 1))
-        with ThreadPoolExecutor(max_workers=workers) as ex:
-            pending, nxt, table = [], 0, None
-            while nxt < len(plan) or pending:   # bounded look-ahead: a few tensors of host memory in flight
-                while nxt < len(plan) and len(pending) < 2 * workers:
-                    pending.append(ex.submit(make, nxt))
-                    nxt += 1
-                name, dims, dt, data, arr = pending.pop(0).result()
-                m.set_param_bytes(name, TensorSpec(dt, dims), data)
-                table = arr if arr is not None else table
+        table = m._fill_random([n for n in m.expected_params() if n != "lm_head"], seed, draw, ["tok_embeddings.weight"])["tok_embeddings.weight"]
         m.set_param("lm_head", np.ascontiguousarray(table.T), m.param_dtype("lm_head"))
         return m
-
-    @property
-    def num_layers(self): return self.config.num_layers
-    @property
-    def context_length(self): return self.config.context_length
 
     # -- graph pieces ----------------------------------------------------------------
     def _norm(self, x: Tensor, P, name: str) -> Tensor:
         """Layer norm of the f32 stream, handed on in the matmul dtype."""
         out, *_ = F.layer_norm(x, P[name + ".gamma"], P[name + ".beta"], self.config.eps)
         return out if self.dtype == "F32" else out.cast(self.dtype)
-
-    def _stack(self, parts: List[Tensor]) -> Tensor:
-        return parts[0] if len(parts) == 1 else Tensor.concat(0, parts)
 
     def _ssm_mixer(self, P, p: str, m: SsmMixerConfig, proj: Tensor, lens, states):
         """proj f32 [rows, z | x | B | C | dt] of all sequences; returns (rows in the matmul dtype, new (conv, state) per sequence)."""
@@ -1277,92 +1365,304 @@ class Dadupel(_ModelBase):
         self._programs[key] = (prog, layout)
         return prog, layout
 
-    # -- forward -----------------------------------------------------------------------
-    def forward_with_decode_cache(self, tokens, position_offset, caches, fixed_capacity=None, last_logits_only=False):
-        """See Gpt.forward_with_decode_cache."""
-        return self.forward_batch([list(tokens)], position_offset, [caches], fixed_capacity, last_logits_only=last_logits_only)
+    # -- what a layer keeps per sequence -------------------------------------------------
+    def _position_args(self, offs):
+        return [self._upload_i32([v for o in offs for v in (0, o, 0)])]
 
-    def forward_decode_device_token(self, token_handle, position_offset, caches, fixed_capacity=None):
-        """See Gpt.forward_decode_device_token."""
-        return self.forward_batch([[None]], position_offset, [caches], fixed_capacity, token_handle=token_handle)
+    def _fresh_slot(self, i, capacity):
+        m = self.config.layers[i].mixer
+        if isinstance(m, SsmMixerConfig):
+            return [self._zeros([m.conv - 1, m.channels], "F32"), self._zeros([m.heads, m.state, m.vdim], "F32")]
+        return [self._zeros([1, capacity, m.row_width])] if m.kv_from is None else []
 
-    def forward_batch(self, token_rows, position_offset, caches, fixed_capacity=None, token_handle=None, last_logits_only=False,
-                      logit_rows: Optional[Sequence[int]] = None):
-        """Independent sequences of any lengths.  `position_offset`: one for all or one per sequence.  The batch either starts
-        (empty caches, offset 0) or goes on by one token each; `caches[b]` is updated in place.  `logit_rows`: the stacked rows
-        whose logits are wanted (default: all, or each sequence's last with `last_logits_only`)."""
-        cfg, B = self.config, len(token_rows)
-        lens = tuple(len(r) for r in token_rows)
-        if B == 0 or min(lens) == 0:
-            raise ValueError("token sequence must contain at least one element")
-        offs = [int(position_offset)] * B if isinstance(position_offset, (int, np.integer)) else [int(o) for o in position_offset]
-        if len(offs) != B or len(caches) != B or any(len(c) != cfg.num_layers for c in caches):
-            raise ValueError(f"expected an offset and {cfg.num_layers} cache slots (one per layer) for every sequence")
-        have = caches[0][0] is not None
-        if any((slot is not None) != have for c in caches for slot in c):
-            raise ValueError("the sequences of a batch either all start or all go on")
-        if have and max(lens) != 1:
-            raise ValueError("decode with an existing cache supports one token per sequence")
-        if not have and any(offs):
-            raise ValueError("a sequence without a cache starts at position 0")
-        if token_handle is not None and max(lens) != 1:
-            raise ValueError("device tokens feed one step (one token per sequence)")
-        if token_handle is None:
-            for row in token_rows:
-                for t in row:
-                    if not 0 <= t < cfg.vocab_size:
-                        raise ValueError(f"token index {t} out of range")
-        totals = [o + n for o, n in zip(offs, lens)]
-        need = max(totals)
-        if need > cfg.context_length:
-            raise ValueError(f"token sequence length {need} exceeds model context length {cfg.context_length}")
-        if fixed_capacity is not None:
-            if not 0 < fixed_capacity <= cfg.context_length or fixed_capacity < need:
-                raise ValueError(f"decode cache capacity {fixed_capacity} invalid for sequence length {need}")
-            capacity = fixed_capacity
-        else:
-            capacity = decode_cache_capacity(need, cfg.context_length)
-        if have:
-            for c, o in zip(caches, offs):
-                for slot in c:
-                    if slot.len != o:
-                        raise ValueError(f"decode cache length {slot.len} must match position offset {o}")
-            # the sequences of a step share one capacity: the largest any of them has or needs
-            capacity = max([capacity] + [s.capacity for c in caches for s in c if isinstance(s, DecodeLatentCache)])
-            for c in caches:
-                for i, s in enumerate(c):
-                    if isinstance(s, DecodeLatentCache) and s.capacity < capacity:
-                        c[i] = DecodeLatentCache(self._grow_rows(s.rows, (1, s.capacity, cfg.layers[i].mixer.row_width), capacity), s.len, capacity)
-        prog, _ = self._build(lens, capacity, have, last_logits_only, None if logit_rows is None else len(logit_rows))
-        tok_arg = token_handle if token_handle is not None else self._upload_i32([t for row in token_rows for t in row])
-        args = [tok_arg, self._upload_i32([o + j for o, n in zip(offs, lens) for j in range(n)]), self._upload_i32([v for o in offs for v in (0, o, 0)])]
-        if logit_rows is not None:
-            args.append(self._upload_i32(logit_rows))
-        held = []
-        for c in caches:
-            for L, slot in zip(cfg.layers, c):
-                m = L.mixer
-                if isinstance(m, SsmMixerConfig):
-                    held += [slot.conv, slot.state] if have else [self._zeros([m.conv - 1, m.channels], "F32"), self._zeros([m.heads, m.state, m.vdim], "F32")]
-                elif m.kv_from is None:
-                    held.append(slot.rows if have else self._zeros([1, capacity, m.row_width]))
-        outs = self._run(prog, args + held, [False] * len(args) + [True] * len(held))
-        it = iter(outs[:-1])
-        for b in range(B):
-            for i, L in enumerate(cfg.layers):
-                m = L.mixer
-                if isinstance(m, SsmMixerConfig):
-                    caches[b][i] = DecodeSsmState(next(it), next(it), totals[b])
-                elif m.kv_from is None:
-                    caches[b][i] = DecodeLatentCache(next(it), totals[b], capacity)
-                else:
-                    caches[b][i] = SharedLayerCache(m.kv_from, totals[b])
-        return outs[-1]
+    def _slot_handles(self, slot):
+        return [slot.conv, slot.state] if isinstance(slot, DecodeSsmState) else [slot.rows] if isinstance(slot, DecodeLatentCache) else []
+
+    def _grown_slot(self, i, slot, capacity):
+        if not isinstance(slot, DecodeLatentCache) or slot.capacity >= capacity:
+            return slot
+        return DecodeLatentCache(self._grow_rows(slot.rows, (1, slot.capacity, self.config.layers[i].mixer.row_width), capacity), slot.len, capacity)
+
+    def _new_slot(self, i, handles, length, capacity):
+        m = self.config.layers[i].mixer
+        if isinstance(m, SsmMixerConfig):
+            return DecodeSsmState(next(handles), next(handles), length)
+        return DecodeLatentCache(next(handles), length, capacity) if m.kv_from is None else SharedLayerCache(m.kv_from, length)
+
+
+# ================================================================================ Fuzazen
+@dataclass
+class ChunkedMixerConfig:
+    """A grouped-query attention mixer whose positions see their own chunk of `chunk` positions only."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot_dims: int
+    rope_base: float
+    chunk: int
+
+    @property
+    def keys(self): return self.kv_heads * self.dim
+    @property
+    def values(self): return self.kv_heads * self.vdim
+    @property
+    def projection(self): return self.heads * self.dim + self.keys + self.values + self.heads    # q | k | v | gate
+
+    def rows(self, capacity: int) -> int:
+        """Cache rows of a sequence of at most `capacity` positions: a position's row is its place in its chunk."""
+        return min(capacity, self.chunk)
+
+
+@dataclass
+class FuzazenLayer:
+    mixer: ChunkedMixerConfig
+    ffn_dim: Optional[int] = None       # None: no feed-forward
+    weights_of: Optional[int] = None    # the layer whose tensors this one uses (None: its own)
+
+
+@dataclass
+class FuzazenConfig:
+    vocab_size: int
+    embed_dim: int
+    eps: float
+    layers: List[FuzazenLayer]
+    embedding_scale: float = 1.0
+    residual_mult: float = 1.0
+    logit_softcap: Optional[float] = None
+    context_length: int = 1 << 20       # the design states no limit; this one bounds the caches
+
+    @property
+    def num_layers(self): return len(self.layers)
+
+    def owner(self, i: int) -> int:
+        """The layer whose tensors layer i uses."""
+        seen = set()
+        while self.layers[i].weights_of is not None:
+            if i in seen or not 0 <= self.layers[i].weights_of < len(self.layers):
+                raise ValueError(f"layer {i}: weights_of must lead to a layer with weights of its own")
+            seen.add(i)
+            i = self.layers[i].weights_of
+        return i
+
+
+class Fuzazen(_RaggedModel):
+    """Decoder of chunked grouped-query attention (pairwise rotation, unit-RMS queries and keys, a sink and an output gate per
+    head) and SwiGLU layers that read the residual stream itself; the norm stands on a sublayer's output: x + m * rms_norm(f(x)).
+    Layers may share their weights.  Soft-capped logits.
+
+    The residual stream, the norms, the packed projection q | k | v | gate and the logits are f32; matmul operands and the caches
+    are in the model dtype.  A cache holds the rows of the current chunk only: position p's row is p % chunk."""
+
+    namespace = "fuzazen"
+
+    def __init__(self, config: FuzazenConfig, backend, dtype: str = "Bf16", context_length: Optional[int] = None):
+        super().__init__(backend, dtype)
+        self.config = config
+        if context_length is not None:
+            config.context_length = int(context_length)
+        for i, L in enumerate(config.layers):
+            m, own = L.mixer, config.layers[config.owner(i)]
+            if m.kv_heads < 1 or m.heads % m.kv_heads or m.rot_dims % 2 or not 0 <= m.rot_dims <= m.dim or m.chunk < 1:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads, rot.dims even and at most dim, the chunk at least 1")
+            if (m, L.ffn_dim) != (own.mixer, own.ffn_dim):
+                raise ValueError(f"layer {i}: a layer that uses another's weights has its sizes")
+        self.chunks = sorted({L.mixer.chunk for L in config.layers})
+
+    # -- configuration and parameters ---------------------------------------------------
+    @staticmethod
+    def config_from_json(c) -> FuzazenConfig:
+        layers = []
+        for L in c["layers"]:
+            if L["type"] != "attention":
+                raise ValueError(f"unknown layer type {L['type']!r}")
+            m, mlp = L["mixer"], L.get("mlp")
+            if mlp is not None and mlp["kind"] != "dense":
+                raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+            mixer = ChunkedMixerConfig(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), scale=float(m["scale"]),
+                                       rot_dims=int(m["rot"]["dims"]), rope_base=float(m["rot"]["base"]), chunk=int(m["mask"]["size"]))
+            layers.append(FuzazenLayer(mixer, None if mlp is None else int(mlp["ff"]), None if L.get("weights_of") is None else int(L["weights_of"])))
+        cap = c.get("logit_softcap")
+        return FuzazenConfig(vocab_size=int(c["vocab"]), embed_dim=int(c["width"]), eps=float(c["norm"]["eps"]), layers=layers,
+                             embedding_scale=float(c["embedding"]["scale"]), residual_mult=float(c["residual_mult"]),
+                             logit_softcap=None if cap is None else float(cap), context_length=int(c.get("context_length", 1 << 20)))
+
+    def checkpoint_config(self) -> Dict[str, object]:
+        c, layers = self.config, []
+        for L in c.layers:
+            m = L.mixer
+            e = {"type": "attention", "mlp": None if L.ffn_dim is None else {"kind": "dense", "ff": L.ffn_dim},
+                 "mixer": dict(heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, scale=m.scale, rot={"dims": m.rot_dims, "base": m.rope_base},
+                               mask={"size": m.chunk})}
+            if L.weights_of is not None:
+                e["weights_of"] = L.weights_of
+            layers.append(e)
+        return {"architecture": "Fuzazen", "vocab": c.vocab_size, "width": c.embed_dim, "norm": {"eps": c.eps}, "embedding": {"scale": c.embedding_scale},
+                "residual_mult": c.residual_mult, "logit_softcap": c.logit_softcap, "layers": layers}
+
+    @staticmethod
+    def _param_plan(c: FuzazenConfig) -> Dict[str, Tuple[tuple, object, bool]]:
+        """parameter -> (shape, tensor of a model folder or the tensors stacked in it, transposed there)."""
+        d = c.embed_dim
+        out = {"tok_embeddings.weight": ((c.vocab_size, d), "embed", False)}
+        for i, L in enumerate(c.layers):
+            if L.weights_of is not None:
+                continue
+            p, t, m = f"blocks.{i}.", f"l{i}.", L.mixer
+            out[p + "mixer.w_qkvg"] = ((d, m.projection), tuple(t + "mix." + n for n in "qkvg"), True)
+            out[p + "mixer.sink"] = ((m.heads,), t + "mix.sink", False)
+            out[p + "mixer.w_out"] = ((m.heads * m.vdim, d), t + "mix.o", True)
+            out[p + "norm_1.gamma"] = ((d,), t + "norm1", False)
+            if L.ffn_dim is not None:
+                out[p + "feed_forward.w_gate"] = ((d, L.ffn_dim), t + "mlp.gate", True)
+                out[p + "feed_forward.w_up"] = ((d, L.ffn_dim), t + "mlp.up", True)
+                out[p + "feed_forward.w_down"] = ((L.ffn_dim, d), t + "mlp.down", True)
+                out[p + "norm_2.gamma"] = ((d,), t + "norm2", False)
+        out["final_norm.gamma"] = ((d,), "final.norm", False)
+        out["lm_head"] = ((d, c.vocab_size), "head", True)
+        return out
+
+    @classmethod
+    def random(cls, config: FuzazenConfig, backend, seed: int = 0, dtype: str = "Bf16", context_length: Optional[int] = None) -> "Fuzazen":
+        """Random weights of the right shapes and of sensible sizes, one numpy stream per tensor."""
+        m = cls(config, backend, dtype, context_length)
+
+        def draw(rng, name, dims):
+            leaf = name.rsplit(".", 1)[-1]
+            if leaf == "gamma":
+                return (1.0 + 0.1 * rng.standard_normal(dims)).astype(np.float32)
+            if leaf == "sink":
+                return rng.standard_normal(dims).astype(np.float32)
+            arr = rng.standard_normal(dims, dtype=np.float32)
+            if leaf != "weight":
+                arr *= np.float32(dims[0] ** -0.5)
+            return arr
+
+        m._fill_random(m.expected_params(), seed, draw)
+        return m
+
+    # -- graph ---------------------------------------------------------------------------
+    def _operand(self, x: Tensor) -> Tensor:
+        """The f32 stream as an operand of matrix products."""
+        return x if self.dtype == "F32" else x.cast(self.dtype)
+
+    def _build(self, lens: Tuple[int, ...], capacity: int, decode: bool, last_only: bool = False, n_logit_rows: Optional[int] = None):
+        """One program for a forward of len(lens) sequences, sequence b bringing lens[b] rows (decode: one each).
+        last_only: the head runs on every sequence's last row; n_logit_rows: on that many rows, named by an argument."""
+        last_only = last_only and not decode
+        key = (lens, capacity, decode, last_only, n_logit_rows)
+        if key in self._programs:
+            return self._programs[key]
+        cfg, dt, B, rows = self.config, self.dtype, len(lens), sum(lens)
+        fb = FunctionBuilder("main", dt)
+        tok = fb.param("Si32", [rows])
+        pos = fb.param("Si32", [rows])
+        # [0, row, 0] of every sequence: where its new cache rows go, one argument per size of chunk
+        starts = {n: fb.param("Si32", [3 * B]) for n in self.chunks}
+        layout = {"args": ["tokens", "positions"] + [f"starts_{n}" for n in self.chunks]}
+        pick = None
+        if n_logit_rows is not None:
+            pick = fb.param("Si32", [n_logit_rows])
+            layout["args"].append("logit_rows")
+        held = [[(fb.param(dt, [L.mixer.kv_heads, L.mixer.rows(capacity), L.mixer.dim]), fb.param(dt, [L.mixer.kv_heads, L.mixer.rows(capacity), L.mixer.vdim]))
+                 for L in cfg.layers] for _ in range(B)]
+        layout["n_args"] = len(fb.params)
+        P = self._declare_params(fb)
+        tables: Dict[bytes, Tensor] = {}
+
+        def table_of(m: ChunkedMixerConfig) -> Tensor:
+            f = F.pair_frequencies(m.rot_dims, m.rope_base)
+            k = f.tobytes()
+            if k not in tables:
+                tables[k] = F.rope_table(pos, fb.constant(TensorSpec("F32", f.shape), f.astype("<f4").tobytes()))
+            return tables[k]
+
+        def part(t: Tensor, b: int) -> Tensor:   # the rows of sequence b
+            return t if B == 1 else t.slice([sum(lens[:b]), 0], [lens[b], t.dims[1]])
+
+        for L in cfg.layers:
+            if L.mixer.rot_dims:
+                table_of(L.mixer)
+        hidden = F.embedding_lookup(P["tok_embeddings.weight"], tok)
+        if dt != "F32":
+            hidden = hidden.cast("F32")
+        if cfg.embedding_scale != 1.0:
+            hidden = hidden * float(cfg.embedding_scale)
+        new = [[()] * cfg.num_layers for _ in range(B)]
+        for i, L in enumerate(cfg.layers):
+            p, m = f"blocks.{cfg.owner(i)}.", L.mixer
+            q = p + "mixer."
+            proj = F.linear(self._operand(hidden), P[q + "w_qkvg"], out_dtype="F32")
+            cols = [0, m.heads * m.dim, m.keys, m.values, m.heads]
+            qs, ks, vs, gate = (proj.slice([0, sum(cols[:j + 1])], [rows, cols[j + 1]]) for j in range(4))
+            qs, ks = (F.rope_pairs(t, table_of(m), n, 0) if m.rot_dims else t for t, n in ((qs, m.heads), (ks, m.kv_heads)))
+            qs, ks = (F.head_rms_norm(t, n, cfg.eps, dt) for t, n in ((qs, m.heads), (ks, m.kv_heads)))
+            vs = self._operand(vs)
+            ctxs = []
+            for b in range(B):
+                kb, vb, sink = part(ks, b), part(vs, b), P[q + "sink"]
+                first = 0 if decode else (lens[b] - 1) // m.chunk * m.chunk   # the rows of the chunk that the next token may go on with
+                at = starts[m.chunk] if B == 1 else starts[m.chunk].slice([3 * b], [3])
+                slot = []
+                for t, width, base in ((kb, m.dim, held[b][i][0]), (vb, m.vdim, held[b][i][1])):
+                    n = lens[b] - first
+                    t = t if first == 0 else t.slice([first, 0], [n, t.dims[1]])
+                    slot.append(F.dynamic_update_slice_into(base, t.reshape([n, m.kv_heads, width]).transpose([1, 0, 2]), at))
+                new[b][i] = tuple(slot)
+                if decode:
+                    ctxs.append(F.chunk_attention_cache(part(qs, b), slot[0], slot[1], sink, pos if B == 1 else pos.slice([b], [1]), m.heads, m.chunk, m.scale))
+                else:   # a prompt starts at its first token: its keys and values are the rows at hand
+                    ctxs.append(F.chunk_attention(part(qs, b), kb, vb, sink, m.heads, m.kv_heads, m.chunk, m.scale))
+            ctx = F.head_gate(self._stack(ctxs), gate, m.heads)
+            y = F.linear(ctx, P[q + "w_out"], out_dtype="F32")
+            hidden = F.post_norm_add(hidden, y, P[p + "norm_1.gamma"], cfg.residual_mult, cfg.eps)
+            if L.ffn_dim is not None:
+                f, h = p + "feed_forward.", self._operand(hidden)
+                act = F.swiglu(F.linear(h, P[f + "w_gate"]), F.linear(h, P[f + "w_up"]))
+                y = F.linear(act, P[f + "w_down"], out_dtype="F32")
+                hidden = F.post_norm_add(hidden, y, P[p + "norm_2.gamma"], cfg.residual_mult, cfg.eps)
+        if pick is not None:
+            hidden = hidden.take(pick)
+        elif last_only:
+            hidden = self._stack([hidden.slice([sum(lens[:b + 1]) - 1, 0], [1, cfg.embed_dim]) for b in range(B)])
+        normed, *_ = F.rms_norm(hidden, P["final_norm.gamma"], cfg.eps)
+        logits = F.linear(self._operand(normed), P["lm_head"], out_dtype="F32")
+        if cfg.logit_softcap is not None:
+            logits = F.softcap(logits, cfg.logit_softcap)
+        fb.set_results([t for b in range(B) for slot in new[b] for t in slot] + [logits])
+        prog = Program(fb)
+        self._programs[key] = (prog, layout)
+        return prog, layout
+
+    # -- what a layer keeps per sequence -------------------------------------------------
+    def _position_args(self, offs):
+        return [self._upload_i32([v for o in offs for v in (0, o % n, 0)]) for n in self.chunks]
+
+    def _slot_dims(self, i, rows):
+        m = self.config.layers[i].mixer
+        return (m.kv_heads, rows, m.dim), (m.kv_heads, rows, m.vdim)
+
+    def _fresh_slot(self, i, capacity):
+        return [self._zeros(d) for d in self._slot_dims(i, self.config.layers[i].mixer.rows(capacity))]
+
+    def _slot_handles(self, slot):
+        return [slot.keys, slot.values]
+
+    def _grown_slot(self, i, slot, capacity):
+        rows = self.config.layers[i].mixer.rows(capacity)
+        if slot.capacity >= rows:
+            return slot
+        return DecodeKvCache(*(self._grow_rows(h, d, rows) for h, d in zip((slot.keys, slot.values), self._slot_dims(i, slot.capacity))), slot.len, rows)
+
+    def _new_slot(self, i, handles, length, capacity):
+        return DecodeKvCache(next(handles), next(handles), length, self.config.layers[i].mixer.rows(capacity))
 
 
 # kind of a checkpoint -> (class, default storage dtype); `architecture` of a model folder's config.json -> kind
-MODEL_KINDS = {"gpt": (Gpt, "F32"), "ministral": (Ministral, "Bf16"), "dadupel": (Dadupel, "Bf16")}
-KIND_OF_ARCHITECTURE = {"Dadupel": "dadupel"}
+MODEL_KINDS = {"gpt": (Gpt, "F32"), "ministral": (Ministral, "Bf16"), "dadupel": (Dadupel, "Bf16"), "fuzazen": (Fuzazen, "Bf16")}
+KIND_OF_ARCHITECTURE = {"Dadupel": "dadupel", "Fuzazen": "fuzazen"}
 
 
 # ================================================================================ BatchGenerator
