@@ -1260,12 +1260,14 @@ int gptrs_hip_fusion_report(const char* program_json, size_t json_len, const int
             if (in.dead) continue;
             text += in.op_name;
             if (in.op == gptrs::OpKind::FLinear) {
+                if (in.post) text += "+post_norm_add";
                 if (in.norm) text += in.norm_ln ? "+layer_norm" : "+rms_norm";
                 if (in.has_bias) text += "+bias";
                 if (in.act == 1) text += "+gelu";
                 if (in.act == 2) text += in.glu ? "+clamped_glu" : "+swiglu";
                 if (in.has_scale) text += "+colscale";
                 if (in.has_residual) text += "+residual";
+                if (in.softcap != 0.f) text += "+softcap";
                 text += in.mfma ? " [gemm]" : in.tiled ? " [stream]" : " [generic]";
             }
             if (in.op == gptrs::OpKind::FAttnDecode && in.rot_half > 0) text += "+rope";

@@ -34,6 +34,7 @@ __device__ __forceinline__ float glu_combine(float g, float u, int kind, float l
     return (g / (1.0f + expf(g * -1.0f))) * u;
 }
 __device__ __forceinline__ float silu_f32(float x) { return x / (1.0f + expf(-x)); }
+__device__ __forceinline__ float softcap_f32(float x, float cap) { return cap * tanhf(x / cap); }
 // log(1 + e^x) without overflow and without losing small values
 __device__ __forceinline__ float softplus_f32(float x) { return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x))); }
 

@@ -321,6 +321,65 @@ struct Fuser {
         reindex();
     }
 
+    // x + mult * rms_norm(y) of f32 rows -> Mix::PostNorm (x, y, gain) -> (sum[, the sum in bf16: a Cast of it taken in]).
+    void pass_post_norm() {
+        const std::vector<int> uses = count_uses();
+        for (size_t i = 0; i < fn.body.size(); ++i) {
+            if (fn.body[i].dead || fn.body[i].op != OpKind::Binary || fn.body[i].binary != BinaryOp::Add || fn.body[i].scalar_rhs) continue;
+            const Instr add = fn.body[i];
+            const Spec& out = add.out_specs[0];
+            if (out.dtype != DType::F32 || out.rank() != 2) continue;
+            for (int side = 0; side < 2; ++side) {
+                const int x = add.operands[1 - side].value;
+                int nv = add.operands[side].value, a, b;
+                float mult = 1.0f;
+                if (x < 0 || nv < 0 || def[nv] < 0 || uses[nv] != 1) continue;
+                if (binary(nv, BinaryOp::Mul, a, b) && scalar(b, mult)) nv = a;
+                else mult = 1.0f;
+                const Instr* nrm = producer(nv);
+                if (!nrm || nrm->dead || nrm->op != OpKind::FRmsNorm || uses[nv] != 1) continue;
+                const Spec* xs = spec_of(x);
+                const Spec* ys = spec_of(nrm->operands[0].value);
+                const Spec* gs = spec_of(nrm->operands[1].value);
+                if (!xs || !ys || !gs || *xs != out || *ys != out || gs->dtype != DType::F32 || nrm->out_specs[0] != out) continue;
+                Instr ni = make(OpKind::FMixer, "fused.post_norm_add", {x, nrm->operands[0].value, nrm->operands[1].value}, add.out_ids[0], out);
+                ni.mix = Mix::PostNorm;
+                ni.post_mult = mult;
+                ni.eps = nrm->eps;
+                ni.scale = nrm->scale;
+                for (Instr& c : fn.body)
+                    if (!c.dead && c.op == OpKind::Cast && c.operands[0].value == add.out_ids[0] && c.out_specs[0].dtype == DType::BF16) {
+                        add_out(ni, c.out_ids[0], c.out_specs[0]);
+                        c.dead = true;
+                        break;
+                    }
+                replace_root(add.out_ids[0], ni);
+                reindex();
+                break;
+            }
+        }
+    }
+
+    // cap * tanh(x / cap) of f32 values -> Mix::Softcap
+    void pass_softcap() {
+        const std::vector<int> uses = count_uses();
+        for (size_t i = 0; i < fn.body.size(); ++i) {
+            const Instr in = fn.body[i];
+            if (in.dead || in.op != OpKind::Binary || in.out_specs[0].dtype != DType::F32) continue;
+            const int v = in.out_ids[0];
+            int t, s1, q, x, s2;
+            float c1, c2;
+            if (!binary(v, BinaryOp::Mul, t, s1) || !scalar(s1, c1) || !unary(t, UnaryOp::Tanh, q) || !binary(q, BinaryOp::Div, x, s2) || !scalar(s2, c2) ||
+                c1 != c2 || !(c1 > 0.0f) || uses[t] != 1 || uses[q] != 1)
+                continue;
+            Instr ni = make(OpKind::FMixer, "fused.softcap", {x}, v, in.out_specs[0]);
+            ni.mix = Mix::Softcap;
+            ni.softcap = c1;
+            replace_root(v, ni);
+        }
+        reindex();
+    }
+
     Instr make(OpKind op, const char* name, std::vector<int> ins, int out_id, const Spec& out_spec) const {
         Instr ni;
         ni.op = op;
@@ -998,6 +1057,151 @@ struct Fuser {
         }
     }
 
+    // A matrix value as a block of another: through Slices, and through casts from f32 (which the kernels' own stores do).
+    struct Block { int base = -1; int64_t row = 0, col = 0, rows = 0, cols = 0; };
+    Block block_of(int v, bool through_casts) const {
+        Block b;
+        const Spec* s = spec_of(v);
+        if (!s || s->rank() != 2) return b;
+        b.rows = s->dims[0];
+        b.cols = s->dims[1];
+        for (;;) {
+            const Instr* p = producer(v);
+            if (p && !p->dead && p->op == OpKind::Slice && p->operands[0].value >= 0) { b.row += p->a[0]; b.col += p->a[1]; v = p->operands[0].value; continue; }
+            if (through_casts && p && !p->dead && p->op == OpKind::Cast && p->operands[0].value >= 0) {
+                const Spec* from = spec_of(p->operands[0].value);
+                if (from && from->dtype == DType::F32) { v = p->operands[0].value; continue; }
+            }
+            break;
+        }
+        b.base = v;
+        return b;
+    }
+    // q or k of all rows: head_rms_norm(rope_pairs(columns of proj)) or head_rms_norm(columns of proj)
+    bool m_chunk_heads(int v, int proj, int64_t col, int64_t heads, float eps, bool first, int& table, float& eps_out) const {
+        const Instr* nm = mixer(v, Mix::HeadNorm);
+        if (!nm || nm->mx.heads != heads) return false;
+        int x = nm->operands[0].value, tab = -1;
+        if (const Instr* rp = mixer(x, Mix::RopePairs)) {
+            if (rp->mx.heads != heads || rp->mx.col != 0) return false;
+            x = rp->operands[0].value;
+            tab = rp->operands[1].value;
+        }
+        const Block b = block_of(x, false);
+        if (b.base != proj || b.row != 0 || b.col != col || b.cols != heads * nm->mx.dim) return false;
+        if (first) { table = tab; eps_out = nm->eps; return true; }
+        return tab == table && nm->eps == eps;
+    }
+    // Chunked attention: the head gate over the stacked attentions of a batch, the preparation of their queries, keys and values
+    // from one projection and the update of the caches -> Mix::ChunkDecode / ChunkPrefill
+    //   (proj, sink, pos, starts, [table,] keys_0, values_0, ..) -> (ctx, keys'_0, values'_0, ..)
+    void pass_chunked() {
+        for (size_t gi = 0; gi < fn.body.size(); ++gi) {
+            if (fn.body[gi].dead || fn.body[gi].op != OpKind::FMixer || fn.body[gi].mix != Mix::HeadGate) continue;
+            const Instr root = fn.body[gi];
+            const std::vector<int> uses = count_uses();
+            const int x = root.operands[0].value;
+            const Block gb = block_of(root.operands[1].value, false);
+            const int proj = gb.base;
+            const Spec* ps = spec_of(proj);
+            const std::vector<int> parts = stacked(x);
+            if (parts.empty() || uses[x] != 1 || !ps || ps->dtype != DType::F32 || ps->rank() != 2 || gb.row != 0 || gb.rows != ps->dims[0]) continue;
+            const Instr* a0 = producer(parts[0]);
+            if (!a0 || a0->dead || a0->op != OpKind::FMixer || (a0->mix != Mix::ChunkAttn && a0->mix != Mix::ChunkAttnCache)) continue;
+            const bool cached = a0->mix == Mix::ChunkAttnCache;
+            Instr::MixAttrs m = a0->mx;
+            const int64_t H = m.heads, G = m.groups, D = m.dim, V = m.vdim, colk = H * D, colv = colk + G * D, colg = colv + G * V;
+            bool ok = root.mx.heads == H && root.mx.vdim == V && gb.col == colg && gb.cols == H && ps->dims[1] == colg + H;
+            if (!ok) continue;
+            const Block qb = block_of(a0->operands[0].value, false);
+            int table = -1, kbase = -1, pos = -1, starts = -1;
+            float eps = 0.f;
+            ok = m_chunk_heads(qb.base, proj, 0, H, 0.f, true, table, eps);
+            std::vector<int> bases, outs, dead;
+            std::vector<int64_t> lens;
+            int64_t row = 0;
+            const int64_t B = (int64_t)parts.size();
+            for (int64_t b = 0; b < B && ok; ++b) {
+                const Instr* at = mixer(parts[b], a0->mix);
+                ok = at && uses[parts[b]] == 1 && at->mx.heads == H && at->mx.groups == G && at->mx.dim == D && at->mx.vdim == V && at->mx.chunk == m.chunk &&
+                     at->scale == a0->scale && at->operands[3].value == a0->operands[3].value;
+                if (!ok) break;
+                const Block q = block_of(at->operands[0].value, false);
+                ok = q.base == qb.base && q.row == row && q.col == 0 && q.cols == H * D;
+                const int64_t len = q.rows, keep = cached ? 1 : (m.chunk > 0 ? (len - 1) % m.chunk + 1 : len);
+                ok = ok && (!cached || len == 1);
+                if (!ok) break;
+                int caches[2] = {-1, -1};
+                if (cached) {
+                    if (b == 0) pos = vector_source(at->operands[4].value);
+                    const Spec* vs = spec_of(pos);
+                    ok = elements_of(at->operands[4].value, pos, b, 1) && vs && vs->dims == std::vector<int64_t>{B};
+                    caches[0] = at->operands[1].value;
+                    caches[1] = at->operands[2].value;
+                } else {
+                    const Block k = block_of(at->operands[1].value, false), v = block_of(at->operands[2].value, true);
+                    if (b == 0) kbase = k.base;
+                    ok = k.base == kbase && k.row == row && k.col == 0 && k.cols == G * D && v.base == proj && v.row == row && v.col == colv && v.cols == G * V;
+                    // the caches: updates with this sequence's last rows that nothing else explains
+                    for (const Instr& du : fn.body) {
+                        if (!ok || du.dead || du.op != OpKind::DynamicUpdateSlice || du.operands[1].value < 0) continue;
+                        int tr, rs;
+                        if (!transpose102(du.operands[1].value, tr) || !reshape_of(tr, rs)) continue;
+                        const Block u = block_of(rs, true);
+                        if (u.row != row + len - keep || u.rows != keep) continue;
+                        if (u.base == kbase && u.cols == G * D) { ok = caches[0] < 0; caches[0] = du.out_ids[0]; }
+                        else if (u.base == proj && u.col == colv && u.cols == G * V) { ok = caches[1] < 0; caches[1] = du.out_ids[0]; }
+                    }
+                    ok = ok && caches[0] >= 0 && caches[1] >= 0;
+                }
+                for (int kv = 0; kv < 2 && ok; ++kv) {
+                    const Instr* du = producer(caches[kv]);
+                    int tr = -1, rs = -1;
+                    ok = du && !du->dead && du->op == OpKind::DynamicUpdateSlice && du->operands[0].value >= 0 && du->operands[2].value >= 0 &&
+                         du->a == std::vector<int64_t>{G, keep, kv ? V : D} && transpose102(du->operands[1].value, tr) && reshape_of(tr, rs);
+                    if (!ok) break;
+                    const Block u = block_of(rs, kv == 1);
+                    if (kv == 0 && b == 0 && cached) kbase = u.base;
+                    ok = u.row == row + len - keep && u.rows == keep && (kv ? u.base == proj && u.col == colv && u.cols == G * V : u.base == kbase && u.col == 0 && u.cols == G * D);
+                    if (kv == 0 && b == 0) starts = vector_source(du->operands[2].value);
+                    const Spec* ss = spec_of(starts);
+                    ok = ok && elements_of(du->operands[2].value, starts, 3 * b, 3) && ss && ss->dims == std::vector<int64_t>{3 * B};
+                    const Spec* cs = spec_of(caches[kv]);
+                    ok = ok && cs && cs->rank() == 3 && cs->dims == std::vector<int64_t>{G, spec_of(caches[0])->dims[1], kv ? V : D} && cs->dtype == root.out_specs[0].dtype &&
+                         cs->dims[1] >= keep && (b == 0 || cs->dims[1] == spec_of(outs[0])->dims[1]);
+                    if (!ok) break;
+                    bases.push_back(du->operands[0].value);
+                    outs.push_back(caches[kv]);
+                    dead.push_back(caches[kv]);
+                }
+                row += len;
+                lens.push_back(len);
+                dead.push_back(parts[b]);
+            }
+            ok = ok && row == ps->dims[0] && m_chunk_heads(kbase, proj, colk, G, eps, false, table, eps);
+            if (!ok) continue;
+            // a cache that something besides this layer's attention reads must not be taken apart from its update: it is not, the
+            // fused instruction defines the same values
+            m.rot = 0;
+            if (table >= 0) m.rot = spec_of(table)->dims[1];
+            if (!cached) pos = starts;   // (unused)
+            Instr ni = make(OpKind::FMixer, cached ? "fused.chunk_decode" : "fused.chunk_prefill", {proj, a0->operands[3].value, pos, starts}, root.out_ids[0], root.out_specs[0]);
+            ni.mix = cached ? Mix::ChunkDecode : Mix::ChunkPrefill;
+            ni.mx = m;
+            ni.scale = a0->scale;
+            ni.eps = eps;
+            ni.lens = lens;
+            auto add = [&](int v) { Operand o; o.value = v; ni.operands.push_back(o); };
+            if (table >= 0) add(table);
+            for (size_t i = 0; i < bases.size(); ++i) { add(bases[i]); add_out(ni, outs[i], *spec_of(outs[i])); }
+            for (int v : dead) kill(v);
+            if (parts[0] != x) kill(x);
+            fn.body[gi] = ni;
+            ++fused;
+            reindex();
+        }
+    }
+
     // ---------------------------------------------------------------- linear layers
     std::vector<int> count_uses() const {
         std::vector<int> uses(fn.max_value_id + 1, 0);
@@ -1077,8 +1281,20 @@ struct Fuser {
                 auto linear_of = [&](int q) -> Instr* {
                     if (q < 0 || def[q] < 0) return nullptr;
                     Instr* p = &fn.body[def[q]];
-                    return (p->op == OpKind::FLinear && !p->dead && uses[q] == 1) ? p : nullptr;
+                    return (p->op == OpKind::FLinear && !p->dead && uses[q] == 1 && p->softcap == 0.f) ? p : nullptr;
                 };
+                if (in.op == OpKind::FMixer && in.mix == Mix::Softcap) {
+                    Instr* lin = linear_of(in.operands[0].value);
+                    if (!lin || lin->quant || lin->act != 0 || lin->has_bias || lin->has_scale || lin->has_residual || lin->softcap != 0.f || !fast_linear(*lin)) continue;
+                    Instr ni = *lin;
+                    ni.softcap = in.softcap;
+                    ni.out_ids = {v};
+                    lin->dead = true;
+                    fn.body[i] = ni;
+                    reindex();
+                    changed = true;
+                    continue;
+                }
                 if (in.op == OpKind::Binary && in.binary == BinaryOp::Add && !in.scalar_rhs) {
                     const int a = in.operands[0].value, b = in.operands[1].value;
                     if (a < 0 || b < 0) continue;
@@ -1224,6 +1440,32 @@ struct Fuser {
                 c->scale = nrm.scale;
             }
             nrm.dead = true;
+            ++fused;
+        }
+        reindex();
+        // A one-row residual update whose sum feeds one decode linear, as bf16 or through a folded RMS norm, becomes that layer's
+        // prologue; the f32 sum is then the layer's second output where something else reads it.
+        const std::vector<int> uses2 = count_uses();
+        for (auto& pn : fn.body) {
+            if (pn.dead || pn.op != OpKind::FMixer || pn.mix != Mix::PostNorm || pn.out_specs[0].dims[0] != 1) continue;
+            const int sum = pn.out_ids[0], low = pn.out_ids.size() > 1 && uses2[pn.out_ids[1]] > 0 ? pn.out_ids[1] : -1;
+            const int feed = low >= 0 ? low : sum;
+            Instr* lin = nullptr;
+            int found = 0;
+            for (auto& c : fn.body)
+                if (!c.dead && c.op == OpKind::FLinear && c.tiled && !c.quant && !c.post && c.operands[0].value == feed) { lin = &c; ++found; }
+            if (found != 1 || is_result[feed] || spec_of(lin->operands[1].value)->dtype != DType::BF16) continue;
+            if (low >= 0 ? (lin->norm || uses2[low] != 1) : (!lin->norm || lin->norm_ln || !lin->x_f32 || uses2[sum] != 1)) continue;
+            lin->operands[0] = pn.operands[1];
+            lin->operands.push_back(pn.operands[2]);
+            lin->operands.push_back(pn.operands[0]);
+            lin->post = true;
+            lin->x_f32 = true;
+            lin->post_mult = pn.post_mult;
+            lin->post_eps = pn.eps;
+            lin->scale = pn.scale;   // 1 / row length, of both norms
+            if (low >= 0 && uses2[sum] > 0) add_out(*lin, sum, pn.out_specs[0]);
+            pn.dead = true;
             ++fused;
         }
         reindex();
@@ -1494,6 +1736,9 @@ int fuse_function(Function& fn) {
     f.pass_split_slices();
     f.pass_elementwise();
     f.dce();
+    f.pass_post_norm();
+    f.pass_softcap();
+    f.dce();
     f.pass_norm_cast();
     f.dce();
     f.pass_rope();
@@ -1505,6 +1750,7 @@ int fuse_function(Function& fn) {
     f.dce();
     f.pass_ssm();
     f.pass_latent();
+    f.pass_chunked();
     f.dce();
     f.pass_linear();
     f.dce();

@@ -78,8 +78,8 @@ void sample_temperature_last_row(hipStream_t s, int dtype, const void* logits, i
 // How a gate / up pair is combined (see glu_combine in device_utils.hpp)
 struct GluParams { int kind = 0; float limit = 0.f, alpha = 1.f, shift = 0.f; };
 // What the unquantised linear kernels apply besides bias, GELU and residual: factors per output column (f32, between bias and
-// residual) and the kind of pair
-struct EpiExtra { const float* colscale = nullptr; GluParams glu; };
+// residual), the kind of pair, and c * tanh(y / c) of the result (softcap c > 0; the weight-streaming kernels only)
+struct EpiExtra { const float* colscale = nullptr; GluParams glu; float softcap = 0.f; };
 
 // ---- fused kernels (kernels_fused.hip) --------------------------------------------------
 // y[r] = LN(x[r]) * gamma + beta over the last axis, two-pass (mean, then centred variance):
@@ -95,6 +95,10 @@ void rms_norm(hipStream_t s, int dtype, const void* x, const void* gamma, void* 
 // the same over f32 rows and gains with a bf16 result (the f32 value rounded once)
 void rms_norm_f32_to_bf16(hipStream_t s, const void* x, const void* gamma, void* y, int64_t rows, int64_t n, float inv_n,
                           float eps);
+// out = x + mult * (y * rsqrt(mean(y^2) + eps) * gain) over f32 rows; out16 (may be null): the same rounded to bf16
+void post_norm_add(hipStream_t s, const float* x, const float* y, const float* gain, float* out, void* out16, int64_t rows, int64_t n, float mult,
+                   float inv_n, float eps);
+void softcap(hipStream_t s, const float* x, float* y, int64_t n, float cap);
 void softmax_rows(hipStream_t s, int dtype, const void* x, void* y, int64_t rows, int64_t n);
 void gelu(hipStream_t s, int dtype, const void* x, void* y, int64_t n, float half, float inv_div, float one);
 void swiglu(hipStream_t s, int dtype, const void* gate, const void* up, void* y, int64_t n);  // up==nullptr: silu
@@ -194,7 +198,10 @@ constexpr size_t kChainBarrierBytes = (kChainCounters * 64 + 64) * sizeof(unsign
 // rounded to bf16 once as it is staged.
 // kChainLayerNorm (with kChainNorm, f32 phases or kChainXF32): LayerNorm with gains `gamma` and offsets `beta` instead of RMSNorm.
 enum : int { kChainNorm = 1, kChainDual = 2, kChainGelu = 4, kChainResidual = 8, kChainBias = 16, kChainOutF32 = 32, kChainXF32 = 64,
-             kChainLayerNorm = 128, kChainAttnFinal = 256, kChainColScale = 512, kChainClampedGlu = 1024 };
+             kChainLayerNorm = 128, kChainAttnFinal = 256, kChainColScale = 512, kChainClampedGlu = 1024, kChainPostNorm = 2048, kChainSoftcap = 4096 };
+// kChainPostNorm (bf16 weights, with kChainXF32): x is a sublayer's f32 output, the phase's input is r = post_res + post_mult *
+// rms_norm(x) * post_gain, left in post_y as well when that is given; with kChainNorm the RMS norm of r (gains `gamma`).
+// kChainSoftcap: y <- softcap * tanh(y / softcap), a layer without bias, residual and factors.
 // weight format of a linear phase; kChainW32: f32 weights (16-byte word = 4 columns x 1 k) with f32 activations,
 // bias, residual and output (the launch's attention phases then read f32 rows and caches as well)
 enum : int { kChainW16 = 0, kChainW8 = 1, kChainW4 = 2, kChainW32 = 3 };
@@ -215,14 +222,18 @@ struct ChainPhase {
     int wfmt, lds_total;   // lds_total: lds_bytes plus what the phase stages behind the activations
     const void* wscale; const void* wscale2;
     // attention: x = packed qkv row [(n_q + 2 n_kv) * head_dim], y = context row [n_q * head_dim]
-    void* k_cache; void* v_cache;              // [n_kv, capacity, head_dim], updated in place
+    union { void* k_cache; void* post_y; };    // [n_kv, capacity, head_dim], updated in place
+    void* v_cache;
     const int32_t* update_starts;              // si32[3]
     const int32_t* query_start;                // si32[1]
-    const void* cos; const void* sin;          // RoPE rows of this position, or null (qkv already rotated)
+    union { const void* cos; const void* post_gain; };   // RoPE rows of this position, or null (qkv already rotated)
+    union { const void* sin; const void* post_res; };    // (post_*: kChainPostNorm, linear phases)
     float* part;                               // [n_q][nch][head_dim + 2] f32
-    int n_q, n_kv, head_dim, capacity, rot_half, nch;
-    float scale;
-    float glu_limit;                           // kChainClampedGlu (with kChainDual): see glu_combine
+    int n_q, n_kv, head_dim;
+    union { int capacity; float post_eps; };
+    int rot_half, nch;
+    union { float scale; float post_mult; };
+    union { float glu_limit; float softcap; }; // kChainClampedGlu (with kChainDual): see glu_combine; kChainSoftcap
     const void* beta;                          // LayerNorm offsets (kChainLayerNorm)
     const void* colscale;                      // kChainColScale: f32 factor per output column, between bias and residual
     float glu_alpha, glu_shift;
@@ -446,6 +457,42 @@ struct LatentPrefillArgs {
 };
 size_t latent_prefill_scratch_bytes(int dtype, int64_t total, int64_t heads, int64_t dim, int64_t rot, int64_t vdim);
 int latent_prefill(hipStream_t s, const LatentPrefillArgs& a);
+
+// ---- chunked attention (kernels_chunked.hip) --------------------------------------------------------------------------
+// n heads of head_dim values, each divided by its root mean square
+void head_rms_norm(hipStream_t s, int in_dtype, int out_dtype, const void* x, void* y, int64_t n, int64_t head_dim, float eps);
+// y = x * sigmoid(gate): x T [rows, heads * vdim], gate f32 with one value per head, rows `ld` apart
+void head_gate(hipStream_t s, int dtype, const void* x, const float* gate, void* y, int64_t rows, int64_t heads, int64_t vdim, int64_t ld);
+// Grouped-query attention inside chunks with a sink per head: q T [t, heads * dim], keys and values of kv head g in row j at
+// k + g * k_head + j * k_row and v + g * v_head + j * v_row.  Without `position` query i (position i) sees the rows from its
+// chunk's first up to i; with it (t = 1) the rows 0 .. position % chunk of `rows` cached ones.  chunk 0: one chunk.
+struct ChunkAttnArgs {
+    int dtype;
+    const void* q; const void* k; const void* v; const float* sink; const int32_t* position;
+    void* ctx;                     // T [t, heads * vdim]
+    int64_t t, heads, kv_heads, dim, vdim, chunk, rows, k_row, k_head, v_row, v_head;
+    float scale;
+};
+void chunk_attn(hipStream_t s, const ChunkAttnArgs& a);
+// The whole mixer between its projections for up to kMixerBatch sequences (Mix::ChunkDecode, Mix::ChunkPrefill): proj f32
+// [total, ld] = q | k | v | gate per row, table f32 [total, rot] or null, ctx T [total, heads * vdim] gated.  Sequence b owns the
+// rows [row0[b], row0[b] + len[b]); its last keep[b] keys and values go to rows starts[3 b + 1] .. of its caches T [kv_heads,
+// rows, dim] and [kv_heads, rows, vdim].  Decode: one row each at position pos[b].  tickets: kSkinnyTickets zeroed counters.
+struct ChunkSeqArgs {
+    int dtype;
+    const float* proj; const float* table; const float* sink; const int32_t* pos; const int32_t* starts;
+    void* ctx;
+    int64_t total, ld, heads, kv_heads, dim, vdim, rot, rows, chunk;
+    float scale, eps;
+    int nseq;
+    int row0[kMixerBatch], len[kMixerBatch], keep[kMixerBatch];
+    void* kcache[kMixerBatch]; void* vcache[kMixerBatch];
+    void* scratch; unsigned* tickets;
+};
+size_t chunk_decode_scratch_bytes(int dtype, int64_t nseq, int64_t rows, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim);
+int chunk_decode(hipStream_t s, const ChunkSeqArgs& a);
+size_t chunk_prefill_scratch_bytes(int dtype, int64_t total, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim);
+int chunk_prefill(hipStream_t s, const ChunkSeqArgs& a);
 void clamped_glu(hipStream_t s, int dtype, const void* gate, const void* up, void* y, int64_t n, const GluParams& p);
 
 }  // namespace k

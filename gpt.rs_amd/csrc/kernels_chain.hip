@@ -160,20 +160,27 @@ struct PhaseRegs {
     float inv_n, eps, glu_limit, glu_alpha, glu_shift;   // (the last three: control wave only)
     const void *x, *gamma, *beta, *bias, *residual, *wscale, *wscale2, *colscale;
     void* y;
+    const void *post_gain, *post_res;   // (kChainPostNorm, bf16 weights only)
+    float post_mult, post_eps;
 };
-// (LN: phases of the launch's weight format may read LayerNorm offsets; a register pair that nobody reads is not kept)
-template <bool LN>
+// (LN: phases of the launch's weight format may read LayerNorm offsets, POST: they may have a residual prologue; a register pair
+// that nobody reads is not kept)
+template <bool LN, bool POST>
 __device__ __forceinline__ void regs_from_table(PhaseRegs& R, const GPTRS_CONST ChainPhase* D) {
     R.K = uni(D->K); R.N = uni(D->N); R.Kw = uni(D->Kw); R.ntiles = uni(D->ntiles); R.upb = uni(D->upb); R.units = uni(D->units);
     R.lds_bytes = uni(D->lds_bytes); R.flags = uni(D->flags); R.wfmt = uni(D->wfmt);
     R.inv_n = __int_as_float(uni(__float_as_int(D->inv_n))); R.eps = __int_as_float(uni(__float_as_int(D->eps)));
     R.x = uni_ptr(D->x); R.gamma = uni_ptr(D->gamma); R.beta = LN ? uni_ptr(D->beta) : nullptr; R.bias = uni_ptr(D->bias); R.residual = uni_ptr(D->residual);
     R.wscale = uni_ptr(D->wscale); R.wscale2 = uni_ptr(D->wscale2); R.y = uni_ptr(D->y);
+    if (POST) {
+        R.post_gain = uni_ptr(D->post_gain); R.post_res = uni_ptr(D->post_res);
+        R.post_mult = __int_as_float(uni(__float_as_int(D->post_mult))); R.post_eps = __int_as_float(uni(__float_as_int(D->post_eps)));
+    }
 }
 #define GPTRS_PD_INT(field) __builtin_amdgcn_readlane(pd, (int)(offsetof(ChainPhase, field) / 4))
 #define GPTRS_PD_PTR(field) ((const void*)(((unsigned long long)(unsigned)__builtin_amdgcn_readlane(pd, (int)(offsetof(ChainPhase, field) / 4) + 1) << 32) | \
                                           (unsigned)__builtin_amdgcn_readlane(pd, (int)(offsetof(ChainPhase, field) / 4))))
-template <bool LN>
+template <bool LN, bool POST>
 __device__ __forceinline__ void regs_from_lanes(PhaseRegs& R, int pd) {   // pd: dword `lane` of the descriptor
     R.K = GPTRS_PD_INT(K); R.N = GPTRS_PD_INT(N); R.Kw = GPTRS_PD_INT(Kw); R.ntiles = GPTRS_PD_INT(ntiles); R.upb = GPTRS_PD_INT(upb);
     R.units = GPTRS_PD_INT(units); R.lds_bytes = GPTRS_PD_INT(lds_bytes); R.flags = GPTRS_PD_INT(flags); R.wfmt = GPTRS_PD_INT(wfmt);
@@ -182,13 +189,18 @@ __device__ __forceinline__ void regs_from_lanes(PhaseRegs& R, int pd) {   // pd:
     R.wscale = GPTRS_PD_PTR(wscale); R.wscale2 = GPTRS_PD_PTR(wscale2); R.y = const_cast<void*>(GPTRS_PD_PTR(y));
     R.colscale = GPTRS_PD_PTR(colscale); R.glu_limit = __int_as_float(GPTRS_PD_INT(glu_limit));
     R.glu_alpha = __int_as_float(GPTRS_PD_INT(glu_alpha)); R.glu_shift = __int_as_float(GPTRS_PD_INT(glu_shift));
+    if (POST) {
+        R.post_gain = GPTRS_PD_PTR(post_gain); R.post_res = GPTRS_PD_PTR(post_res);
+        R.post_mult = __int_as_float(GPTRS_PD_INT(post_mult)); R.post_eps = __int_as_float(GPTRS_PD_INT(post_eps));
+    }
 }
 
 // ---------------------------------------------------------------------------- staging (all waves)
 // xs[j] = (x[2j], x[2j+1]) as a bf16 pair, zero beyond K; with norm: the value the stand-alone
 // RMSNorm kernels store, ((x * inv_rms) * gamma) -> bf16 (normalization.rs:183-217).
+// Returns 1 / rms of the sublayer's output where the phase has a residual prologue.
 template <int FMT>
-__device__ __forceinline__ void stage_block(const PhaseRegs& P, unsigned* xs, float* ssq) {
+__device__ __forceinline__ float stage_block(const PhaseRegs& P, unsigned* xs, float* ssq) {
     const int t = local_tid(), lane = t & 63, wave = uni(t >> 6);
     const int K = P.K;
     const int n = K / 4;                     // 8-byte items holding data (K % 4 == 0)
@@ -213,7 +225,72 @@ __device__ __forceinline__ void stage_block(const PhaseRegs& P, unsigned* xs, fl
             sv[u] = i < sc_n ? gload2(sc_src + i) : make_uint2(0u, 0u);
         }
     }
-    if (FMT == kChainW16 && (P.flags & (kChainNorm | kChainXF32 | kChainLayerNorm)) == (kChainNorm | kChainXF32 | kChainLayerNorm)) {
+    float post_inv = 0.f;
+    if (FMT == kChainW16 && (P.flags & kChainPostNorm)) {
+        // r = post_res + mult * rms_norm(x) * post_gain in f32, rounded to bf16 once; with kChainNorm the RMS norm of r instead
+        constexpr int MF = MAXI / 2;
+        f32x4 v[MF], rr[MF], gg[MF];
+#pragma unroll
+        for (int u = 0; u < MF; ++u) {
+            const int i = u * NT + t;
+            v[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+            rr[u] = v[u];
+            gg[u] = v[u];
+            if (u * NT < n && i < n) {
+                const unsigned long long a = cload8(x + 16 * (size_t)i), b = cload8(x + 16 * (size_t)i + 8);
+                const char* rp = (const char*)P.post_res + 16 * (size_t)i;
+                const unsigned long long c = cload8(rp), d = cload8(rp + 8);
+                v[u] = f32x4{__uint_as_float((unsigned)a), __uint_as_float((unsigned)(a >> 32)), __uint_as_float((unsigned)b), __uint_as_float((unsigned)(b >> 32))};
+                rr[u] = f32x4{__uint_as_float((unsigned)c), __uint_as_float((unsigned)(c >> 32)), __uint_as_float((unsigned)d), __uint_as_float((unsigned)(d >> 32))};
+                gg[u] = *(const GPTRS_GLOBAL f32x4*)((const char*)P.post_gain + 16 * (size_t)i);
+            }
+        }
+        float q = 0.f;
+#pragma unroll
+        for (int u = 0; u < MF; ++u)
+            if (u * NT < n) { q += v[u].x * v[u].x; q += v[u].y * v[u].y; q += v[u].z * v[u].z; q += v[u].w * v[u].w; }
+        const float ws = wave_sum(q);
+        if (lane == 0) ssq[wave] = ws;
+        wg_barrier();
+        float tot = 0.f;
+#pragma unroll
+        for (int w = 0; w < NT / 64; ++w) tot += ssq[w];
+        post_inv = 1.0f / sqrtf(tot * P.inv_n + P.post_eps);
+        const float mult = P.post_mult;
+#pragma unroll
+        for (int u = 0; u < MF; ++u) {   // (padding stays zero)
+            rr[u].x += ((v[u].x * post_inv) * gg[u].x) * mult; rr[u].y += ((v[u].y * post_inv) * gg[u].y) * mult;
+            rr[u].z += ((v[u].z * post_inv) * gg[u].z) * mult; rr[u].w += ((v[u].w * post_inv) * gg[u].w) * mult;
+        }
+        if (P.flags & kChainNorm) {
+            float q2 = 0.f;
+#pragma unroll
+            for (int u = 0; u < MF; ++u) {
+                const int i = u * NT + t;
+                if (u * NT < n) {
+                    q2 += rr[u].x * rr[u].x; q2 += rr[u].y * rr[u].y; q2 += rr[u].z * rr[u].z; q2 += rr[u].w * rr[u].w;
+                    if (i < n) gg[u] = *(const GPTRS_GLOBAL f32x4*)((const char*)P.gamma + 16 * (size_t)i);
+                }
+            }
+            const float w2 = wave_sum(q2);
+            if (lane == 0) ssq[16 + wave] = w2;
+            wg_barrier();
+            float tot2 = 0.f;
+#pragma unroll
+            for (int w = 0; w < NT / 64; ++w) tot2 += ssq[16 + w];
+            const float inv2 = 1.0f / sqrtf(tot2 * P.inv_n + P.eps);
+#pragma unroll
+            for (int u = 0; u < MF; ++u) {
+                rr[u].x = (rr[u].x * inv2) * gg[u].x; rr[u].y = (rr[u].y * inv2) * gg[u].y;
+                rr[u].z = (rr[u].z * inv2) * gg[u].z; rr[u].w = (rr[u].w * inv2) * gg[u].w;
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < MF; ++u) {
+            const int i = u * NT + t;
+            if (u * NT < npad && i < npad) *reinterpret_cast<uint2*>(&xs[2 * i]) = make_uint2(pack_hw(rr[u].x, rr[u].y), pack_hw(rr[u].z, rr[u].w));
+        }
+    } else if (FMT == kChainW16 && (P.flags & (kChainNorm | kChainXF32 | kChainLayerNorm)) == (kChainNorm | kChainXF32 | kChainLayerNorm)) {
         // LayerNorm of an f32 row (f32 gains and offsets), rounded to bf16 once: mean, then the variance of the centred row
         constexpr int MF = MAXI / 2;
         f32x4 v[MF], gg[MF];
@@ -384,6 +461,7 @@ __device__ __forceinline__ void stage_block(const PhaseRegs& P, unsigned* xs, fl
         }
     }
     wg_barrier();
+    return post_inv;
 }
 
 
@@ -1177,7 +1255,7 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
         } else if (u0 < u1) {
             if (lane == 0) lds_st(&sh.go, ph);
             PhaseRegs P;
-            regs_from_lanes<FMT == kChainW32 || FMT == kChainW16>(P, pd);
+            regs_from_lanes<FMT == kChainW32 || FMT == kChainW16, FMT == kChainW16>(P, pd);
             const int flags = P.flags, ntiles = P.ntiles, N = P.N;
             const bool dual = flags & kChainDual;
             const int cpt = dual ? 2 : 4;              // output columns per tile
@@ -1231,8 +1309,32 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
             const bool has_epi = bias || resid || sg || cscale;
             unsigned e_bw = 0u, e_rw = 0u, e_ga = 0u, e_gb = 0u;
             if (has_epi) epi_load(lane * 2, e_bw, e_rw, e_ga, e_gb);
+            // residual prologue: the workgroups of the phase leave the sum in memory, a share each.  What a lane's first element
+            // needs is requested ahead of the staging.
+            const bool post = wfmt == kChainW16 && (flags & kChainPostNorm);
+            float* post_y = post ? (float*)const_cast<void*>(GPTRS_PD_PTR(post_y)) : nullptr;
+            int post_i = 0, post_end = 0;
+            float post_v = 0.f, post_r = 0.f, post_g = 0.f;
+            auto post_load = [&](int i) {
+                post_v = __uint_as_float(cload4((const float*)P.x + i));
+                post_r = __uint_as_float(cload4((const float*)P.post_res + i));
+                post_g = gload((const float*)P.post_gain + i);
+            };
+            if (post_y) {
+                const int active = (units + upb - 1) / upb, share = (P.K + active - 1) / active;
+                post_i = blk * share + lane;
+                post_end = min(blk * share + share, P.K);
+                if (post_i < post_end) post_load(post_i);
+            }
+            float post_inv = 0.f;
             if (wfmt == kChainW32) stage_block_f32(P, xs, sh.ssq);
-            else stage_block<FMT>(P, xs, sh.ssq);
+            else post_inv = stage_block<FMT>(P, xs, sh.ssq);
+            if (post_y) {
+                for (int i = post_i; i < post_end; i += 64) {
+                    if (i != post_i) post_load(i);
+                    cstore4(post_y + i, __float_as_uint(post_r + ((post_v * post_inv) * post_g) * P.post_mult));
+                }
+            }
             if (has_epi) {
                 epi_store(lane * 2, e_bw, e_rw, e_ga, e_gb);
                 for (int i = lane * 2 + 128; i < ncols; i += 128) {
@@ -1304,6 +1406,10 @@ __device__ void control_wave(Shared& sh, unsigned* xs, const ChainPhase* phases,
                         float o[4];
 #pragma unroll
                         for (int c = 0; c < 4; ++c) o[c] = finish(s[c], flags, bi[c], re[c], sc[c]);
+                        if (wfmt == kChainW16 && (flags & kChainSoftcap)) {
+#pragma unroll
+                            for (int c = 0; c < 4; ++c) o[c] = softcap_f32(o[c], P.glu_limit);   // (softcap shares the field)
+                        }
                         if (tile * 4 + 4 > N) {   // the last tile of a width that is not a multiple of 4: its real columns one by one
 #pragma unroll
                             for (int c = 0; c < 4; ++c) {
@@ -1500,7 +1606,7 @@ __device__ void compute_waves(Shared& sh, const unsigned* xs, PhaseTable table, 
             c_Kv = (uni(D->K) + kpw - 1) / kpw;
             c_sidx = 0;   // int4: entry of the unit's first tile and group in the staged scales ...
             c_soff = uni(D->lds_bytes) >> 2;   // ... which sit behind the activations
-            regs_from_table<FMT == kChainW32 || FMT == kChainW16>(R, D);
+            regs_from_table<FMT == kChainW32 || FMT == kChainW16, FMT == kChainW16>(R, D);
             return true;   // (the caller waits for the phase to open and stages its input)
         }
     };

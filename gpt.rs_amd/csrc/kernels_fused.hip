@@ -203,6 +203,69 @@ __global__ void rms_norm_f32_bf16_kernel(const float* __restrict__ x, const floa
         for (int64_t i = threadIdx.x; i < n; i += blockDim.x) out[i] = f32_to_bf16((row[i] * inv_rms) * gamma[i]);
     }
 }
+// out = x + mult * (y * inv_rms(y) * gain), f32 rows; the sum in bf16 as well when out16 is given.  ONE: a thread holds all it
+// handles (n <= 8 per thread), so y is read once and x and the gains are requested ahead of the statistic.
+template <bool ONE>
+__global__ __launch_bounds__(1024) void post_norm_add_kernel(const float* __restrict__ x, const float* __restrict__ y, const float* __restrict__ gain,
+                                                             float* __restrict__ out, bf16_t* __restrict__ out16, int64_t n, float mult, float inv_n, float eps) {
+    __shared__ float red[16];
+    const int64_t base = (int64_t)blockIdx.x * n;
+    if (ONE) {
+        const int64_t i = (int64_t)threadIdx.x * 8;
+        float4 a[2], r[2], g[2];
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            a[e] = r[e] = g[e] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (i < n) {
+                a[e] = *reinterpret_cast<const float4*>(y + base + i + 4 * e);
+                r[e] = *reinterpret_cast<const float4*>(x + base + i + 4 * e);
+                g[e] = *reinterpret_cast<const float4*>(gain + i + 4 * e);
+            }
+        }
+        float q = 0.f;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) { q += a[e].x * a[e].x; q += a[e].y * a[e].y; q += a[e].z * a[e].z; q += a[e].w * a[e].w; }
+        const float inv = 1.0f / sqrtf(block_sum(q, red) * inv_n + eps);
+        if (i >= n) return;
+        fused_u32x4_t w;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            float4 o;
+            o.x = r[e].x + ((a[e].x * inv) * g[e].x) * mult;
+            o.y = r[e].y + ((a[e].y * inv) * g[e].y) * mult;
+            o.z = r[e].z + ((a[e].z * inv) * g[e].z) * mult;
+            o.w = r[e].w + ((a[e].w * inv) * g[e].w) * mult;
+            *reinterpret_cast<float4*>(out + base + i + 4 * e) = o;
+            w[2 * e] = pack_bf16x2(o.x, o.y);
+            w[2 * e + 1] = pack_bf16x2(o.z, o.w);
+        }
+        if (out16) *reinterpret_cast<fused_u32x4_t*>(out16 + base + i) = w;
+        return;
+    }
+    float q = 0.f;
+    for (int64_t i = threadIdx.x; i < n; i += blockDim.x) { const float v = y[base + i]; q += v * v; }
+    const float inv = 1.0f / sqrtf(block_sum(q, red) * inv_n + eps);
+    for (int64_t i = threadIdx.x; i < n; i += blockDim.x) {
+        const float o = x[base + i] + ((y[base + i] * inv) * gain[i]) * mult;
+        out[base + i] = o;
+        if (out16) out16[base + i] = f32_to_bf16(o);
+    }
+}
+void post_norm_add(hipStream_t s, const float* x, const float* y, const float* gain, float* out, void* out16, int64_t rows, int64_t n, float mult,
+                   float inv_n, float eps) {
+    if (rows <= 0 || n <= 0) return;
+    const bool one = n % 8 == 0 && n <= 8192 && ((((uintptr_t)x | (uintptr_t)y | (uintptr_t)gain | (uintptr_t)out | (uintptr_t)out16) & 15u) == 0);
+    const int threads = (int)std::min<int64_t>(one ? cdiv(n / 8, 64) * 64 : cdiv(n, 64) * 64, 1024);
+    if (one) post_norm_add_kernel<true><<<(unsigned)rows, threads, 0, s>>>(x, y, gain, out, (bf16_t*)out16, n, mult, inv_n, eps);
+    else post_norm_add_kernel<false><<<(unsigned)rows, threads, 0, s>>>(x, y, gain, out, (bf16_t*)out16, n, mult, inv_n, eps);
+}
+__global__ __launch_bounds__(256) void softcap_kernel(const float* x, float* y, int64_t n, float cap) {   // (y may be x)
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i < n) y[i] = softcap_f32(x[i], cap);
+}
+void softcap(hipStream_t s, const float* x, float* y, int64_t n, float cap) {
+    if (n > 0) softcap_kernel<<<(unsigned)cdiv(n, 256), 256, 0, s>>>(x, y, n, cap);
+}
 void rms_norm_f32_to_bf16(hipStream_t s, const void* x, const void* gamma, void* y, int64_t rows, int64_t n, float inv_n,
                           float eps) {
     if (rows <= 0 || n <= 0) return;

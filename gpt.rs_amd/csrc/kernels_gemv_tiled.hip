@@ -248,7 +248,8 @@ __global__ __launch_bounds__(256) void gemv_tiled_kernel(const T* __restrict__ x
         // out_f32: the f32 accumulator (plus an f32 residual) is stored as it is
         const float r = residual ? (out_f32 ? reinterpret_cast<const float*>(residual)[(int64_t)m * N + col]
                                             : ldf(residual, (int64_t)m * N + col)) : 0.f;
-        const float res = tiled_finish(tot, tot2, DUAL, act, b, residual != nullptr, r, extra.glu, cs);
+        float res = tiled_finish(tot, tot2, DUAL, act, b, residual != nullptr, r, extra.glu, cs);
+        if (extra.softcap != 0.f) res = softcap_f32(res, extra.softcap);
         if (out_f32) reinterpret_cast<float*>(y)[(int64_t)m * N + col] = res;
         else stf(y, (int64_t)m * N + col, res);
     }

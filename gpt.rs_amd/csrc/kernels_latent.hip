@@ -45,6 +45,21 @@ __global__ __launch_bounds__(256) void rope_pairs_kernel(const T* __restrict__ x
     Elem<T>::st(y, 2 * i + 1, v);
 }
 
+// The same one element per thread, for heads of an odd size
+template <typename T>
+__global__ __launch_bounds__(256) void rope_pairs_any_kernel(const T* __restrict__ x, const float* __restrict__ table, T* __restrict__ y, int64_t n,
+                                                             int64_t per_row, int64_t head_dim, int64_t offset, int64_t half) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    const int64_t r = i / per_row, d = i % per_row % head_dim - offset;
+    float v = Elem<T>::ld(x, i);
+    if (d >= 0 && d < 2 * half) {
+        const float c = table[r * 2 * half + d / 2], s = table[r * 2 * half + half + d / 2], w = Elem<T>::ld(x, d & 1 ? i - 1 : i + 1);
+        v = d & 1 ? v * c + w * s : v * c - w * s;
+    }
+    Elem<T>::st(y, i, v);
+}
+
 // Workgroup = row.  starts (one row): the row goes to place starts[1] of y, which holds `capacity` rows.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_rows_kernel(const float* __restrict__ raw, const float* __restrict__ gain, const float* __restrict__ table,
@@ -626,7 +641,13 @@ void rope_table(hipStream_t s, const int32_t* positions, const float* freqs, flo
 void rope_pairs(hipStream_t s, int dtype, const void* x, const float* table, void* y, int64_t rows, int64_t heads, int64_t head_dim, int64_t offset,
                 int64_t half) {
     const int64_t per_row = heads * head_dim, pairs = rows * per_row / 2;
-    if (pairs <= 0) return;
+    if (rows * per_row <= 0) return;
+    if (head_dim % 2 || offset % 2) {
+        const unsigned ge = (unsigned)cdiv_l(rows * per_row, 256);
+        if (dtype == 0) rope_pairs_any_kernel<float><<<ge, 256, 0, s>>>((const float*)x, table, (float*)y, rows * per_row, per_row, head_dim, offset, half);
+        else rope_pairs_any_kernel<bf16_t><<<ge, 256, 0, s>>>((const bf16_t*)x, table, (bf16_t*)y, rows * per_row, per_row, head_dim, offset, half);
+        return;
+    }
     const unsigned g = (unsigned)cdiv_l(pairs, 256);
     if (dtype == 0) rope_pairs_kernel<float><<<g, 256, 0, s>>>((const float*)x, table, (float*)y, pairs, per_row, head_dim, offset, half);
     else rope_pairs_kernel<bf16_t><<<g, 256, 0, s>>>((const bf16_t*)x, table, (bf16_t*)y, pairs, per_row, head_dim, offset, half);

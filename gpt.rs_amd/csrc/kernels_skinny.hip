@@ -186,7 +186,8 @@ __global__ __launch_bounds__(256) void skinny_gemm_kernel(const T* __restrict__ 
         // out_f32: the f32 accumulator (plus an f32 residual) is stored as it is
         const float r = residual ? (out_f32 ? reinterpret_cast<const float*>(residual)[(int64_t)m * N + n]
                                             : SkinnyT<T>::ld(residual, (int64_t)m * N + n)) : 0.f;
-        const float o = skinny_finish(g[i], up[i], DUAL, act, bv, residual != nullptr, r, extra.glu, cs);
+        float o = skinny_finish(g[i], up[i], DUAL, act, bv, residual != nullptr, r, extra.glu, cs);
+        if (extra.softcap != 0.f) o = softcap_f32(o, extra.softcap);
         if (out_f32) reinterpret_cast<float*>(y)[(int64_t)m * N + n] = o;
         else SkinnyT<T>::st(y, (int64_t)m * N + n, o);
     }

@@ -14,6 +14,12 @@
 //   ssm_state(xbc, p, dt_bias, a_log, state) {groups, dt_col}                           -> state's shape
 //   gated_rms_norm(y T[R, n], p[R, W], gain[n]) {groups, col, eps}                      -> T[R, n]
 //   clamped_glu(gate T, up T) {limit, alpha, shift}                                     -> T, gate's shape
+//   head_rms_norm(x T[R, heads * hd]) {heads, eps}                                      -> T' [R, heads * hd]
+//   head_gate(x T[R, heads * vd], gate[R, heads]) {heads}                               -> T, x's shape
+//   chunk_attention(q T[R, heads * D], k T[R, G * D], v T[R, G * V], sink[heads])
+//                    {heads, kv_heads = G, chunk, scale}                                -> T[R, heads * V]
+//   chunk_attention_cache(q T[1, heads * D], keys T[G, C, D], values T[G, C, V], sink[heads], position si32[1])
+//                    {heads, chunk, scale}                                              -> T[1, heads * V]
 //
 // latent_attention: query i stands at position start + i.  latent_attention_expanded: the queries are the last R of the L
 // positions.  p is the f32 result of an input projection whose columns hold several inputs of the mixer.
@@ -67,7 +73,8 @@ void lower_mixer_calls(Function& fn) {
         auto need = [&](bool ok, const char* what) { if (!ok) fail_spec(in.target + ": " + what); };
         static const std::map<Mix, size_t> kArity = {{Mix::RopeTable, 2}, {Mix::RopePairs, 2}, {Mix::LatentRows, 3}, {Mix::LatentAttn, 5},
                                                      {Mix::LatentAttnX, 4}, {Mix::ConvSilu, 4}, {Mix::ConvState, 2}, {Mix::SsmScan, 6},
-                                                     {Mix::SsmState, 5}, {Mix::GatedNorm, 3}, {Mix::Glu, 2}};
+                                                     {Mix::SsmState, 5}, {Mix::GatedNorm, 3}, {Mix::Glu, 2}, {Mix::HeadNorm, 1},
+                                                     {Mix::HeadGate, 2}, {Mix::ChunkAttn, 4}, {Mix::ChunkAttnCache, 5}};
         need(in.operands.size() == kArity.at(mix), "wrong number of operands");
         std::vector<const Spec*> s;
         for (const Operand& o : in.operands) {
@@ -94,7 +101,7 @@ void lower_mixer_calls(Function& fn) {
                 m.dim = s[0]->dims[1] / m.heads;
                 need(s[1]->rank() == 2 && f32(*s[1], {s[0]->dims[0], s[1]->dims[1]}) && s[1]->dims[1] % 2 == 0, "table must be f32[R, 2 half]");
                 m.rot = s[1]->dims[1];
-                need(m.dim % 2 == 0 && m.col % 2 == 0 && m.col >= 0 && m.col + m.rot <= m.dim, "the rotated part must lie in the head, at even places");
+                need(m.col >= 0 && m.col + m.rot <= m.dim, "the rotated part must lie in the head");
                 break;
             }
             case Mix::LatentRows:
@@ -186,6 +193,47 @@ void lower_mixer_calls(Function& fn) {
                 in.fparam[1] = attr_float(in, "alpha");
                 in.fparam[2] = attr_float(in, "shift");
                 break;
+            case Mix::HeadNorm:
+                m.heads = attr_int(in, "heads");
+                in.eps = attr_float(in, "eps");
+                need(rows2(*s[0]) && dtype_is_float(s[0]->dtype) && dtype_is_float(out.dtype) && out.dims == s[0]->dims, "x must be a float matrix, the output has its shape");
+                need(m.heads > 0 && s[0]->dims[1] % m.heads == 0, "row length must be heads * head_dim");
+                m.dim = s[0]->dims[1] / m.heads;
+                break;
+            case Mix::HeadGate:
+                m.heads = attr_int(in, "heads");
+                need(rows2(*s[0]) && dtype_is_float(s[0]->dtype) && out == *s[0], "x must be a float matrix, the output has its type");
+                need(m.heads > 0 && s[0]->dims[1] % m.heads == 0, "row length must be heads * vdim");
+                m.vdim = s[0]->dims[1] / m.heads;
+                need(f32(*s[1], {s[0]->dims[0], m.heads}), "gate must be f32[R, heads]");
+                break;
+            case Mix::ChunkAttn:
+            case Mix::ChunkAttnCache: {
+                const bool cached = mix == Mix::ChunkAttnCache;
+                m.heads = attr_int(in, "heads");
+                m.chunk = attr_int(in, "chunk");
+                in.scale = attr_float(in, "scale");
+                need(m.heads > 0 && m.chunk >= 0, "heads must be positive, chunk not negative");
+                const DType dt = s[0]->dtype;
+                need(dtype_is_float(dt) && rows2(*s[0]) && s[0]->dims[1] % m.heads == 0, "q must be a float matrix [R, heads * D]");
+                m.dim = s[0]->dims[1] / m.heads;
+                if (cached) {
+                    need(s[1]->rank() == 3 && s[2]->rank() == 3 && s[1]->dims[0] >= 1 && s[1]->dims[1] >= 1 && s[2]->dims[2] >= 1, "caches must be of rank 3");
+                    m.groups = s[1]->dims[0];
+                    m.vdim = s[2]->dims[2];
+                    need(is(*s[1], dt, {m.groups, s[1]->dims[1], m.dim}) && is(*s[2], dt, {m.groups, s[1]->dims[1], m.vdim}), "caches must be T[G, C, D] and T[G, C, V]");
+                    need(s[0]->dims[0] == 1 && is(*s[4], DType::SI32, {1}), "one query at position si32[1]");
+                } else {
+                    m.groups = attr_int(in, "kv_heads");
+                    need(m.groups > 0 && rows2(*s[1]) && rows2(*s[2]) && s[2]->dims[1] % m.groups == 0, "keys and values must be matrices of kv_heads parts");
+                    m.vdim = s[2]->dims[1] / m.groups;
+                    need(is(*s[1], dt, {s[0]->dims[0], m.groups * m.dim}) && is(*s[2], dt, {s[0]->dims[0], m.groups * m.vdim}), "k must be T[R, G * D], v T[R, G * V]");
+                }
+                need(m.heads % m.groups == 0, "heads must be a multiple of the key / value heads");
+                need(f32(*s[3], {m.heads}), "sink must be f32[heads]");
+                need(is(out, dt, {s[0]->dims[0], m.heads * m.vdim}), "output must be T[R, heads * V]");
+                break;
+            }
             default:
                 fail_spec(in.target + ": not a call target");
         }
@@ -195,6 +243,9 @@ void lower_mixer_calls(Function& fn) {
     }
 }
 
+// operands of Mix::ChunkDecode / ChunkPrefill: proj, sink, pos, starts, [table,] keys_0, values_0, keys_1, ..
+static size_t chunk_cache_operand(const Instr& in, int64_t b) { return (size_t)(4 + (in.mx.rot > 0 ? 1 : 0) + 2 * b); }
+
 size_t mixer_scratch_bytes(const Instr& in, const std::vector<const Spec*>& operands) {
     const Instr::MixAttrs& m = in.mx;
     const int dt = (int)in.out_specs[0].dtype;
@@ -203,6 +254,9 @@ size_t mixer_scratch_bytes(const Instr& in, const std::vector<const Spec*>& oper
     if (in.mix == Mix::LatentDecode)
         return k::latent_decode_scratch_bytes(dt, std::min<int64_t>(rows, k::kMixerBatch), operands[in.append ? 8 : 5]->dims[1], m.heads, m.dim, m.rot, m.rank, m.vdim);
     if (in.mix == Mix::LatentPrefill) return k::latent_prefill_scratch_bytes(dt, rows, m.heads, m.dim, m.rot, m.vdim);
+    if (in.mix == Mix::ChunkDecode)
+        return k::chunk_decode_scratch_bytes(dt, std::min<int64_t>(rows, k::kMixerBatch), operands[chunk_cache_operand(in, 0)]->dims[1], m.heads, m.groups, m.dim, m.vdim);
+    if (in.mix == Mix::ChunkPrefill) return k::chunk_prefill_scratch_bytes(dt, rows, m.heads, m.groups, m.dim, m.vdim);
     return 0;
 }
 
@@ -212,6 +266,8 @@ std::vector<std::pair<int, int>> mixer_inplace_pairs(const Instr& in) {
         for (int b = 0; b < (int)in.lens.size(); ++b) { out.push_back({7 + 2 * b, 1 + 2 * b}); out.push_back({8 + 2 * b, 2 + 2 * b}); }
     if (in.mix == Mix::LatentDecode && in.append)
         for (int b = 0; b < (int)in.lens.size(); ++b) out.push_back({8 + b, 1 + b});
+    if (in.mix == Mix::ChunkDecode || in.mix == Mix::ChunkPrefill)
+        for (int i = 0; i < 2 * (int)in.lens.size(); ++i) out.push_back({(int)chunk_cache_operand(in, 0) + i, 1 + i});
     return out;
 }
 
@@ -365,6 +421,76 @@ void run_mixer(const Plan& plan, const Step& st, ExecCtx& cx) {
             }
             break;
         }
+        case Mix::HeadNorm:
+            k::head_rms_norm(s, (int)spec(0).dtype, dt, ptr(0), dst, out.dims[0] * m.heads, m.dim, in.eps);
+            ++cx.launches;
+            break;
+        case Mix::HeadGate:
+            k::head_gate(s, dt, ptr(0), f(1), dst, out.dims[0], m.heads, m.vdim, m.heads);
+            ++cx.launches;
+            break;
+        case Mix::ChunkAttn:
+        case Mix::ChunkAttnCache: {
+            k::ChunkAttnArgs a{};
+            a.dtype = dt;
+            a.q = ptr(0); a.k = ptr(1); a.v = ptr(2); a.sink = f(3); a.ctx = dst;
+            a.t = out.dims[0]; a.heads = m.heads; a.kv_heads = m.groups; a.dim = m.dim; a.vdim = m.vdim; a.chunk = m.chunk; a.scale = in.scale;
+            if (in.mix == Mix::ChunkAttnCache) {
+                a.position = (const int32_t*)ptr(4);
+                a.rows = spec(1).dims[1];
+                a.k_row = m.dim; a.k_head = a.rows * m.dim; a.v_row = m.vdim; a.v_head = a.rows * m.vdim;
+            } else {
+                a.rows = a.t;
+                a.k_row = m.groups * m.dim; a.k_head = m.dim; a.v_row = m.groups * m.vdim; a.v_head = m.vdim;
+            }
+            k::chunk_attn(s, a);
+            ++cx.launches;
+            break;
+        }
+        case Mix::ChunkDecode:
+        case Mix::ChunkPrefill: {
+            int64_t row = 0;
+            for (size_t b0 = 0; b0 < in.lens.size(); b0 += k::kMixerBatch) {
+                k::ChunkSeqArgs a{};
+                a.dtype = dt;
+                a.proj = f(0); a.sink = f(1); a.pos = (const int32_t*)ptr(2) + b0; a.starts = (const int32_t*)ptr(3) + 3 * b0;
+                if (m.rot > 0) a.table = f(4);
+                a.ctx = dst;
+                a.total = out.dims[0]; a.ld = spec(0).dims[1];
+                a.heads = m.heads; a.kv_heads = m.groups; a.dim = m.dim; a.vdim = m.vdim; a.rot = m.rot; a.chunk = m.chunk; a.scale = in.scale; a.eps = in.eps;
+                a.rows = spec(chunk_cache_operand(in, 0)).dims[1];
+                a.nseq = (int)std::min<size_t>(in.lens.size() - b0, k::kMixerBatch);
+                for (int b = 0; b < a.nseq; ++b) {
+                    const size_t q = b0 + b;
+                    a.row0[b] = (int)row;
+                    a.len[b] = (int)in.lens[q];
+                    a.keep[b] = m.chunk > 0 ? (int)((in.lens[q] - 1) % m.chunk + 1) : (int)in.lens[q];
+                    row += in.lens[q];
+                    for (int kv = 0; kv < 2; ++kv) {
+                        const size_t ci = chunk_cache_operand(in, q) + kv;
+                        const void* from = ptr(ci);
+                        void* to = cx.ptr[st.dst[1 + 2 * q + kv]];
+                        if (to != from) {   // a cache that was not donated is copied first
+                            GPTRS_HIP_CHECK(hipMemcpyAsync(to, from, spec(ci).bytes(), hipMemcpyDeviceToDevice, s));
+                            ++cx.launches;
+                        }
+                        (kv ? a.vcache : a.kcache)[b] = to;
+                    }
+                }
+                a.scratch = cx.ws + st.scratch_off;
+                a.tickets = cx.be->skinny_tickets();
+                cx.launches += in.mix == Mix::ChunkDecode ? k::chunk_decode(s, a) : k::chunk_prefill(s, a);
+            }
+            break;
+        }
+        case Mix::PostNorm:
+            k::post_norm_add(s, f(0), f(1), f(2), (float*)dst, st.dst.size() > 1 ? cx.ptr[st.dst[1]] : nullptr, out.dims[0], out.dims[1], in.post_mult, in.scale, in.eps);
+            ++cx.launches;
+            break;
+        case Mix::Softcap:
+            k::softcap(s, f(0), (float*)dst, out.count(), in.softcap);
+            ++cx.launches;
+            break;
         default:
             fail_unimpl(in.op_name, "no kernel bound to this operation");
     }

@@ -572,6 +572,7 @@ void Builder::describe(Step& st) {
                 }
             }
             if (in.mfma) st.scratch_bytes = k::mfma_workspace_bytes((int)ldt, x.dims[0], x.dims[1], w.dims[1], in.act == 2, in.quant);
+            if (in.post) st.scratch_bytes = align_up((size_t)x.dims[1] * 4) + align_up((size_t)x.dims[1] * 2);   // outside a chain: the sum, and its bf16 copy
             if (in.tiled && x.dims[0] >= 2) {
                 // batched decode normalises into scratch first (the matrix-core kernel reads plain rows); layers with
                 // few column tiles add the partial sums of their K splits
@@ -802,7 +803,8 @@ void Builder::build() {
         const int wfmt = chain_format(in, ldt);
         if (in.norm_ln && wfmt != k::kChainW32 && !(wfmt == k::kChainW16 && in.x_f32)) return 0;   // LayerNorm is staged from f32 rows only
         if (wfmt == k::kChainW32 && (in.norm && !in.norm_ln)) return 0;   // ... and RMSNorm for the others
-        if (!k::chain_supported((int)ldt, x.dims[0], x.dims[1], w.dims[1], dual, in.norm, wfmt, in.x_f32, !in.has_bias && !in.has_residual && !in.has_scale)) return 0;
+        if (!k::chain_supported((int)ldt, x.dims[0], x.dims[1], w.dims[1], dual, in.norm || in.post, wfmt, in.x_f32, !in.has_bias && !in.has_residual && !in.has_scale)) return 0;
+        if (in.softcap != 0.f && (wfmt != k::kChainW16 || dual || in.has_bias || in.has_residual || in.has_scale)) return 0;
         k::ChainPhase p{};
         return k::chain_fill_phase(p, x.dims[1], w.dims[1], dual, wfmt) ? 1 : 0;
     };
@@ -949,6 +951,17 @@ static bool run_chain(const Plan& plan, const Step& head, ExecCtx& cx) {
         if (in.has_residual) { p.residual = src_ptr(st, cx, oi++); p.flags |= k::kChainResidual; }
         if (in.norm) { p.gamma = src_ptr(st, cx, oi++); p.inv_n = in.scale; p.eps = in.eps; p.flags |= k::kChainNorm; }
         if (in.norm && in.norm_ln) { p.beta = src_ptr(st, cx, oi++); p.flags |= k::kChainLayerNorm; }
+        if (in.post) {
+            p.flags |= k::kChainPostNorm;
+            p.post_gain = src_ptr(st, cx, oi++);
+            p.post_res = src_ptr(st, cx, oi++);
+            p.post_y = st.dst.size() > 1 ? cx.ptr[st.dst[1]] : nullptr;
+            p.post_mult = in.post_mult;
+            p.post_eps = in.post_eps;
+            p.inv_n = in.scale;
+            if (((uintptr_t)p.post_gain | (uintptr_t)p.post_res | (uintptr_t)p.post_y) & 15) fail_exec("decode chain: f32 rows and gains must be 16-byte aligned");
+        }
+        if (in.softcap != 0.f) { p.flags |= k::kChainSoftcap; p.softcap = in.softcap; }
         if (in.act == 1) p.flags |= k::kChainGelu;
         if (in.act == 2 && in.glu) { p.flags |= k::kChainClampedGlu; p.glu_limit = in.fparam[0]; p.glu_alpha = in.fparam[1]; p.glu_shift = in.fparam[2]; }
         if (in.out_f32 || wfmt == k::kChainW32) p.flags |= k::kChainOutF32;
@@ -1172,6 +1185,7 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                     GPTRS_HIP_CHECK(hipEventRecord(e0, s));
                 }
                 k::mfma_gemm(s, ma);
+                if (in.softcap != 0.f) { k::softcap(s, (const float*)dst, (float*)dst, out.count(), in.softcap); ++cx.launches; }
                 if (cx.profile) {
                     GPTRS_HIP_CHECK(hipEventRecord(e1, s));
                     cx.be->prof_events.emplace_back(e0, e1);
@@ -1205,6 +1219,7 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                 if (in.has_bias) sa.bias = src_ptr(st, cx, oi++);
                 if (in.has_scale) sa.extra.colscale = (const float*)src_ptr(st, cx, oi++);
                 sa.extra.glu = linear_glu(in);
+                sa.extra.softcap = in.softcap;
                 if (in.has_residual) sa.residual = src_ptr(st, cx, oi++);
                 const size_t norm_bytes = in.norm ? align_up((size_t)x.count() * dtype_size(x.dtype)) : 0;
                 if (in.norm) {
@@ -1261,9 +1276,19 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                 if (in.has_bias) ta.bias = src_ptr(st, cx, oi++);
                 if (in.has_scale) ta.extra.colscale = (const float*)src_ptr(st, cx, oi++);
                 ta.extra.glu = linear_glu(in);
+                ta.extra.softcap = in.softcap;
                 if (in.has_residual) ta.residual = src_ptr(st, cx, oi++);
                 if (in.norm) { ta.gamma = src_ptr(st, cx, oi++); ta.inv_n = in.scale; ta.eps = in.eps; }
                 if (in.norm_ln) ta.beta = src_ptr(st, cx, oi++);
+                if (in.post) {   // (one row) the residual update on its own; the layer then reads the bf16 copy, or norms the sum
+                    float* sum = st.dst.size() > 1 ? (float*)cx.ptr[st.dst[1]] : (float*)(cx.ws + st.scratch_off);
+                    void* low = cx.ws + st.scratch_off + align_up((size_t)ta.k * 4);
+                    k::post_norm_add(s, (const float*)src_ptr(st, cx, oi + 1), (const float*)ta.x, (const float*)src_ptr(st, cx, oi), sum, in.norm ? nullptr : low, 1, ta.k,
+                                     in.post_mult, in.scale, in.post_eps);
+                    ++cx.launches;
+                    ta.x = in.norm ? (const void*)sum : low;
+                    ta.x_f32 = in.norm;
+                }
                 ta.y = dst;
                 ta.act = in.act == 1 ? 1 : 0;
                 hipEvent_t e0 = nullptr, e1 = nullptr;
@@ -1283,7 +1308,7 @@ void run_step(const Plan& plan, const Step& st, ExecCtx& cx) {
                 break;
             }
             // (an absorbed column factor or clamped pair runs on the kernels above only: the fusion pass sees to it)
-            if (in.has_scale || in.glu) fail_exec("linear: column factors or a clamped pair on the generic kernel");
+            if (in.has_scale || in.glu || in.post || in.softcap != 0.f) fail_exec("linear: column factors, a clamped pair, a residual prologue or a soft cap on the generic kernel");
             k::LinearArgs a{};
             a.dtype = (int)ldt;
             a.x = src_ptr(st, cx, 0);

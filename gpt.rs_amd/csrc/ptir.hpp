@@ -75,11 +75,12 @@ enum class OpKind {
     FMixer,   // sequence-mixer targets (mixers.cpp): `Instr::mix` says which
     Unsupported
 };
-// What an FMixer instruction computes.  The first block are CustomCall targets (mixer_call_target); the last three are
-// formed by the fusion pass from those and serve every sequence of a batch.
+// What an FMixer instruction computes.  The first block are CustomCall targets (mixer_call_target); the last line is
+// formed by the fusion pass, from those (every sequence of a batch) or from the sequences of post_norm_add and softcap.
 enum class Mix {
     None, RopeTable, RopePairs, LatentRows, LatentAttn, LatentAttnX, ConvSilu, ConvState, SsmScan, SsmState, GatedNorm, Glu,
-    SsmSeq, LatentDecode, LatentPrefill
+    HeadNorm, HeadGate, ChunkAttn, ChunkAttnCache,
+    SsmSeq, LatentDecode, LatentPrefill, ChunkDecode, ChunkPrefill, PostNorm, Softcap
 };
 enum class UnaryOp { Neg, Abs, Exp, Log, Tanh, Erf, Rsqrt, Reciprocal };
 enum class BinaryOp { Add, Sub, Mul, Div, Maximum, Minimum };
@@ -145,10 +146,16 @@ struct Instr {
     int glu = 0;
     // FLinear: every output column is multiplied by an f32 factor (operand behind the bias, ahead of the residual)
     bool has_scale = false;
+    // FLinear (one row, bf16 weights): x is a sublayer's f32 output y, and the layer reads r + post_mult * rms_norm(y) * gain
+    // (last two operands: gain, r; inv_n = `scale`, post_eps), with `norm` the RMS norm of that; the sum is the second output
+    // when there is one
+    bool post = false;
+    float post_mult = 1.f, post_eps = 0.f;
+    float softcap = 0.f;                     // FLinear: softcap * tanh(y / softcap) of an f32 result (0: none)
     // FMixer: attributes of the call (only those of `mix` are meaningful)
     Mix mix = Mix::None;
     struct MixAttrs {
-        int64_t heads = 0, groups = 0, state = 0, vdim = 0, dim = 0, rot = 0, rank = 0, taps = 0, col = 0, dt_col = 0, z_col = 0;
+        int64_t heads = 0, groups = 0, state = 0, vdim = 0, dim = 0, rot = 0, rank = 0, taps = 0, col = 0, dt_col = 0, z_col = 0, chunk = 0;
     } mx;
     std::vector<int64_t> lens;               // FMixer over a batch: rows of each sequence, in order
     bool append = false;                     // Mix::LatentDecode: the step's cache rows are written by the call itself
@@ -186,7 +193,9 @@ inline Mix mixer_call_target(const std::string& t) {
         {"gpt_rs.hip.latent_attention_expanded.v1", Mix::LatentAttnX}, {"gpt_rs.hip.causal_conv_silu.v1", Mix::ConvSilu},
         {"gpt_rs.hip.causal_conv_state.v1", Mix::ConvState}, {"gpt_rs.hip.ssm_scan.v1", Mix::SsmScan},
         {"gpt_rs.hip.ssm_state.v1", Mix::SsmState}, {"gpt_rs.hip.gated_rms_norm.v1", Mix::GatedNorm},
-        {"gpt_rs.hip.clamped_glu.v1", Mix::Glu}};
+        {"gpt_rs.hip.clamped_glu.v1", Mix::Glu}, {"gpt_rs.hip.head_rms_norm.v1", Mix::HeadNorm},
+        {"gpt_rs.hip.head_gate.v1", Mix::HeadGate}, {"gpt_rs.hip.chunk_attention.v1", Mix::ChunkAttn},
+        {"gpt_rs.hip.chunk_attention_cache.v1", Mix::ChunkAttnCache}};
     for (auto& e : kTargets)
         if (t == e.first) return e.second;
     return Mix::None;
