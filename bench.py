@@ -508,7 +508,7 @@ DADUPEL_SIZES = {   # shapes that resemble a model's layers: width, ff, state-sp
     "3072": dict(width=3072, ff=9216, ssm=(96, 64, 128, 8), att=(32, 128, 64, 128, 1536, 512)),
     "4096": dict(width=4096, ff=12288, ssm=(128, 64, 128, 8), att=(32, 128, 64, 128, 1536, 512)),
 }
-DADUPEL_VOCAB = 32768
+DESIGN_VOCAB = 32768
 
 
 def dadupel_config(size: str, layers: int = 4):
@@ -525,7 +525,7 @@ def dadupel_config(size: str, layers: int = 4):
             mix = models.LatentMixerConfig(heads=heads, dim=dim, rot_dim=rot, vdim=vdim, q_rank=qr, kv_rank=kvr, scale=(dim + rot) ** -0.5, rope_base=1e4,
                                            rope_scaling=(4.0, 4096.0, 32.0, 1.0), kv_from=1 if i > 1 else None)
         out.append(models.DadupelLayer(mix, z["ff"], 7.0))
-    return models.DadupelConfig(vocab_size=DADUPEL_VOCAB, embed_dim=z["width"], eps=1e-5, layers=out)
+    return models.DadupelConfig(vocab_size=DESIGN_VOCAB, embed_dim=z["width"], eps=1e-5, layers=out)
 
 
 def _time_model(be, model, prompt_len: int, vocab: int, batch: int, steps: int, warmup: int, capacity: int):
@@ -564,57 +564,98 @@ def _time_model(be, model, prompt_len: int, vocab: int, batch: int, steps: int, 
     return t_prefill, one, many, launches
 
 
-def dadupel_record(args, be):
-    """Prefill and decode rates of the Dadupel design (random weights) beside a Ministral of equal width, feed-forward, depth
-    and vocabulary, both timed in turn in one process."""
+def dadupel_work(cfg, size: str, T: int, kv_len: int):
+    """(matrix elements, state and cache bytes a decode step of a sequence reads, flops of a prompt of T)"""
     from gptrs_amd import models
-    out, L, capacity = [], args.dadupel_layers, max(1280, args.prompt + 256)
+    z = DADUPEL_SIZES[size]
+    H, V, N, G = z["ssm"]
+    heads, dim, rot, vdim, qr, kvr = z["att"]
+    mats = sum(int(np.prod(s[0])) for n, s in models.Dadupel._param_plan(cfg).items() if len(s[0]) == 2 and not n.endswith(("conv", "tok_embeddings.weight")))
+    per_seq = sum(2 * 4 * H * N * V if isinstance(x.mixer, models.SsmMixerConfig) else 2 * (kvr + rot) * kv_len for x in cfg.layers)
+    # flops of a prompt: matrices over every row (the head once), causal attention over (dim + rot) and vdim, the chunked
+    # recurrence counted as N x V products in and out of the state
+    head = cfg.embed_dim * cfg.vocab_size
+    flops = 2.0 * T * (mats - head) + 2.0 * head + sum(
+        4.0 * T * H * N * V if isinstance(x.mixer, models.SsmMixerConfig) else 1.0 * heads * T * T * (dim + rot + vdim) for x in cfg.layers)
+    return mats, per_seq, flops
+
+
+FUZAZEN_SIZES = {   # width, ff, query heads (8 key / value heads, 128 values each)
+    "1536": dict(width=1536, ff=4608, heads=16),
+    "3072": dict(width=3072, ff=9216, heads=32),
+    "4096": dict(width=4096, ff=12288, heads=32),
+}
+
+
+def fuzazen_config(size: str, layers: int, chunk: int):
+    from gptrs_amd import models
+    z = FUZAZEN_SIZES[size]
+    mix = models.ChunkedMixerConfig(heads=z["heads"], kv_heads=8, dim=128, vdim=128, scale=0.1, rot_dims=128, rope_base=5e5, chunk=chunk)
+    return models.FuzazenConfig(vocab_size=DESIGN_VOCAB, embed_dim=z["width"], eps=1e-5, layers=[models.FuzazenLayer(mix, z["ff"]) for _ in range(layers)],
+                                embedding_scale=0.5, residual_mult=0.3, logit_softcap=30.0)
+
+
+def fuzazen_work(cfg, size: str, T: int, kv_len: int):
+    from gptrs_amd import models
+    mats = sum(int(np.prod(s[0])) for n, s in models.Fuzazen._param_plan(cfg).items() if len(s[0]) == 2 and not n.endswith("tok_embeddings.weight"))
+    head, per_seq, att = cfg.embed_dim * cfg.vocab_size, 0, 0.0
+    for x in cfg.layers:
+        m = x.mixer
+        per_seq += 2 * ((kv_len - 1) % m.chunk + 1) * (m.keys + m.values)
+        att += m.heads * (m.dim + m.vdim) * sum(min(m.chunk, T - c) ** 2 for c in range(0, T, m.chunk))
+    return mats, per_seq, 2.0 * T * (mats - head) + 2.0 * head + att
+
+
+def design_record(args, be):
+    """Prefill and decode rates of a design without a reference counterpart (--model dadupel | fuzazen; random weights) beside a
+    Ministral of equal width, feed-forward, depth and vocabulary, both timed in turn in one process."""
+    from gptrs_amd import models
+    name = args.model
+    out, capacity = [], max(1280, args.prompt + 256)
+    L, sizes = (args.dadupel_layers, args.dadupel_sizes) if name == "dadupel" else (args.fuzazen_layers, args.fuzazen_sizes)
     batch = args.batch if args.batch > 1 else 8
     steps, warmup = min(args.steps, 64), min(args.warmup, 8)
-    for size in args.dadupel_sizes.split(","):
-        cfg = dadupel_config(size, L)
-        z = DADUPEL_SIZES[size]
-        H, V, N, G = z["ssm"]
-        heads, dim, rot, vdim, qr, kvr = z["att"]
-        d, T = z["width"], args.prompt
-        model = models.Dadupel.random(cfg, be, seed=5)
-        pf, one, many, launches = _time_model(be, model, T, DADUPEL_VOCAB, batch, steps, warmup, capacity)
+    T, kv_len = args.prompt, args.prompt + warmup + steps // 2
+    for size in sizes.split(","):
+        if name == "dadupel":
+            cls, cfg, work = models.Dadupel, dadupel_config(size, L), dadupel_work
+            ff, heads = DADUPEL_SIZES[size]["ff"], DADUPEL_SIZES[size]["att"][0]
+        else:
+            cls, cfg, work = models.Fuzazen, fuzazen_config(size, L, args.fuzazen_chunk), fuzazen_work
+            ff, heads = FUZAZEN_SIZES[size]["ff"], FUZAZEN_SIZES[size]["heads"]
+        d = cfg.embed_dim
+        model = cls.random(cfg, be, seed=5)
+        pf, one, many, launches = _time_model(be, model, T, DESIGN_VOCAB, batch, steps, warmup, capacity)
         del model
         be.set_option("drop_derived_weights", 1)
-        mats = sum(int(np.prod(s[0])) for n, s in models.Dadupel._param_plan(cfg).items() if len(s[0]) == 2 and not n.endswith(("conv", "tok_embeddings.weight")))
-        kv_len = T + warmup + steps // 2
-        per_seq = sum(2 * 4 * H * N * V if isinstance(x.mixer, models.SsmMixerConfig) else 2 * (kvr + rot) * kv_len for x in cfg.layers)
-        # flops of a prompt: matrices over every row (the head once), causal attention over (dim + rot) and vdim, the chunked
-        # recurrence counted as N x V products in and out of the state
-        flops = 2.0 * T * (mats - d * DADUPEL_VOCAB) + 2.0 * d * DADUPEL_VOCAB + sum(
-            4.0 * T * H * N * V if isinstance(x.mixer, models.SsmMixerConfig) else 1.0 * heads * T * T * (dim + rot + vdim) for x in cfg.layers)
+        mats, per_seq, flops = work(cfg, size, T, kv_len)
         rec = {"width": d, "layers": L, "prompt": T, "prefill_ms": round(pf * 1e3, 3), "prefill_tokens_per_s": round(T / pf, 1),
                "prefill_mfma_frac": round(flops / pf / 1e12 / MFMA_PEAK_TFLOPS, 4),
                "decode_b1_ms": round(one * 1e3, 4), "decode_b1_tokens_per_s": round(1 / one, 1),
                "decode_b1_hbm_frac": round((2 * mats + per_seq) / one / 1e9 / HBM_PEAK_GBPS, 4),
                "decode_b%d_ms" % batch: round(many * 1e3, 4), "decode_b%d_tokens_per_s" % batch: round(batch / many, 1),
                "decode_b%d_hbm_frac" % batch: round((2 * mats + batch * per_seq) / many / 1e9 / HBM_PEAK_GBPS, 4), "launches_b1": launches}
-        mc = models.MinistralConfig(vocab_size=DADUPEL_VOCAB, embed_dim=d, num_layers=L, ffn_dim=z["ff"], num_heads=heads, num_kv_heads=8)
+        mc = models.MinistralConfig(vocab_size=DESIGN_VOCAB, embed_dim=d, num_layers=L, ffn_dim=ff, num_heads=heads, num_kv_heads=8)
         model = models.Ministral.random(mc, be, seed=5, residual_dtype="F32")
-        pf, one, many, launches = _time_model(be, model, T, DADUPEL_VOCAB, batch, steps, warmup, capacity)
+        pf, one, many, launches = _time_model(be, model, T, DESIGN_VOCAB, batch, steps, warmup, capacity)
         del model
         be.set_option("drop_derived_weights", 1)
         a = mc.attention_config()
         lin = d * a.total_projection_dim + a.query_projection_dim * d + 3 * d * mc.ffn_dim
         kv = L * 2 * 2 * a.key_value_projection_dim * kv_len
-        wb = 2 * (L * lin + d * DADUPEL_VOCAB)
-        flops = L * (2.0 * T * lin + 2.0 * mc.num_heads * T * T * mc.head_dim) + 2.0 * d * DADUPEL_VOCAB
+        wb = 2 * (L * lin + d * DESIGN_VOCAB)
+        flops = L * (2.0 * T * lin + 2.0 * mc.num_heads * T * T * mc.head_dim) + 2.0 * d * DESIGN_VOCAB
         rec["ministral"] = {"prefill_ms": round(pf * 1e3, 3), "prefill_mfma_frac": round(flops / pf / 1e12 / MFMA_PEAK_TFLOPS, 4),
                             "decode_b1_ms": round(one * 1e3, 4), "decode_b1_hbm_frac": round((wb + kv) / one / 1e9 / HBM_PEAK_GBPS, 4),
                             "decode_b%d_ms" % batch: round(many * 1e3, 4),
                             "decode_b%d_hbm_frac" % batch: round((wb + batch * kv) / many / 1e9 / HBM_PEAK_GBPS, 4), "launches_b1": launches}
         out.append(rec)
         print(json.dumps(rec), file=sys.stderr, flush=True)
-    first = out[0]
-    print(json.dumps({"metric": "decode tokens/s of the Dadupel design at the first size, batch 1 (side workload; every size under `sizes`)",
+    first, title = out[0], name.capitalize()
+    print(json.dumps({"metric": "decode tokens/s of the %s design at the first size, batch 1 (side workload; every size under `sizes`)" % title,
                       "value": first["decode_b1_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
                       "ms_per_step": first["decode_b1_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
-                      "data": "synthetic", "config": {"workload": "Dadupel, random weights, prompt %d, %d layers" % (args.prompt, L)}, "sizes": out}))
+                      "data": "synthetic", "config": {"workload": "%s, random weights, prompt %d, %d layers" % (title, args.prompt, L)}, "sizes": out}))
 
 
 def batched_decode(args, be, cfg, model, capacity):
@@ -696,11 +737,14 @@ def main():
     ap.add_argument("--batch", type=int, default=1,
                     help="B > 1: batched decode of B independent sequences (rows stacked through the linear layers, one attention "
                          "launch per layer for all of them); a side workload, NOT the headline metric (which is batch 1)")
-    ap.add_argument("--model", choices=["ministral", "gpt2", "dadupel"], default="ministral",
-                    help="dadupel: prefill and decode of the Dadupel design at a few sizes beside a Ministral of equal size; gpt2: the reference's own published workload (GPT-2 small f32, generate 64 tokens); --steps then counts "
+    ap.add_argument("--model", choices=["ministral", "gpt2", "dadupel", "fuzazen"], default="ministral",
+                    help="dadupel, fuzazen: prefill and decode of that design at a few sizes beside a Ministral of equal size; gpt2: the reference's own published workload (GPT-2 small f32, generate 64 tokens); --steps then counts "
                          "whole generate calls (default 8)")
     ap.add_argument("--dadupel-sizes", default=",".join(DADUPEL_SIZES), help="widths to run with --model dadupel, with commas between them")
     ap.add_argument("--dadupel-layers", type=int, default=4)
+    ap.add_argument("--fuzazen-sizes", default=",".join(FUZAZEN_SIZES), help="widths to run with --model fuzazen, with commas between them")
+    ap.add_argument("--fuzazen-layers", type=int, default=4)
+    ap.add_argument("--fuzazen-chunk", type=int, default=8192, help="positions of an attention chunk with --model fuzazen (the default prompt lies in one)")
     ap.add_argument("--microbench", action="store_true",
                     help="single-op programs of BASELINE configs[1] (dot_general / softmax / layer_norm, f32 and bf16) and the "
                          "Ministral prefill GEMM shapes; prints one JSON line with a result per shape")
@@ -758,8 +802,8 @@ def main():
         rec.update({"n_gpus": 1, "higher_is_better": True, "scaling": "weak", "roofline": None})
         print(json.dumps(rec))
         return
-    if args.model == "dadupel":
-        return dadupel_record(args, be)
+    if args.model in ("dadupel", "fuzazen"):
+        return design_record(args, be)
     cfg = models.MinistralConfig(num_layers=args.layers)
     f32_stream = args.residual == "f32"
     total_len = args.prompt + args.warmup + args.steps + 1

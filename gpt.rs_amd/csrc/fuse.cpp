@@ -360,6 +360,56 @@ struct Fuser {
         }
     }
 
+    // The f32 rows of an embedding, taken, widened and scaled, and the same rounded to bf16 -> Mix::EmbedRows (table, indices) ->
+    // (rows f32[, rows bf16]).  Only where it saves something besides the widening: a scale or the rounded copy.
+    void pass_embed() {
+        for (size_t i = 0; i < fn.body.size(); ++i) {
+            const Instr take = fn.body[i];
+            if (take.dead || take.op != OpKind::Take || take.out_specs[0].rank() != 2 || !dtype_is_float(take.out_specs[0].dtype)) continue;
+            const Spec* ts = spec_of(take.operands[0].value);
+            const Spec* is = spec_of(take.operands[1].value);
+            if (!ts || ts->rank() != 2 || !is || is->rank() != 1) continue;
+            const std::vector<int> uses = count_uses();
+            auto reader = [&](int v) -> int {   // the instruction that alone reads v
+                if (uses[v] != 1) return -1;
+                for (size_t j = 0; j < fn.body.size(); ++j)
+                    if (!fn.body[j].dead)
+                        for (const Operand& o : fn.body[j].operands)
+                            if (o.value == v) return (int)j;
+                return -1;
+            };
+            int root = take.out_ids[0];
+            if (take.out_specs[0].dtype == DType::BF16) {
+                const int c = reader(root);
+                if (c < 0 || fn.body[c].op != OpKind::Cast || fn.body[c].out_specs[0].dtype != DType::F32) continue;
+                root = fn.body[c].out_ids[0];
+            }
+            float scale = 1.0f;
+            bool scaled = false;
+            const int mi = reader(root);
+            int a, b;
+            if (mi >= 0 && binary(fn.body[mi].out_ids[0], BinaryOp::Mul, a, b) && a == root && scalar(b, scale)) {
+                root = fn.body[mi].out_ids[0];
+                scaled = true;
+            } else {
+                scale = 1.0f;
+            }
+            int low = -1;
+            for (size_t j = 0; j < fn.body.size() && low < 0; ++j)
+                if (!fn.body[j].dead && fn.body[j].op == OpKind::Cast && fn.body[j].operands[0].value == root && fn.body[j].out_specs[0].dtype == DType::BF16) low = (int)j;
+            if (!scaled && low < 0) continue;
+            Instr ni = make(OpKind::FMixer, "fused.embed_rows", {take.operands[0].value, take.operands[1].value}, root, *spec_of(root));
+            ni.mix = Mix::EmbedRows;
+            ni.scale = scale;
+            if (low >= 0) {
+                add_out(ni, fn.body[low].out_ids[0], fn.body[low].out_specs[0]);
+                fn.body[low].dead = true;
+            }
+            replace_root(root, ni);
+            reindex();
+        }
+    }
+
     // cap * tanh(x / cap) of f32 values -> Mix::Softcap
     void pass_softcap() {
         const std::vector<int> uses = count_uses();
@@ -1737,6 +1787,7 @@ int fuse_function(Function& fn) {
     f.pass_elementwise();
     f.dce();
     f.pass_post_norm();
+    f.pass_embed();
     f.pass_softcap();
     f.dce();
     f.pass_norm_cast();

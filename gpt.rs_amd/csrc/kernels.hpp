@@ -99,6 +99,9 @@ void rms_norm_f32_to_bf16(hipStream_t s, const void* x, const void* gamma, void*
 void post_norm_add(hipStream_t s, const float* x, const float* y, const float* gain, float* out, void* out16, int64_t rows, int64_t n, float mult,
                    float inv_n, float eps);
 void softcap(hipStream_t s, const float* x, float* y, int64_t n, float cap);
+// rows of `table` [vocab, n] by index, as f32 times scale; out16 (may be null): the same rounded to bf16.  Indices as in take().
+void embed_rows(hipStream_t s, int dtype, const void* table, const int32_t* idx, float* out, void* out16, int64_t n_idx, int64_t vocab, int64_t n,
+                float scale, int* err_flag);
 void softmax_rows(hipStream_t s, int dtype, const void* x, void* y, int64_t rows, int64_t n);
 void gelu(hipStream_t s, int dtype, const void* x, void* y, int64_t n, float half, float inv_div, float one);
 void swiglu(hipStream_t s, int dtype, const void* gate, const void* up, void* y, int64_t n);  // up==nullptr: silu

@@ -148,6 +148,69 @@ __global__ __launch_bounds__(256) void chunk_rows_kernel(ChunkSeqArgs a, int ski
     }
 }
 
+// The keys and values of whole prompts in bf16, sizes of up to 8 * 16 * U values and multiples of 8: 16 lanes to a head, 8 values
+// of it per lane and round, all of them requested before the first is used.
+template <int U>
+__global__ __launch_bounds__(256) void chunk_rows16_kernel(ChunkSeqArgs a, bf16_t* __restrict__ ko, bf16_t* __restrict__ vo) {
+    const int b = blockIdx.z, l16 = threadIdx.x & 15;
+    const int H = (int)a.heads, G = (int)a.kv_heads, D = (int)a.dim, V = (int)a.vdim, rot = (int)a.rot;
+    const int w = (int)blockIdx.x * 16 + (int)(threadIdx.x >> 4);
+    if (w >= a.len[b] * 2 * G) return;                                // (16 lanes at a time)
+    const int lr = w / (2 * G), u = w % (2 * G), g = u % G;
+    const bool key = u < G;
+    const int n = key ? D : V;
+    const int64_t row = a.row0[b] + lr;
+    const float* x = a.proj + row * a.ld + (int64_t)H * D + (key ? (int64_t)g * D : (int64_t)G * D + (int64_t)g * V);
+    const float* tab = a.table + row * rot;
+    f32x4_m v[U][2];
+    f32x4_m cs[U], sn[U];
+#pragma unroll
+    for (int i = 0; i < U; ++i) {
+        const int d = 8 * (l16 + 16 * i);
+        v[i][0] = v[i][1] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+        if (d < n) {
+            v[i][0] = *reinterpret_cast<const f32x4_u*>(x + d);
+            v[i][1] = *reinterpret_cast<const f32x4_u*>(x + d + 4);
+        }
+        cs[i] = f32x4_m{1.f, 1.f, 1.f, 1.f};
+        sn[i] = f32x4_m{0.f, 0.f, 0.f, 0.f};
+        if (key) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (d + 2 * e < rot) { cs[i][e] = tab[d / 2 + e]; sn[i][e] = tab[rot / 2 + d / 2 + e]; }
+        }
+    }
+    float f = 1.0f;
+    if (key) {
+        float q = 0.f;
+#pragma unroll
+        for (int i = 0; i < U; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float p = v[i][e >> 1][2 * (e & 1)], r = v[i][e >> 1][2 * (e & 1) + 1];
+                const float y = p * cs[i][e] - r * sn[i][e], z = r * cs[i][e] + p * sn[i][e];
+                v[i][e >> 1][2 * (e & 1)] = y;
+                v[i][e >> 1][2 * (e & 1) + 1] = z;
+                q += y * y + z * z;
+            }
+        f = 1.0f / sqrtf(row16_sum(q) / (float)D + a.eps);
+    }
+    const int cl = lr - (a.len[b] - a.keep[b]);
+    bf16_t* y = (key ? ko : vo) + (row * G + g) * n;
+    bf16_t* c = nullptr;
+    if (cl >= 0) c = (bf16_t*)(key ? a.kcache[b] : a.vcache[b]) + ((int64_t)g * a.rows + clamp_row(a.starts[3 * b + 1], (int)a.rows - a.keep[b]) + cl) * n;
+#pragma unroll
+    for (int i = 0; i < U; ++i) {
+        const int d = 8 * (l16 + 16 * i);
+        if (d >= n) break;
+        u32x4_m o;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = pack_bf16_hw(v[i][e >> 1][2 * (e & 1)] * f, v[i][e >> 1][2 * (e & 1) + 1] * f);
+        *reinterpret_cast<u32x4_m*>(y + d) = o;
+        if (c) *reinterpret_cast<u32x4_m*>(c + d) = o;
+    }
+}
+
 // ---------------------------------------------------------------------------- decode (bf16)
 constexpr int kDecTile = 32;     // cache rows per wave and step
 constexpr int kDecHeads = 16;    // query heads per workgroup (of one key / value head)
@@ -379,8 +442,8 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkSeqArgs a, float
 constexpr int kQTile = 128;      // queries per workgroup: 16 per wave
 constexpr int kKTile = 64;       // keys per step
 
-// Workgroup = 128 queries x head x sequence, 8 waves; keys from the first query's chunk on.  Keys and values of a step in LDS, the
-// next step's words in registers meanwhile.  Queries come from the projection, rotated and normed on the way in.  Everything is
+// Workgroup = 128 queries (16 per wave) x head x sequence; keys from the first query's chunk on.  Keys and values of a step in LDS,
+// the next step's words in registers meanwhile.  Queries come from the projection, rotated and normed on the way in.  Everything is
 // transposed (scores: rows = keys, columns = queries; result: rows = values), so a lane works on one query: softmax in f32
 // registers, started from the sink (maximum = sink, weight 1: always finite, also for a step of which a query sees nothing); the
 // weights go from there into the product with the values, as a bf16 value and its remainder.
@@ -667,9 +730,11 @@ int chunk_prefill(hipStream_t s, const ChunkSeqArgs& a) {
     char* k = (char*)a.scratch;
     char* v = k + chunk_align((size_t)(a.total * a.kv_heads * a.dim) * es);
     if (chunk_prefill_fast(a.dtype, a.total, a.kv_heads, a.dim, a.vdim)) {
-        chunk_rows(s, a, a.heads, nullptr, k, v);
         int64_t longest = 0;
         for (int b = 0; b < a.nseq; ++b) longest = std::max<int64_t>(longest, a.len[b]);
+        const dim3 rows((unsigned)cdiv_c(longest * 2 * a.kv_heads, 16), 1, (unsigned)a.nseq);
+        if (std::max(a.dim, a.vdim) <= 128) chunk_rows16_kernel<1><<<rows, 256, 0, s>>>(a, (bf16_t*)k, (bf16_t*)v);
+        else chunk_rows16_kernel<2><<<rows, 256, 0, s>>>(a, (bf16_t*)k, (bf16_t*)v);
         const int64_t ks = cdiv_c(a.dim, 32);
         if (ks <= 2) launch_prefill_v<2>(s, a, k, v, longest);
         else if (ks <= 4) launch_prefill_v<4>(s, a, k, v, longest);

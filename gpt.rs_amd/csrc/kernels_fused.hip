@@ -259,6 +259,44 @@ void post_norm_add(hipStream_t s, const float* x, const float* y, const float* g
     if (one) post_norm_add_kernel<true><<<(unsigned)rows, threads, 0, s>>>(x, y, gain, out, (bf16_t*)out16, n, mult, inv_n, eps);
     else post_norm_add_kernel<false><<<(unsigned)rows, threads, 0, s>>>(x, y, gain, out, (bf16_t*)out16, n, mult, inv_n, eps);
 }
+template <typename T>
+__global__ __launch_bounds__(256) void embed_rows_kernel(const T* __restrict__ table, const int32_t* __restrict__ idx, float* __restrict__ out,
+                                                         bf16_t* __restrict__ out16, int64_t vocab, int64_t n, float scale, int* err_flag) {
+    const int64_t r = blockIdx.x;
+    const int32_t id = idx[r];
+    const bool ok = id >= 0 && (int64_t)id < vocab;
+    if (!ok && threadIdx.x == 0) atomicExch(err_flag, 1);
+    const T* src = table + (int64_t)(ok ? id : 0) * n;
+    const float f = ok ? scale : 0.f;
+    if (sizeof(T) == 2 && n % 8 == 0) {   // (rows of a tensor: 16-byte aligned)
+        for (int64_t i = (int64_t)threadIdx.x * 8; i < n; i += 2048) {
+            const fused_u32x4_t w = *reinterpret_cast<const fused_u32x4_t*>(src + i);
+            fused_u32x4_t o;
+            float v[8];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                v[2 * e] = bf16lo(w[e]) * f;
+                v[2 * e + 1] = bf16hi(w[e]) * f;
+                o[e] = pack_bf16x2(v[2 * e], v[2 * e + 1]);
+            }
+            *reinterpret_cast<float4*>(out + r * n + i) = make_float4(v[0], v[1], v[2], v[3]);
+            *reinterpret_cast<float4*>(out + r * n + i + 4) = make_float4(v[4], v[5], v[6], v[7]);
+            if (out16) *reinterpret_cast<fused_u32x4_t*>(out16 + r * n + i) = o;
+        }
+        return;
+    }
+    for (int64_t i = threadIdx.x; i < n; i += 256) {
+        const float v = Elem<T>::ld(src, i) * f;
+        out[r * n + i] = v;
+        if (out16) out16[r * n + i] = f32_to_bf16(v);
+    }
+}
+void embed_rows(hipStream_t s, int dtype, const void* table, const int32_t* idx, float* out, void* out16, int64_t n_idx, int64_t vocab, int64_t n,
+                float scale, int* err_flag) {
+    if (n_idx <= 0 || n <= 0) return;
+    if (dtype == 0) embed_rows_kernel<float><<<(unsigned)n_idx, 256, 0, s>>>((const float*)table, idx, out, (bf16_t*)out16, vocab, n, scale, err_flag);
+    else embed_rows_kernel<bf16_t><<<(unsigned)n_idx, 256, 0, s>>>((const bf16_t*)table, idx, out, (bf16_t*)out16, vocab, n, scale, err_flag);
+}
 __global__ __launch_bounds__(256) void softcap_kernel(const float* x, float* y, int64_t n, float cap) {   // (y may be x)
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i < n) y[i] = softcap_f32(x[i], cap);

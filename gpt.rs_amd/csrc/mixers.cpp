@@ -487,6 +487,11 @@ void run_mixer(const Plan& plan, const Step& st, ExecCtx& cx) {
             k::post_norm_add(s, f(0), f(1), f(2), (float*)dst, st.dst.size() > 1 ? cx.ptr[st.dst[1]] : nullptr, out.dims[0], out.dims[1], in.post_mult, in.scale, in.eps);
             ++cx.launches;
             break;
+        case Mix::EmbedRows:
+            k::embed_rows(s, (int)spec(0).dtype, ptr(0), (const int32_t*)ptr(1), (float*)dst, st.dst.size() > 1 ? cx.ptr[st.dst[1]] : nullptr, out.dims[0],
+                          spec(0).dims[0], out.dims[1], in.scale, cx.err_flag);
+            ++cx.launches;
+            break;
         case Mix::Softcap:
             k::softcap(s, f(0), (float*)dst, out.count(), in.softcap);
             ++cx.launches;

@@ -76,11 +76,12 @@ enum class OpKind {
     Unsupported
 };
 // What an FMixer instruction computes.  The first block are CustomCall targets (mixer_call_target); the last line is
-// formed by the fusion pass, from those (every sequence of a batch) or from the sequences of post_norm_add and softcap.
+// formed by the fusion pass, from those (every sequence of a batch) or from the sequences of post_norm_add, softcap
+// and a scaled embedding.
 enum class Mix {
     None, RopeTable, RopePairs, LatentRows, LatentAttn, LatentAttnX, ConvSilu, ConvState, SsmScan, SsmState, GatedNorm, Glu,
     HeadNorm, HeadGate, ChunkAttn, ChunkAttnCache,
-    SsmSeq, LatentDecode, LatentPrefill, ChunkDecode, ChunkPrefill, PostNorm, Softcap
+    SsmSeq, LatentDecode, LatentPrefill, ChunkDecode, ChunkPrefill, PostNorm, Softcap, EmbedRows
 };
 enum class UnaryOp { Neg, Abs, Exp, Log, Tanh, Erf, Rsqrt, Reciprocal };
 enum class BinaryOp { Add, Sub, Mul, Div, Maximum, Minimum };

@@ -217,4 +217,4 @@ def test_a_layer_is_a_handful_of_fused_steps(tmp_path, lens, decode, dtype):
         assert sum("swiglu" in r for r in rep) == 3
         # one row: every residual update is some layer's prologue; more rows: an instruction that leaves the bf16 copy as well
         assert sum("+post_norm_add" in r for r in rep) == (6 if lens == (1,) else 0) and rep.count("fused.post_norm_add") == (0 if lens == (1,) else 6)
-        assert rep.count("Cast") == 2   # both of the embedding
+        assert rep.count("fused.embed_rows") == 1 and "Cast" not in rep

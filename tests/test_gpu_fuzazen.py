@@ -125,6 +125,21 @@ def test_post_norm_add(hip, rows, n, mult, fusion):
     assert np.array_equal(U.bf16(got[0]).reshape(rows, n), got[1])
 
 
+@pytest.mark.parametrize("fusion", [1, 0])
+@pytest.mark.parametrize("dt", ["F32", "Bf16"])
+@pytest.mark.parametrize("rows,n,scale", [(1, 64, 0.37), (7, 37, 0.37), (40, 3000, 5.0), (3, 64, 1.0)])
+def test_scaled_embedding(hip, dt, rows, n, scale, fusion):
+    idx = np.random.default_rng(0).integers(0, 19, rows).astype(np.int32)
+
+    def emit(fb, t, i):
+        x = F.embedding_lookup(t, i)
+        x = x if dt == "F32" else x.cast("F32")
+        x = x if scale == 1.0 else x * scale
+        return [x, x.cast("Bf16")]
+    got, want = both(hip, emit, [(rn(1, 19, n), dt), (idx, "Si32")], fusion=fusion)
+    assert np.array_equal(got[0], want[0]) and np.array_equal(got[1], want[1])
+
+
 @pytest.mark.parametrize("dt", ["F32", "Bf16"])
 @pytest.mark.parametrize("M", [1, 3, 16, 17, 130])
 @pytest.mark.parametrize("K,N", [(64, 96), (128, 37), (100, 50)])
@@ -242,6 +257,7 @@ def test_prompt_and_single_keys(hip, dt, shape, lens, chunk):
         r0 += n
     proj = projection(1, local, H, G, D, V, rot, 30.0, q, dirs)
     sink = rn(2, H)
+    sink[0] = 6.0   # as much as the keys that stand out
     starts = np.zeros(3 * len(lens), np.int32)
     args = [(proj, "F32"), (sink, "F32"), (local.astype(np.int32), "Si32"), (starts, "Si32"), (F.pair_frequencies(rot, 30.0) if rot else np.zeros(1, np.float32), "F32")]
     for b in range(len(lens)):
@@ -282,7 +298,9 @@ def test_decode_of_a_batch_and_single_rows(hip, dt, shape, pos, cap, chunk):
         vc[b][:, n + 1:] += 50.0
     proj = projection(1, np.array(pos), H, G, D, V, rot, 30.0, q, k)
     starts = np.array([v for n in place for v in (0, n, 0)], np.int32)
-    args = [(proj, "F32"), (rn(2, H), "F32"), (np.array(pos, np.int32), "Si32"), (starts, "Si32"), (F.pair_frequencies(rot, 30.0) if rot else np.zeros(1, np.float32), "F32")]
+    sink = rn(2, H)
+    sink[0] = 6.0   # as much as the row that stands out
+    args = [(proj, "F32"), (sink, "F32"), (np.array(pos, np.int32), "Si32"), (starts, "Si32"), (F.pair_frequencies(rot, 30.0) if rot else np.zeros(1, np.float32), "F32")]
     for b in range(B):
         args += [(kc[b], dt), (vc[b], dt)]
     if any(p % chunk >= cap for p in pos):
