@@ -592,7 +592,7 @@ def fuzazen_config(size: str, layers: int, chunk: int):
     z = FUZAZEN_SIZES[size]
     mix = models.ChunkedMixerConfig(heads=z["heads"], kv_heads=8, dim=128, vdim=128, scale=0.1, rot_dims=128, rope_base=5e5, chunk=chunk)
     return models.FuzazenConfig(vocab_size=DESIGN_VOCAB, embed_dim=z["width"], eps=1e-5, layers=[models.FuzazenLayer(mix, z["ff"]) for _ in range(layers)],
-                                embedding_scale=0.5, residual_mult=0.3, logit_softcap=30.0)
+                                embedding_scale=1.5, residual_mult=0.25, logit_softcap=20.0)
 
 
 def fuzazen_work(cfg, size: str, T: int, kv_len: int):

@@ -5,7 +5,7 @@ The directory name carries a dot, so Python cannot import it by name; load it wi
 
     ptir        PTIR program model + builder DSL + serde-JSON wire form
     functional  emitters for the LM functionals, op for op as the reference emits them
-    models      GPT-2 / Ministral / Dadupel drivers and the generators, generic over a backend
+    models      GPT-2 / Ministral / Dadupel / Fuzazen drivers and the generators, generic over a backend
     loader      checkpoints and model folders, weight streaming
     trace       replay of given token ids
     quant       weight-only int8 / int4-g128 packing

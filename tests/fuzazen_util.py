@@ -68,7 +68,7 @@ _wide = [layer(heads=40, kv_heads=2, dim=40, vdim=72, rot=24, chunk=50, scale=0.
 _shared = [layer(chunk=16, weights_of=2), layer(heads=2, chunk=9, base=50.0, ff=None), layer(chunk=16)]
 STACKS = {
     "mixed": config(_mixed + [same(_mixed, 1), same(_mixed, 0)]),
-    "tiled": config(_tiled + [same(_tiled, 0)], width=128, vocab=160, scale=1.0, mult=0.25, cap=30.0),
+    "tiled": config(_tiled + [same(_tiled, 0)], width=128, vocab=160, scale=1.0, mult=0.25, cap=25.0),
     "odd": config([layer(heads=3, kv_heads=1, dim=10, vdim=7, rot=4, chunk=5, ff=36), layer(heads=2, kv_heads=2, dim=7, vdim=5, rot=6, chunk=1, ff=None),
                    layer(heads=5, kv_heads=5, dim=9, vdim=11, rot=8, chunk=1000, ff=52)], width=36, vocab=50, eps=1e-3, mult=1.0, cap=5.0),
     "wide": config(_wide, width=96, vocab=101),

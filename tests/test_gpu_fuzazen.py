@@ -111,7 +111,7 @@ def test_attention_over_a_cached_chunk(hip, dt, pos, C, chunk):
 
 # ------------------------------------------------------------------------------------------ residual updates, soft cap
 @pytest.mark.parametrize("fusion", [1, 0])
-@pytest.mark.parametrize("mult", [0.3, 1.0])
+@pytest.mark.parametrize("mult", [0.35, 1.0])
 @pytest.mark.parametrize("rows,n", [(1, 64), (5, 100), (3, 37), (2, 8200), (130, 1024)])
 def test_post_norm_add(hip, rows, n, mult, fusion):
     y = rn(2, rows, n) * (10.0 ** np.arange(-3, 2))[np.arange(rows) % 5, None].astype(np.float32)
